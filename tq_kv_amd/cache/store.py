@@ -121,9 +121,8 @@ class KVGroup:
 
     def first_needed(self, length):
         """First position a query at or after `length` can still see."""
-        if self.need.window is None:
-            return 0
-        return max(0, length + 1 - self.need.window)
+        lo = 0 if self.need.window is None else max(0, length + 1 - self.need.window)
+        return max(lo, length - length % self.need.chunk) if self.need.chunk else lo
 
 
 class StateGroup:

@@ -1,13 +1,13 @@
 // Attention whose heads have values of another size than their keys, with what some designs put
 // around the softmax: a norm of every query and key head before the rotation, values mixed with
 // those of an earlier layer, a cap on the scores, a window that keeps a sequence's first
-// positions, and a sink in the softmax's denominator.  float32 arithmetic throughout, any sizes;
+// positions or chunks of positions that see nothing before them, and a sink in the softmax's denominator.  float32 arithmetic throughout, any sizes;
 // the kernels for the matrix cores are in attention_masked_mfma.hip.
 //
 //   q_h <- rot(q_h / rms(q_h) * w_q),  k_g <- rot(k_g / rms(k_g) * w_k)      (rms with eps inside the root)
 //   v_g <- (1 - lambda) v_g + lambda v'_g                                      (v' another layer's values of the token)
 //   s_ij = scale q_i . k_j;  s_ij <- cap tanh(s_ij / cap)
-//   i sees j  iff  j <= i and (window == 0 or i - j < window or j < keep_first)
+//   i sees j  iff  j <= i and (window == 0 or i - j < window or j < keep_first), and, with chunks, floor(j / chunk) = floor(i / chunk)
 //   p_ij = exp(s_ij) / (sum_j' exp(s_ij') + exp(sink_h))
 //
 // Cache pages: keys [kv head][position][key_dim], values [kv head][value_dim][place of the position]
@@ -20,15 +20,16 @@
 
 // ---- norm of heads, rotation, value mixing, cache write ---------------------------------------------
 // A wave per head of a token: heads 0..H-1 are queries, then G key heads, then G value heads; a row of qkv is
-// [H * dk | G * dk | G * dv].
+// [H * dk | G * dk | G * dv], or [H * dk | G * dk] where the values are the keys as the product gave them (values_are_keys).
+// Biases (with a row's layout) are added first; style 1 turns in halves, 2 in neighbouring pairs.
 template <typename TA, typename TW>
 __global__ __launch_bounds__(AM_WAVES * TQK_WAVE)
-void normed_rope_store_kernel(const TA* __restrict__ qkv, const TW* __restrict__ q_norm_w, const TW* __restrict__ k_norm_w, float eps,
-                              const float* __restrict__ cos_table, const float* __restrict__ sin_table, int rot_dim, int max_positions,
+void normed_rope_store_kernel(const TA* __restrict__ qkv, const TW* __restrict__ bias, const TW* __restrict__ q_norm_w, const TW* __restrict__ k_norm_w, float eps,
+                              const float* __restrict__ cos_table, const float* __restrict__ sin_table, int rot_dim, int style, int max_positions,
                               const TW* __restrict__ mix, const TA* __restrict__ mix_with, TA* __restrict__ mix_keep,
                               const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos,
                               const int32_t* __restrict__ page_table, int table_width, TA* __restrict__ keys, TA* __restrict__ values,
-                              TA* __restrict__ q_out, int n_heads, int n_kv_heads, int dk, int dv, int write_kv) {
+                              TA* __restrict__ q_out, int n_heads, int n_kv_heads, int dk, int dv, int write_kv, int values_are_keys) {
     const int t = blockIdx.x;
     const int head = blockIdx.y * AM_WAVES + threadIdx.x / TQK_WAVE;
     const int lane = threadIdx.x % TQK_WAVE;
@@ -36,7 +37,7 @@ void normed_rope_store_kernel(const TA* __restrict__ qkv, const TW* __restrict__
     const int pos = tok_pos[t];
     const int kind = head < n_heads ? 0 : (head < n_heads + n_kv_heads ? 1 : 2);
     if (kind != 0 && !write_kv) return;
-    const size_t total = (size_t)(n_heads + n_kv_heads) * dk + (size_t)n_kv_heads * dv;
+    const size_t total = (size_t)(n_heads + n_kv_heads) * dk + (values_are_keys ? 0 : (size_t)n_kv_heads * dv);
     const TA* row = qkv + (size_t)t * total;
     int page = -1;
     if (kind != 0) {
@@ -45,11 +46,12 @@ void normed_rope_store_kernel(const TA* __restrict__ qkv, const TW* __restrict__
     }
     if (kind == 2) {
         const int g = head - n_heads - n_kv_heads;
-        const TA* src = row + (size_t)(n_heads + n_kv_heads) * dk + (size_t)g * dv;
+        const size_t off = values_are_keys ? (size_t)(n_heads + g) * dk : (size_t)(n_heads + n_kv_heads) * dk + (size_t)g * dv;
+        const TA* src = row + off;
         TA* dst = values + ((size_t)page * n_kv_heads + g) * TQK_PAGE * dv + value_place(pos % TQK_PAGE);
         const float lam = mix && mix_with ? to_float(mix[0]) : 0.f;
         for (int i = lane; i < dv; i += TQK_WAVE) {
-            float v = to_float(src[i]);
+            float v = to_float(src[i]) + (bias ? to_float(bias[off + i]) : 0.f);
             const size_t at = ((size_t)t * n_kv_heads + g) * dv + i;
             if (mix_with) v = (1.f - lam) * v + lam * to_float(mix_with[at]);
             const TA stored = from_float<TA>(v);
@@ -59,11 +61,12 @@ void normed_rope_store_kernel(const TA* __restrict__ qkv, const TW* __restrict__
         return;
     }
     const TA* src = row + (size_t)head * dk;
+    const TW* hb = bias ? bias + (size_t)head * dk : nullptr;
     const TW* w = kind == 0 ? q_norm_w : k_norm_w;
     float inv = 1.f;
     if (w) {
         float ss = 0.f;
-        for (int i = lane; i < dk; i += TQK_WAVE) { const float v = to_float(src[i]); ss = fmaf(v, v, ss); }
+        for (int i = lane; i < dk; i += TQK_WAVE) { const float v = to_float(src[i]) + (hb ? to_float(hb[i]) : 0.f); ss = fmaf(v, v, ss); }
         inv = 1.f / sqrtf(wave_sum(ss) / (float)dk + eps);
     }
     TA* dst = kind == 0 ? q_out + ((size_t)t * n_heads + head) * dk
@@ -71,11 +74,11 @@ void normed_rope_store_kernel(const TA* __restrict__ qkv, const TW* __restrict__
     const int half = rot_dim / 2;
     const bool rotate = rot_dim > 0 && pos < max_positions;
     for (int i = lane; i < dk; i += TQK_WAVE) {
-        float x = to_float(src[i]) * inv * (w ? to_float(w[i]) : 1.f);
+        float x = (to_float(src[i]) + (hb ? to_float(hb[i]) : 0.f)) * inv * (w ? to_float(w[i]) : 1.f);
         if (rotate && i < rot_dim) {
-            const bool first = i < half;
-            const int p = first ? i : i - half, partner = first ? i + half : i - half;
-            const float y = to_float(src[partner]) * inv * (w ? to_float(w[partner]) : 1.f);
+            const bool first = style == 2 ? (i & 1) == 0 : i < half;
+            const int p = style == 2 ? i / 2 : (first ? i : i - half), partner = style == 2 ? (i ^ 1) : (first ? i + half : i - half);
+            const float y = (to_float(src[partner]) + (hb ? to_float(hb[partner]) : 0.f)) * inv * (w ? to_float(w[partner]) : 1.f);
             const float c = cos_table[(size_t)pos * half + p], s = sin_table[(size_t)pos * half + p];
             x = first ? x * c - y * s : x * c + y * s;
         }
@@ -260,27 +263,32 @@ void biased_values_store_vec_kernel(const bf16_t* __restrict__ qkv, const TB* __
 // head's pieces meet in LDS; the piece a rotated one turns with is read once more (it is in the caches).
 template <typename TW>
 __global__ __launch_bounds__(256)
-void normed_rope_qk_vec_kernel(const bf16_t* __restrict__ qkv, const TW* __restrict__ q_norm_w, const TW* __restrict__ k_norm_w, float eps,
-                               const float* __restrict__ cos_table, const float* __restrict__ sin_table, int rot_dim, int max_positions,
+void normed_rope_qk_vec_kernel(const bf16_t* __restrict__ qkv, const TW* __restrict__ bias, const TW* __restrict__ q_norm_w, const TW* __restrict__ k_norm_w, float eps,
+                               const float* __restrict__ cos_table, const float* __restrict__ sin_table, int rot_dim, int style, int max_positions,
                                const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ page_table,
                                int table_width, bf16_t* __restrict__ keys, bf16_t* __restrict__ q_out, int n_heads, int n_kv_heads, int dk, int dv,
-                               int write_kv) {
+                               int write_kv, int values_are_keys) {
     extern __shared__ float piece_ss[];
     const int t = blockIdx.x;
     const int per_head = dk / 8, n_pieces = (n_heads + (write_kv ? n_kv_heads : 0)) * per_head;
-    const size_t total = (size_t)(n_heads + n_kv_heads) * dk + (size_t)n_kv_heads * dv;
+    const size_t total = (size_t)(n_heads + n_kv_heads) * dk + (values_are_keys ? 0 : (size_t)n_kv_heads * dv);
     const bf16_t* row = qkv + (size_t)t * total;
-    auto load8 = [&](const bf16_t* p, float* v) {
-        const uint4 raw = *reinterpret_cast<const uint4*>(p);
+    // eight neighbouring elements of the row from `at`, biases added
+    auto load8 = [&](size_t at, float* v) {
+        const uint4 raw = *reinterpret_cast<const uint4*>(row + at);
         const uint32_t u[4] = {raw.x, raw.y, raw.z, raw.w};
 #pragma unroll
         for (int j = 0; j < 4; ++j) { v[2 * j] = __uint_as_float(u[j] << 16); v[2 * j + 1] = __uint_as_float(u[j] & 0xffff0000u); }
+        if (bias) {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) v[j] += to_float(bias[at + j]);
+        }
     };
     const bool normed = q_norm_w != nullptr;
     if (normed) {
         for (int c = threadIdx.x; c < n_pieces; c += blockDim.x) {
             float x[8], ss = 0.f;
-            load8(row + (size_t)c * 8, x);
+            load8((size_t)c * 8, x);
 #pragma unroll
             for (int j = 0; j < 8; ++j) ss = fmaf(x[j], x[j], ss);
             piece_ss[c] = ss;
@@ -304,14 +312,24 @@ void normed_rope_qk_vec_kernel(const bf16_t* __restrict__ qkv, const TW* __restr
             inv = 1.f / sqrtf(ss / (float)dk + eps);
         }
         float x[8];
-        load8(row + (size_t)c * 8, x);
+        load8((size_t)c * 8, x);
 #pragma unroll
         for (int j = 0; j < 8; ++j) x[j] *= inv * (normed ? to_float(w[off + j]) : 1.f);
-        if (rotate && off < rot_dim) {
+        if (rotate && style == 2) {
+            // (a piece holds whole pairs, and the rotated elements are an even number)
+#pragma unroll
+            for (int j = 0; j < 8; j += 2) {
+                if (off + j >= rot_dim) continue;
+                const float cs = cos_table[(size_t)pos * half + (off + j) / 2], sn = sin_table[(size_t)pos * half + (off + j) / 2];
+                const float u = x[j], v = x[j + 1];
+                x[j] = u * cs - v * sn;
+                x[j + 1] = v * cs + u * sn;
+            }
+        } else if (rotate && off < rot_dim) {
             const bool first = off < half;
             const int other = first ? off + half : off - half, p = first ? off : off - half;
             float y[8];
-            load8(row + (size_t)head * dk + other, y);
+            load8((size_t)head * dk + other, y);
             // (half and p are multiples of 8: the eight angles of a piece are two aligned loads of 16 bytes from each table)
             const float4* ct = reinterpret_cast<const float4*>(cos_table + (size_t)pos * half + p);
             const float4* st = reinterpret_cast<const float4*>(sin_table + (size_t)pos * half + p);
@@ -339,10 +357,10 @@ void normed_rope_qk_vec_kernel(const bf16_t* __restrict__ qkv, const TW* __restr
 // of 128 bytes.  Every lane finds its own page and place, so nothing depends on the tokens being neighbours.
 template <typename TW>
 __global__ __launch_bounds__(256)
-void mixed_values_store_vec_kernel(const bf16_t* __restrict__ qkv, const TW* __restrict__ mix, const bf16_t* __restrict__ mix_with,
+void mixed_values_store_vec_kernel(const bf16_t* __restrict__ qkv, const TW* __restrict__ bias, const TW* __restrict__ mix, const bf16_t* __restrict__ mix_with,
                                    bf16_t* __restrict__ mix_keep, const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos,
                                    const int32_t* __restrict__ page_table, int table_width, bf16_t* __restrict__ values, int n_tokens, int n_heads,
-                                   int n_kv_heads, int dk, int dv) {
+                                   int n_kv_heads, int dk, int dv, int values_are_keys) {
     const int lane = threadIdx.x % TQK_WAVE, wave = threadIdx.x / TQK_WAVE, n_waves = blockDim.x / TQK_WAVE;
     const int t = (blockIdx.x / n_kv_heads) * TQK_WAVE + lane, g = blockIdx.x % n_kv_heads;
     if (t >= n_tokens) return;
@@ -350,8 +368,9 @@ void mixed_values_store_vec_kernel(const bf16_t* __restrict__ qkv, const TW* __r
     const int page = page_table[(size_t)tok_seq[t] * table_width + pos / TQK_PAGE];
     if (page < 0) return;                               // the host never lets this happen
     bf16_t* dst = values + ((size_t)page * n_kv_heads + g) * TQK_PAGE * dv + value_place(pos % TQK_PAGE);
-    const size_t total = (size_t)(n_heads + n_kv_heads) * dk + (size_t)n_kv_heads * dv;
-    const bf16_t* src = qkv + (size_t)t * total + (size_t)(n_heads + n_kv_heads) * dk + (size_t)g * dv;
+    const size_t total = (size_t)(n_heads + n_kv_heads) * dk + (values_are_keys ? 0 : (size_t)n_kv_heads * dv);
+    const size_t off = values_are_keys ? (size_t)(n_heads + g) * dk : (size_t)(n_heads + n_kv_heads) * dk + (size_t)g * dv;
+    const bf16_t* src = qkv + (size_t)t * total + off;
     const float lam = mix && mix_with ? to_float(mix[0]) : 0.f;
     for (int c = wave * 8; c < dv; c += n_waves * 8) {
         const uint4 raw = *reinterpret_cast<const uint4*>(src + c);
@@ -359,6 +378,10 @@ void mixed_values_store_vec_kernel(const bf16_t* __restrict__ qkv, const TW* __r
         float v[8];
 #pragma unroll
         for (int j = 0; j < 4; ++j) { v[2 * j] = __uint_as_float(u[j] << 16); v[2 * j + 1] = __uint_as_float(u[j] & 0xffff0000u); }
+        if (bias) {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) v[j] += to_float(bias[off + c + j]);
+        }
         const size_t at = ((size_t)t * n_kv_heads + g) * dv + c;
         if (mix_with) {
             const uint4 mr = *reinterpret_cast<const uint4*>(mix_with + at);
@@ -394,7 +417,7 @@ template <typename T, typename TS>
 __global__ __launch_bounds__(AM_WAVES * TQK_WAVE)
 void attention_masked_kernel(const T* __restrict__ q, const T* __restrict__ keys, const T* __restrict__ values,
                              const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos,
-                             const int32_t* __restrict__ page_table, int table_width, int window, int keep_first, float scale, float cap,
+                             const int32_t* __restrict__ page_table, int table_width, int window, int chunk, int keep_first, float scale, float cap,
                              const TS* __restrict__ sink, T* __restrict__ out, int n_tokens, int n_heads, int n_kv_heads, int dk, int dv) {
     __shared__ float q_lds[AM_WAVES][AM_MAX_D];
     const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
@@ -411,7 +434,7 @@ void attention_masked_kernel(const T* __restrict__ q, const T* __restrict__ keys
     const int pos = tok_pos[t];
     const int32_t* pages = page_table + (size_t)tok_seq[t] * table_width;
     const int kvh = head / (n_heads / n_kv_heads);
-    const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+    const int lo = first_seen(pos, window, chunk);
     const int kept = window > 0 ? keep_first : 0;
     const float* qf = q_lds[wave];
 
@@ -464,40 +487,42 @@ void attention_masked_kernel(const T* __restrict__ q, const T* __restrict__ keys
     }
 }
 
-extern "C" int tqk_normed_rope_store(const void* qkv, int act_dtype, const void* q_norm_w, const void* k_norm_w, int w_dtype, float eps,
-                                     const float* cos_table, const float* sin_table, int rot_dim, int max_positions, const void* mix,
+extern "C" int tqk_normed_rope_store(const void* qkv, int act_dtype, const void* bias, const void* q_norm_w, const void* k_norm_w, int w_dtype, float eps,
+                                     const float* cos_table, const float* sin_table, int rot_dim, int style, int max_positions, const void* mix,
                                      const void* mix_with, void* mix_keep, const int32_t* tok_seq, const int32_t* tok_pos,
                                      const int32_t* page_table, int table_width, void* keys, void* values, void* q_out, int n_tokens,
-                                     int n_heads, int n_kv_heads, int key_dim, int value_dim, int write_kv, void* stream) {
+                                     int n_heads, int n_kv_heads, int key_dim, int value_dim, int write_kv, int values_are_keys, void* stream) {
     TQK_REQUIRE(qkv && tok_pos && q_out, "tqk_normed_rope_store: null pointer");
     TQK_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv_heads > 0 && key_dim > 0 && value_dim > 0, "tqk_normed_rope_store: bad sizes");
     TQK_REQUIRE(rot_dim >= 0 && rot_dim % 2 == 0 && rot_dim <= key_dim, "tqk_normed_rope_store: rot_dim %d must be even and <= key_dim %d", rot_dim, key_dim);
     TQK_REQUIRE(rot_dim == 0 || (cos_table && sin_table && max_positions > 0), "tqk_normed_rope_store: rotation without tables");
     TQK_REQUIRE(!write_kv || (tok_seq && page_table && keys && values && table_width > 0), "tqk_normed_rope_store: no cache to write to");
+    TQK_REQUIRE(rot_dim == 0 || style == 1 || style == 2, "tqk_normed_rope_store: unknown rotation style %d", style);
+    TQK_REQUIRE(!values_are_keys || key_dim == value_dim, "tqk_normed_rope_store: keys of %d elements serve as values of %d", key_dim, value_dim);
     TQK_REQUIRE(!mix_with || mix, "tqk_normed_rope_store: values to mix with, but no weight");
     if (n_tokens == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
     // steps of many tokens in bfloat16 whose sizes fall into pieces of 16 bytes: the two launches above
     const long long pieces = (long long)(n_heads + n_kv_heads) * key_dim / 8;
-    if (act_dtype == TQK_BF16 && n_tokens > 64 && key_dim % 8 == 0 && value_dim % 8 == 0 && rot_dim % 16 == 0 && pieces <= 8192 &&
+    if (act_dtype == TQK_BF16 && n_tokens > 64 && key_dim % 8 == 0 && value_dim % 8 == 0 && (style == 2 || rot_dim % 16 == 0) && pieces <= 8192 &&
         (!q_norm_w) == (!k_norm_w)) {
         const size_t lds = (size_t)pieces * sizeof(float);
         const long long v_blocks = (long long)((n_tokens + TQK_WAVE - 1) / TQK_WAVE) * n_kv_heads;
         TQK_REQUIRE(v_blocks <= 0x7fffffff, "tqk_normed_rope_store: too many tokens");
 #define TQK_NRV(TW) \
-        normed_rope_qk_vec_kernel<TW><<<n_tokens, 256, lds, s>>>((const bf16_t*)qkv, (const TW*)q_norm_w, (const TW*)k_norm_w, eps, cos_table, sin_table, rot_dim, \
-            max_positions, tok_seq, tok_pos, page_table, table_width, (bf16_t*)keys, (bf16_t*)q_out, n_heads, n_kv_heads, key_dim, value_dim, write_kv); \
-        if (write_kv) mixed_values_store_vec_kernel<TW><<<(unsigned)v_blocks, 256, 0, s>>>((const bf16_t*)qkv, (const TW*)mix, (const bf16_t*)mix_with, \
-            (bf16_t*)mix_keep, tok_seq, tok_pos, page_table, table_width, (bf16_t*)values, n_tokens, n_heads, n_kv_heads, key_dim, value_dim)
+        normed_rope_qk_vec_kernel<TW><<<n_tokens, 256, lds, s>>>((const bf16_t*)qkv, (const TW*)bias, (const TW*)q_norm_w, (const TW*)k_norm_w, eps, cos_table, sin_table, rot_dim, style, \
+            max_positions, tok_seq, tok_pos, page_table, table_width, (bf16_t*)keys, (bf16_t*)q_out, n_heads, n_kv_heads, key_dim, value_dim, write_kv, values_are_keys); \
+        if (write_kv) mixed_values_store_vec_kernel<TW><<<(unsigned)v_blocks, 256, 0, s>>>((const bf16_t*)qkv, (const TW*)bias, (const TW*)mix, (const bf16_t*)mix_with, \
+            (bf16_t*)mix_keep, tok_seq, tok_pos, page_table, table_width, (bf16_t*)values, n_tokens, n_heads, n_kv_heads, key_dim, value_dim, values_are_keys)
         if (w_dtype == TQK_F32) { TQK_NRV(float); } else if (w_dtype == TQK_BF16) { TQK_NRV(bf16_t); } else return tqk_fail("tqk_normed_rope_store: unknown dtype %d", w_dtype);
 #undef TQK_NRV
         return tqk_check_launch("tqk_normed_rope_store");
     }
     dim3 grid(n_tokens, (n_heads + 2 * n_kv_heads + AM_WAVES - 1) / AM_WAVES);
 #define TQK_NRS(TA, TW) \
-    normed_rope_store_kernel<TA, TW><<<grid, AM_WAVES * TQK_WAVE, 0, s>>>((const TA*)qkv, (const TW*)q_norm_w, (const TW*)k_norm_w, eps, cos_table, sin_table, \
-        rot_dim, max_positions, (const TW*)mix, (const TA*)mix_with, (TA*)mix_keep, tok_seq, tok_pos, page_table, table_width, (TA*)keys, (TA*)values, \
-        (TA*)q_out, n_heads, n_kv_heads, key_dim, value_dim, write_kv)
+    normed_rope_store_kernel<TA, TW><<<grid, AM_WAVES * TQK_WAVE, 0, s>>>((const TA*)qkv, (const TW*)bias, (const TW*)q_norm_w, (const TW*)k_norm_w, eps, cos_table, sin_table, \
+        rot_dim, style, max_positions, (const TW*)mix, (const TA*)mix_with, (TA*)mix_keep, tok_seq, tok_pos, page_table, table_width, (TA*)keys, (TA*)values, \
+        (TA*)q_out, n_heads, n_kv_heads, key_dim, value_dim, write_kv, values_are_keys)
     if (act_dtype == TQK_F32 && w_dtype == TQK_F32) TQK_NRS(float, float);
     else if (act_dtype == TQK_F32 && w_dtype == TQK_BF16) TQK_NRS(float, bf16_t);
     else if (act_dtype == TQK_BF16 && w_dtype == TQK_F32) TQK_NRS(bf16_t, float);
@@ -553,7 +578,7 @@ extern "C" int tqk_attention_masked_max_dim(void) { return AM_MAX_D; }
 
 extern "C" int tqk_attention_masked(const void* q, const void* keys, const void* values, int act_dtype, const int32_t* tok_seq,
                                     const int32_t* tok_pos, const int32_t* page_table, int table_width, int n_seqs, int n_pages, int window,
-                                    int keep_first, float scale, float cap, const void* sink, int sink_dtype, void* out, int n_tokens,
+                                    int chunk, int keep_first, float scale, float cap, const void* sink, int sink_dtype, void* out, int n_tokens,
                                     int n_heads, int n_kv_heads, int key_dim, int value_dim, void* stream) {
     TQK_REQUIRE(q && keys && values && tok_seq && tok_pos && page_table && out, "tqk_attention_masked: null pointer");
     TQK_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv_heads > 0 && key_dim > 0 && value_dim > 0, "tqk_attention_masked: bad sizes");
@@ -561,13 +586,13 @@ extern "C" int tqk_attention_masked(const void* q, const void* keys, const void*
     TQK_REQUIRE(key_dim <= AM_MAX_D && value_dim <= AM_MAX_D, "tqk_attention_masked: head sizes %d and %d, the kernel takes up to %d", key_dim, value_dim, AM_MAX_D);
     TQK_REQUIRE(n_heads <= 65535, "tqk_attention_masked: too many heads for the grid");
     TQK_REQUIRE(table_width > 0 && n_pages > 0 && n_seqs > 0, "tqk_attention_masked: empty page table");
-    TQK_REQUIRE(window >= 0 && keep_first >= 0 && cap >= 0.f, "tqk_attention_masked: negative window, kept positions or cap");
+    TQK_REQUIRE(window >= 0 && chunk >= 0 && keep_first >= 0 && cap >= 0.f, "tqk_attention_masked: negative window, chunk, kept positions or cap");
     if (n_tokens == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
     dim3 grid((n_tokens + AM_WAVES - 1) / AM_WAVES, n_heads);
 #define TQK_AM(T, TS) \
     attention_masked_kernel<T, TS><<<grid, AM_WAVES * TQK_WAVE, 0, s>>>((const T*)q, (const T*)keys, (const T*)values, tok_seq, tok_pos, page_table, \
-        table_width, window, keep_first, scale, cap, (const TS*)sink, (T*)out, n_tokens, n_heads, n_kv_heads, key_dim, value_dim)
+        table_width, window, chunk, keep_first, scale, cap, (const TS*)sink, (T*)out, n_tokens, n_heads, n_kv_heads, key_dim, value_dim)
     if (act_dtype == TQK_F32 && (!sink || sink_dtype == TQK_F32)) TQK_AM(float, float);
     else if (act_dtype == TQK_F32 && sink_dtype == TQK_BF16) TQK_AM(float, bf16_t);
     else if (act_dtype == TQK_BF16 && (!sink || sink_dtype == TQK_BF16)) TQK_AM(bf16_t, bf16_t);

@@ -1,6 +1,6 @@
 // The attention of attention_masked.hip on the matrix cores (bfloat16 in, float32 softmax): keys of key_dim and
-// values of value_dim per head, a cap on the scores, a window that keeps a sequence's first positions, a sink in
-// the softmax's denominator.  One body serves two kinds of step.
+// values of value_dim per head, a cap on the scores, a window that keeps a sequence's first positions, chunks of positions
+// that see nothing before them, a sink in the softmax's denominator.  One body serves two kinds of step.
 //
 // A wave computes 16 columns against a page of 64 keys at a time (v_mfma_f32_16x16x32_bf16, the mapping of
 // attention_decode.hip: scores^T[key][column] = K . Q^T, out^T[element][column] = V^T . P^T with P staying in the
@@ -28,7 +28,7 @@ namespace {
 struct MaskedArgs {
     const bf16_t *q, *keys, *values;
     const int32_t *tok_pos, *page_table;
-    int table_width, window, keep_first;
+    int table_width, window, chunk, keep_first;
     float scale, cap;
     const void* sink;               // [heads] or null
     int sink_f32;
@@ -115,9 +115,9 @@ void attention_masked_mfma_kernel(const MaskedArgs a) {
     }
     const int window = a.window;
     const int kept = window > 0 ? a.keep_first : 0;
-    const int lo_c = window > 0 ? max(0, pos_c - window + 1) : 0;
-    const int lo_min = window > 0 ? max(0, pos_first - window + 1) : 0;      // the first column's: the smallest
-    const int lo_max = window > 0 ? max(0, pos_max - window + 1) : 0;
+    const int lo_c = first_seen(pos_c, window, a.chunk);
+    const int lo_min = first_seen(pos_first, window, a.chunk);              // the first column's: the smallest
+    const int lo_max = first_seen(pos_max, window, a.chunk);
     const float scale = a.scale, cap = a.cap;
     const float scale2 = scale * LOG2E;
     const float cap2 = cap * LOG2E, scale_over_cap = cap > 0.f ? scale / cap : 0.f;
@@ -331,11 +331,11 @@ void attention_masked_block_kernel(const MaskedArgs a) {
         const int i = sub * SUB + c * 16 + col;
         live[c] = active && i < count;
         pos_c[c] = live[c] ? pos0 + i : w_first;
-        lo_c[c] = window > 0 ? max(0, pos_c[c] - window + 1) : 0;
+        lo_c[c] = first_seen(pos_c[c], window, a.chunk);
         qrow[c] = (size_t)(tok0 + (live[c] ? i : 0)) * a.n_heads + head;
     }
-    const int w_lo_min = window > 0 ? max(0, w_first - window + 1) : 0, w_lo_max = window > 0 ? max(0, w_max - window + 1) : 0;
-    const int lo_min = window > 0 ? max(0, pos0 - window + 1) : 0;
+    const int w_lo_min = first_seen(w_first, window, a.chunk), w_lo_max = first_seen(w_max, window, a.chunk);
+    const int lo_min = first_seen(pos0, window, a.chunk);
     const int pos_max = pos0 + count - 1;
     const float scale = a.scale, cap = a.cap;
     const float scale2 = scale * LOG2E;
@@ -588,7 +588,7 @@ extern "C" int tqk_attention_masked_mfma_tile(int n_tokens, int n_heads, int n_k
  * page_table row r, in n_parts partitions (part_out float32 [rows, heads, n_parts, value_dim], part_ml [rows, heads, n_parts, 2]
  * where n_parts > 1). */
 extern "C" int tqk_attention_masked_mfma(const void* q, const void* keys, const void* values, const int32_t* tok_pos, const int32_t* page_table,
-                                         int table_width, int n_pages, int window, int keep_first, float scale, float cap, const void* sink,
+                                         int table_width, int n_pages, int window, int chunk, int keep_first, float scale, float cap, const void* sink,
                                          int sink_dtype, const int32_t* tile_seq, const int32_t* tile_tok0, const int32_t* tile_count, int n_tiles,
                                          int tile_queries, int n_rows, int n_parts, void* part_out, void* part_ml, void* out, int n_heads, int n_kv_heads,
                                          int key_dim, int value_dim, void* stream) {
@@ -596,7 +596,7 @@ extern "C" int tqk_attention_masked_mfma(const void* q, const void* keys, const 
     TQK_REQUIRE(n_heads > 0 && n_kv_heads > 0 && n_heads % n_kv_heads == 0, "tqk_attention_masked_mfma: %d heads and %d kv heads", n_heads, n_kv_heads);
     TQK_REQUIRE(tqk_attention_masked_mfma_supported(key_dim, value_dim), "tqk_attention_masked_mfma: head sizes %d and %d are not taken", key_dim, value_dim);
     TQK_REQUIRE(table_width > 0 && n_pages > 0, "tqk_attention_masked_mfma: empty page table");
-    TQK_REQUIRE(window >= 0 && keep_first >= 0 && cap >= 0.f, "tqk_attention_masked_mfma: negative window, kept positions or cap");
+    TQK_REQUIRE(window >= 0 && chunk >= 0 && keep_first >= 0 && cap >= 0.f, "tqk_attention_masked_mfma: negative window, chunk, kept positions or cap");
     TQK_REQUIRE(!sink || sink_dtype == TQK_F32 || sink_dtype == TQK_BF16, "tqk_attention_masked_mfma: unknown dtype %d of the sink", sink_dtype);
     const bool tiles = n_tiles > 0;
     if (tiles) TQK_REQUIRE(tile_seq && tile_tok0 && tile_count && tile_queries >= 16, "tqk_attention_masked_mfma: tiles without their lists or their size");
@@ -608,7 +608,7 @@ extern "C" int tqk_attention_masked_mfma(const void* q, const void* keys, const 
     MaskedArgs a = {};
     a.q = (const bf16_t*)q; a.keys = (const bf16_t*)keys; a.values = (const bf16_t*)values;
     a.tok_pos = tok_pos; a.page_table = page_table; a.table_width = table_width;
-    a.window = window; a.keep_first = keep_first; a.scale = scale; a.cap = cap;
+    a.window = window; a.chunk = chunk; a.keep_first = keep_first; a.scale = scale; a.cap = cap;
     a.sink = sink; a.sink_f32 = sink_dtype == TQK_F32;
     a.n_parts = tiles ? 1 : n_parts; a.n_heads = n_heads; a.n_kv_heads = n_kv_heads;
     a.q_blocks = (n_heads / n_kv_heads + 15) / 16;

@@ -100,7 +100,7 @@ struct PrefillArgs {
     const int32_t* tile_count;
     const int32_t* seq_start;
     const int32_t* seq_new;
-    int window;
+    int window, chunk;       // chunk > 0: positions fall into chunks and see nothing of an earlier one
     float scale;
     float cap;               // > 0: scores become cap tanh(scale s / cap)
     bf16_t* out;
@@ -350,7 +350,7 @@ void attention_prefill_kernel(const PrefillArgs p) {
     const bool live = head_local < heads_here && qi < count;
     const int head = head0 + (live ? head_local : 0);
     w.my_pos = live ? pos0 + qi : -1;
-    w.my_lo = p.window > 0 ? max(0, w.my_pos - p.window + 1) : 0;
+    w.my_lo = live ? first_seen(w.my_pos, p.window, p.chunk) : 0;
     // the wave's range of queries (the same for all its heads)
     const int wq_first = (cw * 32) & (tq - 1);
     const int wq_last = min(tq >= 32 ? wq_first + 31 : tq - 1, count - 1);
@@ -359,12 +359,12 @@ void attention_prefill_kernel(const PrefillArgs p) {
     w.wave_live = __builtin_amdgcn_readfirstlane((cw * 32 >> p.tq_shift) < heads_here && wq_first < count);
     w.wave_first = __builtin_amdgcn_readfirstlane(pos0 + wq_first);
     w.wave_last = __builtin_amdgcn_readfirstlane(pos0 + wq_last);
-    w.wave_lo = p.window > 0 ? max(0, w.wave_first - p.window + 1) : 0;            // first key any of its queries sees
-    w.wave_lo_last = p.window > 0 ? max(0, w.wave_last - p.window + 1) : 0;        // first key all of them see
+    w.wave_lo = first_seen(w.wave_first, p.window, p.chunk);            // first key any of its queries sees
+    w.wave_lo_last = first_seen(w.wave_last, p.window, p.chunk);        // first key all of them see
     w.c2 = p.scale * 1.44269504088896340736f;
     w.cap_in = CAP ? p.scale / p.cap : 0.f;
     w.cap_c2 = p.cap * 1.44269504088896340736f;
-    const int tile_lo = p.window > 0 ? max(0, pos0 - p.window + 1) : 0;
+    const int tile_lo = first_seen(pos0, p.window, p.chunk);
     const int first_page = tile_lo / TQK_PAGE;
     w.last_page = (pos0 + count - 1) / TQK_PAGE;
     w.keys = p.keys;
@@ -541,7 +541,7 @@ extern "C" int tqk_attention_prefill_capped(const void* q, const void* keys, con
                                             const int32_t* page_table, int table_width, int n_seqs, int n_pages,
                                             const int32_t* tile_seq, const int32_t* tile_tok0, const int32_t* tile_count,
                                             int n_tiles, int tile_queries, const int32_t* seq_start, const int32_t* seq_new,
-                                            int window, float scale, float cap, void* out, int n_tokens, int n_heads, int n_kv_heads,
+                                            int window, int chunk, float scale, float cap, void* out, int n_tokens, int n_heads, int n_kv_heads,
                                             int head_dim, void* stream) {
     TQK_REQUIRE(cap >= 0.f, "tqk_attention_prefill: negative cap");
     TQK_REQUIRE(q && keys && values && tok_pos && page_table && tile_seq && tile_tok0 && tile_count && seq_start && seq_new && out,
@@ -550,7 +550,7 @@ extern "C" int tqk_attention_prefill_capped(const void* q, const void* keys, con
     TQK_REQUIRE(n_heads % n_kv_heads == 0, "tqk_attention_prefill: %d heads are not a multiple of %d kv heads", n_heads, n_kv_heads);
     TQK_REQUIRE(tqk_attention_prefill_supported(head_dim), "tqk_attention_prefill: head_dim %d is not one of 32, 64, 96, 128", head_dim);
     TQK_REQUIRE(table_width > 0 && n_pages > 0 && n_seqs > 0, "tqk_attention_prefill: empty page table");
-    TQK_REQUIRE(window >= 0, "tqk_attention_prefill: negative window");
+    TQK_REQUIRE(window >= 0 && chunk >= 0, "tqk_attention_prefill: negative window or chunk");
     TQK_REQUIRE(tile_queries == 16 || tile_queries == 32 || tile_queries == 64 || tile_queries == 128,
                 "tqk_attention_prefill: tiles hold 16, 32, 64 or 128 queries, not %d", tile_queries);
     TQK_REQUIRE((((uintptr_t)q | (uintptr_t)keys | (uintptr_t)values | (uintptr_t)out) & 15) == 0,
@@ -560,7 +560,7 @@ extern "C" int tqk_attention_prefill_capped(const void* q, const void* keys, con
     a.q = (const bf16_t*)q; a.keys = (const bf16_t*)keys; a.values = (const bf16_t*)values;
     a.tok_pos = tok_pos; a.page_table = page_table; a.table_width = table_width;
     a.tile_seq = tile_seq; a.tile_tok0 = tile_tok0; a.tile_count = tile_count;
-    a.seq_start = seq_start; a.seq_new = seq_new; a.window = window; a.scale = scale; a.cap = cap;
+    a.seq_start = seq_start; a.seq_new = seq_new; a.window = window; a.chunk = chunk; a.scale = scale; a.cap = cap;
     a.out = (bf16_t*)out; a.n_heads = n_heads; a.n_kv_heads = n_kv_heads; a.n_tiles = n_tiles;
     a.tq_shift = tile_queries == 16 ? 4 : (tile_queries == 32 ? 5 : (tile_queries == 64 ? 6 : 7));
     prefill_heads(n_heads / n_kv_heads, tile_queries, &a.heads_per_block, &a.head_chunks);
@@ -603,5 +603,5 @@ extern "C" int tqk_attention_prefill(const void* q, const void* keys, const void
                                      int window, float scale, void* out, int n_tokens, int n_heads, int n_kv_heads,
                                      int head_dim, void* stream) {
     return tqk_attention_prefill_capped(q, keys, values, tok_pos, page_table, table_width, n_seqs, n_pages, tile_seq, tile_tok0, tile_count, n_tiles,
-                                        tile_queries, seq_start, seq_new, window, scale, 0.f, out, n_tokens, n_heads, n_kv_heads, head_dim, stream);
+                                        tile_queries, seq_start, seq_new, window, 0, scale, 0.f, out, n_tokens, n_heads, n_kv_heads, head_dim, stream);
 }

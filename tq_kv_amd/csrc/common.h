@@ -37,6 +37,14 @@ __device__ __host__ __forceinline__ int value_position(int place) {
     return (place & 32) | (((place >> 2) & 1) << 4) | (((place >> 3) & 3) << 2) | (place & 3);
 }
 
+// ---- which positions a query sees --------------------------------------------------
+// The first position that a query at `pos` sees: the last `window` positions (0: all), and, where positions fall into
+// chunks (chunk > 0), none of an earlier chunk than its own.  Never decreases with pos.
+__device__ __forceinline__ int first_seen(int pos, int window, int chunk) {
+    const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+    return chunk > 0 ? max(lo, pos - pos % chunk) : lo;
+}
+
 // ---- reductions ---------------------------------------------------------------
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll

@@ -32,5 +32,6 @@ void register_nikasun();
 void register_sizudra();
 void register_piditar();
 void register_povipel();
+void register_rasodra();
 
 }  // namespace tq

@@ -47,7 +47,7 @@ TQ_QUERY(int, attention_prefill_supported, int);
 TQ_QUERY(int, attention_prefill_tile, int, int, int, int);
 TQ_KERNEL(attention_prefill, cptr, cptr, cptr, ci32, ci32, int, int, int, ci32, ci32, ci32, int, int, ci32, ci32, int, float, void*, int, int,
           int, int, void*);
-TQ_KERNEL(attention_prefill_capped, cptr, cptr, cptr, ci32, ci32, int, int, int, ci32, ci32, ci32, int, int, ci32, ci32, int, float, float, void*, int,
+TQ_KERNEL(attention_prefill_capped, cptr, cptr, cptr, ci32, ci32, int, int, int, ci32, ci32, ci32, int, int, ci32, ci32, int, int, float, float, void*, int,
           int, int, int, void*);
 TQ_KERNEL(swiglu, cptr, void*, int, int, int, void*);
 TQ_KERNEL(gated_act, cptr, void*, int, int, int, int, float, float, void*);
@@ -55,21 +55,21 @@ TQ_KERNEL(fused_gated_act, cptr, cf32, int, float, cptr, int, void*, int, int, i
 TQ_KERNEL(mid_gated_act, cptr, cptr, void*, int, int, int, void*, int, float, float, void*);
 TQ_QUERY(int, latent_max_rank);
 TQ_QUERY(int, latent_max_row);
-TQ_KERNEL(latent_split, cptr, int, int, int, int, int, int, cptr, cptr, int, float, cf32, cf32, int, int, ci32, ci32, ci32, int, void*, void*, int,
+TQ_KERNEL(latent_split, cptr, int, int, int, int, int, int, cptr, cptr, int, float, cf32, cf32, int, int, int, ci32, ci32, ci32, int, void*, void*, int,
           void*, float*, int, void*);
 TQ_QUERY(int, latent_attention_mfma_supported, int, int);
 TQ_QUERY(int, latent_attention_parts, int, int, int, int);
-TQ_KERNEL(latent_attention_tiles, cf32, cptr, cptr, ci32, ci32, int, int, int, ci32, ci32, ci32, int, int, float, float*, int, int, int, int, void*);
-TQ_KERNEL(latent_attention_mfma, cf32, cptr, cptr, ci32, ci32, ci32, int, int, int, int, float, float*, int, int, int, int, int, float*, float*, void*);
-TQ_KERNEL(latent_absorb, cptr, int, cptr, int, int, int, int, int, cf32, cf32, int, int, ci32, float*, int, int, void*);
-TQ_KERNEL(latent_attention, cf32, cptr, int, ci32, ci32, ci32, int, int, int, int, float, float*, int, int, int, int, void*);
-TQ_KERNEL(latent_values, cf32, cptr, int, cf32, int, int, int, void*, int, int, void*);
+TQ_KERNEL(latent_attention_tiles, cf32, cptr, cptr, ci32, ci32, int, int, int, ci32, ci32, ci32, int, int, float, cf32, float*, int, int, int, int, void*);
+TQ_KERNEL(latent_attention_mfma, cf32, cptr, cptr, ci32, ci32, ci32, int, int, int, int, float, cf32, float*, int, int, int, int, int, float*, float*, void*);
+TQ_KERNEL(latent_absorb, cptr, int, long long, cptr, int, int, int, int, int, cf32, cf32, int, int, int, ci32, float*, int, int, void*);
+TQ_KERNEL(latent_attention, cf32, cptr, int, ci32, ci32, ci32, int, int, int, int, float, cf32, float*, int, int, int, int, void*);
+TQ_KERNEL(latent_values, cf32, cptr, int, cf32, cptr, long long, int, int, int, void*, int, int, void*);
 TQ_QUERY(int, moe_max_experts);
 TQ_QUERY(int, moe_max_tiles, int, int, int);
 TQ_QUERY(int, moe_tile_rows);
 TQ_QUERY(int, grouped_supported, int);
 TQ_KERNEL(moe_product_mfma, cptr, ci32, cptr, long long, void*, int, int, int, int, float, float, ci32, ci32, ci32, ci32, int, int, void*);
-TQ_KERNEL(head_product, cptr, int, long long, long long, cptr, void*, int, long long, long long, cf32, int, int, int, int, void*);
+TQ_KERNEL(head_product, cptr, int, long long, long long, cptr, void*, int, long long, long long, cf32, cptr, int, long long, int, int, int, int, void*);
 TQ_KERNEL(moe_route, cptr, int, cptr, int, int, int, int, float, int, int32_t*, float*, cptr, float*, int, void*);
 TQ_KERNEL(moe_group, ci32, int, int, int, int, int32_t*, int32_t*, int32_t*, int32_t*, int32_t*, int32_t*, void*);
 TQ_KERNEL(moe_product, cptr, int, ci32, cptr, int, long long, void*, int, int, int, int, float, float, ci32, ci32, ci32, ci32, int, void*);
@@ -80,8 +80,8 @@ TQ_KERNEL(remember_tokens, ci32, ci32, ci32, ci32, int32_t*, int, void*);
 TQ_KERNEL(norm_add, float*, cptr, int, cptr, int, float, void*, int, int, void*);
 TQ_KERNEL(unary_act, cptr, void*, int, long long, int, float, float, void*);
 TQ_KERNEL(row_gate, cptr, int, cptr, int, float*, int, int, void*);
-TQ_KERNEL(normed_rope_store, cptr, int, cptr, cptr, int, float, cf32, cf32, int, int, cptr, cptr, void*, ci32, ci32, ci32, int, void*, void*, void*,
-          int, int, int, int, int, int, void*);
+TQ_KERNEL(normed_rope_store, cptr, int, cptr, cptr, cptr, int, float, cf32, cf32, int, int, int, cptr, cptr, void*, ci32, ci32, ci32, int, void*, void*,
+          void*, int, int, int, int, int, int, int, void*);
 TQ_KERNEL(rope_norm_store, cptr, int, cptr, int, cf32, cf32, int, int, int, int, float, ci32, ci32, ci32, int, void*, void*, void*, int, int, int, int,
           int, int, void*);
 TQ_QUERY(int, conv_max_taps);
@@ -102,20 +102,22 @@ TQ_KERNEL(add_rows, float*, cf32, long long, void*);
 TQ_QUERY(int, attention_masked_max_dim);
 TQ_QUERY(int, attention_masked_mfma_supported, int, int);
 TQ_QUERY(int, attention_masked_mfma_tile, int, int, int, int, int);
-TQ_KERNEL(attention_masked_mfma, cptr, cptr, cptr, ci32, ci32, int, int, int, int, float, float, cptr, int, ci32, ci32, ci32, int, int, int, int, void*, void*,
+TQ_KERNEL(attention_masked_mfma, cptr, cptr, cptr, ci32, ci32, int, int, int, int, int, float, float, cptr, int, ci32, ci32, ci32, int, int, int, int, void*, void*,
           void*, int, int, int, int, void*);
-TQ_KERNEL(attention_masked, cptr, cptr, cptr, int, ci32, ci32, ci32, int, int, int, int, int, float, float, cptr, int, void*, int, int, int, int,
+TQ_KERNEL(attention_masked, cptr, cptr, cptr, int, ci32, ci32, ci32, int, int, int, int, int, int, float, float, cptr, int, void*, int, int, int, int,
           int, void*);
 TQ_QUERY(int, streams_max);
 TQ_KERNEL(streams_fill, cf32, float*, int, int, int, void*);
 TQ_KERNEL(streams_step, float*, int, cptr, int, cf32, cf32, cf32, cf32, cf32, float, float*, void*, int, int, int, int, void*);
-TQ_KERNEL(add_layer_norm, float*, cptr, int, ci32, int, cf32, cf32, float, void*, int, int, int, void*);
+TQ_KERNEL(add_layer_norm, float*, cptr, int, ci32, int, cf32, cf32, float, cf32, cf32, float, void*, int, int, int, void*);
 TQ_KERNEL(token_shift, cf32, cf32, float*, long long, ci32, ci32, ci32, ci32, void*, int, int, int, int, void*);
 TQ_KERNEL(shift_remember, cf32, float*, long long, ci32, ci32, ci32, int, int, void*);
 TQ_QUERY(int, linear_attention_max_dim);
-TQ_KERNEL(linear_attention, cptr, cptr, cptr, int, long long, cf32, long long, cf32, float, cf32, float, float, cf32, cf32, int, int, int, ci32, float*,
-          long long, ci32, ci32, ci32, ci32, ci32, float*, float*, float*, int, int, int, int, int, void*);
-TQ_KERNEL(head_norm_gate, cf32, cf32, float, cptr, int, long long, void*, int, int, int, int, void*);
+TQ_KERNEL(linear_attention, cptr, cptr, cptr, int, long long, cf32, long long, cf32, float, cf32, cf32, cf32, cf32, float, float, cf32, cf32, int, int, int,
+          ci32, float*, long long, ci32, ci32, ci32, ci32, ci32, float*, float*, float*, int, int, int, int, int, long long, void*);
+TQ_KERNEL(head_norm_gate, cf32, cf32, int, float, cptr, int, long long, int, void*, int, int, int, int, void*);
+TQ_KERNEL(mlstm_gates, cf32, long long, cf32, float, cptr, cptr, int, long long, float, float*, long long, long long, long long, ci32, ci32, ci32, float*,
+          float*, float*, float*, int, int, int, void*);
 TQ_QUERY(int, pooled_attention_max_dim);
 TQ_QUERY(int, pooled_rows, int);
 TQ_KERNEL(pooled_store, cptr, int, cf32, cf32, int, float, cf32, cf32, int, int, cf32, cf32, int, ci32, ci32, ci32, int, void*, void*, void*, int, int, int,

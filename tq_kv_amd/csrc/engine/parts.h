@@ -63,11 +63,13 @@ struct PartialSums {
 
 // An update of the stream that has not been added yet: nothing, a tensor of the activation
 // dtype, or a product's partial sums (only for a norm that takes those).
+// norm (with a plain tensor): the update is normed by it before it is added; only for a norm that takes such updates.
 struct Pending {
     enum Kind { Nothing, Plain, Sums };
     Kind kind = Nothing;
     Tensor t;
     PartialSums s;
+    Norm* norm = nullptr;
     static Pending of(const Tensor& t) { Pending p; p.kind = t.defined() ? Plain : Nothing; p.t = t; return p; }
     static Pending of(const PartialSums& s) { Pending p; p.kind = Sums; p.s = s; return p; }
 };
@@ -149,6 +151,8 @@ public:
     // out = norm(h[rows] + delta[rows]) for the int32 row indices (on the device); h is left as it is
     virtual void gather_add_norm(StepContext& c, const Tensor& h, const Pending& delta, const int32_t* rows, int64_t n_rows, Tensor& out) = 0;
     virtual bool takes_partial_sums() const { return false; }
+    // whether add_norm and gather_add_norm take an update that `norm` is to be applied to before it is added
+    virtual bool takes_normed_update(const Norm* norm) const { (void)norm; return false; }
     // whether the kernels that add to the stream can prepare this norm, and with what
     virtual bool foldable() const { return false; }
     virtual const Tensor* fold_weight() const { return nullptr; }
@@ -190,6 +194,7 @@ struct CacheEntry {
     int64_t state_offset = 0;       // where in a slot's row the part's own state begins (a part that shares the row with others)
     bool writes = true;             // false: reads another run's cache
     int window = 0;
+    int chunk = 0;
     int keep_first = 0;
 };
 
@@ -241,5 +246,6 @@ void register_recurrent_parts();        // parts_recurrent.cpp; likewise
 void register_streams_parts();          // parts_streams.cpp; likewise
 void register_linear_attention_parts(); // parts_linear_attention.cpp; likewise
 void register_pooled_parts();           // parts_pooled.cpp; likewise
+void register_mlstm_parts();            // parts_mlstm.cpp; likewise
 
 }  // namespace tq

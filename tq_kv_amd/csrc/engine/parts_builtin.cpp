@@ -234,9 +234,11 @@ public:
 // prompt_tile: queries per tile of the prompt kernel (16, 32, 64 or 128).
 //
 // What other designs put around the same attention, all off unless given: value_dim (a head's values are of another
-// size than its keys); qk_norm with eps (every query and key head is divided by its root mean square and multiplied
+// size than its keys); values_are_keys (there is no value projection: the values are the keys as projected, before norm and rotation);
+// qk_norm with eps (every query and key head is divided by its root mean square and multiplied
 // by a weight of head_dim values, before the rotation; with qk_norm_weight false and qk_norm_after_rotation true the heads are divided by
-// their root mean square after the rotation and there is no weight: then the projections may have biases and the rotation may go by pairs); cap (scores become cap tanh(s / cap)); keep_first (with a
+// their root mean square after the rotation and there is no weight); cap (scores become cap tanh(s / cap)); chunk (positions fall into
+// chunks of so many, counted from the sequence's start, and see nothing of an earlier chunk); keep_first (with a
 // window: a sequence's first positions stay visible, at their true places); sink (a learned number per head whose
 // exponential joins the softmax's denominator, with no key and no value); value_mix "source" (the values of the
 // step's tokens are handed to later layers) or "mixed" (v <- (1 - lambda) v + lambda v_source with a learned scalar,
@@ -270,6 +272,10 @@ public:
         qk_norm_weight_ = r.boolean_or("qk_norm_weight", true);
         norm_after_rotation_ = r.boolean_or("qk_norm_after_rotation", false);
         eps_ = qk_norm_ ? (float)r.number("eps") : 0.f;
+        values_are_keys_ = r.boolean_or("values_are_keys", false);
+        if (values_are_keys_ && value_dim_ != head_dim_)
+            raise(TQE_ERR_ARGUMENT, "attention: keys of %d elements cannot serve as values of %d", head_dim_, value_dim_);
+        chunk_ = r.has("chunk") ? (int)r.integer("chunk", 1) : 0;
         cap_ = r.has("cap") ? (float)r.number("cap", true) : 0.f;
         keep_first_ = (int)r.integer_or("keep_first", 0, 0);
         cache_keeps_all_ = r.boolean_or("cache_keeps_all", false);
@@ -281,13 +287,16 @@ public:
         else raise(TQE_ERR_ARGUMENT, "attention: unknown value_mix '%s' (known: none, source, mixed)", mixing.c_str());
         mix_key_ = "attention." + r.string_or("value_mix_key", "values");
         if (keep_first_ > 0 && window_ == 0) raise(TQE_ERR_ARGUMENT, "attention: keep_first %d without a window", keep_first_);
-        extras_ = value_dim_ != head_dim_ || qk_norm_ || cap_ > 0.f || keep_first_ > 0 || has_sink_ || value_mix_ != MIX_NONE;
+        extras_ = value_dim_ != head_dim_ || values_are_keys_ || chunk_ > 0 || qk_norm_ || cap_ > 0.f || keep_first_ > 0 || has_sink_ || value_mix_ != MIX_NONE;
         if (qk_norm_ && qk_norm_weight_ == norm_after_rotation_)
             raise(TQE_ERR_ARGUMENT, "attention: the heads' norm is either weighted and in front of the rotation, or without a weight and after it");
-        // the kernel that adds biases, turns and then norms without a weight stands for every such combination but mixed values
-        const bool turned_ok = extras_ && (!qk_norm_ || norm_after_rotation_) && value_mix_ == MIX_NONE;
-        if (extras_ && (out_bias_ || (qkv_bias_ && !turned_ok)))
-            raise(TQE_ERR_ARGUMENT, "attention: with value_dim, cap, keep_first or sink the projections may have biases where the heads' norm has no weight and values are not mixed; the output has none");
+        // the kernel that adds biases, turns and then norms without a weight stands for every such combination but mixed values and
+        // values that are the keys; the one that norms in front of the rotation for every other
+        const bool turned_ok = extras_ && (!qk_norm_ || norm_after_rotation_) && value_mix_ == MIX_NONE && !values_are_keys_;
+        if (extras_ && norm_after_rotation_ && qk_norm_ && !turned_ok)
+            raise(TQE_ERR_ARGUMENT, "attention: a heads' norm after the rotation goes with values of their own that are not mixed");
+        if (extras_ && out_bias_)
+            raise(TQE_ERR_ARGUMENT, "attention: with value_dim, values_are_keys, chunk, qk_norm, cap, keep_first, sink or value_mix the output has no bias");
         {
             const Json& names = spec.params["names"];
             auto name = [&](const char* role, const char* fallback) { return names[role].is_string() ? names[role].as_string() : std::string(fallback); };
@@ -317,8 +326,8 @@ public:
         if (extras_) {
             const Position::Tables tb = position_->tables();
             turned_first_ = turned_ok && (qkv_bias_ || norm_after_rotation_ || tb.style == STYLE_PAIRS);
-            if (position_->has_apply() || tb.rot_dim > head_dim_ || (tb.style != STYLE_NONE && tb.style != STYLE_HALVES && !turned_ok))
-                raise(TQE_ERR_ARGUMENT, "attention: with value_dim, qk_norm, cap, keep_first, sink or value_mix the position part must turn from tables (in halves where the heads' norm has a weight or values are mixed)");
+            if (position_->has_apply() || tb.rot_dim > head_dim_)
+                raise(TQE_ERR_ARGUMENT, "attention: with value_dim, values_are_keys, chunk, qk_norm, cap, keep_first, sink or value_mix the position part must turn from tables");
         }
     }
 
@@ -326,8 +335,9 @@ public:
         const int64_t q = (int64_t)n_heads_ * head_dim_, kv = (int64_t)n_kv_heads_ * head_dim_;
         auto w = [](int64_t a, int64_t b) { TensorSpec t; t.shape = {a, b}; return t; };
         auto b = [](int64_t a) { TensorSpec t; t.shape = {a}; return t; };
-        TensorSpecs t = {{n_q_, w(q, hidden_)}, {n_k_, w(kv, hidden_)}, {n_v_, w((int64_t)n_kv_heads_ * value_dim_, hidden_)},
-                         {n_o_, w(hidden_, (int64_t)n_heads_ * value_dim_)}};
+        TensorSpecs t = {{n_q_, w(q, hidden_)}, {n_k_, w(kv, hidden_)}};
+        if (!values_are_keys_) t.push_back({n_v_, w((int64_t)n_kv_heads_ * value_dim_, hidden_)});
+        t.push_back({n_o_, w(hidden_, (int64_t)n_heads_ * value_dim_)});
         if (qk_norm_ && qk_norm_weight_) {
             TensorSpec n = b(head_dim_);
             n.init = "one_plus_normal";
@@ -338,7 +348,11 @@ public:
         if (has_sink_) { TensorSpec s = b(n_heads_); s.std_dev = 1.0; t.push_back({n_sink_, s}); }
         // the source layer of a mix has the scalar too, and does not use it
         if (value_mix_ != MIX_NONE) { TensorSpec s; s.shape = {}; s.std_dev = 0.3; t.push_back({n_mix_, s}); }
-        if (qkv_bias_) { t.push_back({n_qb_, b(q)}); t.push_back({n_kb_, b(kv)}); t.push_back({n_vb_, b((int64_t)n_kv_heads_ * value_dim_)}); }
+        if (qkv_bias_) {
+            t.push_back({n_qb_, b(q)});
+            t.push_back({n_kb_, b(kv)});
+            if (!values_are_keys_) t.push_back({n_vb_, b((int64_t)n_kv_heads_ * value_dim_)});
+        }
         if (out_bias_) t.push_back({"o_proj.bias", b(hidden_)});
         return t;
     }
@@ -346,11 +360,16 @@ public:
     static OwnedPtr stacked(const std::vector<OwnedPtr>& parts, hipStream_t stream) { return stack_rows(parts, stream); }
 
     void load(Loaded& t, hipStream_t stream) override {
-        OwnedPtr qkv = stacked({take(t, n_q_.c_str()), take(t, n_k_.c_str()), take(t, n_v_.c_str())}, stream);
+        auto stack_of = [&](const std::string& q, const std::string& k, const std::string& v) {
+            std::vector<OwnedPtr> parts = {take(t, q.c_str()), take(t, k.c_str())};
+            if (!values_are_keys_) parts.push_back(take(t, v.c_str()));
+            return stacked(parts, stream);
+        };
+        OwnedPtr qkv = stack_of(n_q_, n_k_, n_v_);
         if (qk_norm_ && qk_norm_weight_) { q_norm_ = take(t, n_q_norm_.c_str()); k_norm_ = take(t, n_k_norm_.c_str()); }
         if (has_sink_) sink_ = take(t, n_sink_.c_str());
         if (value_mix_ != MIX_NONE) mix_ = take(t, n_mix_.c_str());
-        if (qkv_bias_) b_qkv_ = stacked({take(t, n_qb_.c_str()), take(t, n_kb_.c_str()), take(t, n_vb_.c_str())}, stream);
+        if (qkv_bias_) b_qkv_ = stack_of(n_qb_, n_kb_, n_vb_);
         if (out_bias_) b_o_ = take(t, "o_proj.bias");
         w_qkv_ = make_weight(qkv, 1, false, stream);
         w_o_ = make_weight(take(t, n_o_.c_str()), 1, b_o_ != nullptr, stream);
@@ -369,7 +388,7 @@ public:
     }
     const char* trace_name() const override { return "attn"; }             // the reference's span, src/models/turbo_generic.rs:1920
     void product_shapes(std::vector<std::pair<int64_t, int64_t>>& out) const override {
-        out.push_back({(int64_t)(n_heads_ + n_kv_heads_) * head_dim_ + (int64_t)n_kv_heads_ * value_dim_, hidden_});
+        out.push_back({(int64_t)(n_heads_ + n_kv_heads_) * head_dim_ + (values_are_keys_ ? 0 : (int64_t)n_kv_heads_ * value_dim_), hidden_});
         out.push_back({hidden_, (int64_t)n_heads_ * value_dim_});
     }
 
@@ -382,6 +401,7 @@ public:
         // can share one group of the cache)
         n.window = cache_keeps_all_ ? 0 : window_;
         n.keep_first = cache_keeps_all_ ? 0 : keep_first_;
+        n.chunk = cache_keeps_all_ ? 0 : chunk_;
         return n;
     }
 
@@ -446,7 +466,7 @@ public:
     }
 
 private:
-    // product, then the heads' norm, rotation, value mixing and cache write in one kernel
+    // product, then biases, the heads' norm, rotation, value mixing and cache write in one kernel
     void normed_qkv(StepContext& c, const Tensor& x, const CacheEntry& entry, const StepContext::Table& table, Tensor& q) {
         const int64_t n = x.shape[0];
         Product p = linear(c, x, w_qkv_, nullptr, x.dtype);
@@ -466,15 +486,15 @@ private:
                 raise(TQE_ERR_STATE, "attention: the values an earlier layer left are %s, wanted [%lld, %lld]", it->second.describe().c_str(), (long long)n, (long long)vd);
             mix_with = it->second.data;
         }
-        const int w_dtype = q_norm_ ? q_norm_->t.dtype : mix_ ? mix_->t.dtype : x.dtype;
-        if ((q_norm_ && k_norm_->t.dtype != w_dtype) || (mix_ && mix_->t.dtype != w_dtype))
-            raise(TQE_ERR_STATE, "attention: the heads' norm weights and the mixing scalar are of different types");
+        const int w_dtype = q_norm_ ? q_norm_->t.dtype : mix_ ? mix_->t.dtype : b_qkv_ ? b_qkv_->t.dtype : x.dtype;
+        if ((q_norm_ && k_norm_->t.dtype != w_dtype) || (mix_ && mix_->t.dtype != w_dtype) || (b_qkv_ && b_qkv_->t.dtype != w_dtype))
+            raise(TQE_ERR_STATE, "attention: the heads' norm weights, the biases and the mixing scalar are of different types");
         const bool write = entry.writes;
-        K::normed_rope_store(p.t.data, p.t.dtype, q_norm_ ? q_norm_->t.data : nullptr, k_norm_ ? k_norm_->t.data : nullptr, w_dtype, eps_,
+        K::normed_rope_store(p.t.data, p.t.dtype, b_qkv_ ? b_qkv_->t.data : nullptr, q_norm_ ? q_norm_->t.data : nullptr, k_norm_ ? k_norm_->t.data : nullptr, w_dtype, eps_,
                              turn ? (const float*)tb.cos.data : nullptr, turn ? (const float*)tb.sin.data : nullptr, turn ? tb.rot_dim : 0,
-                             turn ? (int)tb.cos.shape[0] : 0, mix_ ? mix_->t.data : nullptr, mix_with, mix_keep, c.dev.tok_seq, c.dev.tok_pos,
+                             turn ? tb.style : 0, turn ? (int)tb.cos.shape[0] : 0, mix_ ? mix_->t.data : nullptr, mix_with, mix_keep, c.dev.tok_seq, c.dev.tok_pos,
                              write ? table.dev : nullptr, write ? table.width : 0, write ? entry.keys.data : nullptr, write ? entry.values.data : nullptr,
-                             q.data, (int)n, n_heads_, n_kv_heads_, head_dim_, value_dim_, write ? 1 : 0, c.stream);
+                             q.data, (int)n, n_heads_, n_kv_heads_, head_dim_, value_dim_, write ? 1 : 0, values_are_keys_ ? 1 : 0, c.stream);
     }
 
     // product, then biases, rotation (halves or pairs), the heads' norm without a weight after it, and the cache write in one kernel
@@ -511,13 +531,14 @@ private:
                     k_gather_rows(c, whole, c.dev.last_seq, n, gathered);
                     row_table = (const int32_t*)gathered.data;
                 }
-                const int n_parts = partitions(n, table.width);
+                // (no more pages than a chunk can touch are ever visited)
+                const int n_parts = partitions(n, chunk_ > 0 ? std::min(table.width, (chunk_ + TQE_PAGE - 2) / TQE_PAGE + 1) : table.width);
                 Tensor part_out, part_ml;
                 if (n_parts > 1) {
                     part_out = c.alloc(F32, {n, n_heads_, n_parts, value_dim_});
                     part_ml = c.alloc(F32, {n, n_heads_, n_parts, 2});
                 }
-                K::attention_masked_mfma(q.data, entry.keys.data, entry.values.data, tok_pos, row_table, table.width, n_pages, window_, keep_first_, scale_,
+                K::attention_masked_mfma(q.data, entry.keys.data, entry.values.data, tok_pos, row_table, table.width, n_pages, window_, chunk_, keep_first_, scale_,
                                          cap_, sink, sink_dtype, nullptr, nullptr, nullptr, 0, 0, n, n_parts, part_out.data, part_ml.data, out.data, n_heads_,
                                          n_kv_heads_, head_dim_, value_dim_, c.stream);
                 return;
@@ -529,21 +550,21 @@ private:
                 const int tile = tile_for(c);
                 const Tiles t = last_rows ? c.last_tiles(tile) : c.query_tiles(tile);
                 K::attention_prefill_capped(q.data, entry.keys.data, entry.values.data, tok_pos, table.dev, table.width, c.n_seqs, n_pages, t.seq, t.tok0,
-                                            t.count, t.n, tile, c.dev.seq_start, c.dev.seq_new, window_, scale_, cap_, out.data, n, n_heads_, n_kv_heads_,
+                                            t.count, t.n, tile, c.dev.seq_start, c.dev.seq_new, window_, chunk_, scale_, cap_, out.data, n, n_heads_, n_kv_heads_,
                                             head_dim_, c.stream);
                 return;
             }
             if (!rows && policy().prefill_mfma) {
                 const int tile = K::attention_masked_mfma_tile.raw(n, n_heads_, n_kv_heads_, head_dim_, value_dim_);
                 const Tiles t = last_rows ? c.last_tiles(tile) : c.query_tiles(tile);
-                K::attention_masked_mfma(q.data, entry.keys.data, entry.values.data, tok_pos, table.dev, table.width, n_pages, window_, keep_first_, scale_,
+                K::attention_masked_mfma(q.data, entry.keys.data, entry.values.data, tok_pos, table.dev, table.width, n_pages, window_, chunk_, keep_first_, scale_,
                                          cap_, sink, sink_dtype, t.seq, t.tok0, t.count, t.n, tile, 0, 1, nullptr, nullptr, out.data, n_heads_, n_kv_heads_,
                                          head_dim_, value_dim_, c.stream);
                 return;
             }
         }
         K::attention_masked(q.data, entry.keys.data, entry.values.data, q.dtype, tok_seq, tok_pos, table.dev, table.width, c.n_seqs,
-                            (int)entry.keys.shape[0], window_, keep_first_, scale_, cap_, sink_ ? sink_->t.data : nullptr, sink_ ? sink_->t.dtype : 0,
+                            (int)entry.keys.shape[0], window_, chunk_, keep_first_, scale_, cap_, sink_ ? sink_->t.data : nullptr, sink_ ? sink_->t.dtype : 0,
                             out.data, (int)q.shape[0], n_heads_, n_kv_heads_, head_dim_, value_dim_, c.stream);
     }
 
@@ -687,8 +708,8 @@ private:
     bool qkv_bias_, out_bias_;
     float scale_;
     enum { MIX_NONE = 0, MIX_SOURCE = 1, MIX_MIXED = 2 };
-    int value_dim_, keep_first_, value_mix_ = MIX_NONE;
-    bool qk_norm_ = false, has_sink_ = false, extras_ = false, cache_keeps_all_ = false;
+    int value_dim_, chunk_ = 0, keep_first_, value_mix_ = MIX_NONE;
+    bool qk_norm_ = false, has_sink_ = false, extras_ = false, cache_keeps_all_ = false, values_are_keys_ = false;
     bool qk_norm_weight_ = true, norm_after_rotation_ = false, turned_first_ = false;
     float eps_ = 0.f, cap_ = 0.f;
     std::string mix_key_, n_q_, n_k_, n_v_, n_o_, n_q_norm_, n_k_norm_, n_sink_, n_mix_, n_qb_, n_kb_, n_vb_;
@@ -780,7 +801,8 @@ private:
 // pieces of K pending: the norm's kernel adds those up too).  In small decoding steps the
 // framework's parts go further: a product that consumes a norm computes it itself (LazyNorm) and a
 // part's last product adds its result to the stream in its epilogue, so that the norm kernels
-// disappear; parts that do not offer this are simply given tensors.
+// disappear; parts that do not offer this are simply given tensors.  An output norm (post_mixer_norm, post_ff_norm) whose kind the
+// next norm knows is left to that norm's kernel too: output norm, sum and next norm are one pass.
 //
 // params: mixer, feed_forward, mixer_norm, ff_norm (part specs); optional post_mixer_norm,
 // post_ff_norm; names: part -> tensor-name prefix inside the layer (e.g. {"mixer": "self_attn."}).
@@ -845,13 +867,14 @@ public:
     Mixer* mixer() override { return mixer_.get(); }
 
     Stream* forward(StepContext& c, Stream* stream, const CacheEntry& entry, Norm* next_norm, bool last) override {
-        if (last && c.prune_last && policy().prune_last && mixer_->takes_rows) return forward_last_rows(c, stream, entry);
+        if (last && c.prune_last && policy().prune_last && mixer_->takes_rows) return forward_last_rows(c, stream, entry, next_norm);
         Activation x = normed(c, *mixer_norm_, *stream, mixer_->folds_norm(c));
         {
             Span span(mixer_->trace_name());
             const bool adds = (c.fuse_small || c.fuse_mid) && !post_mixer_norm_ && mixer_->adds_to_stream(c);
             if (adds) stream->next_norm = feed_forward_ ? ff_norm_.get() : next_norm;
-            settle(c, *stream, mixer_->forward(c, x, entry, adds ? stream : nullptr, false), post_mixer_norm_.get());
+            settle(c, *stream, mixer_->forward(c, x, entry, adds ? stream : nullptr, false), post_mixer_norm_.get(),
+                   feed_forward_ ? ff_norm_.get() : next_norm);
         }
         if (!feed_forward_) return stream;
         x = normed(c, *ff_norm_, *stream, feed_forward_->folds_norm(c));
@@ -859,7 +882,7 @@ public:
             Span span(feed_forward_->trace_name());
             const bool adds = (c.fuse_small || c.fuse_mid) && !post_ff_norm_ && feed_forward_->adds_to_stream(c);
             if (adds) stream->next_norm = next_norm;
-            settle(c, *stream, feed_forward_->forward(c, x, adds ? stream : nullptr), post_ff_norm_.get());
+            settle(c, *stream, feed_forward_->forward(c, x, adds ? stream : nullptr), post_ff_norm_.get(), next_norm);
         }
         return stream;
     }
@@ -882,18 +905,20 @@ private:
         return a;
     }
     // a part's output that it did not add to the stream itself is left pending for the next norm's kernel
-    void settle(StepContext& c, Stream& stream, Tensor out, Norm* post_norm) {
+    void settle(StepContext& c, Stream& stream, Tensor out, Norm* post_norm, const Norm* next_norm) {
         if (!out.defined()) return;
-        if (post_norm) {
+        const bool together = post_norm && next_norm && next_norm->takes_normed_update(post_norm);
+        if (post_norm && !together) {
             Tensor y = c.alloc(out.dtype, {out.shape[0], out.shape[1]});
             post_norm->forward(c, out, y);
             out = y;
         }
         stream.pending = Pending::of(out);
+        if (together) stream.pending.norm = post_norm;
         stream.invalidate();
     }
 
-    Stream* forward_last_rows(StepContext& c, Stream* stream, const CacheEntry& entry) {
+    Stream* forward_last_rows(StepContext& c, Stream* stream, const CacheEntry& entry, const Norm* next_norm) {
         Activation x;
         {
             Span span(mixer_norm_->trace_name());
@@ -911,7 +936,7 @@ private:
         sub->h = c.alloc(F32, {c.n_last, stream->h.shape[1]});
         if (c.n_last == 0) return sub;
         k_gather_rows(c, stream->h, c.dev.last_rows, c.n_last, sub->h);
-        settle(c, *sub, y, post_mixer_norm_.get());
+        settle(c, *sub, y, post_mixer_norm_.get(), feed_forward_ ? ff_norm_.get() : next_norm);
         if (!feed_forward_) return sub;
         {
             Span span(ff_norm_->trace_name());
@@ -924,7 +949,7 @@ private:
             Span span(feed_forward_->trace_name());
             out = feed_forward_->forward(c, x, nullptr);
         }
-        settle(c, *sub, out, post_ff_norm_.get());
+        settle(c, *sub, out, post_ff_norm_.get(), next_norm);
         return sub;
     }
 
@@ -950,6 +975,7 @@ void register_builtin_parts() {
         register_streams_parts();
         register_linear_attention_parts();
         register_pooled_parts();
+        register_mlstm_parts();
         register_kind("block", "pre_norm", [](const PartSpec& s, BuildEnv& e) { return std::make_shared<PreNormBlock>(s, e); });
     });
 }

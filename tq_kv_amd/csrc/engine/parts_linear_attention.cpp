@@ -171,9 +171,9 @@ public:
         const float inv_tau = per_channel_ ? (float)(1.0 / tau_) : 0.f;
         Tensor o = c.alloc(F32, {n, heads_, dv_});
         auto run = [&](int mode, int items, const Chunks* ch, float* cs, float* cd) {
-            K::linear_attention(in.data, at(in, qk), at(in, 2 * qk), dtype, row_, zp, qk, zb, inv_tau, hd, q_scale_, k_scale_, cos, sin, turn ? tb.rot_dim : 0,
+            K::linear_attention(in.data, at(in, qk), at(in, 2 * qk), dtype, row_, zp, qk, zb, inv_tau, hd, nullptr, nullptr, nullptr, q_scale_, k_scale_, cos, sin, turn ? tb.rot_dim : 0,
                                 turn ? tb.style : 0, max_pos, c.dev.tok_pos, state, row, c.dev.cu, c.dev.seq_new, c.dev.seq_slot, ch ? ch->row0 : nullptr,
-                                ch ? ch->count : nullptr, cs, cd, (float*)o.data, mode, items, heads_, d_, dv_, c.stream);
+                                ch ? ch->count : nullptr, cs, cd, (float*)o.data, mode, items, heads_, d_, dv_, (long long)d_ * dv_, c.stream);
         };
         if (dtype == BF16 && !c.all_decode && !c.capturing && c.max_new >= CHUNKED_FROM && !null_device()) {
             const Chunks ch = c.chunks(SCAN_CHUNK);
@@ -186,7 +186,7 @@ public:
             run(0, c.n_seqs, nullptr, nullptr, nullptr);
         }
         Tensor gated = c.alloc(dtype, {n, vv});
-        K::head_norm_gate((const float*)o.data, norm_w_ ? (const float*)norm_w_->t.data : nullptr, eps_, at(in, 2 * qk + vv), dtype, row_, gated.data, dtype, (int)n,
+        K::head_norm_gate((const float*)o.data, norm_w_ ? (const float*)norm_w_->t.data : nullptr, 0, eps_, at(in, 2 * qk + vv), dtype, row_, 0, gated.data, dtype, (int)n,
                           heads_, dv_, c.stream);
         return linear(c, gated, w_o_, nullptr, dtype).t;
     }

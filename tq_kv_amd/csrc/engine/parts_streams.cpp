@@ -1,8 +1,9 @@
-// A layer norm with weight and bias, and a block that keeps the residual stream in several copies.
+// A layer norm with weight and (optional) bias, and a block that keeps the residual stream in several copies.
 //
 //   norm  layer_norm   (x - mean) / sqrt(var + eps) w + b, the variance the mean of the squared deviations; float32 arithmetic.
-//                      params: size, eps; optional tensor (the weight's name, "weight" unless given; may be empty) and bias_tensor
-//                      ("bias" unless given).
+//                      params: size, eps; optional tensor (the weight's name, "weight" unless given; may be empty), bias (false: the norm has
+//                      none) and bias_tensor ("bias" unless given).  An update of the stream that is to be normed by another layer_norm before
+//                      it is added takes one kernel with the sum and this norm.
 //   block multi_stream pre-norm around a mixer and an optional feed-forward, with `streams` copies X[0..S) of the stream in place of
 //                      the one.  A sublayer reads u = sum_s in[s] X[s], computes y = part(norm(u)), and all copies are updated at
 //                      once from the old ones: X'[r] = sum_s mix[s, r] X[s] + out[r] y.  Every copy starts as the stream the block
@@ -56,18 +57,20 @@ public:
         eps_ = (float)r.number("eps");
         n_w_ = r.string_or("tensor", "weight");
         n_b_ = r.string_or("bias_tensor", "bias");
-        if (n_w_ == n_b_) raise(TQE_ERR_ARGUMENT, "layer_norm: weight and bias under one name '%s'", n_w_.c_str());
+        has_bias_ = r.boolean_or("bias", true);
+        if (has_bias_ && n_w_ == n_b_) raise(TQE_ERR_ARGUMENT, "layer_norm: weight and bias under one name '%s'", n_w_.c_str());
         graph_safe = true;
     }
     TensorSpecs tensors() const override {
         TensorSpec w; w.shape = {size_}; w.init = "one_plus_normal"; w.std_dev = 0.1;
         TensorSpec b; b.shape = {size_}; b.std_dev = 0.1;
+        if (!has_bias_) return {{n_w_, w}};
         return {{n_w_, w}, {n_b_, b}};
     }
     void load(Loaded& t, hipStream_t stream) override {
         stored_ = t;
         w_ = as_floats(take(t, n_w_), stream);
-        b_ = as_floats(take(t, n_b_), stream);
+        if (has_bias_) b_ = as_floats(take(t, n_b_), stream);
     }
     OwnedPtr held(const std::string& name) const override {
         auto it = stored_.find(name);
@@ -76,27 +79,35 @@ public:
     const char* trace_name() const override { return "rms-norm"; }
     int64_t size() const override { return size_; }
     const float* weight() const { return (const float*)w_->t.data; }
-    const float* bias() const { return (const float*)b_->t.data; }
+    const float* bias() const { return b_ ? (const float*)b_->t.data : nullptr; }
     float eps() const { return eps_; }
 
     void forward(StepContext& c, const Tensor& x, Tensor& out) override {
-        K::add_layer_norm(nullptr, x.data, x.dtype, nullptr, (int)x.shape[0], weight(), bias(), eps_, out.data, out.dtype, (int)size_, 0, c.stream);
+        K::add_layer_norm(nullptr, x.data, x.dtype, nullptr, (int)x.shape[0], weight(), bias(), eps_, nullptr, nullptr, 0.f, out.data, out.dtype, (int)size_, 0, c.stream);
+    }
+    bool takes_normed_update(const Norm* norm) const override {
+        const LayerNorm* n = dynamic_cast<const LayerNorm*>(norm);
+        return n && n->size_ == size_;
     }
     void add_norm(StepContext& c, Tensor& h, const Pending& delta, Tensor& out) override {
-        if (delta.kind == Pending::Sums) raise(TQE_ERR_STATE, "layer_norm takes no unfinished product");
-        const bool d = delta.kind == Pending::Plain;
-        K::add_layer_norm((float*)h.data, d ? delta.t.data : nullptr, d ? delta.t.dtype : 0, nullptr, (int)h.shape[0], weight(), bias(), eps_, out.data, out.dtype,
-                          (int)size_, d ? 1 : 0, c.stream);
+        run(c, h, delta, nullptr, h.shape[0], out, delta.kind == Pending::Plain);
     }
     void gather_add_norm(StepContext& c, const Tensor& h, const Pending& delta, const int32_t* rows, int64_t n_rows, Tensor& out) override {
-        if (delta.kind == Pending::Sums) raise(TQE_ERR_STATE, "layer_norm takes no unfinished product");
-        const bool d = delta.kind == Pending::Plain;
-        K::add_layer_norm((float*)h.data, d ? delta.t.data : nullptr, d ? delta.t.dtype : 0, rows, (int)n_rows, weight(), bias(), eps_, out.data, out.dtype,
-                          (int)size_, 0, c.stream);
+        run(c, h, delta, rows, n_rows, out, false);
     }
 
 private:
+    void run(StepContext& c, const Tensor& h, const Pending& delta, const int32_t* rows, int64_t n_rows, Tensor& out, bool write_back) {
+        if (delta.kind == Pending::Sums) raise(TQE_ERR_STATE, "layer_norm takes no unfinished product");
+        const bool d = delta.kind == Pending::Plain;
+        const LayerNorm* n = d && delta.norm ? dynamic_cast<const LayerNorm*>(delta.norm) : nullptr;
+        if (d && delta.norm && !n) raise(TQE_ERR_STATE, "layer_norm: an update that is to be normed by a part of kind '%s' first", delta.norm->kind.c_str());
+        K::add_layer_norm((float*)h.data, d ? delta.t.data : nullptr, d ? delta.t.dtype : 0, rows, (int)n_rows, weight(), bias(), eps_, n ? n->weight() : nullptr,
+                          n ? n->bias() : nullptr, n ? n->eps() : 0.f, out.data, out.dtype, (int)size_, write_back ? 1 : 0, c.stream);
+    }
+
     int act_dtype_;
+    bool has_bias_ = true;
     int64_t size_;
     float eps_;
     std::string n_w_, n_b_;

@@ -70,6 +70,7 @@ Json CacheNeed::to_json() const {
         j.set("key_page", shape_json(key_page));
         j.set("value_page", shape_json(value_page));
         j.set("window", window > 0 ? Json(window) : Json());
+        if (chunk > 0) j.set("chunk", chunk);
         if (keep_first > 0) j.set("keep_first", keep_first);
         if (has_state()) {
             j.set("state_shape", shape_json(state_shape));
@@ -93,6 +94,8 @@ CacheNeed CacheNeed::from_json(const Json& j) {
         n.value_page = shape_from(j["value_page"], "cache need");
         if (j["window"].is_int()) n.window = (int)j["window"].as_int();
         if (n.window < 0) raise(TQE_ERR_ARGUMENT, "cache need: window %d", n.window);
+        if (j["chunk"].is_int()) n.chunk = (int)j["chunk"].as_int();
+        if (n.chunk < 0) raise(TQE_ERR_ARGUMENT, "cache need: chunk %d", n.chunk);
         if (j["keep_first"].is_int()) n.keep_first = (int)j["keep_first"].as_int();
         if (n.keep_first < 0) raise(TQE_ERR_ARGUMENT, "cache need: keep_first %d", n.keep_first);
         if (!j["state_shape"].is_null()) {

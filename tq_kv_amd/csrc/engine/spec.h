@@ -52,14 +52,15 @@ struct CacheNeed {
     int kind = None;
     std::vector<int64_t> key_page, value_page;
     int window = 0;
+    int chunk = 0;               // positions fall into chunks of so many, and only those of the newest position's chunk are ever read again
     int keep_first = 0;          // with a window: the sequence's first positions that stay visible whatever the window
     std::vector<int64_t> state_shape;
     int state_dtype = F32;
     bool has_state() const { return !state_shape.empty(); }
-    bool same_pages(const CacheNeed& o) const { return key_page == o.key_page && value_page == o.value_page && window == o.window && keep_first == o.keep_first; }
+    bool same_pages(const CacheNeed& o) const { return key_page == o.key_page && value_page == o.value_page && window == o.window && chunk == o.chunk && keep_first == o.keep_first; }
     bool same_state(const CacheNeed& o) const { return state_shape == o.state_shape && state_dtype == o.state_dtype; }
     bool operator==(const CacheNeed& o) const {
-        return kind == o.kind && key_page == o.key_page && value_page == o.value_page && window == o.window && keep_first == o.keep_first &&
+        return kind == o.kind && key_page == o.key_page && value_page == o.value_page && window == o.window && chunk == o.chunk && keep_first == o.keep_first &&
                state_shape == o.state_shape && state_dtype == o.state_dtype;
     }
     Json to_json() const;

@@ -67,6 +67,8 @@ CacheStore::CacheStore(const std::vector<CacheNeed>& needs, const std::vector<in
     if (!book) throw Error(TQE_ERR_ARGUMENT, tqe_last_error());
     for (size_t g = 0; g < page_groups.size(); ++g)
         if (page_groups[g].need.keep_first > 0) check_status(tqe_cache_keep_first(book, (int)g, page_groups[g].need.keep_first));
+    for (size_t g = 0; g < page_groups.size(); ++g)
+        if (page_groups[g].need.chunk > 0) check_status(tqe_cache_chunk(book, (int)g, page_groups[g].need.chunk));
 
     // what each run sees
     entries_.assign(n_runs, CacheEntry());
@@ -93,6 +95,7 @@ CacheStore::CacheStore(const std::vector<CacheNeed>& needs, const std::vector<in
             const PageGroup& g = page_groups[(size_t)p.page_group];
             e.group = p.page_group;
             e.window = need.window;
+            e.chunk = need.chunk;
             e.keep_first = need.keep_first;
             e.keys = g.keys->t.slice(p.page_index, p.page_index + 1);
             e.values = g.values->t.slice(p.page_index, p.page_index + 1);

@@ -40,6 +40,9 @@ struct GroupedArgs {
     long long y_row_stride, y_group_stride;
     const float* row_scale;         // y[row, group] is multiplied by row_scale[row * scale_row_stride + group] (or null)
     long long scale_row_stride;
+    const void* out_gate;           // y[row, group, n] is multiplied by the sigmoid of out_gate[row * gate_row_stride + group * N + n] (or null)
+    int out_gate_f32;
+    long long gate_row_stride;
     int N, K;
     int gate;
     float gate_limit, gate_alpha;
@@ -211,6 +214,11 @@ void grouped_mfma_kernel(GroupedArgs p) {
                     v = act_value(p.gate, p.gate_limit, p.gate_alpha, to_float(from_float<bf16_t>(v)));
                 }
                 v *= scale;
+                if (p.out_gate) {
+                    const long long ga = row * p.gate_row_stride + (long long)group * p.N + n;
+                    const float z = p.out_gate_f32 ? ((const float*)p.out_gate)[ga] : to_float(((const bf16_t*)p.out_gate)[ga]);
+                    v *= 1.f / (1.f + expf(-z));
+                }
                 const long long at = row * p.y_row_stride + (long long)group * p.y_group_stride + n;
                 if (p.y_f32) ((float*)p.y)[at] = v;
                 else ((bf16_t*)p.y)[at] = from_float<bf16_t>(v);
@@ -260,10 +268,11 @@ extern "C" int tqk_moe_product_mfma(const void* x, const int32_t* x_rows, const 
 
 /* y[t, h, :N] = scale[t, h] * W_h x[t, h, :K] for every token t and head h.  x: [tokens, heads, x_head_stride...] rows of
  * x_row_stride values, bfloat16 or float32 (x_f32); w: [heads][N][K] bfloat16; y likewise with its own strides;
- * scale [tokens, heads] float32 or null. */
+ * scale [tokens, heads] float32 or null; gate (bfloat16, or float32 with gate_f32; rows gate_stride apart, [heads][N]) or null: y is
+ * multiplied element by element by its sigmoid. */
 extern "C" int tqk_head_product(const void* x, int x_f32, long long x_row_stride, long long x_head_stride, const void* w, void* y, int y_f32,
-                                long long y_row_stride, long long y_head_stride, const float* scale, int n_tokens, int n_heads, int N, int K,
-                                void* stream) {
+                                long long y_row_stride, long long y_head_stride, const float* scale, const void* gate, int gate_f32, long long gate_stride,
+                                int n_tokens, int n_heads, int N, int K, void* stream) {
     TQK_REQUIRE(x && w && y, "tqk_head_product: null pointer");
     TQK_REQUIRE(n_tokens >= 0 && n_heads > 0 && N > 0 && K > 0 && K % 8 == 0, "tqk_head_product: bad sizes (N %d, K %d)", N, K);
     TQK_REQUIRE(x_row_stride % 8 == 0 && x_head_stride % 8 == 0 && ((((uintptr_t)x) | ((uintptr_t)w)) & 15) == 0,
@@ -274,6 +283,7 @@ extern "C" int tqk_head_product(const void* x, int x_f32, long long x_row_stride
     a.w = (const bf16_t*)w; a.w_group_stride = (long long)N * K;
     a.y = y; a.y_f32 = y_f32; a.y_row_stride = y_row_stride; a.y_group_stride = y_head_stride;
     a.row_scale = scale; a.scale_row_stride = n_heads;
+    a.out_gate = gate; a.out_gate_f32 = gate_f32; a.gate_row_stride = gate_stride;
     a.N = N; a.K = K;
     a.n_groups = n_heads; a.n_rows = n_tokens;
     a.tile_rows_max = n_tokens > 32 ? 64 : n_tokens > 16 ? 32 : 16;

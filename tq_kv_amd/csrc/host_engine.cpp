@@ -161,6 +161,7 @@ struct PagePool {
 struct Group {
     PagePool pool;
     int window = 0;                                   // 0: every position stays
+    int chunk = 0;                                    // positions fall into chunks: those of an earlier chunk than the next query's are let go
     int keep_first = 0;                               // with a window: pages that hold any of the first keep_first positions stay too
     std::vector<std::vector<int32_t>> pages;          // per slot: page of positions 64 i .. , -1 where given back
     std::vector<uint8_t> known;                       // per slot: whether the slot has a list at all
@@ -229,6 +230,13 @@ int tqe_cache_keep_first(tqe_cache_t* c, int group, int positions) {
     if (!c || group < 0 || group >= (int)c->groups.size() || positions < 0)
         return fail(TQE_ERR_ARGUMENT, "tqe_cache_keep_first: group %d, %d positions", group, positions);
     c->groups[group].keep_first = positions;
+    return TQE_OK;
+}
+
+int tqe_cache_chunk(tqe_cache_t* c, int group, int positions) {
+    if (!c || group < 0 || group >= (int)c->groups.size() || positions < 0)
+        return fail(TQE_ERR_ARGUMENT, "tqe_cache_chunk: group %d, %d positions", group, positions);
+    c->groups[group].chunk = positions;
     return TQE_OK;
 }
 
@@ -328,12 +336,13 @@ int tqe_cache_commit(tqe_cache_t* c, int n, const int32_t* slots, const int32_t*
         const int s = slots[i];
         c->lengths[s] += n_new[i];
         for (Group& g : c->groups) {
-            if (g.window <= 0) continue;
-            // pages whose positions are all out of the window of the next query go back
+            if (g.window <= 0 && g.chunk <= 0) continue;
+            // pages whose positions are all out of the window of the next query, or in an earlier chunk than its own, go back
             std::vector<int32_t>& have = g.pages[s];
-            const int first_needed = std::max(0, c->lengths[s] + 1 - g.window);
+            int first_needed = g.window > 0 ? std::max(0, c->lengths[s] + 1 - g.window) : 0;
+            if (g.chunk > 0) first_needed = std::max(first_needed, c->lengths[s] - c->lengths[s] % g.chunk);
             const int dead = std::min(first_needed / TQE_PAGE, (int)have.size());
-            for (int k = pages_for(g.keep_first); k < dead; ++k)
+            for (int k = pages_for(g.window > 0 ? g.keep_first : 0); k < dead; ++k)
                 if (have[k] >= 0) { g.pool.give_back(have[k]); have[k] = -1; }
         }
     }

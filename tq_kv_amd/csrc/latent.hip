@@ -11,7 +11,8 @@
 //              -> the cache row of the token's position; sigmoid of the gate logits -> gate [T, H]
 //   absorb     q [T, H, dn + dr] -> qa [T, H, rk + dr]: qa[:rk] = W_uk,h^T q[:dn], qa[rk:] = rotated q[dn:]
 //   attention  softmax((qa . row) * scale) over the window, times row[:rk] -> o [T, H, rk]
-//   values     y[t, h, :] = gate[t, h] * W_uv,h o[t, h, :]
+//   values     y[t, h, :] = gate[t, h] * W_uv,h o[t, h, :], or with a gate for every element
+// The softmax's denominator may hold exp(sink_h) too, a number per head with no key and no value.
 //
 // Norms, angles, scores, softmax weights, gates and all sums are float32; qa and o stay float32
 // between the kernels.  The order of a query's operations depends on its position alone.
@@ -25,12 +26,19 @@
 #define LAT_MAX_DK 640          // largest cache row (latent + rotated part)
 #define LAT_TT 8                // tokens a block of the absorb and values kernels takes
 
+// which element element i turns with, by which angle of the table's row (style 1: in halves, 2: in neighbouring pairs)
+struct Turn { bool first; int partner, angle; };
+__device__ __forceinline__ Turn turn_of(int i, int half, int style) {
+    if (style == 2) return {(i & 1) == 0, i ^ 1, i >> 1};
+    return {i < half, i < half ? i + half : i - half, i < half ? i : i - half};
+}
+
 // ---- split -----------------------------------------------------------------------------------
 template <typename TA, typename TW>
 __global__ __launch_bounds__(256)
 void latent_split_kernel(const TA* __restrict__ proj, int row_stride, int q_rank, int kv_rank, int rot_dim, int n_gate,
                          const TW* __restrict__ q_norm_w, const TW* __restrict__ kv_norm_w, float eps,
-                         const float* __restrict__ cos_table, const float* __restrict__ sin_table, int rot_dims, int max_positions,
+                         const float* __restrict__ cos_table, const float* __restrict__ sin_table, int rot_dims, int style, int max_positions,
                          const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos,
                          const int32_t* __restrict__ page_table, int table_width, TA* __restrict__ cache, TA* __restrict__ turned,
                          int n_pages, TA* __restrict__ cq_out, float* __restrict__ gate_out) {
@@ -38,13 +46,15 @@ void latent_split_kernel(const TA* __restrict__ proj, int row_stride, int q_rank
     const int t = blockIdx.x;
     const int kv_cols = kv_rank > 0 ? kv_rank + rot_dim : 0;
     const TA* row = proj + (size_t)t * row_stride;
-    // the query's latent
+    // the query's latent (where the queries have one)
     float ss = 0.f;
-    for (int i = threadIdx.x; i < q_rank; i += blockDim.x) { const float v = to_float(row[i]); ss = fmaf(v, v, ss); }
-    ss = block_sum(ss, scratch);
-    const float inv_q = 1.f / sqrtf(ss / (float)q_rank + eps);
-    for (int i = threadIdx.x; i < q_rank; i += blockDim.x)
-        cq_out[(size_t)t * q_rank + i] = from_float<TA>(to_float(row[i]) * inv_q * to_float(q_norm_w[i]));
+    if (cq_out) {
+        for (int i = threadIdx.x; i < q_rank; i += blockDim.x) { const float v = to_float(row[i]); ss = fmaf(v, v, ss); }
+        ss = block_sum(ss, scratch);
+        const float inv_q = 1.f / sqrtf(ss / (float)q_rank + eps);
+        for (int i = threadIdx.x; i < q_rank; i += blockDim.x)
+            cq_out[(size_t)t * q_rank + i] = from_float<TA>(to_float(row[i]) * inv_q * to_float(q_norm_w[i]));
+    }
     // the gates
     for (int i = threadIdx.x; i < n_gate; i += blockDim.x)
         gate_out[(size_t)t * n_gate + i] = 1.f / (1.f + expf(-to_float(row[q_rank + kv_cols + i])));
@@ -72,10 +82,10 @@ void latent_split_kernel(const TA* __restrict__ proj, int row_stride, int q_rank
         const float v = to_float(kv[kv_rank + i]);
         float r = v;
         if (i < rot_dims) {
-            const int j = i < half ? i : i - half;
-            const float c = cos_table[(size_t)p * half + j], s = sin_table[(size_t)p * half + j];
-            const float other = to_float(kv[kv_rank + (i < half ? i + half : i - half)]);
-            r = i < half ? v * c - other * s : v * c + other * s;
+            const Turn tn = turn_of(i, half, style);
+            const float c = cos_table[(size_t)p * half + tn.angle], s = sin_table[(size_t)p * half + tn.angle];
+            const float other = to_float(kv[kv_rank + tn.partner]);
+            r = tn.first ? v * c - other * s : v * c + other * s;
         }
         dst[kv_rank + i] = from_float<TA>(r);
     }
@@ -86,15 +96,15 @@ void latent_split_kernel(const TA* __restrict__ proj, int row_stride, int q_rank
 // of W_uk are read along their columns, so a wave's loads are contiguous.
 template <typename TA, typename TW>
 __global__ __launch_bounds__(128)
-void latent_absorb_kernel(const TA* __restrict__ q, const TW* __restrict__ w_uk, int n_heads, int dn, int dr, int rk,
-                          const float* __restrict__ cos_table, const float* __restrict__ sin_table, int rot_dims, int max_positions,
+void latent_absorb_kernel(const TA* __restrict__ q, long long q_stride, const TW* __restrict__ w_uk, int n_heads, int dn, int dr, int rk,
+                          const float* __restrict__ cos_table, const float* __restrict__ sin_table, int rot_dims, int style, int max_positions,
                           const int32_t* __restrict__ tok_pos, float* __restrict__ qa, int n_tokens, int tail_only) {
     extern __shared__ float q_lds[];            // [LAT_TT][dn + dr]
     const int head = blockIdx.y, t0 = blockIdx.x * LAT_TT, d = dn + dr;
     const int n_t = min(LAT_TT, n_tokens - t0);
     for (int i = threadIdx.x; i < LAT_TT * d; i += blockDim.x) {
         const int tt = i / d, c = i % d;
-        q_lds[i] = tt < n_t ? to_float(q[((size_t)(t0 + tt) * n_heads + head) * d + c]) : 0.f;
+        q_lds[i] = tt < n_t ? to_float(q[(size_t)(t0 + tt) * q_stride + (size_t)head * d + c]) : 0.f;
     }
     __syncthreads();
     const TW* w = w_uk + (size_t)head * dn * rk;
@@ -118,9 +128,9 @@ void latent_absorb_kernel(const TA* __restrict__ q, const TW* __restrict__ w_uk,
         float r = qr[c];
         if (c < rot_dims) {
             const int p = min(tok_pos[t0 + tt], max_positions - 1);
-            const int j = c < half ? c : c - half;
-            const float cs = cos_table[(size_t)p * half + j], sn = sin_table[(size_t)p * half + j];
-            r = c < half ? qr[c] * cs - qr[c + half] * sn : qr[c] * cs + qr[c - half] * sn;
+            const Turn tn = turn_of(c, half, style);
+            const float cs = cos_table[(size_t)p * half + tn.angle], sn = sin_table[(size_t)p * half + tn.angle];
+            r = tn.first ? qr[c] * cs - qr[tn.partner] * sn : qr[c] * cs + qr[tn.partner] * sn;
         }
         qa[((size_t)(t0 + tt) * n_heads + head) * (rk + dr) + rk + c] = r;
     }
@@ -135,7 +145,8 @@ template <typename TA>
 __global__ __launch_bounds__(LAT_WAVES * TQK_WAVE)
 void latent_attention_kernel(const float* __restrict__ qa, const TA* __restrict__ cache, const int32_t* __restrict__ tok_seq,
                              const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ page_table, int table_width,
-                             int window, float scale, float* __restrict__ out, int n_tokens, int n_heads, int rk, int dk) {
+                             int window, float scale, const float* __restrict__ sink, float* __restrict__ out, int n_tokens, int n_heads, int rk,
+                             int dk) {
     __shared__ float q_lds[LAT_WAVES][LAT_MAX_DK];
     const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
     const int t = blockIdx.x * LAT_WAVES + wave;
@@ -155,7 +166,8 @@ void latent_attention_kernel(const float* __restrict__ qa, const TA* __restrict_
     float acc[NACC];
 #pragma unroll
     for (int i = 0; i < NACC; ++i) acc[i] = 0.f;
-    float m = -INFINITY, l = 0.f;
+    // the sink is a key of score sink_h without a value: the running maximum and sum start from it
+    float m = sink ? sink[head] : -INFINITY, l = sink ? 1.f : 0.f;
     for (int kb = (lo / TQK_PAGE) * TQK_PAGE; kb <= pos; kb += TQK_PAGE) {
         const int page = pages[kb / TQK_PAGE];
         const int j = kb + lane;
@@ -221,7 +233,7 @@ template <int KS, int NCT, int WAVES>
 __global__ __launch_bounds__(WAVES * TQK_WAVE)
 void latent_attention_mfma_kernel(const float* __restrict__ qa, const bf16_t* __restrict__ cache, const bf16_t* __restrict__ turned,
                                   const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos,
-                                  const int32_t* __restrict__ page_table, int table_width, int window, float scale,
+                                  const int32_t* __restrict__ page_table, int table_width, int window, float scale, const float* __restrict__ sink,
                                   float* __restrict__ out, int n_tokens, int n_heads, int n_chunks, int rk, int dk, int n_parts,
                                   float* __restrict__ part_o, float* __restrict__ part_ml) {
     __shared__ uint4 q_lds[WAVES][KS][TQK_WAVE];
@@ -255,7 +267,9 @@ void latent_attention_mfma_kernel(const float* __restrict__ qa, const bf16_t* __
     lat_floatx4_t o[NCT];
 #pragma unroll
     for (int ct = 0; ct < NCT; ++ct) o[ct] = lat_floatx4_t{0.f, 0.f, 0.f, 0.f};
-    float m = -INFINITY, l = 0.f;
+    // the sink is a key of score sink_h without a value: the running maximum and sum start from it (with several parts the merge adds it)
+    const bool sunk = sink && n_parts == 1;
+    float m = sunk ? sink[min(head, n_heads - 1)] : -INFINITY, l = sunk ? 1.f : 0.f;
 
     for (int kb = (lo / TQK_PAGE + part) * TQK_PAGE; kb <= pos; kb += TQK_PAGE * n_parts) {
         const int page = max(0, pages[kb / TQK_PAGE]);
@@ -366,7 +380,7 @@ template <int KS, int NCT>
 __global__ __launch_bounds__(4 * TQK_WAVE)
 void latent_attention_page_kernel(const float* __restrict__ qa, const bf16_t* __restrict__ cache, const bf16_t* __restrict__ turned,
                                   const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos,
-                                  const int32_t* __restrict__ page_table, int table_width, int window, float scale,
+                                  const int32_t* __restrict__ page_table, int table_width, int window, float scale, const float* __restrict__ sink,
                                   float* __restrict__ out, int n_heads, int n_chunks, int rk, int dk, int n_parts,
                                   float* __restrict__ part_o, float* __restrict__ part_ml) {
     constexpr int CT = NCT / 4;                         // 16-element blocks of the latent a wave takes
@@ -401,7 +415,9 @@ void latent_attention_page_kernel(const float* __restrict__ qa, const bf16_t* __
     lat_floatx4_t o[CT];
 #pragma unroll
     for (int c = 0; c < CT; ++c) o[c] = lat_floatx4_t{0.f, 0.f, 0.f, 0.f};
-    float m = -INFINITY, l = 0.f;
+    // the sink is a key of score sink_h without a value: the running maximum and sum start from it (with several parts the merge adds it)
+    const bool sunk = sink && n_parts == 1;
+    float m = sunk ? sink[min(head, n_heads - 1)] : -INFINITY, l = sunk ? 1.f : 0.f;
 
     for (int kb = (lo / TQK_PAGE + part) * TQK_PAGE; kb <= pos; kb += TQK_PAGE * n_parts) {
         const int page = max(0, pages[kb / TQK_PAGE]);
@@ -496,7 +512,8 @@ void latent_attention_page_kernel(const float* __restrict__ qa, const bf16_t* __
 // the parts of a (token, head) in their order: out = sum_p o_p e^(m_p - M) / sum_p l_p e^(m_p - M)
 #define LAT_MAX_PARTS 128
 __global__ __launch_bounds__(128)
-void latent_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, int n_parts, int rk, float* __restrict__ out) {
+void latent_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, int n_parts, int rk, int n_heads,
+                         const float* __restrict__ sink, float* __restrict__ out) {
     __shared__ float wgt[LAT_MAX_PARTS];
     __shared__ float total;
     const size_t row = blockIdx.x;
@@ -506,13 +523,14 @@ void latent_merge_kernel(const float* __restrict__ part_o, const float* __restri
     const float mine_l = threadIdx.x < n_parts ? ml[2 * threadIdx.x + 1] : 0.f;
     if (threadIdx.x < LAT_MAX_PARTS) wgt[threadIdx.x] = mine;
     __syncthreads();
-    float M = -INFINITY;
+    const float sk = sink ? sink[row % n_heads] : -INFINITY;
+    float M = sk;
     for (int p = 0; p < n_parts; ++p) M = fmaxf(M, wgt[p]);
     __syncthreads();
     if (threadIdx.x < LAT_MAX_PARTS) wgt[threadIdx.x] = threadIdx.x < n_parts ? expf(mine - M) : 0.f;
     __syncthreads();
     if (threadIdx.x == 0) {
-        float L = 0.f;
+        float L = sink ? expf(sk - M) : 0.f;
         for (int p = 0; p < n_parts; ++p) L += part_ml[(row * n_parts + p) * 2 + 1] * wgt[p];
         total = L;
     }
@@ -541,7 +559,8 @@ __global__ __launch_bounds__(4 * TQK_WAVE)
 void latent_attention_tile_kernel(const float* __restrict__ qa, const bf16_t* __restrict__ cache, const bf16_t* __restrict__ turned,
                                   const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ page_table, int table_width,
                                   const int32_t* __restrict__ tile_seq, const int32_t* __restrict__ tile_tok0,
-                                  const int32_t* __restrict__ tile_count, int window, float scale, float* __restrict__ out, int n_heads,
+                                  const int32_t* __restrict__ tile_count, int window, float scale, const float* __restrict__ sink,
+                                  float* __restrict__ out, int n_heads,
                                   int rk, int dk) {
     constexpr int KP = (128 * KS + 255) / 256;          // 16-byte pieces of half a page of rows a thread brings
     constexpr int VP = NCT / 4;                         // and of turned latents
@@ -577,7 +596,7 @@ void latent_attention_tile_kernel(const float* __restrict__ qa, const bf16_t* __
     lat_floatx4_t o[NCT];
 #pragma unroll
     for (int ct = 0; ct < NCT; ++ct) o[ct] = lat_floatx4_t{0.f, 0.f, 0.f, 0.f};
-    float m = -INFINITY, l = 0.f;
+    float m = sink ? sink[min(head, n_heads - 1)] : -INFINITY, l = sink ? 1.f : 0.f;       // (the sink: a key without a value)
 
     // A thread's pieces of half a page are those whose places in LDS follow one another from thread to thread (its
     // writes to LDS then meet no bank twice); in memory a wave's pieces are 64 contiguous bytes of each of 16 rows.
@@ -711,8 +730,8 @@ void latent_attention_tile_kernel(const float* __restrict__ qa, const bf16_t* __
 // W_uv (contiguous loads) and their partial sums are added up in a fixed order.
 template <typename TA, typename TW>
 __global__ __launch_bounds__(256)
-void latent_values_kernel(const float* __restrict__ o, const TW* __restrict__ w_uv, const float* __restrict__ gate, int n_heads, int rk,
-                          int dv, TA* __restrict__ y, int n_tokens) {
+void latent_values_kernel(const float* __restrict__ o, const TW* __restrict__ w_uv, const float* __restrict__ gate,
+                          const TA* __restrict__ element_gate, long long gate_stride, int n_heads, int rk, int dv, TA* __restrict__ y, int n_tokens) {
     extern __shared__ float o_lds[];            // [LAT_TT][rk]
     const int head = blockIdx.y, t0 = blockIdx.x * LAT_TT;
     const int n_t = min(LAT_TT, n_tokens - t0);
@@ -739,7 +758,8 @@ void latent_values_kernel(const float* __restrict__ o, const TW* __restrict__ w_
 #pragma unroll
             for (int tt = 0; tt < LAT_TT; ++tt) v = lane == tt ? acc[tt] : v;
             const int t = t0 + lane;
-            const float g = gate ? gate[(size_t)t * n_heads + head] : 1.f;
+            float g = gate ? gate[(size_t)t * n_heads + head] : 1.f;
+            if (element_gate) g *= 1.f / (1.f + expf(-to_float(element_gate[(size_t)t * gate_stride + (size_t)head * dv + n])));
             y[((size_t)t * n_heads + head) * dv + n] = from_float<TA>(v * g);
         }
     }
@@ -751,23 +771,23 @@ extern "C" int tqk_latent_max_row(void) { return LAT_MAX_DK; }
 
 extern "C" int tqk_latent_split(const void* proj, int act_dtype, int row_stride, int q_rank, int kv_rank, int rot_dim, int n_gate, const void* q_norm_w,
                                 const void* kv_norm_w, int norm_dtype, float eps, const float* cos_table, const float* sin_table,
-                                int rot_dims, int max_positions, const int32_t* tok_seq, const int32_t* tok_pos,
+                                int rot_dims, int style, int max_positions, const int32_t* tok_seq, const int32_t* tok_pos,
                                 const int32_t* page_table, int table_width, void* cache, void* turned, int n_pages, void* cq_out,
                                 float* gate_out, int n_tokens, void* stream) {
-    TQK_REQUIRE(proj && q_norm_w && cq_out, "tqk_latent_split: null pointer");
-    TQK_REQUIRE(q_rank > 0 && kv_rank >= 0 && rot_dim >= 0 && n_gate >= 0 && n_tokens >= 0, "tqk_latent_split: bad sizes");
+    TQK_REQUIRE(proj && (!cq_out || (q_norm_w && q_rank > 0)), "tqk_latent_split: null pointer");
+    TQK_REQUIRE(q_rank >= 0 && kv_rank >= 0 && rot_dim >= 0 && n_gate >= 0 && n_tokens >= 0, "tqk_latent_split: bad sizes");
     TQK_REQUIRE(n_gate == 0 || gate_out, "tqk_latent_split: no place for the gates");
     TQK_REQUIRE(row_stride >= q_rank + (kv_rank > 0 ? kv_rank + rot_dim : 0) + n_gate, "tqk_latent_split: rows of %d values are too short", row_stride);
     if (kv_rank > 0) {
         TQK_REQUIRE(kv_norm_w && cache && tok_seq && tok_pos && page_table && table_width > 0 && n_pages > 0, "tqk_latent_split: no cache to write");
         TQK_REQUIRE(rot_dims >= 0 && rot_dims <= rot_dim && rot_dims % 2 == 0, "tqk_latent_split: %d of %d elements rotate", rot_dims, rot_dim);
-        TQK_REQUIRE(rot_dims == 0 || (cos_table && sin_table && max_positions > 0), "tqk_latent_split: no angle tables");
+        TQK_REQUIRE(rot_dims == 0 || (cos_table && sin_table && max_positions > 0 && (style == 1 || style == 2)), "tqk_latent_split: no angle tables, or an unknown style");
     }
     if (n_tokens == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
 #define TQK_SPLIT(TA, TW)                                                                                                              \
     latent_split_kernel<TA, TW><<<n_tokens, 256, 0, s>>>((const TA*)proj, row_stride, q_rank, kv_rank, rot_dim, n_gate, (const TW*)q_norm_w,       \
-                                                         (const TW*)kv_norm_w, eps, cos_table, sin_table, rot_dims, max_positions,     \
+                                                         (const TW*)kv_norm_w, eps, cos_table, sin_table, rot_dims, style, max_positions, \
                                                          tok_seq, tok_pos, page_table, table_width, (TA*)cache, (TA*)turned, n_pages,  \
                                                          (TA*)cq_out, gate_out)
     if (act_dtype == TQK_F32 && norm_dtype == TQK_F32) TQK_SPLIT(float, float);
@@ -779,21 +799,22 @@ extern "C" int tqk_latent_split(const void* proj, int act_dtype, int row_stride,
     return tqk_check_launch("tqk_latent_split");
 }
 
-extern "C" int tqk_latent_absorb(const void* q, int act_dtype, const void* w_uk, int w_dtype, int n_heads, int dn, int dr, int rk,
-                                 const float* cos_table, const float* sin_table, int rot_dims, int max_positions,
+extern "C" int tqk_latent_absorb(const void* q, int act_dtype, long long q_stride, const void* w_uk, int w_dtype, int n_heads, int dn, int dr, int rk,
+                                 const float* cos_table, const float* sin_table, int rot_dims, int style, int max_positions,
                                  const int32_t* tok_pos, float* qa, int n_tokens, int tail_only, void* stream) {
     TQK_REQUIRE(q && (w_uk || tail_only) && qa && tok_pos, "tqk_latent_absorb: null pointer");
     TQK_REQUIRE(n_heads > 0 && n_heads <= 65535 && dn > 0 && dr >= 0 && rk > 0 && n_tokens >= 0, "tqk_latent_absorb: bad sizes");
     TQK_REQUIRE(rot_dims >= 0 && rot_dims <= dr && rot_dims % 2 == 0, "tqk_latent_absorb: %d of %d elements rotate", rot_dims, dr);
-    TQK_REQUIRE(rot_dims == 0 || (cos_table && sin_table && max_positions > 0), "tqk_latent_absorb: no angle tables");
+    TQK_REQUIRE(rot_dims == 0 || (cos_table && sin_table && max_positions > 0 && (style == 1 || style == 2)), "tqk_latent_absorb: no angle tables, or an unknown style");
+    TQK_REQUIRE(q_stride >= (long long)n_heads * (dn + dr), "tqk_latent_absorb: rows of %lld values are too short", q_stride);
     const size_t lds = (size_t)LAT_TT * (dn + dr) * sizeof(float);
     TQK_REQUIRE(lds <= 48 * 1024, "tqk_latent_absorb: a head of %d + %d elements is more than the kernel stages", dn, dr);
     if (n_tokens == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
     dim3 grid((n_tokens + LAT_TT - 1) / LAT_TT, n_heads);
 #define TQK_ABSORB(TA, TW)                                                                                                             \
-    latent_absorb_kernel<TA, TW><<<grid, 128, lds, s>>>((const TA*)q, (const TW*)w_uk, n_heads, dn, dr, rk, cos_table, sin_table,      \
-                                                        rot_dims, max_positions, tok_pos, qa, n_tokens, tail_only)
+    latent_absorb_kernel<TA, TW><<<grid, 128, lds, s>>>((const TA*)q, q_stride, (const TW*)w_uk, n_heads, dn, dr, rk, cos_table, sin_table, \
+                                                        rot_dims, style, max_positions, tok_pos, qa, n_tokens, tail_only)
     if (act_dtype == TQK_F32 && w_dtype == TQK_F32) TQK_ABSORB(float, float);
     else if (act_dtype == TQK_F32 && w_dtype == TQK_BF16) TQK_ABSORB(float, bf16_t);
     else if (act_dtype == TQK_BF16 && w_dtype == TQK_F32) TQK_ABSORB(bf16_t, float);
@@ -815,7 +836,7 @@ extern "C" int tqk_latent_attention_parts(int n_tokens, int n_heads, int table_w
 
 extern "C" int tqk_latent_attention_mfma(const float* qa, const void* cache, const void* turned, const int32_t* tok_seq, const int32_t* tok_pos,
                                          const int32_t* page_table, int table_width, int n_seqs, int n_pages, int window, float scale,
-                                         float* out, int n_tokens, int n_heads, int rk, int dr, int n_parts, float* part_o, float* part_ml,
+                                         const float* sink, float* out, int n_tokens, int n_heads, int rk, int dr, int n_parts, float* part_o, float* part_ml,
                                          void* stream) {
     TQK_REQUIRE(n_parts >= 1 && n_parts <= LAT_MAX_PARTS && (n_parts == 1 || (part_o && part_ml)),
                 "tqk_latent_attention_mfma: %d parts (1 to %d, with memory for them)", n_parts, LAT_MAX_PARTS);
@@ -831,13 +852,13 @@ extern "C" int tqk_latent_attention_mfma(const float* qa, const void* cache, con
     hipStream_t s = (hipStream_t)stream;
 #define TQK_LAT_MFMA(KS, NCT, WAVES)                                                                                                  \
     latent_attention_mfma_kernel<KS, NCT, WAVES><<<(unsigned)((items + WAVES - 1) / WAVES), WAVES * TQK_WAVE, 0, s>>>(                  \
-        qa, (const bf16_t*)cache, (const bf16_t*)turned, tok_seq, tok_pos, page_table, table_width, window, scale, out, n_tokens, n_heads, \
+        qa, (const bf16_t*)cache, (const bf16_t*)turned, tok_seq, tok_pos, page_table, table_width, window, scale, sink, out, n_tokens, n_heads, \
         n_chunks, rk, dk, n_parts, part_o, part_ml)
     // the smallest build that holds the row and the latent (steps and blocks beyond the sizes multiply zeros)
     // a block of four waves per (token, 16 heads, part) wherever that leaves the chip enough blocks; a wave each otherwise
 #define TQK_LAT_PAGE(KS, NCT)                                                                                                          \
     latent_attention_page_kernel<KS, NCT><<<(unsigned)items, 4 * TQK_WAVE, 0, s>>>(qa, (const bf16_t*)cache, (const bf16_t*)turned, tok_seq, \
-                                                                                   tok_pos, page_table, table_width, window, scale, out,    \
+                                                                                   tok_pos, page_table, table_width, window, scale, sink, out, \
                                                                                    n_heads, n_chunks, rk, dk, n_parts, part_o, part_ml)
     const bool by_block = items <= 16384;
     if (rk <= 128 && dk <= 160) { if (by_block) TQK_LAT_PAGE(5, 8); else TQK_LAT_MFMA(5, 8, 4); }
@@ -848,7 +869,7 @@ extern "C" int tqk_latent_attention_mfma(const float* qa, const void* cache, con
 #undef TQK_LAT_MFMA
     if (tqk_check_launch("tqk_latent_attention_mfma")) return -1;
     if (n_parts > 1) {
-        latent_merge_kernel<<<(unsigned)(n_tokens * n_heads), 128, 0, s>>>(part_o, part_ml, n_parts, rk, out);
+        latent_merge_kernel<<<(unsigned)(n_tokens * n_heads), 128, 0, s>>>(part_o, part_ml, n_parts, rk, n_heads, sink, out);
         return tqk_check_launch("tqk_latent_attention_mfma merge");
     }
     return 0;
@@ -858,7 +879,7 @@ extern "C" int tqk_latent_attention_mfma(const float* qa, const void* cache, con
  * sequence tile_seq[i], first packed token tile_tok0[i], tile_count[i] tokens), a block a tile. */
 extern "C" int tqk_latent_attention_tiles(const float* qa, const void* cache, const void* turned, const int32_t* tok_pos,
                                           const int32_t* page_table, int table_width, int n_seqs, int n_pages, const int32_t* tile_seq,
-                                          const int32_t* tile_tok0, const int32_t* tile_count, int n_tiles, int window, float scale,
+                                          const int32_t* tile_tok0, const int32_t* tile_count, int n_tiles, int window, float scale, const float* sink,
                                           float* out, int n_tokens, int n_heads, int rk, int dr, void* stream) {
     TQK_REQUIRE(qa && cache && turned && tok_pos && page_table && out && tile_seq && tile_tok0 && tile_count, "tqk_latent_attention_tiles: null pointer");
     TQK_REQUIRE(n_tokens >= 0 && n_tiles >= 0 && n_heads > 0 && rk > 0 && dr >= 0, "tqk_latent_attention_tiles: bad sizes");
@@ -872,7 +893,7 @@ extern "C" int tqk_latent_attention_tiles(const float* qa, const void* cache, co
     hipStream_t s = (hipStream_t)stream;
 #define TQK_LAT_TILE(KS, NCT)                                                                                                           \
     latent_attention_tile_kernel<KS, NCT><<<grid, 4 * TQK_WAVE, 0, s>>>(qa, (const bf16_t*)cache, (const bf16_t*)turned, tok_pos, page_table, \
-                                                                        table_width, tile_seq, tile_tok0, tile_count, window, scale, out,    \
+                                                                        table_width, tile_seq, tile_tok0, tile_count, window, scale, sink, out, \
                                                                         n_heads, rk, dk)
     if (rk <= 128 && dk <= 160) TQK_LAT_TILE(5, 8);
     else if (rk <= 256 && dk <= 320) TQK_LAT_TILE(10, 16);
@@ -884,7 +905,7 @@ extern "C" int tqk_latent_attention_tiles(const float* qa, const void* cache, co
 
 extern "C" int tqk_latent_attention(const float* qa, const void* cache, int cache_dtype, const int32_t* tok_seq, const int32_t* tok_pos,
                                     const int32_t* page_table, int table_width, int n_seqs, int n_pages, int window, float scale,
-                                    float* out, int n_tokens, int n_heads, int rk, int dr, void* stream) {
+                                    const float* sink, float* out, int n_tokens, int n_heads, int rk, int dr, void* stream) {
     TQK_REQUIRE(qa && cache && tok_seq && tok_pos && page_table && out, "tqk_latent_attention: null pointer");
     TQK_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_heads <= 65535 && rk > 0 && dr >= 0, "tqk_latent_attention: bad sizes");
     TQK_REQUIRE(rk <= LAT_MAX_RK && rk + dr <= LAT_MAX_DK, "tqk_latent_attention: a latent of %d + %d is more than %d + %d", rk, dr, LAT_MAX_RK,
@@ -895,15 +916,15 @@ extern "C" int tqk_latent_attention(const float* qa, const void* cache, int cach
     dim3 grid((n_tokens + LAT_WAVES - 1) / LAT_WAVES, n_heads);
     if (cache_dtype == TQK_F32)
         latent_attention_kernel<float><<<grid, LAT_WAVES * TQK_WAVE, 0, s>>>(qa, (const float*)cache, tok_seq, tok_pos, page_table, table_width,
-                                                                             window, scale, out, n_tokens, n_heads, rk, rk + dr);
+                                                                             window, scale, sink, out, n_tokens, n_heads, rk, rk + dr);
     else if (cache_dtype == TQK_BF16)
         latent_attention_kernel<bf16_t><<<grid, LAT_WAVES * TQK_WAVE, 0, s>>>(qa, (const bf16_t*)cache, tok_seq, tok_pos, page_table, table_width,
-                                                                              window, scale, out, n_tokens, n_heads, rk, rk + dr);
+                                                                              window, scale, sink, out, n_tokens, n_heads, rk, rk + dr);
     else return tqk_fail("tqk_latent_attention: unknown dtype %d", cache_dtype);
     return tqk_check_launch("tqk_latent_attention");
 }
 
-extern "C" int tqk_latent_values(const float* o, const void* w_uv, int w_dtype, const float* gate, int n_heads, int rk, int dv, void* y,
+extern "C" int tqk_latent_values(const float* o, const void* w_uv, int w_dtype, const float* gate, const void* element_gate, long long gate_stride, int n_heads, int rk, int dv, void* y,
                                  int y_dtype, int n_tokens, void* stream) {
     TQK_REQUIRE(o && w_uv && y, "tqk_latent_values: null pointer");
     TQK_REQUIRE(n_heads > 0 && n_heads <= 65535 && rk > 0 && dv > 0 && n_tokens >= 0, "tqk_latent_values: bad sizes");
@@ -913,7 +934,7 @@ extern "C" int tqk_latent_values(const float* o, const void* w_uv, int w_dtype, 
     hipStream_t s = (hipStream_t)stream;
     dim3 grid((n_tokens + LAT_TT - 1) / LAT_TT, n_heads);
 #define TQK_VALUES(TA, TW) \
-    latent_values_kernel<TA, TW><<<grid, 256, lds, s>>>(o, (const TW*)w_uv, gate, n_heads, rk, dv, (TA*)y, n_tokens)
+    latent_values_kernel<TA, TW><<<grid, 256, lds, s>>>(o, (const TW*)w_uv, gate, (const TA*)element_gate, gate_stride, n_heads, rk, dv, (TA*)y, n_tokens)
     if (y_dtype == TQK_F32 && w_dtype == TQK_F32) TQK_VALUES(float, float);
     else if (y_dtype == TQK_F32 && w_dtype == TQK_BF16) TQK_VALUES(float, bf16_t);
     else if (y_dtype == TQK_BF16 && w_dtype == TQK_F32) TQK_VALUES(bf16_t, float);

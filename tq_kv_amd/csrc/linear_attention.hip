@@ -1,6 +1,7 @@
 // Linear attention with a decaying state: per head S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, with S of d rows (key
 // channels) and dv columns in float32.  The decay a_t is one number per head (fixed) or one per key channel and token, formed here
-// from a product z as sigmoid(z + bias)^(1/tau) = exp(logsigmoid(z + bias) / tau).  q and k may be turned by the position (tables of
+// from a product z as sigmoid(z + bias)^(1/tau) = exp(logsigmoid(z + bias) / tau), or one number per head and token given by its
+// logarithm (log_decay; then k may be weighted by exp(log_in) and the output multiplied by out_scale, per head and token too).  q and k may be turned by the position (tables of
 // cos and sin, in halves or neighbouring pairs over the first rot_dim elements) and scaled on their way in; everything after the
 // loads is float32.
 //
@@ -10,7 +11,8 @@
 // long steps chunks of consecutive tokens: local (every chunk from a zero state; its last state and the product of its decays are
 // left for tqk_chunk_carry) and apply (every chunk again from the state it starts from, with the outputs).
 //
-// tqk_head_norm_gate: out = o / rms(o) (per head, times a weight over the head's columns if given) * silu(gate).
+// tqk_head_norm_gate: out = o / rms(o) (per head, times a weight over the head's columns, or all heads' columns, if given) * silu(gate) or
+// sigmoid(gate).
 #include "common.h"
 #include "tq_kernels.h"
 
@@ -27,6 +29,7 @@ struct LaArgs {
     const float* z_bias;
     float inv_tau;
     const float* head_decay;
+    const float *log_decay, *log_in, *out_scale;        // [tokens, heads] or null
     float q_scale, k_scale;
     const float *cos, *sin;
     int rot_dim, style, max_pos;
@@ -38,6 +41,7 @@ struct LaArgs {
     float *chunk_state, *chunk_decay;
     float* out;
     int H, d, dv;
+    long long head_stride;          // elements between the heads' parts of a state
 };
 
 template <typename T, int RT, int MODE>
@@ -53,7 +57,7 @@ void linear_attention_kernel(LaArgs a, int rg_shift) {
     if (MODE == LA_SCAN) { row0 = a.cu[item]; count = a.seq_new[item]; }
     else { row0 = a.chunk_row0[item]; count = a.chunk_count[item]; }
     if (count <= 0) return;
-    const size_t per_head = (size_t)d * dv;
+    const size_t per_head = (size_t)a.head_stride;
     float* sp = MODE == LA_SCAN ? a.state + (size_t)a.seq_slot[item] * a.state_stride + head * per_head
                                 : a.chunk_state + ((size_t)item * H + head) * per_head;
     float S[RT], P[RT];
@@ -97,6 +101,9 @@ void linear_attention_kernel(LaArgs a, int rg_shift) {
                 const float zz = a.z[row * a.z_stride + (size_t)head * d + i] + a.z_bias[(size_t)head * d + i];
                 const float ls = fminf(zz, 0.f) - log1pf(expf(-fabsf(zz)));
                 al = expf(ls * a.inv_tau);
+            } else if (a.log_decay) {
+                al = expf(a.log_decay[row * H + head]);
+                if (a.log_in) lk[e] *= expf(a.log_in[row * H + head]);
             } else al = a.head_decay[head];
             ld[e] = al;
         }
@@ -119,7 +126,7 @@ void linear_attention_kernel(LaArgs a, int rg_shift) {
             }
             if (MODE != LA_LOCAL) {
                 for (int m = RG >> 1; m > 0; m >>= 1) o += __shfl_xor(o, m, TQK_WAVE);
-                if (rg == 0 && col_ok) a.out[((size_t)row * H + head) * dv + col] = o;
+                if (rg == 0 && col_ok) a.out[((size_t)row * H + head) * dv + col] = a.out_scale ? o * a.out_scale[row * H + head] : o;
             }
         }
     }
@@ -149,7 +156,7 @@ void linear_attention_block_kernel(LaArgs a, int rg_shift, int cb) {
     if (MODE == LA_SCAN) { row0 = a.cu[item]; count = a.seq_new[item]; }
     else { row0 = a.chunk_row0[item]; count = a.chunk_count[item]; }
     if (count <= 0) return;
-    const size_t per_head = (size_t)d * dv;
+    const size_t per_head = (size_t)a.head_stride;
     float* sp = MODE == LA_SCAN ? a.state + (size_t)a.seq_slot[item] * a.state_stride + head * per_head
                                 : a.chunk_state + ((size_t)item * H + head) * per_head;
     float S[RT][4], P[RT];
@@ -197,6 +204,9 @@ void linear_attention_block_kernel(LaArgs a, int rg_shift, int cb) {
                     const float zz = a.z[row * a.z_stride + (size_t)head * d + i] + a.z_bias[(size_t)head * d + i];
                     const float ls = fminf(zz, 0.f) - log1pf(expf(-fabsf(zz)));
                     al = expf(ls * a.inv_tau);
+                } else if (a.log_decay) {
+                    al = expf(a.log_decay[row * H + head]);
+                    if (a.log_in) kv *= expf(a.log_in[row * H + head]);
                 } else al = a.head_decay[head];
             }
             lq[e] = qv;
@@ -235,6 +245,11 @@ void linear_attention_block_kernel(LaArgs a, int rg_shift, int cb) {
                         for (int m = RG >> 1; m > 0; m >>= 1) o[c] += __shfl_xor(o[c], m, TQK_WAVE);
                     if (rg == 0 && col_ok) {
                         float* dst = a.out + ((size_t)(row0 + t0 + tt) * H + head) * dv + col0;
+                        if (a.out_scale) {
+                            const float os = a.out_scale[(size_t)(row0 + t0 + tt) * H + head];
+#pragma unroll
+                            for (int c = 0; c < 4; ++c) o[c] *= os;
+                        }
 #pragma unroll
                         for (int c = 0; c < 4; ++c) dst[c] = o[c];
                     }
@@ -254,11 +269,12 @@ void linear_attention_block_kernel(LaArgs a, int rg_shift, int cb) {
     }
 }
 
-// out[t, h, j] = o[t, h, j] / sqrt(mean_j o[t, h]^2 + eps) * w[j] * silu(gate[t, h * dv + j]); a wave per (token, head)
+// out[t, h, j] = o[t, h, j] / sqrt(mean_j o[t, h]^2 + eps) * w[h * w_stride + j] * f(gate[t, h * dv + j]), f silu or the sigmoid alone; a wave
+// per (token, head)
 template <typename TG, typename TO>
 __global__ __launch_bounds__(256)
-void head_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ w, float eps, const TG* __restrict__ gate, long long gate_stride,
-                           TO* __restrict__ out, long long n_pairs, int H, int dv) {
+void head_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ w, int w_stride, float eps, const TG* __restrict__ gate,
+                           long long gate_stride, int sigmoid, TO* __restrict__ out, long long n_pairs, int H, int dv) {
     const long long pair = (long long)blockIdx.x * (256 / TQK_WAVE) + threadIdx.x / TQK_WAVE;
     if (pair >= n_pairs) return;
     const int lane = threadIdx.x % TQK_WAVE;
@@ -272,8 +288,8 @@ void head_norm_gate_kernel(const float* __restrict__ o, const float* __restrict_
     for (int j = lane; j < dv; j += TQK_WAVE) {
         const float g = gate ? to_float(gate[t * gate_stride + (size_t)h * dv + j]) : 0.f;
         float v = orow[j] * inv;
-        if (w) v *= w[j];
-        if (gate) v *= g / (1.f + expf(-g));
+        if (w) v *= w[(size_t)h * w_stride + j];
+        if (gate) v *= (sigmoid ? 1.f : g) / (1.f + expf(-g));
         out[(size_t)pair * dv + j] = from_float<TO>(v);
     }
 }
@@ -281,13 +297,15 @@ void head_norm_gate_kernel(const float* __restrict__ o, const float* __restrict_
 extern "C" int tqk_linear_attention_max_dim(void) { return 512; }
 
 extern "C" int tqk_linear_attention(const void* q, const void* k, const void* v, int act_dtype, long long stride, const float* z, long long z_stride,
-                                    const float* z_bias, float inv_tau, const float* head_decay, float q_scale, float k_scale, const float* cos,
+                                    const float* z_bias, float inv_tau, const float* head_decay, const float* log_decay, const float* log_in,
+                                    const float* out_scale, float q_scale, float k_scale, const float* cos,
                                     const float* sin, int rot_dim, int style, int max_pos, const int32_t* tok_pos, float* state, long long state_stride,
                                     const int32_t* cu, const int32_t* seq_new, const int32_t* seq_slot, const int32_t* chunk_row0,
                                     const int32_t* chunk_count, float* chunk_state, float* chunk_decay, float* out, int mode, int n_items, int heads,
-                                    int d, int dv, void* stream) {
+                                    int d, int dv, long long head_stride, void* stream) {
     TQK_REQUIRE(q && k && v, "tqk_linear_attention: null pointer");
-    TQK_REQUIRE((z && z_bias) || head_decay, "tqk_linear_attention: neither a decay per channel nor one per head");
+    TQK_REQUIRE((z && z_bias) || head_decay || log_decay, "tqk_linear_attention: neither a decay per channel nor one per head");
+    TQK_REQUIRE(head_stride >= (long long)d * dv, "tqk_linear_attention: heads' states overlap");
     TQK_REQUIRE(mode >= LA_SCAN && mode <= LA_APPLY, "tqk_linear_attention: unknown mode %d", mode);
     TQK_REQUIRE(mode == LA_SCAN ? (state && cu && seq_new && seq_slot) : (chunk_row0 && chunk_count && chunk_state && chunk_decay),
                 "tqk_linear_attention: mode %d lacks its arrays", mode);
@@ -297,8 +315,8 @@ extern "C" int tqk_linear_attention(const void* q, const void* k, const void* v,
     TQK_REQUIRE(!cos || (sin && tok_pos && rot_dim > 0 && rot_dim % 2 == 0 && rot_dim <= d && max_pos > 0 && (style == LA_STYLE_HALVES || style == LA_STYLE_PAIRS)),
                 "tqk_linear_attention: bad rotation");
     if (n_items == 0) return 0;
-    LaArgs a = {q, k, v, stride, z, z_stride, z_bias, inv_tau, head_decay, q_scale, k_scale, cos, sin, rot_dim, style, max_pos, tok_pos, state, state_stride,
-                cu, seq_new, seq_slot, chunk_row0, chunk_count, chunk_state, chunk_decay, out, heads, d, dv};
+    LaArgs a = {q, k, v, stride, z, z_stride, z_bias, inv_tau, head_decay, log_decay, log_in, out_scale, q_scale, k_scale, cos, sin, rot_dim, style, max_pos, tok_pos,
+                state, state_stride, cu, seq_new, seq_slot, chunk_row0, chunk_count, chunk_state, chunk_decay, out, heads, d, dv, head_stride};
     hipStream_t s = (hipStream_t)stream;
     if (d % 4 == 0 && dv % 4 == 0 && dv >= 16 && (((uintptr_t)out) & 15) == 0) {
         // a thread holds rt rows by four columns: rt = 16 where the head has the rows for it, and as many row groups as cover the head
@@ -348,7 +366,8 @@ extern "C" int tqk_linear_attention(const void* q, const void* k, const void* v,
     return tqk_check_launch("tqk_linear_attention");
 }
 
-extern "C" int tqk_head_norm_gate(const float* o, const float* weight, float eps, const void* gate, int gate_dtype, long long gate_stride, void* out,
+extern "C" int tqk_head_norm_gate(const float* o, const float* weight, int weight_stride, float eps, const void* gate, int gate_dtype, long long gate_stride,
+                                  int sigmoid, void* out,
                                   int out_dtype, int n_tokens, int heads, int dv, void* stream) {
     TQK_REQUIRE(o && out, "tqk_head_norm_gate: null pointer");
     TQK_REQUIRE(n_tokens >= 0 && heads > 0 && dv > 0, "tqk_head_norm_gate: bad sizes");
@@ -357,7 +376,7 @@ extern "C" int tqk_head_norm_gate(const float* o, const float* weight, float eps
     const long long blocks = (pairs + 3) / 4;
     TQK_REQUIRE(blocks <= 0x7fffffff, "tqk_head_norm_gate: too many rows");
     hipStream_t s = (hipStream_t)stream;
-#define TQK_HNG(TG, TO) head_norm_gate_kernel<TG, TO><<<(unsigned)blocks, 256, 0, s>>>(o, weight, eps, (const TG*)gate, gate_stride, (TO*)out, pairs, heads, dv)
+#define TQK_HNG(TG, TO) head_norm_gate_kernel<TG, TO><<<(unsigned)blocks, 256, 0, s>>>(o, weight, weight_stride, eps, (const TG*)gate, gate_stride, sigmoid, (TO*)out, pairs, heads, dv)
     if (gate_dtype == TQK_F32 && out_dtype == TQK_F32) TQK_HNG(float, float);
     else if (gate_dtype == TQK_BF16 && out_dtype == TQK_BF16) TQK_HNG(bf16_t, bf16_t);
     else if (gate_dtype == TQK_F32 && out_dtype == TQK_BF16) TQK_HNG(float, bf16_t);

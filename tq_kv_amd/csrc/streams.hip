@@ -6,7 +6,9 @@
 //                       X'[t, r] = sum_s mix[s, r] X[t, s] + out[r] y[t]; then (where `in` is given) what the next part reads,
 //                       u = sum_s in[s] X'[t, s], left as it is in u_out and / or normed, (u - mean) / sqrt(var + eps) w + b, in n_out.
 //                       The variance is the mean of the squared deviations from the mean (two passes over a row kept in LDS).
-//   tqk_add_layer_norm  out[i] = LN(h[rows[i]] + delta[rows[i]]) (rows null: row i; h or delta may be missing; write_back: h keeps the sum)
+//   tqk_add_layer_norm  out[i] = LN(h[rows[i]] + delta[rows[i]]) (rows null: row i; h or delta may be missing; write_back: h keeps the sum);
+//                       the update may be normed itself before it is added: a part's output norm, the residual sum and the next part's norm
+//                       in one pass.  A norm's bias may be missing.
 //   tqk_token_shift     out[t] = n[t] + (n[t - 1] - n[t]) mu, the row before a sequence's first token of the step taken from the
 //                       sequence's state (zeros before its first token); `remember` (steps of one token a sequence) also leaves n[t] there
 //   tqk_shift_remember  state of sequence s = n[last token the step brings of s]
@@ -80,29 +82,159 @@ void streams_step_kernel(float* __restrict__ X, int S, const TY* __restrict__ y,
     float ss = 0.f;
     for (int e = threadIdx.x; e < W; e += blockDim.x) { const float dlt = row_u[e] - mean; ss = fmaf(dlt, dlt, ss); }
     const float inv = 1.f / sqrtf(block_sum(ss, scratch) / (float)W + eps);
-    for (int e = threadIdx.x; e < W; e += blockDim.x) n_out[t * W + e] = from_float<TN>((row_u[e] - mean) * inv * nw[e] + nb[e]);
+    for (int e = threadIdx.x; e < W; e += blockDim.x) n_out[t * W + e] = from_float<TN>((row_u[e] - mean) * inv * nw[e] + (nb ? nb[e] : 0.f));
 }
+
+// The update of a row may be normed itself before it is added (pw given): h += (d - mean d) / sqrt(var d + peps) pw + pb.
+struct LayerNormArgs {
+    float* h;
+    const void* delta;
+    const int32_t* rows;
+    const float *w, *b;
+    float eps;
+    const float *pw, *pb;
+    float peps;
+    void* out;
+    int W, write_back;
+};
 
 template <typename TD, typename TO>
 __global__ __launch_bounds__(256)
-void add_layer_norm_kernel(float* __restrict__ h, const TD* __restrict__ delta, const int32_t* __restrict__ rows, const float* __restrict__ w,
-                           const float* __restrict__ b, float eps, TO* __restrict__ out, int W, int write_back) {
+void add_layer_norm_kernel(const LayerNormArgs a) {
     extern __shared__ float row_u[];
     __shared__ float scratch[4];
-    const size_t i = blockIdx.x, r = rows ? (size_t)rows[i] : i;
+    const int W = a.W;
+    const size_t i = blockIdx.x, r = a.rows ? (size_t)a.rows[i] : i;
+    const TD* delta = (const TD*)a.delta;
+    float pmean = 0.f, pinv = 1.f;
+    if (a.pw) {
+        float sum = 0.f;
+        for (int e = threadIdx.x; e < W; e += blockDim.x) sum += to_float(delta[r * W + e]);
+        pmean = block_sum(sum, scratch) / (float)W;
+        float ss = 0.f;
+        for (int e = threadIdx.x; e < W; e += blockDim.x) { const float dlt = to_float(delta[r * W + e]) - pmean; ss = fmaf(dlt, dlt, ss); }
+        pinv = 1.f / sqrtf(block_sum(ss, scratch) / (float)W + a.peps);
+    }
     float sum = 0.f;
     for (int e = threadIdx.x; e < W; e += blockDim.x) {
-        float v = h ? h[r * W + e] : 0.f;
-        if (delta) v += to_float(delta[r * W + e]);
-        if (write_back && h) h[r * W + e] = v;
+        float v = a.h ? a.h[r * W + e] : 0.f;
+        if (delta) {
+            float d = to_float(delta[r * W + e]);
+            if (a.pw) d = (d - pmean) * pinv * a.pw[e] + (a.pb ? a.pb[e] : 0.f);
+            v += d;
+        }
+        if (a.write_back && a.h) a.h[r * W + e] = v;
         row_u[e] = v;
         sum += v;
     }
     const float mean = block_sum(sum, scratch) / (float)W;
     float ss = 0.f;
     for (int e = threadIdx.x; e < W; e += blockDim.x) { const float dlt = row_u[e] - mean; ss = fmaf(dlt, dlt, ss); }
-    const float inv = 1.f / sqrtf(block_sum(ss, scratch) / (float)W + eps);
-    for (int e = threadIdx.x; e < W; e += blockDim.x) out[i * W + e] = from_float<TO>((row_u[e] - mean) * inv * w[e] + b[e]);
+    const float inv = 1.f / sqrtf(block_sum(ss, scratch) / (float)W + a.eps);
+    TO* out = (TO*)a.out;
+    for (int e = threadIdx.x; e < W; e += blockDim.x) out[i * W + e] = from_float<TO>((row_u[e] - mean) * inv * a.w[e] + (a.b ? a.b[e] : 0.f));
+}
+
+// The same for rows that fall into pieces of four elements, a thread NV of them: the update and the sum stay in registers between the
+// sums over the row, whose partial results meet in LDS behind one barrier each.
+__device__ __forceinline__ void load4(const float* p, float (&v)[4]) {
+    const float4 x = *reinterpret_cast<const float4*>(p);
+    v[0] = x.x; v[1] = x.y; v[2] = x.z; v[3] = x.w;
+}
+__device__ __forceinline__ void load4(const bf16_t* p, float (&v)[4]) {
+    const uint2 x = *reinterpret_cast<const uint2*>(p);
+    v[0] = __uint_as_float(x.x << 16); v[1] = __uint_as_float(x.x & 0xffff0000u);
+    v[2] = __uint_as_float(x.y << 16); v[3] = __uint_as_float(x.y & 0xffff0000u);
+}
+__device__ __forceinline__ void store4(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+__device__ __forceinline__ void store4(bf16_t* p, const float (&v)[4]) {
+    *reinterpret_cast<uint2*>(p) = make_uint2((uint32_t)float_to_bf16_bits(v[0]) | ((uint32_t)float_to_bf16_bits(v[1]) << 16),
+                                              (uint32_t)float_to_bf16_bits(v[2]) | ((uint32_t)float_to_bf16_bits(v[3]) << 16));
+}
+// (slots: a place of its own for every sum of the kernel, so that one barrier is enough)
+__device__ __forceinline__ float row_sum(float v, float* slots) {
+    v = wave_sum(v);
+    if ((threadIdx.x & (TQK_WAVE - 1)) == 0) slots[threadIdx.x / TQK_WAVE] = v;
+    __syncthreads();
+    float total = 0.f;
+    for (int w = 0; w < (int)(blockDim.x / TQK_WAVE); ++w) total += slots[w];
+    return total;
+}
+
+template <typename TD, typename TO, int NV>
+__global__ __launch_bounds__(1024)
+void add_layer_norm_vec_kernel(const LayerNormArgs a) {
+    __shared__ float slots[4][16];
+    const int W = a.W, n4 = W / 4;
+    const size_t i = blockIdx.x, r = a.rows ? (size_t)a.rows[i] : i;
+    const TD* delta = a.delta ? (const TD*)a.delta + r * W : nullptr;
+    float* h = a.h ? a.h + r * W : nullptr;
+    float d[NV][4], x[NV][4];
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+        const int c = threadIdx.x + k * blockDim.x;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) d[k][j] = x[k][j] = 0.f;
+        if (c < n4) {
+            if (delta) load4(delta + 4 * c, d[k]);
+            if (h) load4(h + 4 * c, x[k]);
+        }
+    }
+    if (a.pw) {
+        float sum = 0.f;
+#pragma unroll
+        for (int k = 0; k < NV; ++k)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) sum += d[k][j];
+        const float mean = row_sum(sum, slots[0]) / (float)W;
+        float ss = 0.f;
+#pragma unroll
+        for (int k = 0; k < NV; ++k)
+            if (threadIdx.x + k * blockDim.x < n4) {
+#pragma unroll
+                for (int j = 0; j < 4; ++j) { const float dlt = d[k][j] - mean; ss = fmaf(dlt, dlt, ss); }
+            }
+        const float inv = 1.f / sqrtf(row_sum(ss, slots[1]) / (float)W + a.peps);
+#pragma unroll
+        for (int k = 0; k < NV; ++k) {
+            const int c = threadIdx.x + k * blockDim.x;
+            if (c >= n4) continue;
+            float w4[4], b4[4] = {0.f, 0.f, 0.f, 0.f};
+            load4(a.pw + 4 * c, w4);
+            if (a.pb) load4(a.pb + 4 * c, b4);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) d[k][j] = (d[k][j] - mean) * inv * w4[j] + b4[j];
+        }
+    }
+    float sum = 0.f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+        const int c = threadIdx.x + k * blockDim.x;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) { x[k][j] += d[k][j]; sum += x[k][j]; }
+        if (c < n4 && a.write_back && h) store4(h + 4 * c, x[k]);
+    }
+    const float mean = row_sum(sum, slots[2]) / (float)W;
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k)
+        if (threadIdx.x + k * blockDim.x < n4) {
+#pragma unroll
+            for (int j = 0; j < 4; ++j) { const float dlt = x[k][j] - mean; ss = fmaf(dlt, dlt, ss); }
+        }
+    const float inv = 1.f / sqrtf(row_sum(ss, slots[3]) / (float)W + a.eps);
+    TO* out = (TO*)a.out + i * W;
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+        const int c = threadIdx.x + k * blockDim.x;
+        if (c >= n4) continue;
+        float w4[4], b4[4] = {0.f, 0.f, 0.f, 0.f}, y[4];
+        load4(a.w + 4 * c, w4);
+        if (a.b) load4(a.b + 4 * c, b4);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) y[j] = (x[k][j] - mean) * inv * w4[j] + b4[j];
+        store4(out + 4 * c, y);
+    }
 }
 
 template <typename TO>
@@ -148,7 +280,7 @@ extern "C" int tqk_streams_step(float* X, int n_streams, const void* y, int y_dt
     TQK_REQUIRE(X, "tqk_streams_step: null pointer");
     TQK_REQUIRE(n_streams > 0 && n_streams <= STREAMS_MAX, "tqk_streams_step: %d copies of the stream, the kernel takes up to %d", n_streams, STREAMS_MAX);
     TQK_REQUIRE(!y || (mix && out_w), "tqk_streams_step: an update without its weights");
-    TQK_REQUIRE(!n_out || (in_w && norm_w && norm_b), "tqk_streams_step: a norm without its weights");
+    TQK_REQUIRE(!n_out || (in_w && norm_w), "tqk_streams_step: a norm without its weights");
     TQK_REQUIRE(!u_out || in_w, "tqk_streams_step: a sum without its weights");
     TQK_REQUIRE(n_tokens >= 0 && width > 0 && width <= 12288, "tqk_streams_step: bad sizes");
     if (n_tokens == 0 || (!y && !in_w)) return 0;
@@ -172,20 +304,32 @@ extern "C" int tqk_streams_step(float* X, int n_streams, const void* y, int y_dt
 }
 
 extern "C" int tqk_add_layer_norm(float* h, const void* delta, int delta_dtype, const int32_t* rows, int n_rows, const float* weight, const float* bias,
-                                  float eps, void* out, int out_dtype, int width, int write_back, void* stream) {
-    TQK_REQUIRE((h || delta) && weight && bias && out, "tqk_add_layer_norm: null pointer");
+                                  float eps, const float* delta_weight, const float* delta_bias, float delta_eps, void* out, int out_dtype, int width,
+                                  int write_back, void* stream) {
+    TQK_REQUIRE((h || delta) && weight && out, "tqk_add_layer_norm: null pointer");
     TQK_REQUIRE(n_rows >= 0 && width > 0 && width <= 12288, "tqk_add_layer_norm: bad sizes");
     TQK_REQUIRE(!(write_back && rows), "tqk_add_layer_norm: chosen rows are not written back");
+    TQK_REQUIRE(!delta_weight || delta, "tqk_add_layer_norm: a norm of an update that is not there");
     if (n_rows == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
-    const size_t lds = (size_t)width * sizeof(float);
-#define TQK_ALN(TD, TO) add_layer_norm_kernel<TD, TO><<<n_rows, 256, lds, s>>>(h, (const TD*)delta, rows, weight, bias, eps, (TO*)out, width, write_back)
+    const LayerNormArgs a = {h, delta, rows, weight, bias, eps, delta_weight, delta_bias, delta_eps, out, width, write_back};
     const int dd = delta ? delta_dtype : TQK_F32;
+    TQK_REQUIRE((dd == TQK_F32 || dd == TQK_BF16) && (out_dtype == TQK_F32 || out_dtype == TQK_BF16), "tqk_add_layer_norm: unknown dtypes %d, %d", delta_dtype, out_dtype);
+    const uintptr_t all = (uintptr_t)h | (uintptr_t)delta | (uintptr_t)weight | (uintptr_t)bias | (uintptr_t)delta_weight | (uintptr_t)delta_bias | (uintptr_t)out;
+    const bool vec = width % 4 == 0 && (all & 15) == 0;
+    const size_t lds = (size_t)width * sizeof(float);
+    // threads by the width alone, so that a row's sums have one order whatever the step holds
+    int threads = (width / 4 + TQK_WAVE - 1) / TQK_WAVE * TQK_WAVE;
+    threads = threads < TQK_WAVE ? TQK_WAVE : threads > 1024 ? 1024 : threads;
+    const int nv = (width / 4 + threads - 1) / threads;
+#define TQK_ALN(TD, TO) do { if (!vec) add_layer_norm_kernel<TD, TO><<<n_rows, 256, lds, s>>>(a); \
+        else if (nv <= 1) add_layer_norm_vec_kernel<TD, TO, 1><<<n_rows, threads, 0, s>>>(a); \
+        else if (nv <= 2) add_layer_norm_vec_kernel<TD, TO, 2><<<n_rows, threads, 0, s>>>(a); \
+        else add_layer_norm_vec_kernel<TD, TO, 3><<<n_rows, threads, 0, s>>>(a); } while (0)
     if (dd == TQK_F32 && out_dtype == TQK_F32) TQK_ALN(float, float);
-    else if (dd == TQK_F32 && out_dtype == TQK_BF16) TQK_ALN(float, bf16_t);
-    else if (dd == TQK_BF16 && out_dtype == TQK_F32) TQK_ALN(bf16_t, float);
-    else if (dd == TQK_BF16 && out_dtype == TQK_BF16) TQK_ALN(bf16_t, bf16_t);
-    else return tqk_fail("tqk_add_layer_norm: unknown dtypes %d, %d", delta_dtype, out_dtype);
+    else if (dd == TQK_F32) TQK_ALN(float, bf16_t);
+    else if (out_dtype == TQK_F32) TQK_ALN(bf16_t, float);
+    else TQK_ALN(bf16_t, bf16_t);
 #undef TQK_ALN
     return tqk_check_launch("tqk_add_layer_norm");
 }

@@ -20,7 +20,7 @@ extern "C" {
 #endif
 
 #define TQE_PAGE 64             /* positions per cache page (the kernel library is asked for its own and must agree) */
-#define TQE_KERNEL_ABI 22       /* the version of the kernel library's interface (tqk_abi_version) this engine is written against */
+#define TQE_KERNEL_ABI 23       /* the version of the kernel library's interface (tqk_abi_version) this engine is written against */
 #define TQE_MAX_GROUPS 16       /* groups of cached runs a cache may have */
 
 enum {
@@ -61,6 +61,11 @@ void tqe_cache_free(tqe_cache_t* cache);
 /* A group with a window also keeps the pages that hold any of a sequence's first `positions` positions (set before the
  * cache is used; 0, the default: the window alone decides). */
 int tqe_cache_keep_first(tqe_cache_t* cache, int group, int positions);
+
+/* The positions of a group fall into chunks of `positions`, counted from a sequence's start, and a query reads its own chunk
+ * only: pages all of whose positions belong to an earlier chunk than the next query's are given back (set before the cache is
+ * used; 0, the default: no chunks). */
+int tqe_cache_chunk(tqe_cache_t* cache, int group, int positions);
 
 /* A free slot with length 0 (TQE_ERR_FULL if there is none); everything a slot holds goes back. */
 int tqe_cache_acquire(tqe_cache_t* cache, int32_t* slot_out);

@@ -173,12 +173,13 @@ int tqk_attention_prefill(const void* q, const void* keys, const void* values, c
                           int n_tiles, int tile_queries, const int32_t* seq_start, const int32_t* seq_new,
                           int window, float scale, void* out, int n_tokens, int n_heads, int n_kv_heads,
                           int head_dim, void* stream);
-/* The same with a cap on the scores: cap > 0 makes them cap tanh(scale q.k / cap) before the softmax. */
+/* The same with a cap on the scores: cap > 0 makes them cap tanh(scale q.k / cap) before the softmax; chunk > 0: a query sees no
+ * position of an earlier chunk of `chunk` positions than its own. */
 int tqk_attention_prefill_capped(const void* q, const void* keys, const void* values, const int32_t* tok_pos,
                                  const int32_t* page_table, int table_width, int n_seqs, int n_pages,
                                  const int32_t* tile_seq, const int32_t* tile_tok0, const int32_t* tile_count,
                                  int n_tiles, int tile_queries, const int32_t* seq_start, const int32_t* seq_new,
-                                 int window, float scale, float cap, void* out, int n_tokens, int n_heads, int n_kv_heads,
+                                 int window, int chunk, float scale, float cap, void* out, int n_tokens, int n_heads, int n_kv_heads,
                                  int head_dim, void* stream);
 
 /* out[t, i] = silu(gate_up[t, i]) * gate_up[t, inter + i] */
@@ -197,26 +198,26 @@ int tqk_mid_gated_act(const void* x, const void* w_packed, void* y, int M, int N
 /* Attention through a low-rank latent (latent.hip).  Every position leaves one cache row [rk + dr]: the normed
  * latent and one rotated key part, shared by all heads; pages are [n_pages][64][rk + dr].
  * tqk_latent_split: row t of proj (row_stride values) begins [q_rank | kv_rank + rot_dim (absent when kv_rank == 0) | n_gate].  cq_out
- * [tokens, q_rank] = RMS norm of the first part times q_norm_w; the second part goes into the cache row of the token's
- * position (RMS norm times kv_norm_w of its first kv_rank values, rotation in halves of the first rot_dims of the
+ * [tokens, q_rank] = RMS norm of the first part times q_norm_w (null: the first part is left alone); the second part goes into the cache row of the token's
+ * position (RMS norm times kv_norm_w of its first kv_rank values, rotation (style 1: in halves, 2: element 2i with 2i + 1) of the first rot_dims of the
  * others by the angle table row tok_pos[t]; `turned`, if given, gets the latent a second time, pages [n_pages][kv_rank][64]
  * with a page's positions at the places of the standard value pages, see tqk_rope_store); gate_out [tokens, n_gate] = sigmoid of the last part, float32. */
 int tqk_latent_max_rank(void);          /* the largest latent (rk) tqk_latent_attention takes */
 int tqk_latent_max_row(void);           /* the largest cache row (rk + dr) it takes */
 int tqk_latent_split(const void* proj, int act_dtype, int row_stride, int q_rank, int kv_rank, int rot_dim, int n_gate, const void* q_norm_w,
                      const void* kv_norm_w, int norm_dtype, float eps, const float* cos_table, const float* sin_table,
-                     int rot_dims, int max_positions, const int32_t* tok_seq, const int32_t* tok_pos,
+                     int rot_dims, int style, int max_positions, const int32_t* tok_seq, const int32_t* tok_pos,
                      const int32_t* page_table, int table_width, void* cache, void* turned, int n_pages, void* cq_out,
                      float* gate_out, int n_tokens, void* stream);
-/* qa [tokens, heads, rk + dr] float32: qa[:rk] = W_uk,h^T q[:dn] (w_uk [heads * dn, rk]), qa[rk:] = q[dn:] rotated;
+/* qa [tokens, heads, rk + dr] float32: qa[:rk] = W_uk,h^T q[:dn] (w_uk [heads * dn, rk]), qa[rk:] = q[dn:] rotated (rows of q q_stride values apart);
  * tail_only: the rotated part alone (the product is someone else's: tqk_head_product) */
-int tqk_latent_absorb(const void* q, int act_dtype, const void* w_uk, int w_dtype, int n_heads, int dn, int dr, int rk,
-                      const float* cos_table, const float* sin_table, int rot_dims, int max_positions,
+int tqk_latent_absorb(const void* q, int act_dtype, long long q_stride, const void* w_uk, int w_dtype, int n_heads, int dn, int dr, int rk,
+                      const float* cos_table, const float* sin_table, int rot_dims, int style, int max_positions,
                       const int32_t* tok_pos, float* qa, int n_tokens, int tail_only, void* stream);
 /* out [tokens, heads, rk] float32 = softmax over the visible positions of (qa . row) * scale, times row[:rk];
- * visible: lo..tok_pos[t], lo = max(0, tok_pos - window + 1) if window > 0 else 0 */
+ * visible: lo..tok_pos[t], lo = max(0, tok_pos - window + 1) if window > 0 else 0; sink [heads] (or null) adds exp(sink_h) to the denominator */
 int tqk_latent_attention(const float* qa, const void* cache, int cache_dtype, const int32_t* tok_seq, const int32_t* tok_pos,
-                         const int32_t* page_table, int table_width, int n_seqs, int n_pages, int window, float scale,
+                         const int32_t* page_table, int table_width, int n_seqs, int n_pages, int window, float scale, const float* sink,
                          float* out, int n_tokens, int n_heads, int rk, int dr, void* stream);
 /* the same on the matrix cores, for a bfloat16 cache with its turned copy, where tqk_latent_attention_mfma_supported says so */
 int tqk_latent_attention_mfma_supported(int rk, int dr);
@@ -224,16 +225,17 @@ int tqk_latent_attention_mfma_supported(int rk, int dr);
  * heads, n_parts, rk] and part_ml [tokens, heads, n_parts, 2] are its scratch.  tqk_latent_attention_parts: a good number. */
 int tqk_latent_attention_parts(int n_tokens, int n_heads, int table_width, int window);
 int tqk_latent_attention_mfma(const float* qa, const void* cache, const void* turned, const int32_t* tok_seq, const int32_t* tok_pos,
-                              const int32_t* page_table, int table_width, int n_seqs, int n_pages, int window, float scale,
+                              const int32_t* page_table, int table_width, int n_seqs, int n_pages, int window, float scale, const float* sink,
                               float* out, int n_tokens, int n_heads, int rk, int dr, int n_parts, float* part_o, float* part_ml,
                               void* stream);
 /* the same for steps of several tokens per sequence: tiles of up to 4 consecutive tokens of one sequence, a block a tile */
 int tqk_latent_attention_tiles(const float* qa, const void* cache, const void* turned, const int32_t* tok_pos,
                                const int32_t* page_table, int table_width, int n_seqs, int n_pages, const int32_t* tile_seq,
-                               const int32_t* tile_tok0, const int32_t* tile_count, int n_tiles, int window, float scale,
+                               const int32_t* tile_tok0, const int32_t* tile_count, int n_tiles, int window, float scale, const float* sink,
                                float* out, int n_tokens, int n_heads, int rk, int dr, void* stream);
-/* y [tokens, heads * dv] = gate[t, h] * W_uv,h o[t, h] (w_uv [heads * dv, rk]; gate may be null) */
-int tqk_latent_values(const float* o, const void* w_uv, int w_dtype, const float* gate, int n_heads, int rk, int dv, void* y,
+/* y [tokens, heads * dv] = gate[t, h] * W_uv,h o[t, h] (w_uv [heads * dv, rk]; gate may be null), times the sigmoid of element_gate
+ * [tokens, heads * dv] (of y's type, rows gate_stride values apart; or null) */
+int tqk_latent_values(const float* o, const void* w_uv, int w_dtype, const float* gate, const void* element_gate, long long gate_stride, int n_heads, int rk, int dv, void* y,
                       int y_dtype, int n_tokens, void* stream);
 
 /* A feed-forward of routed experts (moe.hip).  tqk_moe_route: idx, weight [tokens, top]: the `top` experts with the
@@ -269,7 +271,8 @@ int tqk_moe_product_mfma(const void* x, const int32_t* x_rows, const void* w, lo
                          int gated, int gate, float limit, float alpha, const int32_t* tile_expert, const int32_t* tile_row0,
                          const int32_t* tile_rows, const int32_t* n_tiles, int max_tiles, int tile_m, void* stream);
 int tqk_head_product(const void* x, int x_f32, long long x_row_stride, long long x_head_stride, const void* w, void* y, int y_f32,
-                     long long y_row_stride, long long y_head_stride, const float* scale, int n_tokens, int n_heads, int N, int K,
+                     long long y_row_stride, long long y_head_stride, const float* scale, const void* gate, int gate_f32,
+                     long long gate_stride, int n_tokens, int n_heads, int N, int K,
                      void* stream);
 int tqk_moe_combine(const void* y, int act_dtype, const int32_t* pair_pos, const float* weight, int top, const void* shared,
                     const float* shared_scale, void* out, int n_tokens, int hidden, void* stream);
@@ -293,23 +296,25 @@ int tqk_unary_act(const void* x, void* out, int act_dtype, long long n, int kind
 int tqk_row_gate(const void* x, int act_dtype, const void* w, int w_dtype, float* out, int n_tokens, int hidden, void* stream);
 
 /* Attention with keys of key_dim and values of value_dim per head (attention_masked.hip).  tqk_normed_rope_store: a row of qkv is
- * [heads * key_dim | kv_heads * key_dim | kv_heads * value_dim]; every query and key head is divided by its root mean square
+ * [heads * key_dim | kv_heads * key_dim | kv_heads * value_dim] (values_are_keys: the last part is missing, and the values are the keys as
+ * they come); bias (or null, of w_dtype) has a row's layout and is added first; every query and key head is divided by its root mean square
  * (eps inside the root) and multiplied by q_norm_w / k_norm_w [key_dim] (null: no norm), then its first rot_dim elements are
- * rotated in halves by the angle table row tok_pos[t]; values become (1 - mix[0]) v + mix[0] mix_with[t] where mix_with
+ * turned (style 1: in halves, 2: element 2i with 2i + 1) by the angle table row tok_pos[t]; values become (1 - mix[0]) v + mix[0] mix_with[t] where mix_with
  * [tokens, kv_heads * value_dim] is given, and are written to mix_keep (if given) as they go to the cache.  Pages: keys
  * [n_pages, kv_heads, 64, key_dim], values [n_pages, kv_heads, value_dim, 64] with the places of tqk_rope_store.
- * tqk_attention_masked: a query at position i sees j <= i with i - j < window or j < keep_first (window 0: all); scores
+ * tqk_attention_masked: a query at position i sees j <= i with i - j < window or j < keep_first (window 0: all), and,
+ * with chunk > 0, floor(j / chunk) = floor(i / chunk); scores
  * scale q.k, then cap tanh(s / cap) if cap > 0; sink [heads] (or null) adds exp(sink_h) to the softmax's denominator.
  * One wave per (token, head), float32 throughout; out [tokens, heads * value_dim]. */
-int tqk_normed_rope_store(const void* qkv, int act_dtype, const void* q_norm_w, const void* k_norm_w, int w_dtype, float eps,
-                          const float* cos_table, const float* sin_table, int rot_dim, int max_positions, const void* mix,
+int tqk_normed_rope_store(const void* qkv, int act_dtype, const void* bias, const void* q_norm_w, const void* k_norm_w, int w_dtype, float eps,
+                          const float* cos_table, const float* sin_table, int rot_dim, int style, int max_positions, const void* mix,
                           const void* mix_with, void* mix_keep, const int32_t* tok_seq, const int32_t* tok_pos,
                           const int32_t* page_table, int table_width, void* keys, void* values, void* q_out, int n_tokens,
-                          int n_heads, int n_kv_heads, int key_dim, int value_dim, int write_kv, void* stream);
+                          int n_heads, int n_kv_heads, int key_dim, int value_dim, int write_kv, int values_are_keys, void* stream);
 int tqk_attention_masked_max_dim(void);
 int tqk_attention_masked(const void* q, const void* keys, const void* values, int act_dtype, const int32_t* tok_seq,
                          const int32_t* tok_pos, const int32_t* page_table, int table_width, int n_seqs, int n_pages, int window,
-                         int keep_first, float scale, float cap, const void* sink, int sink_dtype, void* out, int n_tokens,
+                         int chunk, int keep_first, float scale, float cap, const void* sink, int sink_dtype, void* out, int n_tokens,
                          int n_heads, int n_kv_heads, int key_dim, int value_dim, void* stream);
 
 /* The same on the matrix cores (attention_masked_mfma.hip), bfloat16, key_dim a multiple of 8, both sizes up to 256.  n_tiles > 0:
@@ -320,7 +325,7 @@ int tqk_attention_masked(const void* q, const void* keys, const void* values, in
 int tqk_attention_masked_mfma_supported(int key_dim, int value_dim);
 int tqk_attention_masked_mfma_tile(int n_tokens, int n_heads, int n_kv_heads, int key_dim, int value_dim);
 int tqk_attention_masked_mfma(const void* q, const void* keys, const void* values, const int32_t* tok_pos, const int32_t* page_table,
-                              int table_width, int n_pages, int window, int keep_first, float scale, float cap, const void* sink,
+                              int table_width, int n_pages, int window, int chunk, int keep_first, float scale, float cap, const void* sink,
                               int sink_dtype, const int32_t* tile_seq, const int32_t* tile_tok0, const int32_t* tile_count, int n_tiles,
                               int tile_queries, int n_rows, int n_parts, void* part_out, void* part_ml, void* out, int n_heads, int n_kv_heads,
                               int key_dim, int value_dim, void* stream);
@@ -425,7 +430,8 @@ int tqk_sample(const float* logits, int n_rows, int vocab, float temperature, in
  * in_w is given, u = sum_s in_w[s] X'[t, s] goes to u_out (if given) and (u - mean) / sqrt(var + eps) norm_w + norm_b to n_out (if given);
  * wide != 0 lets a row have more threads (another order of its sums than with wide == 0).
  * tqk_add_layer_norm: out[i] = that norm of h[rows[i]] + delta[rows[i]] (rows null: row i; h or delta may be null; write_back leaves
- * the sum in h).  tqk_token_shift: out[t] = n[t] + (n[t - 1] - n[t]) mu, with the sequence's state row in place of n[t - 1] for the first
+ * the sum in h); delta_weight given: the update is normed with it (and delta_bias, delta_eps) before it is added; biases may be null.
+ * tqk_token_shift: out[t] = n[t] + (n[t - 1] - n[t]) mu, with the sequence's state row in place of n[t - 1] for the first
  * token a step brings of it; remember != 0 (steps of one token a sequence) also leaves n[t] in the state.  tqk_shift_remember: the state
  * of every sequence becomes n of the last token the step brings of it. */
 int tqk_streams_max(void);
@@ -434,7 +440,8 @@ int tqk_streams_step(float* X, int n_streams, const void* y, int y_dtype, const 
                      const float* norm_w, const float* norm_b, float eps, float* u_out, void* n_out, int n_dtype, int n_tokens, int width,
                      int wide, void* stream);
 int tqk_add_layer_norm(float* h, const void* delta, int delta_dtype, const int32_t* rows, int n_rows, const float* weight, const float* bias,
-                       float eps, void* out, int out_dtype, int width, int write_back, void* stream);
+                       float eps, const float* delta_weight, const float* delta_bias, float delta_eps, void* out, int out_dtype, int width,
+                       int write_back, void* stream);
 int tqk_token_shift(const float* n, const float* mu, float* state, long long state_stride, const int32_t* tok_seq, const int32_t* tok_pos,
                     const int32_t* seq_start, const int32_t* seq_slot, void* out, int out_dtype, int n_tokens, int width, int remember,
                     void* stream);
@@ -442,22 +449,36 @@ int tqk_shift_remember(const float* n, float* state, long long state_stride, con
                        int n_seqs, int width, void* stream);
 
 /* Linear attention with a decaying state (linear_attention.hip): per head S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, the state
- * of a slot [heads][d][dv] float32.  q, k, v: rows `stride` elements apart, heads side by side.  The decay: z [tokens, heads * d] float32
- * with z_bias gives a = sigmoid(z + bias)^inv_tau per key channel; z null: head_decay[h] for the whole head.  q and k are turned by
+ * of a slot [heads][d][dv] float32, head_stride elements from head to head.  q, k, v: rows `stride` elements apart, heads side by side.  The decay: z [tokens, heads * d] float32
+ * with z_bias gives a = sigmoid(z + bias)^inv_tau per key channel; z null: head_decay[h] for the whole head, or, with
+ * log_decay [tokens, heads], its exponential (k then times exp(log_in), the output times out_scale, both [tokens, heads] or null).  q and k are turned by
  * tok_pos through cos, sin [max_pos, rot_dim / 2] (style 1: halves, 2: pairs; cos null: not turned) and multiplied by q_scale, k_scale.
  * mode 0: every sequence's tokens in order from its state row, which is written back (cu, seq_new, seq_slot; n_items sequences).
  * mode 1 and 2: chunks as tqk_ssm_chunks takes them (chunk_row0, chunk_count; n_items chunks), between them tqk_chunk_carry with
  * p_stride heads * d, p_div dv and per_seq heads * d * dv.  out [tokens, heads, dv] float32.
- * tqk_head_norm_gate: out[t, h] = o[t, h] / rms(o[t, h]) * weight (null: 1) * silu(gate[t, h]) (null: 1). */
+ * tqk_head_norm_gate: out[t, h] = o[t, h] / rms(o[t, h]) * weight[h * weight_stride ..] (null: 1) * silu(gate[t, h]) (null: 1; sigmoid != 0: the
+ * sigmoid alone). */
 int tqk_linear_attention_max_dim(void);
 int tqk_linear_attention(const void* q, const void* k, const void* v, int act_dtype, long long stride, const float* z, long long z_stride,
-                         const float* z_bias, float inv_tau, const float* head_decay, float q_scale, float k_scale, const float* cos,
+                         const float* z_bias, float inv_tau, const float* head_decay, const float* log_decay, const float* log_in,
+                         const float* out_scale, float q_scale, float k_scale, const float* cos,
                          const float* sin, int rot_dim, int style, int max_pos, const int32_t* tok_pos, float* state, long long state_stride,
                          const int32_t* cu, const int32_t* seq_new, const int32_t* seq_slot, const int32_t* chunk_row0,
                          const int32_t* chunk_count, float* chunk_state, float* chunk_decay, float* out, int mode, int n_items, int heads,
-                         int d, int dv, void* stream);
-int tqk_head_norm_gate(const float* o, const float* weight, float eps, const void* gate, int gate_dtype, long long gate_stride, void* out,
+                         int d, int dv, long long head_stride, void* stream);
+int tqk_head_norm_gate(const float* o, const float* weight, int weight_stride, float eps, const void* gate, int gate_dtype, long long gate_stride,
+                       int sigmoid, void* out,
                        int out_dtype, int n_tokens, int heads, int dv, void* stream);
+
+/* The gates of a matrix memory (mlstm.hip): z [tokens] rows z_stride apart, [heads] input gates' products then [heads] forget gates', bias
+ * [2 heads].  a = cap tanh((z_i + b) / cap), f = log sigmoid(cap tanh((z_f + b) / cap)); in the tokens' order m_t = max(f_t + m_(t-1), a_t), kappa
+ * = f + m_(t-1) - m_t, tau = a - m_t, m: all [tokens, heads].  m is carried at state[m_offset + head] of the sequence's slot.  inv_den (or null)
+ * [tokens, heads]: n_t = e^kappa n_(t-1) + e^tau k_t is carried too (the last d of a head's head_stride elements), and 1 / (max(|n_t . q_scale
+ * q_t|, e^(-m_t)) + 1e-6) is left there.  tqk_linear_attention with log_decay kappa, log_in tau, out_scale inv_den is the memory itself. */
+int tqk_mlstm_gates(const float* z, long long z_stride, const float* bias, float cap, const void* q, const void* k, int act_dtype, long long stride,
+                    float q_scale, float* state, long long state_stride, long long head_stride, long long m_offset, const int32_t* cu,
+                    const int32_t* seq_new, const int32_t* seq_slot, float* kappa, float* tau, float* m, float* inv_den, int n_seqs, int heads,
+                    int d, void* stream);
 
 /* Attention over a window plus pooled blocks (pooled_attention.hip).  Pages: keys [kv heads][page + tqk_pooled_rows(pool)][d], values
  * likewise with dv; a block's means lie behind the positions of the page that holds its last position.  tqk_pooled_store: qkv

@@ -12,7 +12,7 @@ import torch
 from ..csrc import build as _build
 
 _LIB = None
-KERNEL_ABI = 22         # tqk_abi_version of the kernel library these wrappers are written against
+KERNEL_ABI = 23         # tqk_abi_version of the kernel library these wrappers are written against
 
 F32, BF16 = 0, 1
 STYLE_NONE, STYLE_HALVES, STYLE_PAIRS = 0, 1, 2
@@ -388,11 +388,12 @@ def attention_prefill_tile(n_tokens, n_heads, n_kv_heads, head_dim):
 
 
 def attention_prefill(q, keys, values, tok_pos, page_table, tile_seq, tile_tok0, tile_count, seq_start, seq_new,
-                      window, scale, out, tile_queries=64, cap=0.0):
+                      window, scale, out, tile_queries=64, cap=0.0, chunk=0):
     """Causal attention of tiles of up to tile_queries (16, 32, 64 or 128) consecutive queries
     (q [T, heads, d] bfloat16) over the paged cache; out [T, heads*d].  tile_count must not
     exceed tile_queries (the caller built the tiles; the kernel covers no more).  cap > 0: the
-    scores become cap tanh(scale q.k / cap) before the softmax."""
+    scores become cap tanh(scale q.k / cap) before the softmax.  chunk > 0: a query sees nothing of an
+    earlier chunk of positions than its own."""
     n, n_heads, head_dim = q.shape
     n_pages, n_kv_heads = keys.shape[0], keys.shape[1]
     n_seqs, width = page_table.shape
@@ -404,7 +405,7 @@ def attention_prefill(q, keys, values, tok_pos, page_table, tile_seq, tile_tok0,
         _dev(tile_seq, "tile_seq", torch.int32, (n_tiles,)), _dev(tile_tok0, "tile_tok0", torch.int32, (n_tiles,)),
         _dev(tile_count, "tile_count", torch.int32, (n_tiles,)), n_tiles, int(tile_queries),
         _dev(seq_start, "seq_start", torch.int32, (n_seqs,)), _dev(seq_new, "seq_new", torch.int32, (n_seqs,)),
-        int(window or 0), ctypes.c_float(scale), ctypes.c_float(cap), _dev(out, "out", torch.bfloat16, (n, n_heads * head_dim)),
+        int(window or 0), int(chunk), ctypes.c_float(scale), ctypes.c_float(cap), _dev(out, "out", torch.bfloat16, (n, n_heads * head_dim)),
         n, n_heads, n_kv_heads, head_dim, _stream()), "attention_prefill")
     return out
 
