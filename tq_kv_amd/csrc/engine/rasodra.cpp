@@ -1,6 +1,6 @@
 // Rasodra: a decoder whose layers are listed one by one in its configuration.  A sublayer has a norm on both sides, x <- x + N_b(part(N_a(x)))
-// with layer norms that have a weight and no bias; a layer is a mixer and an optional feed-forward, down(max(up, 0)^2).  A layer may name an
-// earlier layer whose tensors it uses: then it runs with that layer's weights, with a cache or state of its own.
+// with layer norms that have a weight and no bias; a layer is a mixer and an optional feed-forward, down(max(up, 0)^2).  A layer may name
+// another layer whose tensors it uses: then it runs with that layer's weights, with a cache or state of its own.
 // Three mixers.  "mlstm": a matrix memory with gates kept as logarithms against a running maximum.  "latent_attention": attention through
 // one cached latent and one rotated key part per position, queries straight from the input, a sink, an output gate for every element.
 // "attention": grouped-query attention with biases whose values are its keys as projected, heads normed with a weight in front of a rotation by
@@ -98,17 +98,23 @@ Json rasodra_typed(const Json& raw, const std::string& where) {
         t.set("type", type);
         t.set("mixer", mixer_typed(object_at(l, "mixer", at), at + ".mixer", type));
         t.set("mlp", mlp_typed(l["mlp"], at + ".mlp"));
-        // whose tensors the layer uses: its own, or those of an earlier layer of the same sizes
-        long long source = i;
-        if (lr.has("weights_of")) {
-            const long long of = lr.integer("weights_of", 0);
-            if (of >= i) raise(TQE_ERR_CONFIG, "%s: weights_of %lld is no earlier layer", at.c_str(), of);
-            for (const char* key : {"type", "mixer", "mlp"})
-                if (t[key].dump() != typed[(size_t)of][key].dump()) raise(TQE_ERR_CONFIG, "%s: its %s is not that of layer %lld, whose tensors it uses", at.c_str(), key, of);
-            source = typed[(size_t)of]["source"].as_int();
-        }
-        t.set("source", source);
+        t.set("source", lr.has("weights_of") ? lr.integer("weights_of", 0) : i);
         typed.push_back(t);
+    }
+    // whose tensors a layer uses: its own, or those of another layer of the same sizes (which may itself use another's)
+    const long long n = (long long)typed.size();
+    for (long long i = 0; i < n; ++i) {
+        const std::string at = format("%s: layers[%lld]", where.c_str(), i);
+        long long source = i;
+        for (long long steps = 0; source >= n || typed[(size_t)source]["source"].as_int() != source; ++steps) {
+            if (source >= n || steps == n) raise(TQE_ERR_CONFIG, "%s: weights_of leads to no layer with tensors of its own", at.c_str());
+            source = typed[(size_t)source]["source"].as_int();
+        }
+        Json t = typed[(size_t)i];
+        for (const char* key : {"type", "mixer", "mlp"})
+            if (t[key].dump() != typed[(size_t)source][key].dump())
+                raise(TQE_ERR_CONFIG, "%s: its %s is not that of layer %lld, whose tensors it uses", at.c_str(), key, source);
+        t.set("source", source);
         list.push(t);
     }
     c.set("layers", list);
@@ -154,12 +160,11 @@ ModelSpec rasodra_spec(const Json& c) {
     }
     const bool keep_all = (int)groups.size() > TQE_MAX_GROUPS;
     std::map<long long, int> index;                     // layers with tensors of their own, by their number in the list
-    size_t l = 0;
+    long long number = 0;
     for (const Json& layer : c["layers"].items()) {
         const Json& m = layer["mixer"];
         const Json& mlp = layer["mlp"];
-        const long long source = layer["source"].as_int(), number = (long long)l++;
-        if (source == number) {
+        if (layer["source"].as_int() == number) {
             const std::string type = layer["type"].as_string();
             PartSpec mixer;
             if (type == "mlstm")
@@ -185,8 +190,11 @@ ModelSpec rasodra_spec(const Json& c) {
             index[number] = (int)s.layers.size();
             s.layers.push_back(spec);
         }
+        ++number;
+    }
+    for (const Json& layer : c["layers"].items()) {
         Run run;
-        run.layer = index.at(source);
+        run.layer = index.at(layer["source"].as_int());
         s.order.push_back(run);
     }
     s.final_norm = PartSpec::from_json(norm, "final norm");
