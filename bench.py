@@ -23,7 +23,8 @@ heads, mixed values, and in every other layer a score cap, a window that keeps t
 embedding; norms on the parts' outputs; routed experts without a gate product).  `python bench.py --streams` does it for the Povipel design beside a
 Piditar shape of equal size.  `python bench.py --recurrent` does it for the
 Piditar design (layers of attention, of a real-gated linear recurrent unit and of a selective state-space mixer, each with a dense
-feed-forward).
+feed-forward).  `python bench.py --matrix-memory` does it for the Rasodra design (a matrix memory, latent attention with a sink and an
+element gate, chunked attention whose values are its keys, norms on both sides of every part) beside a Nikasun shape of equal size.
 """
 import argparse
 import gc
@@ -54,6 +55,7 @@ def main():
     ap.add_argument("--masked", action="store_true", help="measure the Sizudra design beside a Qwen2 shape of equal size instead of the default workload")
     ap.add_argument("--recurrent", action="store_true", help="measure the Piditar design beside a Qwen2 shape of equal size instead of the default workload")
     ap.add_argument("--streams", action="store_true", help="measure the Povipel design beside a Piditar shape of equal size instead of the default workload")
+    ap.add_argument("--matrix-memory", action="store_true", help="measure the Rasodra design beside a Nikasun shape of equal size instead of the default workload")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this library runs on one GPU; --gpus %d is not supported" % args.gpus)
@@ -166,6 +168,9 @@ def main():
         return design_comparison("piditar", recurrent_shapes, args, torch, Model, Engine, note, timed_prefill, decode, random_prompts, release)
     if args.streams:
         return design_comparison("povipel", streams_shapes, args, torch, Model, Engine, note, timed_prefill, decode, random_prompts, release, beside="piditar")
+
+    if args.matrix_memory:
+        return design_comparison("rasodra", memory_shapes, args, torch, Model, Engine, note, timed_prefill, decode, random_prompts, release, beside="nikasun")
 
     # -- the headline shape -------------------------------------------------------------------------
     raw = dict(catalog.find(args.shape))
@@ -390,6 +395,31 @@ def streams_shapes(width, layers=4):
     return povipel, piditar, {"width": width, "layers": layers, "heads": heads, "kv_heads": kv_heads, "streams": 4, "window": 1024, "pool": 16,
                               "linear_heads": right["heads"], "linear_dim": 128, "linear_vdim": 256, "retention_heads": retention["heads"],
                               "dense_ff": dense["ff"], "experts": 32, "top": 4, "expert_ff": moe["expert"]["ff"], "beside_ff": base["ff"]}
+
+
+def memory_shapes(width, layers=4):
+    """A Rasodra configuration (matrix memory without a feed-forward, latent attention twice, chunked attention) and a Nikasun one (latent
+    attention in every layer, the first without a feed-forward) of the same width, depth, heads, head sizes and latent, and as many
+    multiply-adds in the feed-forward products."""
+    heads, dim = width // 128, 128
+    kv_heads = max(1, heads // 4)
+    ff = 4 * width
+    rot = {"base": 10000.0, "dims": 64}
+    memory = {"heads": width // 256, "dim": 128, "vdim": 256, "gate_cap": 15.0}
+    latent = {"heads": heads, "dim": dim, "rot_dim": 64, "vdim": dim, "kv_rank": 512, "scale": (dim + 64) ** -0.5, "rot": rot}
+    chunked = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": 1024}, "rot": rot}
+    dense = {"kind": "dense", "ff": ff}
+    kinds = [("mlstm", memory, None), ("latent_attention", latent, dense), ("latent_attention", latent, dense), ("attention", chunked, dense)]
+    lay = [{"type": kinds[l % 4][0], "mixer": kinds[l % 4][1], "mlp": kinds[l % 4][2]} for l in range(layers)]
+    rasodra = {"architecture": "Rasodra", "vocab": 32000, "width": width, "norm": {"eps": 1e-5}, "layers": lay, "max_positions": 8192}
+    # a gated feed-forward is three products, Rasodra's two
+    gated = {"kind": "dense", "ff": 2 * ff // 3 // 256 * 256}
+    other = dict(latent, q_rank=3 * width // 8, mask={"size": 8192})
+    nikasun = {"architecture": "Nikasun", "vocab": 32000, "width": width, "embedding": {"scale": width ** 0.5}, "norm": {"eps": 1e-5}, "max_positions": 8192,
+               "layers": [{"type": "latent_attention", "mixer": other, "mlp": gated if l % 4 else None} for l in range(layers)]}
+    return rasodra, nikasun, {"width": width, "layers": layers, "memory_heads": memory["heads"], "memory_dim": 128, "memory_vdim": 256, "heads": heads,
+                              "kv_heads": kv_heads, "head_dim": dim, "kv_rank": 512, "rot_dim": 64, "chunk": 1024, "ff": ff, "beside_ff": gated["ff"],
+                              "beside_q_rank": other["q_rank"]}
 
 
 def design_comparison(design, shapes, args, torch, Model, Engine, note, timed_prefill, decode, random_prompts, release, beside="qwen2"):

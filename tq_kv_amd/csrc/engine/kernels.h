@@ -116,6 +116,11 @@ TQ_QUERY(int, linear_attention_max_dim);
 TQ_KERNEL(linear_attention, cptr, cptr, cptr, int, long long, cf32, long long, cf32, float, cf32, cf32, cf32, cf32, float, float, cf32, cf32, int, int, int,
           ci32, float*, long long, ci32, ci32, ci32, ci32, ci32, float*, float*, float*, int, int, int, int, int, long long, void*);
 TQ_KERNEL(head_norm_gate, cf32, cf32, int, float, cptr, int, long long, int, void*, int, int, int, int, void*);
+TQ_QUERY(int, mlstm_chunks_supported, int, int);
+TQ_QUERY(int, mlstm_apply_norms, int);
+TQ_KERNEL(mlstm_gate_scan, cf32, long long, cf32, float, float*, long long, long long, ci32, ci32, ci32, float*, float*, float*, int, int, void*);
+TQ_KERNEL(mlstm_local, cptr, cptr, long long, cf32, cf32, ci32, ci32, int, float*, float*, int, int, int, void*);
+TQ_KERNEL(mlstm_apply, cptr, cptr, cptr, long long, cf32, cf32, cf32, float, ci32, ci32, int, float*, float*, cf32, float, cptr, void*, int, int, int, void*);
 TQ_KERNEL(mlstm_gates, cf32, long long, cf32, float, cptr, cptr, int, long long, float, float*, long long, long long, long long, ci32, ci32, ci32, float*,
           float*, float*, float*, int, int, int, void*);
 TQ_QUERY(int, pooled_attention_max_dim);

@@ -10,7 +10,8 @@
 //
 // The state of a sequence is one float32 row of the cache's state groups (zero when a slot is taken): per head S and n one behind the
 // other, then the heads' m.  Gates, maxima, n, S and the heads' norm are float32 whatever the activation type, and so are the gates'
-// products' results; q, k, v and the output gate come from one product with the weights stacked.
+// products' results; q, k, v and the output gate come from one product with the weights stacked.  Steps that bring many tokens of a
+// sequence in bfloat16 run in chunks on the matrix cores (mlstm.hip), with the heads' norm and the gate in the last of their kernels.
 //
 // params: hidden, heads, head_dim, value_dim, gate_cap, eps; optional q_scale (head_dim^(-1/2) unless given), names {q, k, v, g, o, norm, i,
 // i_bias, f, f_bias}.
@@ -110,8 +111,30 @@ public:
         const int64_t qk = (int64_t)heads_ * d_, vv = (int64_t)heads_ * dv_;
         const Tensor in = linear(c, x.x, w_in_, nullptr, dtype).t;                    // [q | k | v | g | padding]
         const Tensor z = linear(c, x.x, w_gates_, nullptr, F32).t;                    // [i | f | padding]
-        Tensor kappa = c.alloc(F32, {n, heads_}), tau = c.alloc(F32, {n, heads_}), m = c.alloc(F32, {n, heads_}), inv_den = c.alloc(F32, {n, heads_});
-        Tensor o = c.alloc(F32, {n, heads_, dv_});
+        Tensor kappa = c.alloc(F32, {n, heads_}), tau = c.alloc(F32, {n, heads_}), m = c.alloc(F32, {n, heads_});
+        Tensor gated = c.alloc(dtype, {n, vv});
+        const float* norm_w = (const float*)norm_w_->t.data;
+        const void* gate = at(in, 2 * qk + vv);
+        Tensor o;
+        if (dtype == BF16 && !c.all_decode && !c.capturing && c.max_new >= CHUNKED_FROM && !null_device() && K::mlstm_chunks_supported.raw(d_, dv_)) {
+            const Chunks ch = c.chunks(CHUNK);
+            Tensor cs = c.alloc(F32, {ch.n, heads_, head_stride()}), cd = c.alloc(F32, {ch.n, heads_});
+            const bool norms = K::mlstm_apply_norms.raw(dv_) != 0;
+            if (!norms) o = c.alloc(F32, {n, heads_, dv_});
+            K::mlstm_gate_scan((const float*)z.data, z.cols(), (const float*)gate_bias_->t.data, cap_, state, row, m_offset, c.dev.cu, c.dev.seq_new,
+                               c.dev.seq_slot, (float*)kappa.data, (float*)tau.data, (float*)m.data, c.n_seqs, heads_, c.stream);
+            K::mlstm_local(at(in, qk), at(in, 2 * qk), row_, (const float*)kappa.data, (const float*)tau.data, ch.row0, ch.count, ch.n, (float*)cs.data,
+                           (float*)cd.data, heads_, d_, dv_, c.stream);
+            K::chunk_carry((const float*)cd.data, heads_, (int)head_stride(), (float*)cs.data, ch.seq_first, c.dev.seq_slot, state, row, c.n_seqs, m_offset,
+                           c.stream);
+            K::mlstm_apply(in.data, at(in, qk), at(in, 2 * qk), row_, (const float*)kappa.data, (const float*)tau.data, (const float*)m.data, q_scale_, ch.row0,
+                           ch.count, ch.n, (float*)cs.data, (float*)o.data, norm_w, eps_, gate, gated.data, heads_, d_, dv_, c.stream);
+            if (!norms)
+                K::head_norm_gate((const float*)o.data, norm_w, dv_, eps_, gate, dtype, row_, 1, gated.data, dtype, (int)n, heads_, dv_, c.stream);
+            return finish(c, gated, stream);
+        }
+        Tensor inv_den = c.alloc(F32, {n, heads_});
+        o = c.alloc(F32, {n, heads_, dv_});
         K::mlstm_gates((const float*)z.data, z.cols(), (const float*)gate_bias_->t.data, cap_, in.data, at(in, qk), dtype, row_, q_scale_, state, row,
                        head_stride(), m_offset, c.dev.cu, c.dev.seq_new, c.dev.seq_slot, (float*)kappa.data, (float*)tau.data, (float*)m.data,
                        (float*)inv_den.data, c.n_seqs, heads_, d_, c.stream);
@@ -119,17 +142,21 @@ public:
                             (const float*)tau.data, (const float*)inv_den.data, q_scale_, 1.f, nullptr, nullptr, 0, 0, 0, c.dev.tok_pos, state, row, c.dev.cu,
                             c.dev.seq_new, c.dev.seq_slot, nullptr, nullptr, nullptr, nullptr, (float*)o.data, 0, c.n_seqs, heads_, d_, dv_, head_stride(),
                             c.stream);
-        Tensor gated = c.alloc(dtype, {n, vv});
-        K::head_norm_gate((const float*)o.data, (const float*)norm_w_->t.data, dv_, eps_, at(in, 2 * qk + vv), dtype, row_, 1, gated.data, dtype, (int)n, heads_,
-                          dv_, c.stream);
+        K::head_norm_gate((const float*)o.data, norm_w, dv_, eps_, gate, dtype, row_, 1, gated.data, dtype, (int)n, heads_, dv_, c.stream);
+        return finish(c, gated, stream);
+    }
+
+private:
+    // steps that bring so many tokens of some sequence run in chunks on the matrix cores, shorter ones token by token
+    static const int CHUNKED_FROM = 32, CHUNK = 64;
+
+    Tensor finish(StepContext& c, const Tensor& gated, Stream* stream) {
         if (stream) {
             add_product(c, *stream, gated, w_o_);
             return Tensor();
         }
-        return linear(c, gated, w_o_, nullptr, dtype).t;
+        return linear(c, gated, w_o_, nullptr, gated.dtype).t;
     }
-
-private:
     int64_t head_stride() const { return (int64_t)d_ * dv_ + d_; }
 
     int64_t hidden_, row_ = 0;

@@ -480,6 +480,23 @@ int tqk_mlstm_gates(const float* z, long long z_stride, const float* bias, float
                     const int32_t* seq_new, const int32_t* seq_slot, float* kappa, float* tau, float* m, float* inv_den, int n_seqs, int heads,
                     int d, void* stream);
 
+/* The same memory for steps of many tokens, bfloat16, on the matrix cores, where tqk_mlstm_chunks_supported(d, dv): tqk_mlstm_gate_scan leaves kappa,
+ * tau and m (in another order of the sums than tqk_mlstm_gates) and carries m in the state.  Chunks of up to 64 tokens as tqk_ssm_chunks takes them:
+ * tqk_mlstm_local leaves a chunk's own part of the state [chunks][heads][d * dv | d] and its decay [chunks][heads]; tqk_chunk_carry (p_stride
+ * heads, p_div d * dv + d) turns that into the state every chunk starts from; tqk_mlstm_apply gives the outputs: out [tokens, heads, dv]
+ * float32, or with out null (where tqk_mlstm_apply_norms(dv)) gated [tokens, heads * dv] bfloat16 = the heads divided by their root mean
+ * square, times norm_weight [heads, dv], times sigmoid(gate) (rows `stride` apart). */
+int tqk_mlstm_chunks_supported(int d, int dv);
+int tqk_mlstm_apply_norms(int dv);
+int tqk_mlstm_gate_scan(const float* z, long long z_stride, const float* bias, float cap, float* state, long long state_stride, long long m_offset,
+                        const int32_t* cu, const int32_t* seq_new, const int32_t* seq_slot, float* kappa, float* tau, float* m, int n_seqs,
+                        int heads, void* stream);
+int tqk_mlstm_local(const void* k, const void* v, long long stride, const float* kappa, const float* tau, const int32_t* chunk_row0,
+                    const int32_t* chunk_count, int n_chunks, float* chunk_state, float* chunk_decay, int heads, int d, int dv, void* stream);
+int tqk_mlstm_apply(const void* q, const void* k, const void* v, long long stride, const float* kappa, const float* tau, const float* m,
+                    float q_scale, const int32_t* chunk_row0, const int32_t* chunk_count, int n_chunks, float* chunk_state, float* out,
+                    const float* norm_weight, float eps, const void* gate, void* gated, int heads, int d, int dv, void* stream);
+
 /* Attention over a window plus pooled blocks (pooled_attention.hip).  Pages: keys [kv heads][page + tqk_pooled_rows(pool)][d], values
  * likewise with dv; a block's means lie behind the positions of the page that holds its last position.  tqk_pooled_store: qkv
  * [tokens, (heads + kv heads) d + kv heads dv]; normed: q and k heads are divided by their root mean square (times q_weight, k_weight
