@@ -398,7 +398,7 @@ def streams_shapes(width, layers=4):
 
 
 def memory_shapes(width, layers=4):
-    """A Rasodra configuration (matrix memory without a feed-forward, latent attention twice, chunked attention) and a Nikasun one (latent
+    """A Rasodra configuration (matrix memory without a feed-forward, latent attention, chunked attention, latent attention) and a Nikasun one (latent
     attention in every layer, the first without a feed-forward) of the same width, depth, heads, head sizes and latent, and as many
     multiply-adds in the feed-forward products."""
     heads, dim = width // 128, 128
@@ -409,7 +409,7 @@ def memory_shapes(width, layers=4):
     latent = {"heads": heads, "dim": dim, "rot_dim": 64, "vdim": dim, "kv_rank": 512, "scale": (dim + 64) ** -0.5, "rot": rot}
     chunked = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": 1024}, "rot": rot}
     dense = {"kind": "dense", "ff": ff}
-    kinds = [("mlstm", memory, None), ("latent_attention", latent, dense), ("latent_attention", latent, dense), ("attention", chunked, dense)]
+    kinds = [("mlstm", memory, None), ("latent_attention", latent, dense), ("attention", chunked, dense), ("latent_attention", latent, dense)]
     lay = [{"type": kinds[l % 4][0], "mixer": kinds[l % 4][1], "mlp": kinds[l % 4][2]} for l in range(layers)]
     rasodra = {"architecture": "Rasodra", "vocab": 32000, "width": width, "norm": {"eps": 1e-5}, "layers": lay, "max_positions": 8192}
     # a gated feed-forward is three products, Rasodra's two

@@ -52,6 +52,8 @@ TQ_KERNEL(attention_prefill_capped, cptr, cptr, cptr, ci32, ci32, int, int, int,
 TQ_KERNEL(swiglu, cptr, void*, int, int, int, void*);
 TQ_KERNEL(gated_act, cptr, void*, int, int, int, int, float, float, void*);
 TQ_KERNEL(fused_gated_act, cptr, cf32, int, float, cptr, int, void*, int, int, int, int, float, float, void*);
+TQ_KERNEL(fused_store_act, cptr, cptr, int, void*, int, int, int, int, float, float, void*);
+TQ_KERNEL(mid_store_act, cptr, cptr, void*, int, int, int, void*, int, float, float, void*);
 TQ_KERNEL(mid_gated_act, cptr, cptr, void*, int, int, int, void*, int, float, float, void*);
 TQ_QUERY(int, latent_max_rank);
 TQ_QUERY(int, latent_max_row);
@@ -110,6 +112,7 @@ TQ_QUERY(int, streams_max);
 TQ_KERNEL(streams_fill, cf32, float*, int, int, int, void*);
 TQ_KERNEL(streams_step, float*, int, cptr, int, cf32, cf32, cf32, cf32, cf32, float, float*, void*, int, int, int, int, void*);
 TQ_KERNEL(add_layer_norm, float*, cptr, int, ci32, int, cf32, cf32, float, cf32, cf32, float, void*, int, int, int, void*);
+TQ_KERNEL(add_layer_norm_sums, float*, cptr, int, cf32, int, int, ci32, int, cf32, cf32, float, cf32, cf32, float, void*, int, int, int, void*);
 TQ_KERNEL(token_shift, cf32, cf32, float*, long long, ci32, ci32, ci32, ci32, void*, int, int, int, int, void*);
 TQ_KERNEL(shift_remember, cf32, float*, long long, ci32, ci32, ci32, int, int, void*);
 TQ_QUERY(int, linear_attention_max_dim);

@@ -273,6 +273,28 @@ Tensor gated_linear(StepContext& c, const Tensor& x, const Weight& w, const Gate
     return act;
 }
 
+Tensor activated_linear(StepContext& c, const Tensor& x, const Weight& w, const Gate& gate) {
+    const int64_t m = x.shape[0];
+    if (skinny_ok(x, w)) {
+        Tensor act = c.alloc(BF16, {m, w.n});
+        int packed = 0;
+        const void* wp = few_ptr(w, &packed);
+        K::fused_store_act(x.data, wp, packed, act.data, (int)m, (int)w.n, (int)w.k, gate.kind, gate.limit, gate.alpha, c.stream);
+        return act;
+    }
+    if (mid_ok(x, w)) {
+        Tensor act = c.alloc(BF16, {m, w.n});
+        const int splits = K::mid_splits.raw((int)w.n, (int)w.k, 0);
+        Tensor scratch;
+        if (splits > 1) scratch = c.alloc(F32, {splits, m, w.n});
+        K::mid_store_act(x.data, w.packed->t.data, act.data, (int)m, (int)w.n, (int)w.k, scratch.data, gate.kind, gate.limit, gate.alpha, c.stream);
+        return act;
+    }
+    Tensor u = linear(c, x, w, nullptr, x.dtype).t;
+    K::unary_act(u.data, u.data, u.dtype, (long long)u.numel(), gate.kind, gate.limit, gate.alpha, c.stream);
+    return u;
+}
+
 // The few-row kernel that adds to the stream keeps one block per tile of 16 features, a block stays on one compute
 // unit, and a compute unit alone pulls about a 256th of what the memory gives when all of them pull.  Where the tiles
 // fall badly on the units (the 320 tiles of a 5120-wide product on 256 units: a quarter of the units work twice as long

@@ -80,6 +80,8 @@ struct Gate {
 // gate(x Wg^T, x Wu^T) with Wg stacked on Wu: [M, K] x [2I, K] -> [M, I]
 Tensor gated_linear(StepContext& c, const Tensor& x, const Weight& w_gate_up, const Gate& gate);
 inline Tensor gated_silu_linear(StepContext& c, const Tensor& x, const Weight& w_gate_up) { return gated_linear(c, x, w_gate_up, Gate()); }
+// f(x W^T) with f the gate's function of one product: [M, K] x [N, K] -> [M, N]
+Tensor activated_linear(StepContext& c, const Tensor& x, const Weight& w, const Gate& gate);
 // Several loaded tensors stacked along their first dimension (float32 if any of them is), then zero rows up to a
 // multiple of pad_rows_to.
 OwnedPtr stack_rows(const std::vector<OwnedPtr>& parts, hipStream_t stream, int64_t pad_rows_to = 1);

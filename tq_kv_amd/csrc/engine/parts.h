@@ -63,7 +63,7 @@ struct PartialSums {
 
 // An update of the stream that has not been added yet: nothing, a tensor of the activation
 // dtype, or a product's partial sums (only for a norm that takes those).
-// norm (with a plain tensor): the update is normed by it before it is added; only for a norm that takes such updates.
+// norm: the update is normed by it before it is added; only for a norm that takes such updates.
 struct Pending {
     enum Kind { Nothing, Plain, Sums };
     Kind kind = Nothing;

@@ -871,16 +871,16 @@ public:
         Activation x = normed(c, *mixer_norm_, *stream, mixer_->folds_norm(c));
         {
             Span span(mixer_->trace_name());
-            const bool adds = (c.fuse_small || c.fuse_mid) && !post_mixer_norm_ && mixer_->adds_to_stream(c);
-            if (adds) stream->next_norm = feed_forward_ ? ff_norm_.get() : next_norm;
-            settle(c, *stream, mixer_->forward(c, x, entry, adds ? stream : nullptr, false), post_mixer_norm_.get(),
-                   feed_forward_ ? ff_norm_.get() : next_norm);
+            Norm* reader = feed_forward_ ? ff_norm_.get() : next_norm;
+            const bool adds = may_add(c, post_mixer_norm_.get(), reader) && mixer_->adds_to_stream(c);
+            if (adds) stream->next_norm = reader;
+            settle(c, *stream, mixer_->forward(c, x, entry, adds ? stream : nullptr, false), post_mixer_norm_.get(), reader);
         }
         if (!feed_forward_) return stream;
         x = normed(c, *ff_norm_, *stream, feed_forward_->folds_norm(c));
         {
             Span span(feed_forward_->trace_name());
-            const bool adds = (c.fuse_small || c.fuse_mid) && !post_ff_norm_ && feed_forward_->adds_to_stream(c);
+            const bool adds = may_add(c, post_ff_norm_.get(), next_norm) && feed_forward_->adds_to_stream(c);
             if (adds) stream->next_norm = next_norm;
             settle(c, *stream, feed_forward_->forward(c, x, adds ? stream : nullptr), post_ff_norm_.get(), next_norm);
         }
@@ -904,9 +904,19 @@ private:
         stream.invalidate();
         return a;
     }
+    // Whether a part may be given the stream.  With an output norm it must not be added yet: only in steps whose products are left pending
+    // (as sums over pieces of K), for a next norm that applies the output norm first.
+    static bool may_add(const StepContext& c, const Norm* post_norm, const Norm* next_norm) {
+        if (!post_norm) return c.fuse_small || c.fuse_mid;
+        return c.fuse_mid && next_norm && next_norm->takes_normed_update(post_norm) && next_norm->takes_partial_sums();
+    }
     // a part's output that it did not add to the stream itself is left pending for the next norm's kernel
+    // (an output norm that goes with the next norm's kernel: what a part left pending on the stream is that norm's to read)
     void settle(StepContext& c, Stream& stream, Tensor out, Norm* post_norm, const Norm* next_norm) {
-        if (!out.defined()) return;
+        if (!out.defined()) {
+            if (post_norm) stream.pending.norm = post_norm;
+            return;
+        }
         const bool together = post_norm && next_norm && next_norm->takes_normed_update(post_norm);
         if (post_norm && !together) {
             Tensor y = c.alloc(out.dtype, {out.shape[0], out.shape[1]});

@@ -10,7 +10,7 @@
 //
 // The state of a sequence is one float32 row of the cache's state groups (zero when a slot is taken): per head S and n one behind the
 // other, then the heads' m.  Gates, maxima, n, S and the heads' norm are float32 whatever the activation type, and so are the gates'
-// products' results; q, k, v and the output gate come from one product with the weights stacked.  Steps that bring many tokens of a
+// products' results; q, k, v, the output gate and the gates come from one product with the weights stacked.  Steps that bring many tokens of a
 // sequence in bfloat16 run in chunks on the matrix cores (mlstm.hip), with the heads' norm and the gate in the last of their kernels.
 //
 // params: hidden, heads, head_dim, value_dim, gate_cap, eps; optional q_scale (head_dim^(-1/2) unless given), names {q, k, v, g, o, norm, i,
@@ -71,9 +71,10 @@ public:
     }
     void load(Loaded& t, hipStream_t stream) override {
         // (rows up to a multiple of 16, so that the products' rows stay at multiples of 16 bytes whatever the sizes)
-        OwnedPtr in = stack_rows({take(t, n_q_), take(t, n_k_), take(t, n_v_), take(t, n_g_)}, stream, 16);
+        OwnedPtr in = stack_rows({take(t, n_q_), take(t, n_k_), take(t, n_v_), take(t, n_g_), take(t, n_i_), take(t, n_f_)}, stream, 16);
         row_ = in->t.shape[0];
         w_in_ = make_weight(in, 1, false, stream);
+        // (the gates' rows a second time, for steps whose other rows are wanted in bfloat16)
         w_gates_ = make_weight(stack_rows({take(t, n_i_), take(t, n_f_)}, stream, 16), 1, false, stream);
         gate_bias_ = as_floats(stack_rows({take(t, n_ib_), take(t, n_fb_)}, stream), stream);
         w_o_ = make_weight(take(t, n_o_), 1, false, stream);
@@ -89,7 +90,7 @@ public:
     }
     const char* trace_name() const override { return "mlstm"; }
     void product_shapes(std::vector<std::pair<int64_t, int64_t>>& out) const override {
-        out.push_back({(2LL * heads_ * d_ + 2LL * heads_ * dv_ + 15) / 16 * 16, hidden_});
+        out.push_back({(2LL * heads_ * d_ + 2LL * heads_ * dv_ + 2LL * heads_ + 15) / 16 * 16, hidden_});
         out.push_back({hidden_, (int64_t)heads_ * dv_});
     }
     CacheNeed cache_need() const override {
@@ -109,14 +110,17 @@ public:
         const long long row = entry.state.cols(), m_offset = heads_ * head_stride();
         float* state = (float*)entry.state.data + entry.state_offset;
         const int64_t qk = (int64_t)heads_ * d_, vv = (int64_t)heads_ * dv_;
-        const Tensor in = linear(c, x.x, w_in_, nullptr, dtype).t;                    // [q | k | v | g | padding]
-        const Tensor z = linear(c, x.x, w_gates_, nullptr, F32).t;                    // [i | f | padding]
+        // many tokens in bfloat16 run in chunks on the matrix cores, whose operands are bfloat16; else one product gives everything in float32
+        const bool chunked = dtype == BF16 && !c.all_decode && !c.capturing && c.max_new >= CHUNKED_FROM && !null_device() &&
+                             K::mlstm_chunks_supported.raw(d_, dv_);
+        const Tensor in = linear(c, x.x, w_in_, nullptr, chunked ? BF16 : F32).t;      // [q | k | v | g | i | f | padding]
+        const Tensor z = chunked ? linear(c, x.x, w_gates_, nullptr, F32).t : Tensor();
         Tensor kappa = c.alloc(F32, {n, heads_}), tau = c.alloc(F32, {n, heads_}), m = c.alloc(F32, {n, heads_});
         Tensor gated = c.alloc(dtype, {n, vv});
         const float* norm_w = (const float*)norm_w_->t.data;
         const void* gate = at(in, 2 * qk + vv);
         Tensor o;
-        if (dtype == BF16 && !c.all_decode && !c.capturing && c.max_new >= CHUNKED_FROM && !null_device() && K::mlstm_chunks_supported.raw(d_, dv_)) {
+        if (chunked) {
             const Chunks ch = c.chunks(CHUNK);
             Tensor cs = c.alloc(F32, {ch.n, heads_, head_stride()}), cd = c.alloc(F32, {ch.n, heads_});
             const bool norms = K::mlstm_apply_norms.raw(dv_) != 0;
@@ -135,14 +139,14 @@ public:
         }
         Tensor inv_den = c.alloc(F32, {n, heads_});
         o = c.alloc(F32, {n, heads_, dv_});
-        K::mlstm_gates((const float*)z.data, z.cols(), (const float*)gate_bias_->t.data, cap_, in.data, at(in, qk), dtype, row_, q_scale_, state, row,
+        K::mlstm_gates((const float*)at(in, 2 * qk + 2 * vv), row_, (const float*)gate_bias_->t.data, cap_, in.data, at(in, qk), F32, row_, q_scale_, state, row,
                        head_stride(), m_offset, c.dev.cu, c.dev.seq_new, c.dev.seq_slot, (float*)kappa.data, (float*)tau.data, (float*)m.data,
                        (float*)inv_den.data, c.n_seqs, heads_, d_, c.stream);
-        K::linear_attention(in.data, at(in, qk), at(in, 2 * qk), dtype, row_, nullptr, 0, nullptr, 0.f, nullptr, (const float*)kappa.data,
+        K::linear_attention(in.data, at(in, qk), at(in, 2 * qk), F32, row_, nullptr, 0, nullptr, 0.f, nullptr, (const float*)kappa.data,
                             (const float*)tau.data, (const float*)inv_den.data, q_scale_, 1.f, nullptr, nullptr, 0, 0, 0, c.dev.tok_pos, state, row, c.dev.cu,
                             c.dev.seq_new, c.dev.seq_slot, nullptr, nullptr, nullptr, nullptr, (float*)o.data, 0, c.n_seqs, heads_, d_, dv_, head_stride(),
                             c.stream);
-        K::head_norm_gate((const float*)o.data, norm_w, dv_, eps_, gate, dtype, row_, 1, gated.data, dtype, (int)n, heads_, dv_, c.stream);
+        K::head_norm_gate((const float*)o.data, norm_w, dv_, eps_, gate, F32, row_, 1, gated.data, dtype, (int)n, heads_, dv_, c.stream);
         return finish(c, gated, stream);
     }
 

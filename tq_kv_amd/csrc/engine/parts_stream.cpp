@@ -106,11 +106,15 @@ public:
         out.push_back({inter_, hidden_});
         out.push_back({hidden_, inter_});
     }
-    Tensor forward(StepContext& c, const Activation& x, Stream*) override {
+    bool adds_to_stream(const StepContext& c) const override { return fusable(c.n_tokens, w_down_, true) || leaves_sums(c.n_tokens, w_down_); }
+    Tensor forward(StepContext& c, const Activation& x, Stream* stream) override {
         if (x.lazy) raise(TQE_ERR_STATE, "activated takes no folded norm");
-        Tensor u = linear(c, x.x, w_up_, nullptr, x.x.dtype).t;
-        K::unary_act(u.data, u.data, u.dtype, (long long)u.numel(), act_.kind, act_.limit, act_.alpha, c.stream);
-        return linear(c, u, w_down_, nullptr, x.x.dtype).t;
+        const Tensor act = activated_linear(c, x.x, w_up_, act_);
+        if (stream) {
+            add_product(c, *stream, act, w_down_);
+            return Tensor();
+        }
+        return linear(c, act, w_down_, nullptr, x.x.dtype).t;
     }
 
 private:

@@ -3,7 +3,7 @@
 //   norm  layer_norm   (x - mean) / sqrt(var + eps) w + b, the variance the mean of the squared deviations; float32 arithmetic.
 //                      params: size, eps; optional tensor (the weight's name, "weight" unless given; may be empty), bias (false: the norm has
 //                      none) and bias_tensor ("bias" unless given).  An update of the stream that is to be normed by another layer_norm before
-//                      it is added takes one kernel with the sum and this norm.
+//                      it is added takes one kernel with the sum and this norm, and so does a product's sums over pieces of its K.
 //   block multi_stream pre-norm around a mixer and an optional feed-forward, with `streams` copies X[0..S) of the stream in place of
 //                      the one.  A sublayer reads u = sum_s in[s] X[s], computes y = part(norm(u)), and all copies are updated at
 //                      once from the old ones: X'[r] = sum_s mix[s, r] X[s] + out[r] y.  Every copy starts as the stream the block
@@ -85,12 +85,13 @@ public:
     void forward(StepContext& c, const Tensor& x, Tensor& out) override {
         K::add_layer_norm(nullptr, x.data, x.dtype, nullptr, (int)x.shape[0], weight(), bias(), eps_, nullptr, nullptr, 0.f, out.data, out.dtype, (int)size_, 0, c.stream);
     }
+    bool takes_partial_sums() const override { return true; }
     bool takes_normed_update(const Norm* norm) const override {
         const LayerNorm* n = dynamic_cast<const LayerNorm*>(norm);
         return n && n->size_ == size_;
     }
     void add_norm(StepContext& c, Tensor& h, const Pending& delta, Tensor& out) override {
-        run(c, h, delta, nullptr, h.shape[0], out, delta.kind == Pending::Plain);
+        run(c, h, delta, nullptr, h.shape[0], out, delta.kind != Pending::Nothing);
     }
     void gather_add_norm(StepContext& c, const Tensor& h, const Pending& delta, const int32_t* rows, int64_t n_rows, Tensor& out) override {
         run(c, h, delta, rows, n_rows, out, false);
@@ -98,12 +99,15 @@ public:
 
 private:
     void run(StepContext& c, const Tensor& h, const Pending& delta, const int32_t* rows, int64_t n_rows, Tensor& out, bool write_back) {
-        if (delta.kind == Pending::Sums) raise(TQE_ERR_STATE, "layer_norm takes no unfinished product");
-        const bool d = delta.kind == Pending::Plain;
-        const LayerNorm* n = d && delta.norm ? dynamic_cast<const LayerNorm*>(delta.norm) : nullptr;
-        if (d && delta.norm && !n) raise(TQE_ERR_STATE, "layer_norm: an update that is to be normed by a part of kind '%s' first", delta.norm->kind.c_str());
-        K::add_layer_norm((float*)h.data, d ? delta.t.data : nullptr, d ? delta.t.dtype : 0, rows, (int)n_rows, weight(), bias(), eps_, n ? n->weight() : nullptr,
-                          n ? n->bias() : nullptr, n ? n->eps() : 0.f, out.data, out.dtype, (int)size_, write_back ? 1 : 0, c.stream);
+        const bool d = delta.kind == Pending::Plain, sums = delta.kind == Pending::Sums;
+        const LayerNorm* n = (d || sums) && delta.norm ? dynamic_cast<const LayerNorm*>(delta.norm) : nullptr;
+        if ((d || sums) && delta.norm && !n) raise(TQE_ERR_STATE, "layer_norm: an update that is to be normed by a part of kind '%s' first", delta.norm->kind.c_str());
+        if (sums && (delta.s.rows() != h.shape[0] || delta.s.cols() != size_))
+            raise(TQE_ERR_STATE, "layer_norm: the update's sums are [%lld, %lld] for a stream of [%lld, %lld]", (long long)delta.s.rows(), (long long)delta.s.cols(),
+                  (long long)h.shape[0], (long long)size_);
+        K::add_layer_norm_sums((float*)h.data, d ? delta.t.data : nullptr, d ? delta.t.dtype : sums ? delta.s.dtype : 0, sums ? (const float*)delta.s.sums.data : nullptr,
+                               sums ? (int)delta.s.sums.shape[0] : 0, sums ? (int)delta.s.rows() : 0, rows, (int)n_rows, weight(), bias(), eps_,
+                               n ? n->weight() : nullptr, n ? n->bias() : nullptr, n ? n->eps() : 0.f, out.data, out.dtype, (int)size_, write_back ? 1 : 0, c.stream);
     }
 
     int act_dtype_;

@@ -48,6 +48,7 @@ struct MidArgs {
     int M, N, K, k_per_split;   // k_per_split: a multiple of MID_CHUNK
     int gate;                   // gated: which gate (TQK_GATE_*), with its limit and alpha
     float gate_limit, gate_alpha;
+    int activated;              // store: the gate's function of the product itself is applied (act_value)
 };
 
 __device__ __forceinline__ uint2 pack4_bf16(float a, float b, float c, float d) {
@@ -55,10 +56,13 @@ __device__ __forceinline__ uint2 pack4_bf16(float a, float b, float c, float d) 
                       (uint32_t)float_to_bf16_bits(c) | ((uint32_t)float_to_bf16_bits(d) << 16));
 }
 
-struct Gate { int kind; float limit, alpha; };
+struct Gate { int kind; float limit, alpha; int activated; };
 __device__ __forceinline__ float gate_times_up(const Gate& gate, float gate_sum, float up_sum) {
     const float g = to_float(from_float<bf16_t>(gate_sum)), up = to_float(from_float<bf16_t>(up_sum));
     return gate_value(gate.kind, gate.limit, gate.alpha, g, up);
+}
+__device__ __forceinline__ float finished(const Gate& gate, float sum) {
+    return gate.activated ? act_value(gate.kind, gate.limit, gate.alpha, to_float(from_float<bf16_t>(sum))) : sum;
 }
 
 // MT: groups of 16 rows of x (2: up to 32 rows, 4: up to 64, 8: up to 128).  TN: tiles of 16
@@ -270,6 +274,10 @@ void mid_product_kernel(const MidArgs p) {
                 const int n = n_lo0 + 16 * t + nb;
                 if (m >= p.M) continue;
                 TY* dst = y + (size_t)m * p.N + n;
+                if (p.activated) {
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) acc[t][mt][r] = finished(Gate{p.gate, p.gate_limit, p.gate_alpha, 1}, acc[t][mt][r]);
+                }
                 if (vec && n + 3 < p.N) {
                     if constexpr (sizeof(TY) == 4) *reinterpret_cast<floatx4_t*>(dst) = acc[t][mt];
                     else *reinterpret_cast<uint2*>(dst) = pack4_bf16(acc[t][mt][0], acc[t][mt][1], acc[t][mt][2], acc[t][mt][3]);
@@ -289,7 +297,7 @@ void mid_product_kernel(const MidArgs p) {
             if (m >= p.M) continue;
             float o[4];
 #pragma unroll
-            for (int r = 0; r < 4; ++r) o[r] = gate_times_up(Gate{p.gate, p.gate_limit, p.gate_alpha}, acc[0][mt][r], acc[TN - 1][mt][r]);
+            for (int r = 0; r < 4; ++r) o[r] = gate_times_up(Gate{p.gate, p.gate_limit, p.gate_alpha, 0}, acc[0][mt][r], acc[TN - 1][mt][r]);
             bf16_t* dst = y + (size_t)m * n_out + n;
             if (vec && n + 3 < n_out) { *reinterpret_cast<uint2*>(dst) = pack4_bf16(o[0], o[1], o[2], o[3]); continue; }
 #pragma unroll
@@ -313,7 +321,7 @@ __global__ void mid_finish_kernel(const float* __restrict__ partial, void* __res
         if (EPI == MID_GATED) b += src[n_out + n];
     }
     if (EPI == MID_GATED) ((bf16_t*)yv)[i] = from_float<bf16_t>(gate_times_up(gate, a, b));
-    else ((TY*)yv)[i] = from_float<TY>(a);
+    else ((TY*)yv)[i] = from_float<TY>(finished(gate, a));
 }
 
 // How a product of this shape is cut: tiles per wave, waves per block, splits of K.  From N and K
@@ -408,7 +416,7 @@ static int launch_mid(const MidArgs& a, const MidPlan& plan, bool finish, hipStr
     if (tqk_check_launch("tqk_mid product")) return -1;
     if (plan.splits > 1 && finish) {
         const size_t total = (size_t)a.M * (EPI == MID_GATED ? a.N / 2 : a.N);
-        mid_finish_kernel<EPI, TY><<<(unsigned)((total + 255) / 256), 256, 0, s>>>(a.partial, a.y, plan.splits, a.M, a.N, Gate{a.gate, a.gate_limit, a.gate_alpha});
+        mid_finish_kernel<EPI, TY><<<(unsigned)((total + 255) / 256), 256, 0, s>>>(a.partial, a.y, plan.splits, a.M, a.N, Gate{a.gate, a.gate_limit, a.gate_alpha, a.activated});
         return tqk_check_launch("tqk_mid finish");
     }
     return 0;
@@ -443,7 +451,7 @@ static int check_mid(const MidArgs& a, const void* scratch, bool gated, bool fin
  * (for tqk_add_rmsnorm_sums) and y is not written. */
 extern "C" int tqk_mid_store(const void* x, const void* w_packed, void* y, int y_dtype, int M, int N, int K,
                              void* scratch, int finish, void* stream) {
-    MidArgs a = {(const bf16_t*)x, (const bf16_t*)w_packed, y, (float*)scratch, M, N, K, 0, 0, 0.f, 1.f};
+    MidArgs a = {(const bf16_t*)x, (const bf16_t*)w_packed, y, (float*)scratch, M, N, K, 0, 0, 0.f, 1.f, 0};
     if (check_mid(a, scratch, false, finish != 0, "tqk_mid_store")) return -1;
     TQK_REQUIRE(y_dtype == TQK_F32 || y_dtype == TQK_BF16, "tqk_mid_store: unknown output dtype %d", y_dtype);
     if (M == 0) return 0;
@@ -452,6 +460,18 @@ extern "C" int tqk_mid_store(const void* x, const void* w_packed, void* y, int y
     hipStream_t s = (hipStream_t)stream;
     return y_dtype == TQK_F32 ? launch_rows<MID_STORE, float>(a, plan, finish != 0, s)
                               : launch_rows<MID_STORE, bf16_t>(a, plan, finish != 0, s);
+}
+
+/* y[M,N] = f(x w^T) in bfloat16, f a gate's function of one product (TQK_GATE_*: common.h). */
+extern "C" int tqk_mid_store_act(const void* x, const void* w_packed, void* y, int M, int N, int K, void* scratch, int gate, float limit, float alpha,
+                                 void* stream) {
+    TQK_REQUIRE(gate >= 0 && gate < TQK_GATE_KINDS, "tqk_mid_store_act: unknown activation %d", gate);
+    MidArgs a = {(const bf16_t*)x, (const bf16_t*)w_packed, y, (float*)scratch, M, N, K, 0, gate, limit, alpha, 1};
+    if (check_mid(a, scratch, false, true, "tqk_mid_store_act")) return -1;
+    if (M == 0) return 0;
+    const MidPlan plan = mid_plan(N, K, false);
+    a.k_per_split = plan.k_per_split;
+    return launch_rows<MID_STORE, bf16_t>(a, plan, true, (hipStream_t)stream);
 }
 
 /* y[M, N/2] = silu(gate) * up, w = gate rows then up rows, packed in two parts. */
@@ -463,7 +483,7 @@ extern "C" int tqk_mid_gated(const void* x, const void* w_packed, void* y, int M
 extern "C" int tqk_mid_gated_act(const void* x, const void* w_packed, void* y, int M, int N, int K, void* scratch, int gate, float limit,
                                  float alpha, void* stream) {
     TQK_REQUIRE(gate >= 0 && gate < TQK_GATE_KINDS, "tqk_mid_gated: unknown gate %d", gate);
-    MidArgs a = {(const bf16_t*)x, (const bf16_t*)w_packed, y, (float*)scratch, M, N, K, 0, gate, limit, alpha};
+    MidArgs a = {(const bf16_t*)x, (const bf16_t*)w_packed, y, (float*)scratch, M, N, K, 0, gate, limit, alpha, 0};
     if (check_mid(a, scratch, true, true, "tqk_mid_gated")) return -1;
     if (M == 0) return 0;
     const MidPlan plan = mid_plan(N, K, true);

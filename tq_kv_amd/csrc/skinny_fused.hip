@@ -38,7 +38,7 @@
 // sums by sqrt(mean + eps).  The statistics are those of the float32 stream.
 //
 // Back ends:
-//   store     y = result (bfloat16 or float32)
+//   store     y = result (bfloat16 or float32), or an activation of it
 //   gated     rows n and n_out + n of w are gate and up: y = silu(gate) * up
 //             (src/models/turbo_generic.rs:105-111)
 //   residual  h += bfloat16(result) in float32: the residual sum of
@@ -80,6 +80,7 @@ struct FusedArgs {
     void* y;
     int gate;                   // gated: which gate (TQK_GATE_*), with its limit and alpha
     float gate_limit, gate_alpha;
+    int activated;              // store: the gate's function of the product itself is applied (act_value)
     // residual
     float* h;                   // [M, N]
     const bf16_t* next_norm_w;  // [N] weight of the norm that follows, or null
@@ -315,7 +316,9 @@ void skinny_fused_kernel(const FusedArgs p) {
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int n = n_lo0 + 16 * t + nb + r;
-                if (n < p.N) y[(size_t)m * p.N + n] = from_float<TY>(acc[t][r] * inv_rms);
+                float v = acc[t][r] * inv_rms;
+                if (p.activated) v = act_value(p.gate, p.gate_limit, p.gate_alpha, to_float(from_float<bf16_t>(v)));
+                if (n < p.N) y[(size_t)m * p.N + n] = from_float<TY>(v);
             }
     } else if constexpr (EPI == EPI_GATED) {
         bf16_t* y = (bf16_t*)p.y;
@@ -471,6 +474,18 @@ extern "C" int tqk_fused_store(const void* x, const int32_t* x_rows, const float
     }
     if (ss_parts) return y_dtype == TQK_F32 ? launch_tiled<true, EPI_STORE, float>(a, s) : launch_tiled<true, EPI_STORE, bf16_t>(a, s);
     return y_dtype == TQK_F32 ? launch_tiled<false, EPI_STORE, float>(a, s) : launch_tiled<false, EPI_STORE, bf16_t>(a, s);
+}
+
+/* y[M,N] = f(x w^T) in bfloat16, f a gate's function of one product (TQK_GATE_*: common.h). */
+extern "C" int tqk_fused_store_act(const void* x, const void* w, int w_packed, void* y, int M, int N, int K, int gate, float limit, float alpha, void* stream) {
+    TQK_REQUIRE(gate >= 0 && gate < TQK_GATE_KINDS, "tqk_fused_store_act: unknown activation %d", gate);
+    FusedArgs a = {};
+    a.x = (const bf16_t*)x; a.w = (const bf16_t*)w; a.w_packed = w_packed; a.M = M; a.N = N; a.K = K; a.y = y;
+    a.activated = 1; a.gate = gate; a.gate_limit = limit; a.gate_alpha = alpha;
+    if (check_common(a, "tqk_fused_store_act")) return -1;
+    TQK_REQUIRE(y, "tqk_fused_store_act: null output");
+    if (M == 0) return 0;
+    return launch_tiled<false, EPI_STORE, bf16_t>(a, (hipStream_t)stream);
 }
 
 /* y[M, N/2] = silu(gate) * up of the (normalised) product, w = gate rows then up rows. */

@@ -125,6 +125,20 @@ __global__ void unary_act_kernel(const TA* __restrict__ x, TA* __restrict__ out,
     if (i < n) out[i] = from_float<TA>(act_value(kind, limit, alpha, to_float(x[i])));
 }
 
+// the same with eight bfloat16 elements a thread
+__global__ void unary_act_vec_kernel(const uint4* __restrict__ x, uint4* __restrict__ out, long long n8, int kind, float limit, float alpha) {
+    const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= n8) return;
+    const uint4 v = x[i];
+    const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+    uint32_t o[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k)
+        o[k] = (uint32_t)float_to_bf16_bits(act_value(kind, limit, alpha, __uint_as_float(w[k] << 16))) |
+               ((uint32_t)float_to_bf16_bits(act_value(kind, limit, alpha, __uint_as_float(w[k] & 0xffff0000u))) << 16);
+    out[i] = make_uint4(o[0], o[1], o[2], o[3]);
+}
+
 // out[t] = sigmoid(x[t] . w), a wave per token
 template <typename TA, typename TW>
 __global__ __launch_bounds__(256)
@@ -193,6 +207,10 @@ extern "C" int tqk_unary_act(const void* x, void* out, int act_dtype, long long 
     const long long blocks = (n + 255) / 256;
     TQK_REQUIRE(blocks <= 0x7fffffff, "tqk_unary_act: too many elements");
     hipStream_t s = (hipStream_t)stream;
+    if (act_dtype == TQK_BF16 && n % 8 == 0 && (((uintptr_t)x | (uintptr_t)out) & 15) == 0) {
+        unary_act_vec_kernel<<<(unsigned)((n / 8 + 255) / 256), 256, 0, s>>>((const uint4*)x, (uint4*)out, n / 8, kind, limit, alpha);
+        return tqk_check_launch("tqk_unary_act");
+    }
     if (act_dtype == TQK_F32) unary_act_kernel<float><<<(unsigned)blocks, 256, 0, s>>>((const float*)x, (float*)out, n, kind, limit, alpha);
     else if (act_dtype == TQK_BF16) unary_act_kernel<bf16_t><<<(unsigned)blocks, 256, 0, s>>>((const bf16_t*)x, (bf16_t*)out, n, kind, limit, alpha);
     else return tqk_fail("tqk_unary_act: unknown dtype %d", act_dtype);

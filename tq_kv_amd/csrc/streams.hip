@@ -96,6 +96,9 @@ struct LayerNormArgs {
     float peps;
     void* out;
     int W, write_back;
+    const float* sums;              // the update as the sums of a product over pieces of its K, [pieces][rows][W] (then delta is null)
+    int pieces, sums_bf16;          // sums_bf16: the finished product would have been rounded to bfloat16
+    long long piece_stride;
 };
 
 template <typename TD, typename TO>
@@ -106,20 +109,26 @@ void add_layer_norm_kernel(const LayerNormArgs a) {
     const int W = a.W;
     const size_t i = blockIdx.x, r = a.rows ? (size_t)a.rows[i] : i;
     const TD* delta = (const TD*)a.delta;
+    auto update = [&](int e) -> float {
+        if (!a.sums) return delta ? to_float(delta[r * W + e]) : 0.f;
+        float v = 0.f;
+        for (int p = 0; p < a.pieces; ++p) v += a.sums[(size_t)p * a.piece_stride + r * W + e];
+        return a.sums_bf16 ? to_float(from_float<bf16_t>(v)) : v;
+    };
     float pmean = 0.f, pinv = 1.f;
     if (a.pw) {
         float sum = 0.f;
-        for (int e = threadIdx.x; e < W; e += blockDim.x) sum += to_float(delta[r * W + e]);
+        for (int e = threadIdx.x; e < W; e += blockDim.x) sum += update(e);
         pmean = block_sum(sum, scratch) / (float)W;
         float ss = 0.f;
-        for (int e = threadIdx.x; e < W; e += blockDim.x) { const float dlt = to_float(delta[r * W + e]) - pmean; ss = fmaf(dlt, dlt, ss); }
+        for (int e = threadIdx.x; e < W; e += blockDim.x) { const float dlt = update(e) - pmean; ss = fmaf(dlt, dlt, ss); }
         pinv = 1.f / sqrtf(block_sum(ss, scratch) / (float)W + a.peps);
     }
     float sum = 0.f;
     for (int e = threadIdx.x; e < W; e += blockDim.x) {
         float v = a.h ? a.h[r * W + e] : 0.f;
-        if (delta) {
-            float d = to_float(delta[r * W + e]);
+        if (delta || a.sums) {
+            float d = update(e);
             if (a.pw) d = (d - pmean) * pinv * a.pw[e] + (a.pb ? a.pb[e] : 0.f);
             v += d;
         }
@@ -177,6 +186,18 @@ void add_layer_norm_vec_kernel(const LayerNormArgs a) {
         for (int j = 0; j < 4; ++j) d[k][j] = x[k][j] = 0.f;
         if (c < n4) {
             if (delta) load4(delta + 4 * c, d[k]);
+            if (a.sums) {
+                for (int p = 0; p < a.pieces; ++p) {
+                    float v[4];
+                    load4(a.sums + (size_t)p * a.piece_stride + r * W + 4 * c, v);
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) d[k][j] += v[j];
+                }
+                if (a.sums_bf16) {
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) d[k][j] = to_float(from_float<bf16_t>(d[k][j]));
+                }
+            }
             if (h) load4(h + 4 * c, x[k]);
         }
     }
@@ -306,16 +327,26 @@ extern "C" int tqk_streams_step(float* X, int n_streams, const void* y, int y_dt
 extern "C" int tqk_add_layer_norm(float* h, const void* delta, int delta_dtype, const int32_t* rows, int n_rows, const float* weight, const float* bias,
                                   float eps, const float* delta_weight, const float* delta_bias, float delta_eps, void* out, int out_dtype, int width,
                                   int write_back, void* stream) {
+    return tqk_add_layer_norm_sums(h, delta, delta_dtype, nullptr, 0, 0, rows, n_rows, weight, bias, eps, delta_weight, delta_bias, delta_eps, out, out_dtype, width,
+                                   write_back, stream);
+}
+
+extern "C" int tqk_add_layer_norm_sums(float* h, const void* delta, int delta_dtype, const float* sums, int pieces, int sum_rows, const int32_t* rows, int n_rows,
+                                       const float* weight, const float* bias, float eps, const float* delta_weight, const float* delta_bias, float delta_eps,
+                                       void* out, int out_dtype, int width, int write_back, void* stream) {
+    TQK_REQUIRE(!sums || (!delta && pieces > 0 && sum_rows > 0 && (rows || sum_rows == n_rows)), "tqk_add_layer_norm: sums of %d pieces of %d rows", pieces, sum_rows);
     TQK_REQUIRE((h || delta) && weight && out, "tqk_add_layer_norm: null pointer");
     TQK_REQUIRE(n_rows >= 0 && width > 0 && width <= 12288, "tqk_add_layer_norm: bad sizes");
     TQK_REQUIRE(!(write_back && rows), "tqk_add_layer_norm: chosen rows are not written back");
-    TQK_REQUIRE(!delta_weight || delta, "tqk_add_layer_norm: a norm of an update that is not there");
+    TQK_REQUIRE(!delta_weight || delta || sums, "tqk_add_layer_norm: a norm of an update that is not there");
     if (n_rows == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
-    const LayerNormArgs a = {h, delta, rows, weight, bias, eps, delta_weight, delta_bias, delta_eps, out, width, write_back};
+    const LayerNormArgs a = {h, delta, rows, weight, bias, eps, delta_weight, delta_bias, delta_eps, out, width, write_back, sums, pieces, delta_dtype == TQK_BF16,
+                             (long long)sum_rows * width};
     const int dd = delta ? delta_dtype : TQK_F32;
     TQK_REQUIRE((dd == TQK_F32 || dd == TQK_BF16) && (out_dtype == TQK_F32 || out_dtype == TQK_BF16), "tqk_add_layer_norm: unknown dtypes %d, %d", delta_dtype, out_dtype);
-    const uintptr_t all = (uintptr_t)h | (uintptr_t)delta | (uintptr_t)weight | (uintptr_t)bias | (uintptr_t)delta_weight | (uintptr_t)delta_bias | (uintptr_t)out;
+    const uintptr_t all = (uintptr_t)h | (uintptr_t)delta | (uintptr_t)weight | (uintptr_t)bias | (uintptr_t)delta_weight | (uintptr_t)delta_bias | (uintptr_t)out |
+                          (uintptr_t)sums;
     const bool vec = width % 4 == 0 && (all & 15) == 0;
     const size_t lds = (size_t)width * sizeof(float);
     // threads by the width alone, so that a row's sums have one order whatever the step holds

@@ -194,6 +194,10 @@ int tqk_fused_gated_act(const void* x, const float* ss_parts, int n_ss_parts, fl
                         int M, int N, int K, int gate, float limit, float alpha, void* stream);
 int tqk_mid_gated_act(const void* x, const void* w_packed, void* y, int M, int N, int K, void* scratch, int gate, float limit,
                       float alpha, void* stream);
+/* y[M,N] = f(x w^T) in bfloat16 for few and for mid-sized numbers of rows, f one of the gates above as a function of one product (u = 1) */
+int tqk_fused_store_act(const void* x, const void* w, int w_packed, void* y, int M, int N, int K, int gate, float limit, float alpha, void* stream);
+int tqk_mid_store_act(const void* x, const void* w_packed, void* y, int M, int N, int K, void* scratch, int gate, float limit, float alpha,
+                      void* stream);
 
 /* Attention through a low-rank latent (latent.hip).  Every position leaves one cache row [rk + dr]: the normed
  * latent and one rotated key part, shared by all heads; pages are [n_pages][64][rk + dr].
@@ -442,6 +446,11 @@ int tqk_streams_step(float* X, int n_streams, const void* y, int y_dtype, const 
 int tqk_add_layer_norm(float* h, const void* delta, int delta_dtype, const int32_t* rows, int n_rows, const float* weight, const float* bias,
                        float eps, const float* delta_weight, const float* delta_bias, float delta_eps, void* out, int out_dtype, int width,
                        int write_back, void* stream);
+/* The same with the update as a product's sums over pieces of its K, sums [pieces, sum_rows, width] (or null; then delta may be given): added up
+ * in their order and rounded to delta_dtype as the finished product would be. */
+int tqk_add_layer_norm_sums(float* h, const void* delta, int delta_dtype, const float* sums, int pieces, int sum_rows, const int32_t* rows, int n_rows,
+                            const float* weight, const float* bias, float eps, const float* delta_weight, const float* delta_bias, float delta_eps,
+                            void* out, int out_dtype, int width, int write_back, void* stream);
 int tqk_token_shift(const float* n, const float* mu, float* state, long long state_stride, const int32_t* tok_seq, const int32_t* tok_pos,
                     const int32_t* seq_start, const int32_t* seq_slot, void* out, int out_dtype, int n_tokens, int width, int remember,
                     void* stream);
