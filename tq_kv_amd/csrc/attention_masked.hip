@@ -8,7 +8,7 @@
 //   v_g <- (1 - lambda) v_g + lambda v'_g                                      (v' another layer's values of the token)
 //   s_ij = scale q_i . k_j;  s_ij <- cap tanh(s_ij / cap)
 //   i sees j  iff  j <= i and (window == 0 or i - j < window or j < keep_first), and, with chunks, floor(j / chunk) = floor(i / chunk)
-//   p_ij = exp(s_ij) / (sum_j' exp(s_ij') + exp(sink_h))
+//   p_ij = exp(s_ij) / (sum_j' exp(s_ij') + exp(sink_h));  the head's output times head_scale_ih where that is given
 //
 // Cache pages: keys [kv head][position][key_dim], values [kv head][value_dim][place of the position]
 // (value_place in common.h).
@@ -234,7 +234,7 @@ template <typename TB>
 __global__ __launch_bounds__(256)
 void biased_values_store_vec_kernel(const bf16_t* __restrict__ qkv, const TB* __restrict__ bias, const int32_t* __restrict__ tok_seq,
                                     const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ page_table, int table_width,
-                                    bf16_t* __restrict__ values, int n_tokens, int n_heads, int n_kv_heads, int dk, int dv) {
+                                    bf16_t* __restrict__ values, int n_tokens, int n_kv_heads, int dv, size_t row_stride, size_t values_at) {
     const int lane = threadIdx.x % TQK_WAVE, wave = threadIdx.x / TQK_WAVE, n_waves = blockDim.x / TQK_WAVE;
     const int t = (blockIdx.x / n_kv_heads) * TQK_WAVE + lane, g = blockIdx.x % n_kv_heads;
     if (t >= n_tokens) return;
@@ -242,9 +242,8 @@ void biased_values_store_vec_kernel(const bf16_t* __restrict__ qkv, const TB* __
     const int page = page_table[(size_t)tok_seq[t] * table_width + pos / TQK_PAGE];
     if (page < 0) return;                               // the host never lets this happen
     bf16_t* dst = values + ((size_t)page * n_kv_heads + g) * TQK_PAGE * dv + value_place(pos % TQK_PAGE);
-    const size_t total = (size_t)(n_heads + n_kv_heads) * dk + (size_t)n_kv_heads * dv;
-    const size_t off = (size_t)(n_heads + n_kv_heads) * dk + (size_t)g * dv;
-    const bf16_t* src = qkv + (size_t)t * total + off;
+    const size_t off = values_at + (size_t)g * dv;
+    const bf16_t* src = qkv + (size_t)t * row_stride + off;
     for (int c = wave * 8; c < dv; c += n_waves * 8) {
         const uint4 raw = *reinterpret_cast<const uint4*>(src + c);
         const uint32_t u[4] = {raw.x, raw.y, raw.z, raw.w};
@@ -408,6 +407,130 @@ void mixed_values_store_vec_kernel(const bf16_t* __restrict__ qkv, const TW* __r
     }
 }
 
+// ---- bias, a norm over the whole projection, rotation, a gate per head, cache write ---------------------------
+// A block per token.  A row is [H * dk | G * dk | G * dv | ... | H gate products at gate_at], rows row_stride apart; with no keys and values of
+// its own (kv false) a row is [H * dk | ... ] and the cache is left alone.  Biases (the row's layout) first; then all of q, and all of k, are
+// divided by the root mean square of the whole projection and multiplied by a weight of that size (weights null: not); then the heads' first
+// rot_dim elements are turned (style 1: in halves, 2: in neighbouring pairs).  gate_out[t, h] = sigmoid of the head's gate product.
+// VEC elements a load and store: 8 (bfloat16, sizes that fall into such pieces) or 1.  A row's sums are added up in an order that its
+// sizes alone decide.
+struct ProjectionArgs {
+    const void* rows;
+    long long row_stride;
+    const float *bias, *q_norm_w, *k_norm_w;
+    float eps;
+    const float *cos_table, *sin_table;
+    int rot_dim, style, max_positions;
+    const int32_t *tok_seq, *tok_pos, *page_table;
+    int table_width;
+    void *keys, *values, *q_out;
+    float* gate_out;
+    long long gate_at;
+    int n_heads, n_kv_heads, dk, dv, kv, store_values;
+};
+
+template <typename TA, int VEC> struct Piece {
+    __device__ static void load(const TA* p, float* v) { v[0] = to_float(p[0]); }
+    __device__ static void store(TA* p, const float* v) { p[0] = from_float<TA>(v[0]); }
+};
+template <> struct Piece<bf16_t, 8> {
+    __device__ static void load(const bf16_t* p, float* v) {
+        const uint4 raw = *reinterpret_cast<const uint4*>(p);
+        const uint32_t u[4] = {raw.x, raw.y, raw.z, raw.w};
+#pragma unroll
+        for (int j = 0; j < 4; ++j) { v[2 * j] = __uint_as_float(u[j] << 16); v[2 * j + 1] = __uint_as_float(u[j] & 0xffff0000u); }
+    }
+    __device__ static void store(bf16_t* p, const float* v) {
+        uint32_t u[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) u[j] = float_to_bf16_bits(v[2 * j]) | ((uint32_t)float_to_bf16_bits(v[2 * j + 1]) << 16);
+        *reinterpret_cast<uint4*>(p) = make_uint4(u[0], u[1], u[2], u[3]);
+    }
+};
+
+template <typename TA, int VEC>
+__global__ __launch_bounds__(256)
+void projection_store_kernel(const ProjectionArgs a) {
+    __shared__ float scratch[4];
+    const int t = blockIdx.x;
+    const int H = a.n_heads, G = a.n_kv_heads, dk = a.dk, dv = a.dv;
+    const int nq = H * dk, nk = a.kv ? G * dk : 0;
+    const TA* row = (const TA*)a.rows + (size_t)t * a.row_stride;
+    auto load = [&](int at, float* v) {
+        Piece<TA, VEC>::load(row + at, v);
+        if (a.bias) {
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) v[j] += a.bias[at + j];
+        }
+    };
+    if (a.gate_out)
+        for (int h = threadIdx.x; h < H; h += blockDim.x) a.gate_out[(size_t)t * H + h] = 1.f / (1.f + expf(-to_float(row[a.gate_at + h])));
+    float inv_q = 1.f, inv_k = 1.f;
+    if (a.q_norm_w) {
+        float sq = 0.f, sk = 0.f;
+        for (int e = threadIdx.x * VEC; e < nq + nk; e += blockDim.x * VEC) {
+            float v[VEC], ss = 0.f;
+            load(e, v);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) ss = fmaf(v[j], v[j], ss);
+            if (e < nq) sq += ss; else sk += ss;
+        }
+        inv_q = 1.f / sqrtf(block_sum(sq, scratch) / (float)nq + a.eps);
+        if (nk) inv_k = 1.f / sqrtf(block_sum(sk, scratch) / (float)nk + a.eps);
+    }
+    const int pos = a.tok_pos[t];
+    const int half = a.rot_dim / 2;
+    const bool rotate = a.rot_dim > 0 && pos < a.max_positions;
+    int page = -1;
+    if (a.kv) page = a.page_table[(size_t)a.tok_seq[t] * a.table_width + pos / TQK_PAGE];
+    for (int e = threadIdx.x * VEC; e < nq + nk; e += blockDim.x * VEC) {
+        const bool is_q = e < nq;
+        if (!is_q && page < 0) continue;                    // the host never lets this happen
+        const int in_part = is_q ? e : e - nq, head = in_part / dk, off = in_part % dk;
+        const float* w = a.q_norm_w ? (is_q ? a.q_norm_w : a.k_norm_w) : nullptr;
+        const int part_at = is_q ? 0 : nq;
+        const float inv = is_q ? inv_q : inv_k;
+        auto normed = [&](int at, float* v) {
+            load(at, v);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) v[j] *= w ? inv * w[at - part_at + j] : 1.f;
+        };
+        float x[VEC];
+        normed(e, x);
+        if (rotate && off < a.rot_dim) {
+            const float* ct = a.cos_table + (size_t)pos * half;
+            const float* st = a.sin_table + (size_t)pos * half;
+            if (a.style == 2 && VEC > 1) {
+#pragma unroll
+                for (int j = 0; j + 1 < VEC; j += 2) {
+                    if (off + j >= a.rot_dim) continue;
+                    const float c = ct[(off + j) / 2], s = st[(off + j) / 2], u = x[j], v = x[j + 1];
+                    x[j] = u * c - v * s;
+                    x[j + 1] = v * c + u * s;
+                }
+            } else {
+                const bool first = a.style == 2 ? !(off & 1) : off < half;
+                const int partner = a.style == 2 ? (off ^ 1) : first ? off + half : off - half;
+                const int angle = a.style == 2 ? off / 2 : first ? off : off - half;
+                float y[VEC];
+                normed(e - off + partner, y);
+#pragma unroll
+                for (int j = 0; j < VEC; ++j) {
+                    const float c = ct[angle + j], s = st[angle + j];
+                    x[j] = first ? x[j] * c - y[j] * s : x[j] * c + y[j] * s;
+                }
+            }
+        }
+        TA* dst = is_q ? (TA*)a.q_out + (size_t)t * nq + in_part
+                       : (TA*)a.keys + (((size_t)page * G + head) * TQK_PAGE + pos % TQK_PAGE) * dk + off;
+        Piece<TA, VEC>::store(dst, x);
+    }
+    if (!a.kv || !a.store_values || page < 0) return;
+    TA* values = (TA*)a.values + (size_t)page * G * TQK_PAGE * dv + value_place(pos % TQK_PAGE);
+    for (int e = threadIdx.x; e < G * dv; e += blockDim.x)
+        values[(size_t)e * TQK_PAGE] = from_float<TA>(to_float(row[nq + nk + e]) + (a.bias ? a.bias[nq + nk + e] : 0.f));
+}
+
 // ---- attention, a wave per (token, head) --------------------------------------------------------------
 // Keys are taken a page at a time; lane j computes the score of key j of the page, the softmax runs online over the
 // pages, then lane c accumulates output element c (+64, ...).  The order of operations for a query depends on its
@@ -418,7 +541,7 @@ __global__ __launch_bounds__(AM_WAVES * TQK_WAVE)
 void attention_masked_kernel(const T* __restrict__ q, const T* __restrict__ keys, const T* __restrict__ values,
                              const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos,
                              const int32_t* __restrict__ page_table, int table_width, int window, int chunk, int keep_first, float scale, float cap,
-                             const TS* __restrict__ sink, T* __restrict__ out, int n_tokens, int n_heads, int n_kv_heads, int dk, int dv) {
+                             const TS* __restrict__ sink, const float* __restrict__ head_scale, T* __restrict__ out, int n_tokens, int n_heads, int n_kv_heads, int dk, int dv) {
     __shared__ float q_lds[AM_WAVES][AM_MAX_D];
     const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
     const int t = blockIdx.x * AM_WAVES + wave;
@@ -480,10 +603,11 @@ void attention_masked_kernel(const T* __restrict__ q, const T* __restrict__ keys
         }
     }
     T* o = out + ((size_t)t * n_heads + head) * dv;
+    const float hs = head_scale ? head_scale[(size_t)t * n_heads + head] : 1.f;
 #pragma unroll
     for (int a = 0; a < NACC; ++a) {
         const int c = lane + a * TQK_WAVE;
-        if (c < dv) o[c] = from_float<T>(acc[a] / l);
+        if (c < dv) o[c] = from_float<T>(acc[a] / l * hs);
     }
 }
 
@@ -555,7 +679,8 @@ extern "C" int tqk_rope_norm_store(const void* qkv, int act_dtype, const void* b
             max_positions, normed, eps, tok_seq, tok_pos, page_table, table_width, (bf16_t*)keys, (bf16_t*)q_out, n_heads, n_kv_heads, key_dim, value_dim, write_kv)
 #define TQK_RNV_ALL(TB) do { if (key_dim <= 128) TQK_RNV(TB, 2); else TQK_RNV(TB, 4); \
         if (write_kv) biased_values_store_vec_kernel<TB><<<(unsigned)v_blocks, 256, 0, s>>>((const bf16_t*)qkv, (const TB*)bias, tok_seq, tok_pos, page_table, \
-            table_width, (bf16_t*)values, n_tokens, n_heads, n_kv_heads, key_dim, value_dim); } while (0)
+            table_width, (bf16_t*)values, n_tokens, n_kv_heads, value_dim, (size_t)(n_heads + n_kv_heads) * key_dim + (size_t)n_kv_heads * value_dim, \
+            (size_t)(n_heads + n_kv_heads) * key_dim); } while (0)
         if (bias && bias_dtype == TQK_F32) TQK_RNV_ALL(float); else TQK_RNV_ALL(bf16_t);
 #undef TQK_RNV_ALL
 #undef TQK_RNV
@@ -574,12 +699,47 @@ extern "C" int tqk_rope_norm_store(const void* qkv, int act_dtype, const void* b
     return tqk_check_launch("tqk_rope_norm_store");
 }
 
+extern "C" int tqk_projection_store(const void* rows, int act_dtype, long long row_stride, const float* bias, const float* q_norm_w, const float* k_norm_w, float eps,
+                                    const float* cos_table, const float* sin_table, int rot_dim, int style, int max_positions, const int32_t* tok_seq,
+                                    const int32_t* tok_pos, const int32_t* page_table, int table_width, void* keys, void* values, void* q_out,
+                                    float* gate_out, long long gate_at, int n_tokens, int n_heads, int n_kv_heads, int key_dim, int value_dim, int kv,
+                                    void* stream) {
+    TQK_REQUIRE(rows && tok_pos && q_out, "tqk_projection_store: null pointer");
+    TQK_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv_heads > 0 && key_dim > 0 && value_dim > 0 && (long long)n_heads * key_dim <= (1 << 24), "tqk_projection_store: bad sizes");
+    const long long nq = (long long)n_heads * key_dim, nk = kv ? (long long)n_kv_heads * key_dim : 0, nv = kv ? (long long)n_kv_heads * value_dim : 0;
+    TQK_REQUIRE(row_stride >= nq + nk + nv && (!gate_out || (gate_at >= nq + nk + nv && row_stride >= gate_at + n_heads)), "tqk_projection_store: rows too short");
+    TQK_REQUIRE(rot_dim >= 0 && rot_dim % 2 == 0 && rot_dim <= key_dim, "tqk_projection_store: rot_dim %d must be even and <= key_dim %d", rot_dim, key_dim);
+    TQK_REQUIRE(rot_dim == 0 || (cos_table && sin_table && max_positions > 0 && (style == 1 || style == 2)), "tqk_projection_store: rotation without tables, or of an unknown style");
+    TQK_REQUIRE(!kv || (tok_seq && page_table && keys && values && table_width > 0), "tqk_projection_store: no cache to write to");
+    TQK_REQUIRE(!q_norm_w || !kv || k_norm_w, "tqk_projection_store: queries normed and keys not");
+    if (n_tokens == 0) return 0;
+    hipStream_t s = (hipStream_t)stream;
+    ProjectionArgs a = {rows, row_stride, bias, q_norm_w, k_norm_w, eps, cos_table, sin_table, rot_dim, style, max_positions, tok_seq, tok_pos, page_table, table_width,
+                        keys, values, q_out, gate_out, gate_at, n_heads, n_kv_heads, key_dim, value_dim, kv, 1};
+    const bool aligned = row_stride % 8 == 0 && (((uintptr_t)rows | (uintptr_t)keys | (uintptr_t)q_out) & 15) == 0;
+    if (act_dtype == TQK_BF16 && key_dim % 8 == 0 && (rot_dim == 0 || style == 2 || rot_dim % 16 == 0) && aligned) {
+        // steps of many tokens: values with the lanes along the tokens
+        const bool apart = kv && n_tokens > 64 && value_dim % 8 == 0;
+        a.store_values = apart ? 0 : 1;
+        projection_store_kernel<bf16_t, 8><<<n_tokens, 256, 0, s>>>(a);
+        if (apart) {
+            const long long v_blocks = (long long)((n_tokens + TQK_WAVE - 1) / TQK_WAVE) * n_kv_heads;
+            TQK_REQUIRE(v_blocks <= 0x7fffffff, "tqk_projection_store: too many tokens");
+            biased_values_store_vec_kernel<float><<<(unsigned)v_blocks, 256, 0, s>>>((const bf16_t*)rows, bias, tok_seq, tok_pos, page_table, table_width, (bf16_t*)values,
+                                                                                     n_tokens, n_kv_heads, value_dim, (size_t)row_stride, (size_t)(nq + nk));
+        }
+    } else if (act_dtype == TQK_BF16) projection_store_kernel<bf16_t, 1><<<n_tokens, 256, 0, s>>>(a);
+    else if (act_dtype == TQK_F32) projection_store_kernel<float, 1><<<n_tokens, 256, 0, s>>>(a);
+    else return tqk_fail("tqk_projection_store: unknown dtype %d", act_dtype);
+    return tqk_check_launch("tqk_projection_store");
+}
+
 extern "C" int tqk_attention_masked_max_dim(void) { return AM_MAX_D; }
 
 extern "C" int tqk_attention_masked(const void* q, const void* keys, const void* values, int act_dtype, const int32_t* tok_seq,
                                     const int32_t* tok_pos, const int32_t* page_table, int table_width, int n_seqs, int n_pages, int window,
-                                    int chunk, int keep_first, float scale, float cap, const void* sink, int sink_dtype, void* out, int n_tokens,
-                                    int n_heads, int n_kv_heads, int key_dim, int value_dim, void* stream) {
+                                    int chunk, int keep_first, float scale, float cap, const void* sink, int sink_dtype, const float* head_scale,
+                                    void* out, int n_tokens, int n_heads, int n_kv_heads, int key_dim, int value_dim, void* stream) {
     TQK_REQUIRE(q && keys && values && tok_seq && tok_pos && page_table && out, "tqk_attention_masked: null pointer");
     TQK_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv_heads > 0 && key_dim > 0 && value_dim > 0, "tqk_attention_masked: bad sizes");
     TQK_REQUIRE(n_heads % n_kv_heads == 0, "tqk_attention_masked: %d heads are not a multiple of %d kv heads", n_heads, n_kv_heads);
@@ -592,7 +752,7 @@ extern "C" int tqk_attention_masked(const void* q, const void* keys, const void*
     dim3 grid((n_tokens + AM_WAVES - 1) / AM_WAVES, n_heads);
 #define TQK_AM(T, TS) \
     attention_masked_kernel<T, TS><<<grid, AM_WAVES * TQK_WAVE, 0, s>>>((const T*)q, (const T*)keys, (const T*)values, tok_seq, tok_pos, page_table, \
-        table_width, window, chunk, keep_first, scale, cap, (const TS*)sink, (T*)out, n_tokens, n_heads, n_kv_heads, key_dim, value_dim)
+        table_width, window, chunk, keep_first, scale, cap, (const TS*)sink, head_scale, (T*)out, n_tokens, n_heads, n_kv_heads, key_dim, value_dim)
     if (act_dtype == TQK_F32 && (!sink || sink_dtype == TQK_F32)) TQK_AM(float, float);
     else if (act_dtype == TQK_F32 && sink_dtype == TQK_BF16) TQK_AM(float, bf16_t);
     else if (act_dtype == TQK_BF16 && (!sink || sink_dtype == TQK_BF16)) TQK_AM(bf16_t, bf16_t);

@@ -32,6 +32,7 @@ struct MaskedArgs {
     float scale, cap;
     const void* sink;               // [heads] or null
     int sink_f32;
+    const float* head_scale;        // [rows, heads] or null: the outputs are multiplied by it
     int n_parts, n_heads, n_kv_heads, q_blocks, dk, dv;
     const int32_t *tile_seq, *tile_tok0, *tile_count;      // tiles
     float *part_out, *part_ml;      // rows with more than one partition
@@ -218,7 +219,7 @@ void attention_masked_mfma_kernel(const MaskedArgs a) {
     if (TILE) {
         if (!live) return;
         bf16_t* po = a.out + qrow * dv;
-        const float inv = 1.f / l;
+        const float inv = (a.head_scale ? a.head_scale[qrow] : 1.f) / l;
 #pragma unroll
         for (int db = 0; db < DB; ++db)
 #pragma unroll
@@ -269,7 +270,7 @@ void attention_masked_mfma_kernel(const MaskedArgs a) {
             l = l * a1 + __builtin_amdgcn_exp2f(sk - mn);
         }
         bf16_t* po = a.out + qrow * dv;
-        const float inv = 1.f / l;
+        const float inv = (a.head_scale ? a.head_scale[qrow] : 1.f) / l;
 #pragma unroll
         for (int db = 0; db < DB; ++db)
 #pragma unroll
@@ -499,7 +500,7 @@ void attention_masked_block_kernel(const MaskedArgs a) {
         lc += __shfl_xor(lc, 32, TQK_WAVE);
         if (!live[c]) continue;
         bf16_t* po = a.out + qrow[c] * dv;
-        const float inv = 1.f / lc;
+        const float inv = (a.head_scale ? a.head_scale[qrow[c]] : 1.f) / lc;
 #pragma unroll
         for (int db = 0; db < DB; ++db)
 #pragma unroll
@@ -512,7 +513,7 @@ void attention_masked_block_kernel(const MaskedArgs a) {
 
 // out[row, :] = sum_p 2^(m_p - M) o_p / (sum_p 2^(m_p - M) l_p + 2^(sink - M)), partitions in order
 __global__ void attention_masked_merge_kernel(const float* __restrict__ part_out, const float* __restrict__ part_ml, int n_parts, int dv, int n_heads,
-                                              const void* __restrict__ sink, int sink_f32, bf16_t* __restrict__ out) {
+                                              const void* __restrict__ sink, int sink_f32, const float* __restrict__ head_scale, bf16_t* __restrict__ out) {
     const size_t row = blockIdx.x;                     // row * n_heads + head
     const float2* ml = reinterpret_cast<const float2*>(part_ml) + row * n_parts;
     float M = -INFINITY, sk = -INFINITY;
@@ -535,7 +536,7 @@ __global__ void attention_masked_merge_kernel(const float* __restrict__ part_out
             denom += wgt * s.y;
             acc += has ? wgt * v : 0.f;
         }
-        out[row * dv + c] = from_float<bf16_t>(acc / denom);
+        out[row * dv + c] = from_float<bf16_t>(acc / denom * (head_scale ? head_scale[row] : 1.f));
     }
 }
 
@@ -589,8 +590,8 @@ extern "C" int tqk_attention_masked_mfma_tile(int n_tokens, int n_heads, int n_k
  * where n_parts > 1). */
 extern "C" int tqk_attention_masked_mfma(const void* q, const void* keys, const void* values, const int32_t* tok_pos, const int32_t* page_table,
                                          int table_width, int n_pages, int window, int chunk, int keep_first, float scale, float cap, const void* sink,
-                                         int sink_dtype, const int32_t* tile_seq, const int32_t* tile_tok0, const int32_t* tile_count, int n_tiles,
-                                         int tile_queries, int n_rows, int n_parts, void* part_out, void* part_ml, void* out, int n_heads, int n_kv_heads,
+                                         int sink_dtype, const float* head_scale, const int32_t* tile_seq, const int32_t* tile_tok0, const int32_t* tile_count,
+                                         int n_tiles, int tile_queries, int n_rows, int n_parts, void* part_out, void* part_ml, void* out, int n_heads, int n_kv_heads,
                                          int key_dim, int value_dim, void* stream) {
     TQK_REQUIRE(q && keys && values && tok_pos && page_table && out, "tqk_attention_masked_mfma: null pointer");
     TQK_REQUIRE(n_heads > 0 && n_kv_heads > 0 && n_heads % n_kv_heads == 0, "tqk_attention_masked_mfma: %d heads and %d kv heads", n_heads, n_kv_heads);
@@ -609,7 +610,7 @@ extern "C" int tqk_attention_masked_mfma(const void* q, const void* keys, const 
     a.q = (const bf16_t*)q; a.keys = (const bf16_t*)keys; a.values = (const bf16_t*)values;
     a.tok_pos = tok_pos; a.page_table = page_table; a.table_width = table_width;
     a.window = window; a.chunk = chunk; a.keep_first = keep_first; a.scale = scale; a.cap = cap;
-    a.sink = sink; a.sink_f32 = sink_dtype == TQK_F32;
+    a.sink = sink; a.sink_f32 = sink_dtype == TQK_F32; a.head_scale = head_scale;
     a.n_parts = tiles ? 1 : n_parts; a.n_heads = n_heads; a.n_kv_heads = n_kv_heads;
     a.q_blocks = (n_heads / n_kv_heads + 15) / 16;
     TQK_REQUIRE((long long)n_kv_heads * a.q_blocks <= 65535 && n_heads <= 65535, "tqk_attention_masked_mfma: grid too large");
@@ -623,6 +624,6 @@ extern "C" int tqk_attention_masked_mfma(const void* q, const void* keys, const 
     else status = launch_masked_dv<8>(a, tiles, n_tiles, tile_queries, n_rows, s);
     if (status || tiles || n_parts == 1) return status;
     attention_masked_merge_kernel<<<n_rows * n_heads, value_dim >= 128 ? 128 : 64, 0, s>>>((const float*)part_out, (const float*)part_ml, n_parts, value_dim,
-                                                                                            n_heads, sink, a.sink_f32, (bf16_t*)out);
+                                                                                            n_heads, sink, a.sink_f32, head_scale, (bf16_t*)out);
     return tqk_check_launch("tqk_attention_masked_mfma merge");
 }

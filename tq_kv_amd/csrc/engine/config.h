@@ -33,5 +33,6 @@ void register_sizudra();
 void register_piditar();
 void register_povipel();
 void register_rasodra();
+void register_kezasun();
 
 }  // namespace tq

@@ -76,16 +76,20 @@ TQ_KERNEL(moe_route, cptr, int, cptr, int, int, int, int, float, int, int32_t*, 
 TQ_KERNEL(moe_group, ci32, int, int, int, int, int32_t*, int32_t*, int32_t*, int32_t*, int32_t*, int32_t*, void*);
 TQ_KERNEL(moe_product, cptr, int, ci32, cptr, int, long long, void*, int, int, int, int, float, float, ci32, ci32, ci32, ci32, int, void*);
 TQ_KERNEL(moe_scale_rows, cptr, int, ci32, cf32, int, void*, float*, int, int, void*);
-TQ_KERNEL(moe_combine, cptr, int, ci32, cf32, int, cptr, cf32, void*, int, int, void*);
+TQ_KERNEL(moe_route_grouped, cptr, int, cptr, int, int, int, int, cf32, int, int, float, int32_t*, float*, int, void*);
+TQ_KERNEL(moe_combine, cptr, int, ci32, cf32, int, cptr, cptr, cf32, cptr, float, void*, int, int, void*);
 TQ_KERNEL(pair_embed, cptr, int, int, long long, long long, ci32, ci32, ci32, ci32, ci32, int32_t*, float*, int, int, int, void*, int, void*);
 TQ_KERNEL(remember_tokens, ci32, ci32, ci32, ci32, int32_t*, int, void*);
 TQ_KERNEL(norm_add, float*, cptr, int, cptr, int, float, void*, int, int, void*);
 TQ_KERNEL(unary_act, cptr, void*, int, long long, int, float, float, void*);
+TQ_KERNEL(scaled_sum, cptr, cptr, int, float, void*, long long, void*);
 TQ_KERNEL(row_gate, cptr, int, cptr, int, float*, int, int, void*);
 TQ_KERNEL(normed_rope_store, cptr, int, cptr, cptr, cptr, int, float, cf32, cf32, int, int, int, cptr, cptr, void*, ci32, ci32, ci32, int, void*, void*,
           void*, int, int, int, int, int, int, int, void*);
 TQ_KERNEL(rope_norm_store, cptr, int, cptr, int, cf32, cf32, int, int, int, int, float, ci32, ci32, ci32, int, void*, void*, void*, int, int, int, int,
           int, int, void*);
+TQ_KERNEL(projection_store, cptr, int, long long, cf32, cf32, cf32, float, cf32, cf32, int, int, int, ci32, ci32, ci32, int, void*, void*, void*, float*,
+          long long, int, int, int, int, int, int, void*);
 TQ_QUERY(int, conv_max_taps);
 TQ_QUERY(int, ssm_max_state);
 TQ_KERNEL(conv_state, cptr, int, long long, cf32, cf32, cf32, int, int, cf32, long long, ci32, ci32, ci32, ci32, float*, int, int, void*);
@@ -104,9 +108,9 @@ TQ_KERNEL(add_rows, float*, cf32, long long, void*);
 TQ_QUERY(int, attention_masked_max_dim);
 TQ_QUERY(int, attention_masked_mfma_supported, int, int);
 TQ_QUERY(int, attention_masked_mfma_tile, int, int, int, int, int);
-TQ_KERNEL(attention_masked_mfma, cptr, cptr, cptr, ci32, ci32, int, int, int, int, int, float, float, cptr, int, ci32, ci32, ci32, int, int, int, int, void*, void*,
+TQ_KERNEL(attention_masked_mfma, cptr, cptr, cptr, ci32, ci32, int, int, int, int, int, float, float, cptr, int, cf32, ci32, ci32, ci32, int, int, int, int, void*, void*,
           void*, int, int, int, int, void*);
-TQ_KERNEL(attention_masked, cptr, cptr, cptr, int, ci32, ci32, ci32, int, int, int, int, int, int, float, float, cptr, int, void*, int, int, int, int,
+TQ_KERNEL(attention_masked, cptr, cptr, cptr, int, ci32, ci32, ci32, int, int, int, int, int, int, float, float, cptr, int, cf32, void*, int, int, int, int,
           int, void*);
 TQ_QUERY(int, streams_max);
 TQ_KERNEL(streams_fill, cf32, float*, int, int, int, void*);
@@ -116,9 +120,13 @@ TQ_KERNEL(add_layer_norm_sums, float*, cptr, int, cf32, int, int, ci32, int, cf3
 TQ_KERNEL(token_shift, cf32, cf32, float*, long long, ci32, ci32, ci32, ci32, void*, int, int, int, int, void*);
 TQ_KERNEL(shift_remember, cf32, float*, long long, ci32, ci32, ci32, int, int, void*);
 TQ_QUERY(int, linear_attention_max_dim);
-TQ_KERNEL(linear_attention, cptr, cptr, cptr, int, long long, cf32, long long, cf32, float, cf32, cf32, cf32, cf32, float, float, cf32, cf32, int, int, int,
-          ci32, float*, long long, ci32, ci32, ci32, ci32, ci32, float*, float*, float*, int, int, int, int, int, long long, void*);
+TQ_KERNEL(linear_attention, cptr, cptr, cptr, int, long long, cf32, long long, cf32, float, cf32, cf32, cf32, cf32, cf32, cf32, float, float, cf32, cf32, int,
+          int, int, ci32, float*, long long, ci32, ci32, ci32, ci32, ci32, float*, float*, float*, int, int, int, int, int, long long, void*);
 TQ_KERNEL(head_norm_gate, cf32, cf32, int, float, cptr, int, long long, int, void*, int, int, int, int, void*);
+TQ_KERNEL(token_mixes, cptr, int, cf32, int, float*, long long, ci32, ci32, ci32, ci32, void*, int, int, int, void*);
+TQ_KERNEL(rows_remember, cptr, int, float*, long long, ci32, ci32, ci32, int, int, void*);
+TQ_QUERY(int, low_rank_max);
+TQ_KERNEL(low_rank_decay, cf32, cf32, cf32, float*, int, int, int, void*);
 TQ_QUERY(int, mlstm_chunks_supported, int, int);
 TQ_QUERY(int, mlstm_apply_norms, int);
 TQ_KERNEL(mlstm_gate_scan, cf32, long long, cf32, float, float*, long long, long long, ci32, ci32, ci32, float*, float*, float*, int, int, void*);

@@ -216,6 +216,9 @@ public:
     virtual bool folds_norm(const StepContext& c) const { (void)c; return false; }
     virtual bool adds_to_stream(const StepContext& c) const { (void)c; return false; }
     virtual Tensor forward(StepContext& c, const Activation& x, Stream* stream) = 0;
+    // Optional: scale (forward(x) + beside) out of the part's own last kernel (beside: [tokens, hidden], what another part made of the step).
+    virtual bool takes_beside() const { return false; }
+    virtual Tensor forward_beside(StepContext& c, const Activation& x, const Tensor& beside, float scale) { (void)beside; (void)scale; return forward(c, x, nullptr); }
 };
 
 class Block : public Part {
@@ -247,5 +250,7 @@ void register_streams_parts();          // parts_streams.cpp; likewise
 void register_linear_attention_parts(); // parts_linear_attention.cpp; likewise
 void register_pooled_parts();           // parts_pooled.cpp; likewise
 void register_mlstm_parts();            // parts_mlstm.cpp; likewise
+void register_time_mixing_parts();      // parts_time_mixing.cpp; likewise
+void register_joint_parts();            // parts_joint.cpp; likewise
 
 }  // namespace tq

@@ -86,6 +86,15 @@ static OwnedPtr take(Loaded& tensors, const char* name) {
     return it->second;
 }
 
+static OwnedPtr as_floats(const OwnedPtr& p, hipStream_t stream) {
+    if (p->t.dtype == F32) return p;
+    std::vector<int64_t> dims(p->t.shape, p->t.shape + p->t.ndim);
+    OwnedPtr out = make_owned(F32, dims);
+    if (!null_device()) K::convert(p->t.data, p->t.dtype, out->t.data, F32, (long long)p->t.numel(), stream);
+    stream_synchronize(stream);
+    return out;
+}
+
 // ---- RMSNorm -----------------------------------------------------------------------------------
 // As the reference computes it (src/models/turbo_generic.rs:41-51): x / sqrt(mean(x^2) + eps) *
 // weight in float32, cast last; the weight is used as it is stored (no 1 + w).
@@ -164,6 +173,9 @@ private:
 // 1 / base^(2j/d) with base rounded to float32 and the power taken in float32, angle = position *
 // theta_j in float32, cos and sin of it.  Layouts: halves (:417-427, what Qwen2 uses) and pairs
 // (:430-443); rot_dim < head_dim rotates the first rot_dim elements only (:752-761).
+//
+// Optional scaling {factor, low, high, original}: a frequency f with wavelength l = 2 pi / f stays as it is where l < original / high, becomes
+// f / factor where l > original / low, and between the two (1 - s) f / factor + s f with s = (original / l - low) / (high - low).
 class Rotary : public Position {
 public:
     Rotary(const PartSpec& spec, BuildEnv&) {
@@ -184,6 +196,17 @@ public:
         const float base = (float)theta_;
         std::vector<float> inv((size_t)half);
         for (int j = 0; j < half; ++j) inv[(size_t)j] = 1.0f / powf(base, (float)(2 * j) / (float)rot_dim_);
+        if (!spec.params["scaling"].is_null()) {
+            KeyReader sc(spec.params["scaling"], "rotary: scaling", TQE_ERR_ARGUMENT);
+            const double factor = sc.number("factor", true), low = sc.number("low", true), high = sc.number("high", true), original = sc.number("original", true);
+            for (float& f : inv) {
+                const double length = 2.0 * M_PI / (double)f;
+                if (length < original / high) continue;
+                if (length > original / low) { f = (float)((double)f / factor); continue; }
+                const double s = (original / length - low) / (high - low);
+                f = (float)((1.0 - s) * (double)f / factor + s * (double)f);
+            }
+        }
         for (int64_t p = 0; p < max_positions; ++p)
             for (int j = 0; j < half; ++j) {
                 const float angle = (float)p * inv[(size_t)j];
@@ -243,8 +266,12 @@ public:
 // exponential joins the softmax's denominator, with no key and no value); value_mix "source" (the values of the
 // step's tokens are handed to later layers) or "mixed" (v <- (1 - lambda) v + lambda v_source with a learned scalar,
 // before the cache); value_mix_key (which source, "values" unless given); cache_keeps_all (the cache keeps every page although the
-// mixer sees a window); names: the tensors' names inside the
-// part's prefix {q, k, v, o, q_norm, k_norm, sink, mix}.  With any of them the step runs through the kernels of
+// mixer sees a window); cache_window (the cache keeps so many positions although the mixer sees a smaller window: another run reads them);
+// qk_norm_over "projection" (with qk_norm: all of q, and all of k, are divided by the root mean square of the whole projection and multiplied by a
+// weight of its size, before the rotation); sink_score (a number: a sink of that fixed score for every head, without a tensor); gate "head" (a
+// head's output is multiplied by the sigmoid of a product of its own with the mixer's input); own_kv false (no projections of keys and
+// values: the run reads another run's cache); names: the tensors' names inside the
+// part's prefix {q, k, v, o, q_norm, k_norm, sink, mix, gate}.  With any of them the step runs through the kernels of
 // attention_masked.hip.
 //
 // Its pages: keys [kv heads, page, head_dim]; values [kv heads, head_dim, page], transposed inside
@@ -280,6 +307,19 @@ public:
         keep_first_ = (int)r.integer_or("keep_first", 0, 0);
         cache_keeps_all_ = r.boolean_or("cache_keeps_all", false);
         has_sink_ = r.boolean_or("sink", false);
+        fixed_sink_ = r.has("sink_score");
+        if (fixed_sink_) sink_score_ = (float)r.number("sink_score");
+        if (has_sink_ && fixed_sink_) raise(TQE_ERR_ARGUMENT, "attention: a learned sink and one of a fixed score");
+        const std::string norm_over = r.string_or("qk_norm_over", "head");
+        if (norm_over != "head" && norm_over != "projection") raise(TQE_ERR_ARGUMENT, "attention: unknown qk_norm_over '%s' (known: head, projection)", norm_over.c_str());
+        const std::string gate = r.string_or("gate", "none");
+        if (gate != "none" && gate != "head") raise(TQE_ERR_ARGUMENT, "attention: unknown gate '%s' (known: none, head)", gate.c_str());
+        gated_ = gate == "head";
+        own_kv_ = r.boolean_or("own_kv", true);
+        cache_window_ = r.has("cache_window") ? (int)r.integer("cache_window", 1) : window_;
+        if (cache_window_ < window_ || (window_ == 0 && cache_window_ != 0)) raise(TQE_ERR_ARGUMENT, "attention: the cache keeps %d positions, the mixer sees %d", cache_window_, window_);
+        // one kernel puts a norm over the projection, a gate per head and queries alone between the product and the attention
+        projected_ = (qk_norm_ && norm_over == "projection") || gated_ || !own_kv_;
         const std::string mixing = r.string_or("value_mix", "none");
         if (mixing == "none") value_mix_ = MIX_NONE;
         else if (mixing == "source") value_mix_ = MIX_SOURCE;
@@ -287,12 +327,15 @@ public:
         else raise(TQE_ERR_ARGUMENT, "attention: unknown value_mix '%s' (known: none, source, mixed)", mixing.c_str());
         mix_key_ = "attention." + r.string_or("value_mix_key", "values");
         if (keep_first_ > 0 && window_ == 0) raise(TQE_ERR_ARGUMENT, "attention: keep_first %d without a window", keep_first_);
-        extras_ = value_dim_ != head_dim_ || values_are_keys_ || chunk_ > 0 || qk_norm_ || cap_ > 0.f || keep_first_ > 0 || has_sink_ || value_mix_ != MIX_NONE;
+        extras_ = value_dim_ != head_dim_ || values_are_keys_ || chunk_ > 0 || qk_norm_ || cap_ > 0.f || keep_first_ > 0 || has_sink_ || fixed_sink_ || projected_ ||
+                  value_mix_ != MIX_NONE;
+        if (projected_ && (values_are_keys_ || value_mix_ != MIX_NONE || (qk_norm_ && (norm_over != "projection" || !qk_norm_weight_ || norm_after_rotation_))))
+            raise(TQE_ERR_ARGUMENT, "attention: a gate, a norm over the projection or borrowed keys and values go with values of their own that are not mixed, and no norm of heads");
         if (qk_norm_ && qk_norm_weight_ == norm_after_rotation_)
             raise(TQE_ERR_ARGUMENT, "attention: the heads' norm is either weighted and in front of the rotation, or without a weight and after it");
         // the kernel that adds biases, turns and then norms without a weight stands for every such combination but mixed values and
         // values that are the keys; the one that norms in front of the rotation for every other
-        const bool turned_ok = extras_ && (!qk_norm_ || norm_after_rotation_) && value_mix_ == MIX_NONE && !values_are_keys_;
+        const bool turned_ok = extras_ && !projected_ && (!qk_norm_ || norm_after_rotation_) && value_mix_ == MIX_NONE && !values_are_keys_;
         if (extras_ && norm_after_rotation_ && qk_norm_ && !turned_ok)
             raise(TQE_ERR_ARGUMENT, "attention: a heads' norm after the rotation goes with values of their own that are not mixed");
         if (extras_ && out_bias_)
@@ -302,7 +345,7 @@ public:
             auto name = [&](const char* role, const char* fallback) { return names[role].is_string() ? names[role].as_string() : std::string(fallback); };
             n_q_ = name("q", "q_proj.weight"); n_k_ = name("k", "k_proj.weight"); n_v_ = name("v", "v_proj.weight"); n_o_ = name("o", "o_proj.weight");
             n_q_norm_ = name("q_norm", "q_norm.weight"); n_k_norm_ = name("k_norm", "k_norm.weight");
-            n_sink_ = name("sink", "sink"); n_mix_ = name("mix", "value_mix");
+            n_sink_ = name("sink", "sink"); n_mix_ = name("mix", "value_mix"); n_gate_ = name("gate", "gate.weight");
             n_qb_ = name("q_bias", "q_proj.bias"); n_kb_ = name("k_bias", "k_proj.bias"); n_vb_ = name("v_bias", "v_proj.bias");
         }
         if (r.has("prompt_tile") && prompt_tile_ != 16 && prompt_tile_ != 32 && prompt_tile_ != 64 && prompt_tile_ != 128)
@@ -335,41 +378,59 @@ public:
         const int64_t q = (int64_t)n_heads_ * head_dim_, kv = (int64_t)n_kv_heads_ * head_dim_;
         auto w = [](int64_t a, int64_t b) { TensorSpec t; t.shape = {a, b}; return t; };
         auto b = [](int64_t a) { TensorSpec t; t.shape = {a}; return t; };
-        TensorSpecs t = {{n_q_, w(q, hidden_)}, {n_k_, w(kv, hidden_)}};
-        if (!values_are_keys_) t.push_back({n_v_, w((int64_t)n_kv_heads_ * value_dim_, hidden_)});
+        TensorSpecs t = {{n_q_, w(q, hidden_)}};
+        if (own_kv_) t.push_back({n_k_, w(kv, hidden_)});
+        if (own_kv_ && !values_are_keys_) t.push_back({n_v_, w((int64_t)n_kv_heads_ * value_dim_, hidden_)});
+        if (gated_) t.push_back({n_gate_, w(n_heads_, hidden_)});
         t.push_back({n_o_, w(hidden_, (int64_t)n_heads_ * value_dim_)});
         if (qk_norm_ && qk_norm_weight_) {
-            TensorSpec n = b(head_dim_);
+            TensorSpec n = b(projected_ ? q : head_dim_);
             n.init = "one_plus_normal";
             n.std_dev = 0.1;
             t.push_back({n_q_norm_, n});
-            t.push_back({n_k_norm_, n});
+            n.shape = {projected_ ? kv : head_dim_};
+            if (own_kv_) t.push_back({n_k_norm_, n});
         }
         if (has_sink_) { TensorSpec s = b(n_heads_); s.std_dev = 1.0; t.push_back({n_sink_, s}); }
         // the source layer of a mix has the scalar too, and does not use it
         if (value_mix_ != MIX_NONE) { TensorSpec s; s.shape = {}; s.std_dev = 0.3; t.push_back({n_mix_, s}); }
         if (qkv_bias_) {
             t.push_back({n_qb_, b(q)});
-            t.push_back({n_kb_, b(kv)});
-            if (!values_are_keys_) t.push_back({n_vb_, b((int64_t)n_kv_heads_ * value_dim_)});
+            if (own_kv_) t.push_back({n_kb_, b(kv)});
+            if (own_kv_ && !values_are_keys_) t.push_back({n_vb_, b((int64_t)n_kv_heads_ * value_dim_)});
         }
         if (out_bias_) t.push_back({"o_proj.bias", b(hidden_)});
         return t;
     }
 
-    static OwnedPtr stacked(const std::vector<OwnedPtr>& parts, hipStream_t stream) { return stack_rows(parts, stream); }
-
     void load(Loaded& t, hipStream_t stream) override {
         auto stack_of = [&](const std::string& q, const std::string& k, const std::string& v) {
-            std::vector<OwnedPtr> parts = {take(t, q.c_str()), take(t, k.c_str())};
-            if (!values_are_keys_) parts.push_back(take(t, v.c_str()));
-            return stacked(parts, stream);
+            std::vector<OwnedPtr> parts = {take(t, q.c_str())};
+            if (own_kv_) parts.push_back(take(t, k.c_str()));
+            if (own_kv_ && !values_are_keys_) parts.push_back(take(t, v.c_str()));
+            return parts;
         };
-        OwnedPtr qkv = stack_of(n_q_, n_k_, n_v_);
-        if (qk_norm_ && qk_norm_weight_) { q_norm_ = take(t, n_q_norm_.c_str()); k_norm_ = take(t, n_k_norm_.c_str()); }
+        std::vector<OwnedPtr> first = stack_of(n_q_, n_k_, n_v_);
+        if (gated_) first.push_back(take(t, n_gate_.c_str()));
+        // (rows up to a multiple of 16 where the gate's stand behind the others, so that the product's rows stay at multiples of 16 bytes)
+        OwnedPtr qkv = stack_rows(first, stream, projected_ ? 16 : 1);
+        row_ = qkv->t.shape[0];
+        if (qk_norm_ && qk_norm_weight_) { q_norm_ = take(t, n_q_norm_.c_str()); if (own_kv_) k_norm_ = take(t, n_k_norm_.c_str()); }
         if (has_sink_) sink_ = take(t, n_sink_.c_str());
+        if (fixed_sink_) {
+            const std::vector<float> scores((size_t)n_heads_, sink_score_);
+            sink_ = make_owned(F32, {n_heads_});
+            copy_to_device(sink_->t.data, scores.data(), scores.size() * 4, stream);
+            stream_synchronize(stream);
+        }
         if (value_mix_ != MIX_NONE) mix_ = take(t, n_mix_.c_str());
-        if (qkv_bias_) b_qkv_ = stack_of(n_qb_, n_kb_, n_vb_);
+        if (qkv_bias_) b_qkv_ = stack_rows(stack_of(n_qb_, n_kb_, n_vb_), stream);
+        if (projected_) {
+            // (small vectors, read in float32 by the kernel behind the product)
+            if (b_qkv_) bias_f_ = as_floats(b_qkv_, stream);
+            if (q_norm_) q_norm_f_ = as_floats(q_norm_, stream);
+            if (k_norm_) k_norm_f_ = as_floats(k_norm_, stream);
+        }
         if (out_bias_) b_o_ = take(t, "o_proj.bias");
         w_qkv_ = make_weight(qkv, 1, false, stream);
         w_o_ = make_weight(take(t, n_o_.c_str()), 1, b_o_ != nullptr, stream);
@@ -383,12 +444,15 @@ public:
         if (q_norm_ && name == n_q_norm_) return q_norm_;
         if (k_norm_ && name == n_k_norm_) return k_norm_;
         if (has_sink_ && name == n_sink_) return sink_;
+        if (name == "sink.score") return fixed_sink_ ? sink_ : nullptr;
         if (value_mix_ != MIX_NONE && name == n_mix_) return mix_;
         return nullptr;
     }
     const char* trace_name() const override { return "attn"; }             // the reference's span, src/models/turbo_generic.rs:1920
     void product_shapes(std::vector<std::pair<int64_t, int64_t>>& out) const override {
-        out.push_back({(int64_t)(n_heads_ + n_kv_heads_) * head_dim_ + (values_are_keys_ ? 0 : (int64_t)n_kv_heads_ * value_dim_), hidden_});
+        int64_t n = (int64_t)n_heads_ * head_dim_ + (gated_ ? n_heads_ : 0);
+        if (own_kv_) n += (int64_t)n_kv_heads_ * head_dim_ + (values_are_keys_ ? 0 : (int64_t)n_kv_heads_ * value_dim_);
+        out.push_back({projected_ ? (n + 15) / 16 * 16 : n, hidden_});
         out.push_back({hidden_, (int64_t)n_heads_ * value_dim_});
     }
 
@@ -399,7 +463,7 @@ public:
         n.value_page = {n_kv_heads_, value_dim_, TQE_PAGE};
         // (cache_keeps_all: the cache gives no page back although the mixer sees a window, so that layers of many different windows
         // can share one group of the cache)
-        n.window = cache_keeps_all_ ? 0 : window_;
+        n.window = cache_keeps_all_ ? 0 : cache_window_;
         n.keep_first = cache_keeps_all_ ? 0 : keep_first_;
         n.chunk = cache_keeps_all_ ? 0 : chunk_;
         return n;
@@ -430,7 +494,13 @@ public:
         const StepContext::Table& table = c.tables.at((size_t)entry.group);
         Tensor q = c.alloc(dtype, {n, n_heads_, head_dim_});
         const int n_pages = (int)entry.keys.shape[0];
-        if (extras_) {
+        Tensor head_scale;
+        if (entry.writes != own_kv_ && !own_kv_) raise(TQE_ERR_STATE, "attention: a layer without keys and values of its own was given a cache of its own");
+        if (projected_) {
+            if (x.lazy) raise(TQE_ERR_STATE, "attention: this configuration takes no folded norm");
+            if (gated_) head_scale = c.alloc(F32, {n, n_heads_});
+            projected_q(c, x.x, entry, table, q, head_scale);
+        } else if (extras_) {
             if (x.lazy && !turned_first_) raise(TQE_ERR_STATE, "attention: this configuration takes no folded norm");
             if (turned_first_) turned_qkv(c, x, entry, table, q);
             else normed_qkv(c, x.x, entry, table, q);
@@ -452,12 +522,17 @@ public:
             if (c.n_last == 0) return Tensor(nullptr, dtype, {0, hidden_});
             Tensor ql = c.alloc(dtype, {c.n_last, n_heads_, head_dim_});
             k_gather_rows(c, q, c.dev.last_rows, c.n_last, ql);
+            Tensor scale_l;
+            if (head_scale.defined()) {
+                scale_l = c.alloc(F32, {c.n_last, n_heads_});
+                k_gather_rows(c, head_scale, c.dev.last_rows, c.n_last, scale_l);
+            }
             Tensor y = c.alloc(dtype, {c.n_last, qd});
-            attend_rows(c, ql, entry, table, y);
+            attend_rows(c, ql, entry, table, scale_l, y);
             return linear(c, y, w_o_, b_o_ ? &b_o_->t : nullptr, dtype).t;
         }
         Tensor y = c.alloc(dtype, {n, qd});
-        attend(c, q, entry, table, y);
+        attend(c, q, entry, table, head_scale, y);
         if (stream) {
             add_product(c, *stream, y, w_o_);
             return Tensor();
@@ -497,6 +572,21 @@ private:
                              q.data, (int)n, n_heads_, n_kv_heads_, head_dim_, value_dim_, write ? 1 : 0, values_are_keys_ ? 1 : 0, c.stream);
     }
 
+    // product (the gate's rows behind the others), then biases, the norm over the projection, rotation, the gate's sigmoid and the cache write
+    // in one kernel
+    void projected_q(StepContext& c, const Tensor& x, const CacheEntry& entry, const StepContext::Table& table, Tensor& q, Tensor& head_scale) {
+        const Tensor p = linear(c, x, w_qkv_, nullptr, x.dtype).t;
+        const Position::Tables tb = position_->tables();
+        const bool turn = tb.style != STYLE_NONE, write = entry.writes;
+        const long long gate_at = (long long)n_heads_ * head_dim_ + (own_kv_ ? (long long)n_kv_heads_ * (head_dim_ + value_dim_) : 0);
+        auto floats = [](const OwnedPtr& o) { return o ? (const float*)o->t.data : nullptr; };
+        K::projection_store(p.data, p.dtype, row_, floats(bias_f_), floats(q_norm_f_), floats(k_norm_f_), eps_, turn ? (const float*)tb.cos.data : nullptr,
+                            turn ? (const float*)tb.sin.data : nullptr, turn ? tb.rot_dim : 0, turn ? tb.style : 0, turn ? (int)tb.cos.shape[0] : 0, c.dev.tok_seq,
+                            c.dev.tok_pos, write ? table.dev : nullptr, write ? table.width : 0, write ? entry.keys.data : nullptr,
+                            write ? entry.values.data : nullptr, q.data, (float*)head_scale.data, gate_at, (int)x.shape[0], n_heads_, n_kv_heads_, head_dim_,
+                            value_dim_, write ? 1 : 0, c.stream);
+    }
+
     // product, then biases, rotation (halves or pairs), the heads' norm without a weight after it, and the cache write in one kernel
     void turned_qkv(StepContext& c, const Activation& x, const CacheEntry& entry, const StepContext::Table& table, Tensor& q) {
         const int64_t n = x.rows();
@@ -513,14 +603,15 @@ private:
                            write ? 1 : 0, c.stream);
     }
 
-    // Attention of rows (sequence tok_seq[r], position tok_pos[r]) with the cap, the kept first positions and the sink.  bfloat16 on the
+    // Attention of rows (sequence tok_seq[r], position tok_pos[r]) with the cap, the kept first positions, the sink and the heads' gates.  bfloat16 on the
     // matrix cores where the sizes allow: steps of one token a sequence and a few chosen rows with a row's pages dealt out to
     // partitions, other steps in tiles of consecutive queries; else the plain kernel, one wave per (row, head).
     void attend_masked(StepContext& c, const Tensor& q, const CacheEntry& entry, const StepContext::Table& table, const int32_t* tok_seq,
-                       const int32_t* tok_pos, Tensor& out, bool last_rows) {
+                       const int32_t* tok_pos, const Tensor& head_scale, Tensor& out, bool last_rows) {
         const int n = (int)q.shape[0], n_pages = (int)entry.keys.shape[0];
         const void* sink = sink_ ? sink_->t.data : nullptr;
         const int sink_dtype = sink_ ? sink_->t.dtype : 0;
+        const float* hs = (const float*)head_scale.data;
         if (q.dtype == BF16 && K::attention_masked_mfma_supported.raw(head_dim_, value_dim_)) {
             const bool rows = last_rows ? n <= DECODE_KERNEL_ROWS : c.all_decode;
             if (rows && policy().decode_mfma) {
@@ -539,13 +630,13 @@ private:
                     part_ml = c.alloc(F32, {n, n_heads_, n_parts, 2});
                 }
                 K::attention_masked_mfma(q.data, entry.keys.data, entry.values.data, tok_pos, row_table, table.width, n_pages, window_, chunk_, keep_first_, scale_,
-                                         cap_, sink, sink_dtype, nullptr, nullptr, nullptr, 0, 0, n, n_parts, part_out.data, part_ml.data, out.data, n_heads_,
+                                         cap_, sink, sink_dtype, hs, nullptr, nullptr, nullptr, 0, 0, n, n_parts, part_out.data, part_ml.data, out.data, n_heads_,
                                          n_kv_heads_, head_dim_, value_dim_, c.stream);
                 return;
             }
             // keys and values of one size, every earlier position visible (or a plain window), no sink: the prompt kernel of the
             // plain attention takes the cap as an option
-            if (!rows && policy().prefill_mfma && value_dim_ == head_dim_ && keep_first_ == 0 && !sink_ &&
+            if (!rows && policy().prefill_mfma && value_dim_ == head_dim_ && keep_first_ == 0 && !sink_ && !hs &&
                 K::attention_prefill_supported.raw(head_dim_)) {
                 const int tile = tile_for(c);
                 const Tiles t = last_rows ? c.last_tiles(tile) : c.query_tiles(tile);
@@ -558,14 +649,14 @@ private:
                 const int tile = K::attention_masked_mfma_tile.raw(n, n_heads_, n_kv_heads_, head_dim_, value_dim_);
                 const Tiles t = last_rows ? c.last_tiles(tile) : c.query_tiles(tile);
                 K::attention_masked_mfma(q.data, entry.keys.data, entry.values.data, tok_pos, table.dev, table.width, n_pages, window_, chunk_, keep_first_, scale_,
-                                         cap_, sink, sink_dtype, t.seq, t.tok0, t.count, t.n, tile, 0, 1, nullptr, nullptr, out.data, n_heads_, n_kv_heads_,
+                                         cap_, sink, sink_dtype, hs, t.seq, t.tok0, t.count, t.n, tile, 0, 1, nullptr, nullptr, out.data, n_heads_, n_kv_heads_,
                                          head_dim_, value_dim_, c.stream);
                 return;
             }
         }
         K::attention_masked(q.data, entry.keys.data, entry.values.data, q.dtype, tok_seq, tok_pos, table.dev, table.width, c.n_seqs,
                             (int)entry.keys.shape[0], window_, chunk_, keep_first_, scale_, cap_, sink_ ? sink_->t.data : nullptr, sink_ ? sink_->t.dtype : 0,
-                            out.data, (int)q.shape[0], n_heads_, n_kv_heads_, head_dim_, value_dim_, c.stream);
+                            hs, out.data, (int)q.shape[0], n_heads_, n_kv_heads_, head_dim_, value_dim_, c.stream);
     }
 
     // queries per tile of the prompt kernel for this step
@@ -658,9 +749,9 @@ private:
     // head size the MFMA kernels do not take: the plain kernel, one wave per (token, head).
     // bfloat16 and one token per sequence: the partitioned decoding kernel; bfloat16 otherwise: the
     // tiled prompt kernel.
-    void attend(StepContext& c, const Tensor& q, const CacheEntry& entry, const StepContext::Table& table, Tensor& out) {
+    void attend(StepContext& c, const Tensor& q, const CacheEntry& entry, const StepContext::Table& table, const Tensor& head_scale, Tensor& out) {
         const int n = (int)q.shape[0], n_pages = (int)entry.keys.shape[0];
-        if (extras_) return attend_masked(c, q, entry, table, c.dev.tok_seq, c.dev.tok_pos, out, false);
+        if (extras_) return attend_masked(c, q, entry, table, c.dev.tok_seq, c.dev.tok_pos, head_scale, out, false);
         if (q.dtype == BF16 && c.all_decode && policy().decode_mfma && K::attention_decode_supported.raw(head_dim_))
             return decode_kernel(c, q, entry, c.dev.tok_pos, table.dev, table.width, out);
         // (not for steps of one token per sequence: tiles of one query are what the plain kernel does anyway,
@@ -679,9 +770,9 @@ private:
 
     // The same for the step's last_rows alone (q holds their queries): the cache already holds the
     // keys and values of all the step's tokens.
-    void attend_rows(StepContext& c, const Tensor& q, const CacheEntry& entry, const StepContext::Table& table, Tensor& out) {
+    void attend_rows(StepContext& c, const Tensor& q, const CacheEntry& entry, const StepContext::Table& table, const Tensor& head_scale, Tensor& out) {
         const int n = (int)q.shape[0], n_pages = (int)entry.keys.shape[0];
-        if (extras_) return attend_masked(c, q, entry, table, c.dev.last_seq, c.dev.last_pos, out, true);
+        if (extras_) return attend_masked(c, q, entry, table, c.dev.last_seq, c.dev.last_pos, head_scale, out, true);
         if (q.dtype == BF16 && policy().decode_mfma && K::attention_decode_supported.raw(head_dim_) && c.n_last <= DECODE_KERNEL_ROWS) {
             // few rows: the decoding kernel shares a row's keys out over many blocks, where the prompt
             // kernel would walk them in one; a row is a sequence of its own to it
@@ -711,7 +802,12 @@ private:
     int value_dim_, chunk_ = 0, keep_first_, value_mix_ = MIX_NONE;
     bool qk_norm_ = false, has_sink_ = false, extras_ = false, cache_keeps_all_ = false, values_are_keys_ = false;
     bool qk_norm_weight_ = true, norm_after_rotation_ = false, turned_first_ = false;
-    float eps_ = 0.f, cap_ = 0.f;
+    bool projected_ = false, fixed_sink_ = false, gated_ = false, own_kv_ = true;
+    int cache_window_ = 0;
+    int64_t row_ = 0;
+    float eps_ = 0.f, cap_ = 0.f, sink_score_ = 0.f;
+    std::string n_gate_;
+    OwnedPtr bias_f_, q_norm_f_, k_norm_f_;
     std::string mix_key_, n_q_, n_k_, n_v_, n_o_, n_q_norm_, n_k_norm_, n_sink_, n_mix_, n_qb_, n_kb_, n_vb_;
     std::shared_ptr<Position> position_;
     Weight w_qkv_, w_o_;
@@ -986,6 +1082,8 @@ void register_builtin_parts() {
         register_linear_attention_parts();
         register_pooled_parts();
         register_mlstm_parts();
+        register_time_mixing_parts();
+        register_joint_parts();
         register_kind("block", "pre_norm", [](const PartSpec& s, BuildEnv& e) { return std::make_shared<PreNormBlock>(s, e); });
     });
 }

@@ -171,7 +171,7 @@ public:
         const float inv_tau = per_channel_ ? (float)(1.0 / tau_) : 0.f;
         Tensor o = c.alloc(F32, {n, heads_, dv_});
         auto run = [&](int mode, int items, const Chunks* ch, float* cs, float* cd) {
-            K::linear_attention(in.data, at(in, qk), at(in, 2 * qk), dtype, row_, zp, qk, zb, inv_tau, hd, nullptr, nullptr, nullptr, q_scale_, k_scale_, cos, sin, turn ? tb.rot_dim : 0,
+            K::linear_attention(in.data, at(in, qk), at(in, 2 * qk), dtype, row_, zp, qk, zb, inv_tau, hd, nullptr, nullptr, nullptr, nullptr, nullptr, q_scale_, k_scale_, cos, sin, turn ? tb.rot_dim : 0,
                                 turn ? tb.style : 0, max_pos, c.dev.tok_pos, state, row, c.dev.cu, c.dev.seq_new, c.dev.seq_slot, ch ? ch->row0 : nullptr,
                                 ch ? ch->count : nullptr, cs, cd, (float*)o.data, mode, items, heads_, d_, dv_, (long long)d_ * dv_, c.stream);
         };

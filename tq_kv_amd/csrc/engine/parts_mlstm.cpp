@@ -143,7 +143,7 @@ public:
                        head_stride(), m_offset, c.dev.cu, c.dev.seq_new, c.dev.seq_slot, (float*)kappa.data, (float*)tau.data, (float*)m.data,
                        (float*)inv_den.data, c.n_seqs, heads_, d_, c.stream);
         K::linear_attention(in.data, at(in, qk), at(in, 2 * qk), F32, row_, nullptr, 0, nullptr, 0.f, nullptr, (const float*)kappa.data,
-                            (const float*)tau.data, (const float*)inv_den.data, q_scale_, 1.f, nullptr, nullptr, 0, 0, 0, c.dev.tok_pos, state, row, c.dev.cu,
+                            (const float*)tau.data, (const float*)inv_den.data, nullptr, nullptr, q_scale_, 1.f, nullptr, nullptr, 0, 0, 0, c.dev.tok_pos, state, row, c.dev.cu,
                             c.dev.seq_new, c.dev.seq_slot, nullptr, nullptr, nullptr, nullptr, (float*)o.data, 0, c.n_seqs, heads_, d_, dv_, head_stride(),
                             c.stream);
         K::head_norm_gate((const float*)o.data, norm_w, dv_, eps_, gate, F32, row_, 1, gated.data, dtype, (int)n, heads_, dv_, c.stream);

@@ -18,9 +18,15 @@
 // instead of the softmax over all; weight_on "input" multiplies an expert's input by the weight (the output is then the plain sum of
 // E(w x) over the chosen experts, which is not w E(x) since an expert is not linear).
 //
-// params: hidden, inter, n_experts, top, router_scale, gate / limit / alpha, gated, normalize, score, weight_on, shared (a feed-forward
+// Choosing by more than the score: correction names a tensor [experts + identity] that is added to the scores for the choice alone;
+// n_groups and keep_groups cut the experts into equal groups of neighbours, and only experts of the keep_groups best groups (by the largest
+// choice score in them) can be chosen; identity: so many experts more, the router's last, that have no tensors and give back their
+// input.  With any of them the weights are the chosen experts' softmax scores over their sum plus weight_floor (normalize "chosen").
+//
+// params: hidden, inter, n_experts, top, router_scale, gate / limit / alpha, gated, normalize, score, weight_on, identity, correction (a tensor's
+// name, or null), n_groups, keep_groups, weight_floor, shared (a feed-forward
 // part spec, or null), shared_gate (a tensor's name, or null); optional names {router, expert (with %d for the expert's number), gate, up,
-// down, shared}.  Tensors: router [experts, hidden]; per expert gate, up [inter, hidden], down
+// down, shared}.  Tensors: router [experts + identity, hidden]; per expert gate, up [inter, hidden], down
 // [hidden, inter]; the shared expert's own under its prefix.
 #include "kernels.h"
 #include "linear.h"
@@ -34,6 +40,15 @@ OwnedPtr take(Loaded& tensors, const std::string& name) {
     auto it = tensors.find(name);
     if (it == tensors.end() || !it->second) raise(TQE_ERR_WEIGHTS, "a part was not given its tensor '%s'", name.c_str());
     return it->second;
+}
+
+OwnedPtr as_floats(const OwnedPtr& p, hipStream_t stream) {
+    if (p->t.dtype == F32) return p;
+    std::vector<int64_t> dims(p->t.shape, p->t.shape + p->t.ndim);
+    OwnedPtr out = make_owned(F32, dims);
+    if (!null_device()) K::convert(p->t.data, p->t.dtype, out->t.data, F32, (long long)p->t.numel(), stream);
+    stream_synchronize(stream);
+    return out;
 }
 
 class RoutedExperts : public FeedForward {
@@ -57,9 +72,21 @@ public:
         if (weight_on != "output" && weight_on != "input") raise(TQE_ERR_ARGUMENT, "routed_experts: unknown weight_on '%s' (known: input, output)", weight_on.c_str());
         weight_on_input_ = weight_on == "input";
         n_shared_gate_ = r.string_or("shared_gate", "");
-        if (top_ > n_experts_) raise(TQE_ERR_ARGUMENT, "routed_experts: top %d of %d experts", top_, n_experts_);
+        identity_ = (int)r.integer_or("identity", 0, 0);
+        n_correction_ = r.string_or("correction", "");
+        n_groups_ = (int)r.integer_or("n_groups", 1, 1);
+        keep_groups_ = (int)r.integer_or("keep_groups", n_groups_, 1);
+        weight_floor_ = (float)r.number_or("weight_floor", 0.0);
+        const int outputs = n_experts_ + identity_;
+        by_choice_ = identity_ > 0 || !n_correction_.empty() || keep_groups_ < n_groups_ || weight_floor_ != 0.f;
+        if (top_ > outputs) raise(TQE_ERR_ARGUMENT, "routed_experts: top %d of %d experts", top_, outputs);
+        if (outputs % n_groups_ || keep_groups_ > n_groups_) raise(TQE_ERR_ARGUMENT, "routed_experts: %d of %d groups of %d experts", keep_groups_, n_groups_, outputs);
+        if (top_ > keep_groups_ * (outputs / n_groups_))
+            raise(TQE_ERR_ARGUMENT, "routed_experts: top %d of the %d experts that %d groups hold", top_, keep_groups_ * (outputs / n_groups_), keep_groups_);
+        if (by_choice_ && (!renormalize_ || sigmoid_scores_ || !n_shared_gate_.empty() || router_scale_ != 1.f))
+            raise(TQE_ERR_ARGUMENT, "routed_experts: identity, correction, groups and weight_floor go with softmax scores, normalize 'chosen', router_scale 1 and no shared_gate");
         const int most = K::moe_max_experts.raw();
-        if (n_experts_ > most) raise(TQE_ERR_CONFIG, "routed_experts: %d experts are more than the kernels take (%d)", n_experts_, most);
+        if (outputs > most) raise(TQE_ERR_CONFIG, "routed_experts: %d experts are more than the kernels take (%d)", outputs, most);
         const Json& names = spec.params["names"];
         auto name = [&](const char* role, const char* fallback) { return names[role].is_string() ? names[role].as_string() : std::string(fallback); };
         n_router_ = name("router", "router");
@@ -86,7 +113,8 @@ public:
     }
     TensorSpecs tensors() const override {
         auto w = [](int64_t a, int64_t b) { TensorSpec t; t.shape = {a, b}; return t; };
-        TensorSpecs t = {{n_router_, w(n_experts_, hidden_)}};
+        TensorSpecs t = {{n_router_, w(n_experts_ + identity_, hidden_)}};
+        if (!n_correction_.empty()) { TensorSpec c; c.shape = {n_experts_ + identity_}; t.push_back({n_correction_, c}); }
         for (int e = 0; e < n_experts_; ++e) {
             const std::string p = expert_prefix(e);
             if (gated_) t.push_back({p + n_gate_, w(inter_, hidden_)});
@@ -100,6 +128,7 @@ public:
     }
     void load(Loaded& t, hipStream_t stream) override {
         router_ = take(t, n_router_);
+        if (!n_correction_.empty()) correction_ = as_floats(stored_correction_ = take(t, n_correction_), stream);
         // all experts' weights in two tensors: [experts, gate rows then up rows, hidden] and [experts, hidden, inter]
         std::vector<OwnedPtr> gu, down;
         for (int e = 0; e < n_experts_; ++e) {
@@ -119,6 +148,7 @@ public:
     }
     OwnedPtr held(const std::string& name) const override {
         if (name == n_router_) return router_;
+        if (!n_correction_.empty() && name == n_correction_) return stored_correction_;
         if (!n_shared_gate_.empty() && name == n_shared_gate_) return shared_gate_;
         if (name == "experts.gate_up") return gate_up_;
         if (name == "experts.down") return down_;
@@ -130,7 +160,16 @@ public:
         if (shared_) shared_->product_shapes(out);
     }
 
-    Tensor forward(StepContext& c, const Activation& x, Stream*) override {
+    Tensor forward(StepContext& c, const Activation& x, Stream*) override { return run(c, x, nullptr, 1.f); }
+    bool takes_beside() const override { return true; }
+    Tensor forward_beside(StepContext& c, const Activation& x, const Tensor& beside, float scale) override {
+        if (beside.dtype != x.x.dtype || beside.shape[0] != x.x.shape[0] || beside.cols() != hidden_)
+            raise(TQE_ERR_STATE, "routed_experts: what is to be added is %s for a step of [%lld, %lld]", beside.describe().c_str(), (long long)x.x.shape[0], (long long)hidden_);
+        return run(c, x, beside.data, scale);
+    }
+
+private:
+    Tensor run(StepContext& c, const Activation& x, const void* beside, float scale) {
         if (x.lazy) raise(TQE_ERR_STATE, "routed_experts takes no folded norm");
         const int64_t n = x.x.shape[0];
         const int dtype = x.x.dtype;
@@ -151,8 +190,13 @@ public:
         Tensor shared_scale;
         const bool gate_in_route = shared_gate_ && shared_gate_->t.dtype == router_->t.dtype;
         if (shared_gate_) shared_scale = c.alloc(F32, {n});
-        K::moe_route(x.x.data, dtype, router_->t.data, router_->t.dtype, n_experts_, (int)hidden_, top_, router_scale_, (renormalize_ ? 1 : 0) | (sigmoid_scores_ ? 2 : 0), (int32_t*)idx.data,
-                     (float*)weight.data, gate_in_route ? shared_gate_->t.data : nullptr, gate_in_route ? (float*)shared_scale.data : nullptr, (int)n, c.stream);
+        if (by_choice_)
+            K::moe_route_grouped(x.x.data, dtype, router_->t.data, router_->t.dtype, n_experts_ + identity_, (int)hidden_, top_,
+                                 correction_ ? (const float*)correction_->t.data : nullptr, n_groups_, keep_groups_, weight_floor_, (int32_t*)idx.data,
+                                 (float*)weight.data, (int)n, c.stream);
+        else
+            K::moe_route(x.x.data, dtype, router_->t.data, router_->t.dtype, n_experts_, (int)hidden_, top_, router_scale_, (renormalize_ ? 1 : 0) | (sigmoid_scores_ ? 2 : 0), (int32_t*)idx.data,
+                         (float*)weight.data, gate_in_route ? shared_gate_->t.data : nullptr, gate_in_route ? (float*)shared_scale.data : nullptr, (int)n, c.stream);
         K::moe_group((const int32_t*)idx.data, (int)n, top_, n_experts_, tile_m, (int32_t*)pair_pos.data, (int32_t*)sorted_tok.data, tile_expert, tile_row0,
                      tile_rows, (int32_t*)n_tiles.data, c.stream);
         Tensor shared_out;
@@ -191,20 +235,21 @@ public:
                            0, 0.f, 1.f, tile_expert, tile_row0, tile_rows, (const int32_t*)n_tiles.data, max_tiles, c.stream);
         }
         Tensor out = c.alloc(dtype, {n, hidden_});
-        K::moe_combine(y.data, dtype, (const int32_t*)pair_pos.data, sum_weight, top_, shared_out.data,
-                       shared_gate_ ? (const float*)shared_scale.data : nullptr, out.data, (int)n,
-                       (int)hidden_, c.stream);
+        K::moe_combine(y.data, dtype, (const int32_t*)pair_pos.data, sum_weight, top_, identity_ ? x.x.data : nullptr, shared_out.data,
+                       shared_gate_ ? (const float*)shared_scale.data : nullptr, beside, scale, out.data, (int)n, (int)hidden_, c.stream);
         return out;
     }
 
-private:
     int64_t hidden_, inter_;
     int n_experts_, top_;
     float router_scale_;
     Gate gate_;
     bool gated_ = true, renormalize_ = false, sigmoid_scores_ = false, weight_on_input_ = false;
-    std::string n_shared_gate_;
-    OwnedPtr shared_gate_;
+    int identity_ = 0, n_groups_ = 1, keep_groups_ = 1;
+    bool by_choice_ = false;
+    float weight_floor_ = 0.f;
+    std::string n_shared_gate_, n_correction_;
+    OwnedPtr shared_gate_, correction_, stored_correction_;
     std::string n_router_, n_expert_, n_gate_, n_up_, n_down_, n_shared_;
     std::shared_ptr<FeedForward> shared_;
     OwnedPtr router_, gate_up_, down_;

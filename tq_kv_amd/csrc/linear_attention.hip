@@ -1,7 +1,9 @@
 // Linear attention with a decaying state: per head S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, with S of d rows (key
 // channels) and dv columns in float32.  The decay a_t is one number per head (fixed) or one per key channel and token, formed here
 // from a product z as sigmoid(z + bias)^(1/tau) = exp(logsigmoid(z + bias) / tau), or one number per head and token given by its
-// logarithm (log_decay; then k may be weighted by exp(log_in) and the output multiplied by out_scale, per head and token too).  q and k may be turned by the position (tables of
+// logarithm (log_decay; then k may be weighted by exp(log_in) and the output multiplied by out_scale, per head and token too), or given as it
+// is per key channel and token (decay).  With a bonus u [heads, d] a token's output reads the state in front of it, and the token itself through
+// u instead of the state: o_t = S_(t-1)^T q_t + (sum_i u_i k_i q_i) v_t.  q and k may be turned by the position (tables of
 // cos and sin, in halves or neighbouring pairs over the first rot_dim elements) and scaled on their way in; everything after the
 // loads is float32.
 //
@@ -30,6 +32,8 @@ struct LaArgs {
     float inv_tau;
     const float* head_decay;
     const float *log_decay, *log_in, *out_scale;        // [tokens, heads] or null
+    const float* decay;                                 // [tokens, heads * d], or null
+    const float* bonus;                                 // [heads, d], or null
     float q_scale, k_scale;
     const float *cos, *sin;
     int rot_dim, style, max_pos;
@@ -44,10 +48,23 @@ struct LaArgs {
     long long head_stride;          // elements between the heads' parts of a state
 };
 
-template <typename T, int RT, int MODE>
+// With a bonus: the staged tokens' sums of u k q over the head's channels, a wave a token (in LDS, after every thread's pieces of q and k are)
+__device__ __forceinline__ void la_bonus_sums(const float* lq, const float* lk, const float* u, int d, int row, int nt, float* sums) {
+    const int lane = threadIdx.x % TQK_WAVE;
+    __syncthreads();
+    for (int tt = threadIdx.x / TQK_WAVE; tt < nt; tt += blockDim.x / TQK_WAVE) {
+        float s = 0.f;
+        for (int i = lane; i < d; i += TQK_WAVE) s = fmaf(u[i] * lk[tt * row + i], lq[tt * row + i], s);
+        s = wave_sum(s);
+        if (lane == 0) sums[tt] = s;
+    }
+}
+
+template <typename T, int RT, int MODE, bool BONUS>
 __global__ __launch_bounds__(LA_THREADS)
 void linear_attention_kernel(LaArgs a, int rg_shift) {
     extern __shared__ float la_lds[];
+    __shared__ float la_bonus[LA_TB];
     const int d = a.d, dv = a.dv, H = a.H;
     const int head = blockIdx.y, item = blockIdx.z;
     const int RG = 1 << rg_shift, CB = LA_THREADS >> rg_shift;
@@ -97,7 +114,9 @@ void linear_attention_kernel(LaArgs a, int rg_shift) {
             lq[e] = qv * a.q_scale;
             lk[e] = kv * a.k_scale;
             float al;
-            if (a.z) {
+            if (a.decay) {
+                al = a.decay[(row * H + head) * d + i];
+            } else if (a.z) {
                 const float zz = a.z[row * a.z_stride + (size_t)head * d + i] + a.z_bias[(size_t)head * d + i];
                 const float ls = fminf(zz, 0.f) - log1pf(expf(-fabsf(zz)));
                 al = expf(ls * a.inv_tau);
@@ -107,6 +126,7 @@ void linear_attention_kernel(LaArgs a, int rg_shift) {
             } else al = a.head_decay[head];
             ld[e] = al;
         }
+        if (BONUS && MODE != LA_LOCAL) la_bonus_sums(lq, lk, a.bonus + (size_t)head * d, d, d, nt, la_bonus);
         __syncthreads();
         for (int tt = 0; tt < nt; ++tt) {
             const long long row = row0 + t0 + tt;
@@ -119,13 +139,15 @@ void linear_attention_kernel(LaArgs a, int rg_shift) {
             for (int i = 0; i < RT; ++i) {
                 const int r = i * RG + rg;
                 if (r < d) {
+                    if (BONUS) o = fmaf(S[i], q[r], o);
                     S[i] = fmaf(al[r], S[i], k[r] * vv);
-                    o = fmaf(S[i], q[r], o);
+                    if (!BONUS) o = fmaf(S[i], q[r], o);
                     if (MODE == LA_LOCAL) P[i] *= al[r];
                 }
             }
             if (MODE != LA_LOCAL) {
                 for (int m = RG >> 1; m > 0; m >>= 1) o += __shfl_xor(o, m, TQK_WAVE);
+                if (BONUS) o = fmaf(la_bonus[tt], vv, o);
                 if (rg == 0 && col_ok) a.out[((size_t)row * H + head) * dv + col] = a.out_scale ? o * a.out_scale[row * H + head] : o;
             }
         }
@@ -142,10 +164,11 @@ void linear_attention_kernel(LaArgs a, int rg_shift) {
 // The same with a block of the state per thread: RT neighbouring rows by four neighbouring columns, for heads whose sizes are multiples of
 // four.  A token costs a thread three 16-byte LDS reads per four rows (q, k and the decay) and one for its four values, for 4 RT state
 // elements; rows beyond the head's (the padding up to RG * RT) stay zero.
-template <typename T, int RT, int MODE>
+template <typename T, int RT, int MODE, bool BONUS>
 __global__ __launch_bounds__(LA_THREADS)
 void linear_attention_block_kernel(LaArgs a, int rg_shift, int cb) {
     extern __shared__ float la_lds[];
+    __shared__ float la_bonus[LA_TB];
     const int d = a.d, dv = a.dv, H = a.H;
     const int head = blockIdx.y, item = blockIdx.z;
     const int RG = 1 << rg_shift, dpad = RG * RT;
@@ -200,7 +223,9 @@ void linear_attention_block_kernel(LaArgs a, int rg_shift, int cb) {
                 }
                 qv *= a.q_scale;
                 kv *= a.k_scale;
-                if (a.z) {
+                if (a.decay) {
+                    al = a.decay[((size_t)row * H + head) * d + i];
+                } else if (a.z) {
                     const float zz = a.z[row * a.z_stride + (size_t)head * d + i] + a.z_bias[(size_t)head * d + i];
                     const float ls = fminf(zz, 0.f) - log1pf(expf(-fabsf(zz)));
                     al = expf(ls * a.inv_tau);
@@ -217,6 +242,7 @@ void linear_attention_block_kernel(LaArgs a, int rg_shift, int cb) {
             const int tt = e / cb, c = e - tt * cb, col = blockIdx.x * cb + c;
             lv[e] = col < dv ? to_float(vb[(row0 + t0 + tt) * a.stride + col]) : 0.f;
         }
+        if (BONUS && MODE != LA_LOCAL) la_bonus_sums(lq, lk, a.bonus + (size_t)head * d, d, dpad, nt, la_bonus);
         __syncthreads();
         if (cg * 4 < cb) {
             for (int tt = 0; tt < nt; ++tt) {
@@ -233,8 +259,9 @@ void linear_attention_block_kernel(LaArgs a, int rg_shift, int cb) {
                     for (int j = 0; j < 4; ++j) {
 #pragma unroll
                         for (int c = 0; c < 4; ++c) {
+                            if (BONUS) o[c] = fmaf(S[i + j][c], qq[j], o[c]);
                             S[i + j][c] = fmaf(aa[j], S[i + j][c], kk[j] * v4[c]);
-                            o[c] = fmaf(S[i + j][c], qq[j], o[c]);
+                            if (!BONUS) o[c] = fmaf(S[i + j][c], qq[j], o[c]);
                         }
                         if (MODE == LA_LOCAL) P[i + j] *= aa[j];
                     }
@@ -243,6 +270,10 @@ void linear_attention_block_kernel(LaArgs a, int rg_shift, int cb) {
 #pragma unroll
                     for (int c = 0; c < 4; ++c)
                         for (int m = RG >> 1; m > 0; m >>= 1) o[c] += __shfl_xor(o[c], m, TQK_WAVE);
+                    if (BONUS) {
+#pragma unroll
+                        for (int c = 0; c < 4; ++c) o[c] = fmaf(la_bonus[tt], v4[c], o[c]);
+                    }
                     if (rg == 0 && col_ok) {
                         float* dst = a.out + ((size_t)(row0 + t0 + tt) * H + head) * dv + col0;
                         if (a.out_scale) {
@@ -298,13 +329,13 @@ extern "C" int tqk_linear_attention_max_dim(void) { return 512; }
 
 extern "C" int tqk_linear_attention(const void* q, const void* k, const void* v, int act_dtype, long long stride, const float* z, long long z_stride,
                                     const float* z_bias, float inv_tau, const float* head_decay, const float* log_decay, const float* log_in,
-                                    const float* out_scale, float q_scale, float k_scale, const float* cos,
+                                    const float* out_scale, const float* decay, const float* bonus, float q_scale, float k_scale, const float* cos,
                                     const float* sin, int rot_dim, int style, int max_pos, const int32_t* tok_pos, float* state, long long state_stride,
                                     const int32_t* cu, const int32_t* seq_new, const int32_t* seq_slot, const int32_t* chunk_row0,
                                     const int32_t* chunk_count, float* chunk_state, float* chunk_decay, float* out, int mode, int n_items, int heads,
                                     int d, int dv, long long head_stride, void* stream) {
     TQK_REQUIRE(q && k && v, "tqk_linear_attention: null pointer");
-    TQK_REQUIRE((z && z_bias) || head_decay || log_decay, "tqk_linear_attention: neither a decay per channel nor one per head");
+    TQK_REQUIRE((z && z_bias) || head_decay || log_decay || decay, "tqk_linear_attention: neither a decay per channel nor one per head");
     TQK_REQUIRE(head_stride >= (long long)d * dv, "tqk_linear_attention: heads' states overlap");
     TQK_REQUIRE(mode >= LA_SCAN && mode <= LA_APPLY, "tqk_linear_attention: unknown mode %d", mode);
     TQK_REQUIRE(mode == LA_SCAN ? (state && cu && seq_new && seq_slot) : (chunk_row0 && chunk_count && chunk_state && chunk_decay),
@@ -315,7 +346,7 @@ extern "C" int tqk_linear_attention(const void* q, const void* k, const void* v,
     TQK_REQUIRE(!cos || (sin && tok_pos && rot_dim > 0 && rot_dim % 2 == 0 && rot_dim <= d && max_pos > 0 && (style == LA_STYLE_HALVES || style == LA_STYLE_PAIRS)),
                 "tqk_linear_attention: bad rotation");
     if (n_items == 0) return 0;
-    LaArgs a = {q, k, v, stride, z, z_stride, z_bias, inv_tau, head_decay, log_decay, log_in, out_scale, q_scale, k_scale, cos, sin, rot_dim, style, max_pos, tok_pos,
+    LaArgs a = {q, k, v, stride, z, z_stride, z_bias, inv_tau, head_decay, log_decay, log_in, out_scale, decay, bonus, q_scale, k_scale, cos, sin, rot_dim, style, max_pos, tok_pos,
                 state, state_stride, cu, seq_new, seq_slot, chunk_row0, chunk_count, chunk_state, chunk_decay, out, heads, d, dv, head_stride};
     hipStream_t s = (hipStream_t)stream;
     if (d % 4 == 0 && dv % 4 == 0 && dv >= 16 && (((uintptr_t)out) & 15) == 0) {
@@ -330,7 +361,8 @@ extern "C" int tqk_linear_attention(const void* q, const void* k, const void* v,
             threads = (threads + TQK_WAVE - 1) / TQK_WAVE * TQK_WAVE;
             dim3 bgrid((dv + cb - 1) / cb, heads, n_items);
             const size_t blds = (size_t)LA_TB * (3 * (size_t)(rt << shift) + cb) * sizeof(float);
-#define TQK_LAB(T, RT, MODE) linear_attention_block_kernel<T, RT, MODE><<<bgrid, threads, blds, s>>>(a, shift, cb)
+#define TQK_LAB(T, RT, MODE) do { if (bonus) linear_attention_block_kernel<T, RT, MODE, true><<<bgrid, threads, blds, s>>>(a, shift, cb); \
+        else linear_attention_block_kernel<T, RT, MODE, false><<<bgrid, threads, blds, s>>>(a, shift, cb); } while (0)
 #define TQK_LAB_MODE(T, RT) do { if (mode == LA_SCAN) TQK_LAB(T, RT, LA_SCAN); else if (mode == LA_LOCAL) TQK_LAB(T, RT, LA_LOCAL); else TQK_LAB(T, RT, LA_APPLY); } while (0)
 #define TQK_LAB_ROWS(T) do { if (rt == 16) TQK_LAB_MODE(T, 16); else if (rt == 8) TQK_LAB_MODE(T, 8); else TQK_LAB_MODE(T, 4); } while (0)
             if (act_dtype == TQK_F32) TQK_LAB_ROWS(float);
@@ -353,7 +385,8 @@ extern "C" int tqk_linear_attention(const void* q, const void* k, const void* v,
     TQK_REQUIRE(rows <= 64, "tqk_linear_attention: %d rows a thread", rows);
     dim3 grid((dv + cb - 1) / cb, heads, n_items);
     const size_t lds = (size_t)3 * LA_TB * d * sizeof(float);
-#define TQK_LA(T, RT, MODE) linear_attention_kernel<T, RT, MODE><<<grid, LA_THREADS, lds, s>>>(a, rg_shift)
+#define TQK_LA(T, RT, MODE) do { if (bonus) linear_attention_kernel<T, RT, MODE, true><<<grid, LA_THREADS, lds, s>>>(a, rg_shift); \
+        else linear_attention_kernel<T, RT, MODE, false><<<grid, LA_THREADS, lds, s>>>(a, rg_shift); } while (0)
 #define TQK_LA_MODE(T, RT) do { if (mode == LA_SCAN) TQK_LA(T, RT, LA_SCAN); else if (mode == LA_LOCAL) TQK_LA(T, RT, LA_LOCAL); else TQK_LA(T, RT, LA_APPLY); } while (0)
 #define TQK_LA_ROWS(T) do { if (rows <= 1) TQK_LA_MODE(T, 1); else if (rows <= 2) TQK_LA_MODE(T, 2); else if (rows <= 4) TQK_LA_MODE(T, 4); \
         else if (rows <= 8) TQK_LA_MODE(T, 8); else if (rows <= 16) TQK_LA_MODE(T, 16); else if (rows <= 32) TQK_LA_MODE(T, 32); else TQK_LA_MODE(T, 64); } while (0)

@@ -4,14 +4,18 @@
 //   route     z = W_r x in float32, s = softmax(z) over all experts, the `top` largest (the lower index wins
 //             a tie); weight = s * scale, not renormalised.  One wave per token.  Mode bit 1 renormalises over the chosen;
 //             mode bit 2 makes every expert's score sigmoid(z) on its own instead of the softmax.
+//   route_grouped   the same logits over experts and, after them, experts that give back their input; chosen by s + correction within
+//             the best groups of neighbours (a group's rank is its largest s + correction), weights the chosen s over (their sum + floor)
 //   scale     rows[pair_pos[p]] = weight[p] * x[p / top] (for experts whose input, not output, carries the weight), and unit[p] = 1
 //   group     pair p = (token p / top, choice p % top) gets a row of its own among its expert's rows:
 //             pair_pos[p]; sorted_tok[row] names the row's token.  The rows of an expert are cut into tiles of
 //             tile_m rows; the tile list (expert, first row, rows) and its length stay on the device, so the
-//             launches that follow have the same shape whatever the router chose.
+//             launches that follow have the same shape whatever the router chose.  A choice beyond the experts with weights
+//             (an expert that gives back its input) gets no row: pair_pos[p] = -1.
 //   product   for each tile, rows x (gathered through sorted_tok, or as they lie) times the tile's expert's
 //             weight: plain, or gate and up with the gate applied.  Blocks beyond the list's length exit.
-//   combine   out[t] = sum_k weight[t, k] * y[pair_pos[t, k]] (+ what a shared expert gave), in float32.
+//   combine   out[t] = sum_k weight[t, k] * y[pair_pos[t, k]] (+ what a shared expert gave), in float32; the token's own input in
+//             place of a row where there is none; optionally out[t] = scale (that + beside[t]).
 //
 // A row's sums never depend on which rows share its tile, nor on the order the pairs were given rows in.
 #include "common.h"
@@ -27,14 +31,9 @@
 // A block per token: its waves share the experts out for the logits (each a dot product over the lanes, several loads
 // under way at once, added up in a fixed order), then the first wave takes the softmax and the largest.
 template <typename TA, typename TW>
-__global__ __launch_bounds__(MOE_ROUTE_WAVES * TQK_WAVE)
-void moe_route_kernel(const TA* __restrict__ x, const TW* __restrict__ w, int n_experts, int hidden, int top, float scale, int mode,
-                      int32_t* __restrict__ idx, float* __restrict__ weight, const TW* __restrict__ gate_w, float* __restrict__ gate_out) {
-    const int renormalize = mode & 1, sigmoid_scores = mode & 2;
-    __shared__ float z[MOE_MAX_EXPERTS];
+__device__ __forceinline__ void route_logits(const TA* __restrict__ xr, const TW* __restrict__ w, int n_experts, int hidden, const TW* __restrict__ gate_w,
+                                             float* __restrict__ gate_out, float* z) {
     const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
-    const int t = blockIdx.x;
-    const TA* xr = x + (size_t)t * hidden;
     // one row more where a gate is given: sigmoid(x . gate_w) per token, which rides along with the experts' dot products
     for (int e = wave; e < n_experts + (gate_w ? 1 : 0); e += MOE_ROUTE_WAVES) {
         const TW* wr = e < n_experts ? w + (size_t)e * hidden : gate_w;
@@ -67,10 +66,21 @@ void moe_route_kernel(const TA* __restrict__ x, const TW* __restrict__ w, int n_
         const float dot = wave_sum((d0 + d1) + (d2 + d3));
         if (lane == 0) {
             if (e < n_experts) z[e] = dot;
-            else gate_out[t] = 1.f / (1.f + expf(-dot));
+            else *gate_out = 1.f / (1.f + expf(-dot));
         }
     }
     __syncthreads();
+}
+
+template <typename TA, typename TW>
+__global__ __launch_bounds__(MOE_ROUTE_WAVES * TQK_WAVE)
+void moe_route_kernel(const TA* __restrict__ x, const TW* __restrict__ w, int n_experts, int hidden, int top, float scale, int mode,
+                      int32_t* __restrict__ idx, float* __restrict__ weight, const TW* __restrict__ gate_w, float* __restrict__ gate_out) {
+    const int renormalize = mode & 1, sigmoid_scores = mode & 2;
+    __shared__ float z[MOE_MAX_EXPERTS];
+    const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
+    const int t = blockIdx.x;
+    route_logits(x + (size_t)t * hidden, w, n_experts, hidden, gate_w, gate_w ? gate_out + t : nullptr, z);
     if (wave != 0) return;
     float m = -INFINITY;
     for (int e = lane; e < n_experts; e += TQK_WAVE) m = fmaxf(m, z[e]);
@@ -92,6 +102,7 @@ void moe_route_kernel(const TA* __restrict__ x, const TW* __restrict__ w, int n_
             const int oe = __shfl_xor(best_e, o, TQK_WAVE);
             if (ov > best || (ov == best && oe < best_e)) { best = ov; best_e = oe; }
         }
+        if (best_e >= n_experts) best_e = k;                        // (scores that are not numbers: some expert that is there)
         if (lane == best_e % TQK_WAVE) z[best_e] = -INFINITY;       // the lane that reads this expert writes it: no other sees it
         if (lane == 0) {
             idx[(size_t)t * top + k] = best_e;
@@ -107,6 +118,86 @@ void moe_route_kernel(const TA* __restrict__ x, const TW* __restrict__ w, int n_
     }
 }
 
+// The lane's largest of z[lane], z[lane + 64], ... below n, then the wave's: the lower index wins a tie.  In every lane of the wave.
+__device__ __forceinline__ int wave_argmax(const volatile float* z, int n, int lane, float& best) {
+    int at = 0x7fffffff;
+    best = -INFINITY;
+    for (int e = lane; e < n; e += TQK_WAVE) {
+        const float v = z[e];
+        if (v > best) { best = v; at = e; }
+    }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+        const float ov = __shfl_xor(best, o, TQK_WAVE);
+        const int oe = __shfl_xor(at, o, TQK_WAVE);
+        if (ov > best || (ov == best && oe < at)) { best = ov; at = oe; }
+    }
+    return at;
+}
+
+// Choice by score plus correction within the best groups of neighbours.  What the first wave keeps of the experts lies in LDS and is
+// read and written by that wave alone, each element by one lane between two of the wave's exchanges.
+template <typename TA, typename TW>
+__global__ __launch_bounds__(MOE_ROUTE_WAVES * TQK_WAVE)
+void moe_route_grouped_kernel(const TA* __restrict__ x, const TW* __restrict__ w, int n_experts, int hidden, int top, const float* __restrict__ correction,
+                              int n_groups, int keep, float floor, int32_t* __restrict__ idx, float* __restrict__ weight) {
+    __shared__ float z[MOE_MAX_EXPERTS];
+    __shared__ volatile float score[MOE_MAX_EXPERTS], choice[MOE_MAX_EXPERTS], group[MOE_MAX_EXPERTS];
+    const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
+    const int t = blockIdx.x;
+    route_logits(x + (size_t)t * hidden, w, n_experts, hidden, (const TW*)nullptr, (float*)nullptr, z);
+    if (wave != 0) return;
+    float m = -INFINITY;
+    for (int e = lane; e < n_experts; e += TQK_WAVE) m = fmaxf(m, z[e]);
+    m = wave_max(m);
+    float sum = 0.f;
+    for (int e = lane; e < n_experts; e += TQK_WAVE) sum += expf(z[e] - m);
+    sum = wave_sum(sum);
+    for (int e = lane; e < n_experts; e += TQK_WAVE) {
+        const float s = expf(z[e] - m) / sum;
+        score[e] = s;
+        choice[e] = s + (correction ? correction[e] : 0.f);
+    }
+    __threadfence_block();
+    __builtin_amdgcn_wave_barrier();
+    float best;
+    if (keep < n_groups) {
+        const int per = n_experts / n_groups;
+        for (int g = lane; g < n_groups; g += TQK_WAVE) {
+            float b = -INFINITY;
+            for (int i = 0; i < per; ++i) b = fmaxf(b, choice[g * per + i]);
+            group[g] = b;
+        }
+        __threadfence_block();
+        __builtin_amdgcn_wave_barrier();
+        // the kept groups are struck from the list; what is left on it is then closed
+        for (int k = 0; k < keep; ++k) {
+            const int g = wave_argmax(group, n_groups, lane, best);
+            if (g < n_groups && lane == g % TQK_WAVE) group[g] = -INFINITY;
+        }
+        __threadfence_block();
+        __builtin_amdgcn_wave_barrier();
+        for (int e = lane; e < n_experts; e += TQK_WAVE)
+            if (group[e / per] != -INFINITY) choice[e] = -INFINITY;
+        __threadfence_block();
+        __builtin_amdgcn_wave_barrier();
+    }
+    float chosen = 0.f;
+    for (int k = 0; k < top; ++k) {
+        int e = wave_argmax(choice, n_experts, lane, best);
+        e = e < n_experts ? e : k;                          // (scores that are not numbers: some expert that is there)
+        if (lane == e % TQK_WAVE) choice[e] = -INFINITY;
+        const float s = score[e];
+        chosen += s;
+        if (lane == 0) {
+            idx[(size_t)t * top + k] = e;
+            weight[(size_t)t * top + k] = s;
+        }
+    }
+    if (lane == 0)
+        for (int k = 0; k < top; ++k) weight[(size_t)t * top + k] /= chosen + floor;
+}
+
 // ---- group -----------------------------------------------------------------------------------
 __global__ __launch_bounds__(1024)
 void moe_group_kernel(const int32_t* __restrict__ idx, int n_pairs, int top, int n_experts, int tile_m, int32_t* __restrict__ pair_pos,
@@ -115,7 +206,10 @@ void moe_group_kernel(const int32_t* __restrict__ idx, int n_pairs, int top, int
     __shared__ int count[MOE_MAX_EXPERTS], offset[MOE_MAX_EXPERTS], tile_base[MOE_MAX_EXPERTS];
     for (int e = threadIdx.x; e < n_experts; e += blockDim.x) count[e] = 0;
     __syncthreads();
-    for (int p = threadIdx.x; p < n_pairs; p += blockDim.x) pair_pos[p] = atomicAdd(&count[idx[p]], 1);
+    for (int p = threadIdx.x; p < n_pairs; p += blockDim.x) {
+        const int e = idx[p];
+        pair_pos[p] = e < n_experts ? atomicAdd(&count[e], 1) : -1;
+    }
     __syncthreads();
     if (threadIdx.x == 0) {
         int rows = 0, tiles = 0;
@@ -137,7 +231,9 @@ void moe_group_kernel(const int32_t* __restrict__ idx, int n_pairs, int top, int
         }
     }
     for (int p = threadIdx.x; p < n_pairs; p += blockDim.x) {
-        const int row = offset[idx[p]] + pair_pos[p];
+        const int e = idx[p];
+        if (e >= n_experts) continue;
+        const int row = offset[e] + pair_pos[p];
         pair_pos[p] = row;
         sorted_tok[row] = p / top;
     }
@@ -223,7 +319,8 @@ void moe_product_kernel(const TX* __restrict__ x, const int32_t* __restrict__ x_
 template <typename TA>
 __global__ __launch_bounds__(256)
 void moe_combine_kernel(const TA* __restrict__ y, const int32_t* __restrict__ pair_pos, const float* __restrict__ weight, int top,
-                        const TA* __restrict__ shared, const float* __restrict__ shared_scale, TA* __restrict__ out, int hidden) {
+                        const TA* __restrict__ x, const TA* __restrict__ shared, const float* __restrict__ shared_scale, const TA* __restrict__ beside,
+                        float scale, TA* __restrict__ out, int hidden) {
     // the token's rows and weights once, side by side, not one load after the other in front of every element
     __shared__ int32_t row[MOE_MAX_EXPERTS];
     __shared__ float wt[MOE_MAX_EXPERTS];
@@ -237,9 +334,13 @@ void moe_combine_kernel(const TA* __restrict__ y, const int32_t* __restrict__ pa
     for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
         float v = 0.f;
 #pragma unroll 4
-        for (int k = 0; k < top; ++k) v = fmaf(wt[k], to_float(y[(size_t)row[k] * hidden + i]), v);
+        for (int k = 0; k < top; ++k) {
+            const TA* src = row[k] >= 0 || !x ? y + (size_t)row[k] * hidden : x + (size_t)t * hidden;
+            v = fmaf(wt[k], to_float(src[i]), v);
+        }
         if (shared) v = fmaf(ss, to_float(shared[(size_t)t * hidden + i]), v);
-        out[(size_t)t * hidden + i] = from_float<TA>(v);
+        if (beside) v += to_float(beside[(size_t)t * hidden + i]);
+        out[(size_t)t * hidden + i] = from_float<TA>(v * scale);
     }
 }
 
@@ -251,9 +352,11 @@ void moe_scale_rows_kernel(const TA* __restrict__ x, const int32_t* __restrict__
     const size_t p = blockIdx.x;
     const float w = weight[p];
     const TA* src = x + (p / top) * hidden;
-    TA* dst = rows + (size_t)pair_pos[p] * hidden;
+    const int row = pair_pos[p];
+    if (threadIdx.x == 0) unit[p] = row < 0 ? w : 1.f;              // without a row: the input itself, times the weight
+    if (row < 0) return;
+    TA* dst = rows + (size_t)row * hidden;
     for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = from_float<TA>(w * to_float(src[i]));
-    if (threadIdx.x == 0) unit[p] = 1.f;
 }
 
 // ---- entry points ----------------------------------------------------------------------------
@@ -291,6 +394,26 @@ extern "C" int tqk_moe_route(const void* x, int act_dtype, const void* w_router,
     else return tqk_fail("tqk_moe_route: unknown dtypes %d, %d", act_dtype, w_dtype);
 #undef TQK_ROUTE
     return tqk_check_launch("tqk_moe_route");
+}
+
+extern "C" int tqk_moe_route_grouped(const void* x, int act_dtype, const void* w_router, int w_dtype, int n_experts, int hidden, int top, const float* correction,
+                                     int n_groups, int keep, float floor, int32_t* idx, float* weight, int n_tokens, void* stream) {
+    TQK_REQUIRE(x && w_router && idx && weight, "tqk_moe_route_grouped: null pointer");
+    TQK_REQUIRE(n_experts > 0 && n_experts <= MOE_MAX_EXPERTS, "tqk_moe_route_grouped: %d experts, the kernel takes 1 to %d", n_experts, MOE_MAX_EXPERTS);
+    TQK_REQUIRE(n_groups > 0 && n_experts % n_groups == 0 && keep > 0 && keep <= n_groups, "tqk_moe_route_grouped: %d of %d groups of %d experts", keep, n_groups, n_experts);
+    TQK_REQUIRE(top > 0 && top <= keep * (n_experts / n_groups) && hidden > 0 && n_tokens >= 0, "tqk_moe_route_grouped: bad sizes (top %d of %d experts)", top,
+                keep * (n_experts / n_groups));
+    if (n_tokens == 0) return 0;
+    hipStream_t s = (hipStream_t)stream;
+#define TQK_ROUTE(TA, TW) \
+    moe_route_grouped_kernel<TA, TW><<<n_tokens, MOE_ROUTE_WAVES * TQK_WAVE, 0, s>>>((const TA*)x, (const TW*)w_router, n_experts, hidden, top, correction, n_groups, keep, floor, idx, weight)
+    if (act_dtype == TQK_F32 && w_dtype == TQK_F32) TQK_ROUTE(float, float);
+    else if (act_dtype == TQK_F32 && w_dtype == TQK_BF16) TQK_ROUTE(float, bf16_t);
+    else if (act_dtype == TQK_BF16 && w_dtype == TQK_F32) TQK_ROUTE(bf16_t, float);
+    else if (act_dtype == TQK_BF16 && w_dtype == TQK_BF16) TQK_ROUTE(bf16_t, bf16_t);
+    else return tqk_fail("tqk_moe_route_grouped: unknown dtypes %d, %d", act_dtype, w_dtype);
+#undef TQK_ROUTE
+    return tqk_check_launch("tqk_moe_route_grouped");
 }
 
 extern "C" int tqk_moe_group(const int32_t* idx, int n_tokens, int top, int n_experts, int tile_m, int32_t* pair_pos, int32_t* sorted_tok,
@@ -340,16 +463,17 @@ extern "C" int tqk_moe_product(const void* x, int act_dtype, const int32_t* x_ro
     return tqk_fail("tqk_moe_product: unknown dtypes %d, %d", act_dtype, w_dtype);
 }
 
-extern "C" int tqk_moe_combine(const void* y, int act_dtype, const int32_t* pair_pos, const float* weight, int top, const void* shared,
-                               const float* shared_scale, void* out, int n_tokens, int hidden, void* stream) {
+extern "C" int tqk_moe_combine(const void* y, int act_dtype, const int32_t* pair_pos, const float* weight, int top, const void* x, const void* shared,
+                               const float* shared_scale, const void* beside, float scale, void* out, int n_tokens, int hidden, void* stream) {
     TQK_REQUIRE(y && pair_pos && weight && out, "tqk_moe_combine: null pointer");
     TQK_REQUIRE(top > 0 && top <= MOE_MAX_EXPERTS && hidden > 0 && n_tokens >= 0, "tqk_moe_combine: bad sizes");
     if (n_tokens == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
-    if (act_dtype == TQK_F32)
-        moe_combine_kernel<float><<<n_tokens, 256, 0, s>>>((const float*)y, pair_pos, weight, top, (const float*)shared, shared_scale, (float*)out, hidden);
-    else if (act_dtype == TQK_BF16)
-        moe_combine_kernel<bf16_t><<<n_tokens, 256, 0, s>>>((const bf16_t*)y, pair_pos, weight, top, (const bf16_t*)shared, shared_scale, (bf16_t*)out, hidden);
+#define TQK_COMBINE(TA) \
+    moe_combine_kernel<TA><<<n_tokens, 256, 0, s>>>((const TA*)y, pair_pos, weight, top, (const TA*)x, (const TA*)shared, shared_scale, (const TA*)beside, scale, (TA*)out, hidden)
+    if (act_dtype == TQK_F32) TQK_COMBINE(float);
+    else if (act_dtype == TQK_BF16) TQK_COMBINE(bf16_t);
     else return tqk_fail("tqk_moe_combine: unknown dtype %d", act_dtype);
+#undef TQK_COMBINE
     return tqk_check_launch("tqk_moe_combine");
 }

@@ -139,6 +139,13 @@ __global__ void unary_act_vec_kernel(const uint4* __restrict__ x, uint4* __restr
     out[i] = make_uint4(o[0], o[1], o[2], o[3]);
 }
 
+// out = scale (a + b), b may be null: what two parts that ran side by side leave for the stream
+template <typename TA>
+__global__ void scaled_sum_kernel(const TA* __restrict__ a, const TA* __restrict__ b, float scale, TA* __restrict__ out, long long n) {
+    const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) out[i] = from_float<TA>(scale * (to_float(a[i]) + (b ? to_float(b[i]) : 0.f)));
+}
+
 // out[t] = sigmoid(x[t] . w), a wave per token
 template <typename TA, typename TW>
 __global__ __launch_bounds__(256)
@@ -215,6 +222,18 @@ extern "C" int tqk_unary_act(const void* x, void* out, int act_dtype, long long 
     else if (act_dtype == TQK_BF16) unary_act_kernel<bf16_t><<<(unsigned)blocks, 256, 0, s>>>((const bf16_t*)x, (bf16_t*)out, n, kind, limit, alpha);
     else return tqk_fail("tqk_unary_act: unknown dtype %d", act_dtype);
     return tqk_check_launch("tqk_unary_act");
+}
+
+extern "C" int tqk_scaled_sum(const void* a, const void* b, int act_dtype, float scale, void* out, long long n, void* stream) {
+    TQK_REQUIRE(a && out && n >= 0, "tqk_scaled_sum: null pointer");
+    if (n == 0) return 0;
+    const long long blocks = (n + 255) / 256;
+    TQK_REQUIRE(blocks <= 0x7fffffff, "tqk_scaled_sum: too many elements");
+    hipStream_t s = (hipStream_t)stream;
+    if (act_dtype == TQK_F32) scaled_sum_kernel<float><<<(unsigned)blocks, 256, 0, s>>>((const float*)a, (const float*)b, scale, (float*)out, n);
+    else if (act_dtype == TQK_BF16) scaled_sum_kernel<bf16_t><<<(unsigned)blocks, 256, 0, s>>>((const bf16_t*)a, (const bf16_t*)b, scale, (bf16_t*)out, n);
+    else return tqk_fail("tqk_scaled_sum: unknown dtype %d", act_dtype);
+    return tqk_check_launch("tqk_scaled_sum");
 }
 
 extern "C" int tqk_row_gate(const void* x, int act_dtype, const void* w, int w_dtype, float* out, int n_tokens, int hidden, void* stream) {

@@ -250,8 +250,11 @@ int tqk_latent_values(const float* o, const void* w_uv, int w_dtype, const float
  * y [pairs, N]; gated 0: the product alone, 1: gate and up, 2: one product [N, K] with the gate's function of it alone (u = 1:
  * relu2 gives max(z, 0)^2).  tqk_moe_route with renormalize: the chosen weights are divided by their sum (the softmax over
  * the chosen logits alone); with gate_w [hidden] (of the router's type, or null) it also writes gate_out[t] = sigmoid(x[t] . gate_w).
- * tqk_moe_combine: out[t] = sum_k weight[t, k] y[pair_pos[t, k]] + shared_scale[t] * shared[t]
- * (shared may be null; shared_scale null: 1).  tqk_moe_route's mode: bit 1 is that renormalising, bit 2 makes the scores
+ * tqk_moe_route_grouped: s = softmax(W_r x), the `top` with the largest s + correction (correction null: 0) among the `keep` of n_groups groups
+ * of neighbours whose largest s + correction is largest; weight = s / (the chosen s' sum + floor).  tqk_moe_group: a choice idx >= n_experts (an
+ * expert that gives back its input) gets no row, pair_pos -1.
+ * tqk_moe_combine: out[t] = scale (sum_k weight[t, k] y[pair_pos[t, k]] + shared_scale[t] * shared[t] + beside[t])
+ * (shared, beside may be null; shared_scale null: 1), x[t] in place of a row where pair_pos is -1.  tqk_moe_route's mode: bit 1 is that renormalising, bit 2 makes the scores
  * sigmoid(z) of every expert on its own instead of the softmax.  tqk_moe_scale_rows: rows[pair_pos[p]] = weight[p] * x[p / top]
  * and unit[p] = 1, for experts whose input carries the weight. */
 int tqk_moe_scale_rows(const void* x, int act_dtype, const int32_t* pair_pos, const float* weight, int top, void* rows, float* unit,
@@ -261,6 +264,8 @@ int tqk_moe_tile_rows(void);
 int tqk_moe_max_tiles(int n_pairs, int n_experts, int tile_m);
 int tqk_moe_route(const void* x, int act_dtype, const void* w_router, int w_dtype, int n_experts, int hidden, int top, float scale,
                   int mode, int32_t* idx, float* weight, const void* gate_w, float* gate_out, int n_tokens, void* stream);
+int tqk_moe_route_grouped(const void* x, int act_dtype, const void* w_router, int w_dtype, int n_experts, int hidden, int top, const float* correction,
+                          int n_groups, int keep, float floor, int32_t* idx, float* weight, int n_tokens, void* stream);
 int tqk_moe_group(const int32_t* idx, int n_tokens, int top, int n_experts, int tile_m, int32_t* pair_pos, int32_t* sorted_tok,
                   int32_t* tile_expert, int32_t* tile_row0, int32_t* tile_rows, int32_t* n_tiles, void* stream);
 int tqk_moe_product(const void* x, int act_dtype, const int32_t* x_rows, const void* w, int w_dtype, long long expert_stride, void* y,
@@ -278,8 +283,8 @@ int tqk_head_product(const void* x, int x_f32, long long x_row_stride, long long
                      long long y_row_stride, long long y_head_stride, const float* scale, const void* gate, int gate_f32,
                      long long gate_stride, int n_tokens, int n_heads, int N, int K,
                      void* stream);
-int tqk_moe_combine(const void* y, int act_dtype, const int32_t* pair_pos, const float* weight, int top, const void* shared,
-                    const float* shared_scale, void* out, int n_tokens, int hidden, void* stream);
+int tqk_moe_combine(const void* y, int act_dtype, const int32_t* pair_pos, const float* weight, int top, const void* x, const void* shared,
+                    const float* shared_scale, const void* beside, float scale, void* out, int n_tokens, int hidden, void* stream);
 
 /* Around the residual stream (stream_ops.hip).  tqk_pair_embed: h[t] += table[(prev * mul_prev + token * mul_cur) mod buckets],
  * table [buckets + 1, hidden], the last row for a sequence's first token; prev is the token before it in the step or, for the
@@ -297,6 +302,8 @@ int tqk_remember_tokens(const int32_t* tokens, const int32_t* cu, const int32_t*
 int tqk_norm_add(float* h, const void* y, int act_dtype, const void* weight, int weight_dtype, float eps, void* copy, int n_tokens,
                  int hidden, void* stream);
 int tqk_unary_act(const void* x, void* out, int act_dtype, long long n, int kind, float limit, float alpha, void* stream);
+/* out = scale (a + b) over n elements of the activation type (b may be null) */
+int tqk_scaled_sum(const void* a, const void* b, int act_dtype, float scale, void* out, long long n, void* stream);
 int tqk_row_gate(const void* x, int act_dtype, const void* w, int w_dtype, float* out, int n_tokens, int hidden, void* stream);
 
 /* Attention with keys of key_dim and values of value_dim per head (attention_masked.hip).  tqk_normed_rope_store: a row of qkv is
@@ -309,6 +316,7 @@ int tqk_row_gate(const void* x, int act_dtype, const void* w, int w_dtype, float
  * tqk_attention_masked: a query at position i sees j <= i with i - j < window or j < keep_first (window 0: all), and,
  * with chunk > 0, floor(j / chunk) = floor(i / chunk); scores
  * scale q.k, then cap tanh(s / cap) if cap > 0; sink [heads] (or null) adds exp(sink_h) to the softmax's denominator.
+ * head_scale [rows, heads] float32 (or null) multiplies the heads' outputs.
  * One wave per (token, head), float32 throughout; out [tokens, heads * value_dim]. */
 int tqk_normed_rope_store(const void* qkv, int act_dtype, const void* bias, const void* q_norm_w, const void* k_norm_w, int w_dtype, float eps,
                           const float* cos_table, const float* sin_table, int rot_dim, int style, int max_positions, const void* mix,
@@ -318,8 +326,8 @@ int tqk_normed_rope_store(const void* qkv, int act_dtype, const void* bias, cons
 int tqk_attention_masked_max_dim(void);
 int tqk_attention_masked(const void* q, const void* keys, const void* values, int act_dtype, const int32_t* tok_seq,
                          const int32_t* tok_pos, const int32_t* page_table, int table_width, int n_seqs, int n_pages, int window,
-                         int chunk, int keep_first, float scale, float cap, const void* sink, int sink_dtype, void* out, int n_tokens,
-                         int n_heads, int n_kv_heads, int key_dim, int value_dim, void* stream);
+                         int chunk, int keep_first, float scale, float cap, const void* sink, int sink_dtype, const float* head_scale, void* out,
+                         int n_tokens, int n_heads, int n_kv_heads, int key_dim, int value_dim, void* stream);
 
 /* The same on the matrix cores (attention_masked_mfma.hip), bfloat16, key_dim a multiple of 8, both sizes up to 256.  n_tiles > 0:
  * tiles of up to tile_queries = tqk_attention_masked_mfma_tile(...) consecutive queries of one sequence (lists on the device; tok_pos and q by packed
@@ -330,8 +338,8 @@ int tqk_attention_masked_mfma_supported(int key_dim, int value_dim);
 int tqk_attention_masked_mfma_tile(int n_tokens, int n_heads, int n_kv_heads, int key_dim, int value_dim);
 int tqk_attention_masked_mfma(const void* q, const void* keys, const void* values, const int32_t* tok_pos, const int32_t* page_table,
                               int table_width, int n_pages, int window, int chunk, int keep_first, float scale, float cap, const void* sink,
-                              int sink_dtype, const int32_t* tile_seq, const int32_t* tile_tok0, const int32_t* tile_count, int n_tiles,
-                              int tile_queries, int n_rows, int n_parts, void* part_out, void* part_ml, void* out, int n_heads, int n_kv_heads,
+                              int sink_dtype, const float* head_scale, const int32_t* tile_seq, const int32_t* tile_tok0, const int32_t* tile_count,
+                              int n_tiles, int tile_queries, int n_rows, int n_parts, void* part_out, void* part_ml, void* out, int n_heads, int n_kv_heads,
                               int key_dim, int value_dim, void* stream);
 
 /* Bias, rotation, then a norm without a weight (attention_masked.hip): rows of qkv are [heads * key_dim | kv heads * key_dim | kv heads *
@@ -341,6 +349,17 @@ int tqk_rope_norm_store(const void* qkv, int act_dtype, const void* bias, int bi
                         int rot_dim, int style, int max_positions, int normed, float eps, const int32_t* tok_seq, const int32_t* tok_pos,
                         const int32_t* page_table, int table_width, void* keys, void* values, void* q_out, int n_tokens, int n_heads,
                         int n_kv_heads, int key_dim, int value_dim, int write_kv, void* stream);
+
+/* Bias, a norm over the whole projection, rotation, a gate per head (attention_masked.hip).  rows: [heads * key_dim | kv heads * key_dim | kv
+ * heads * value_dim], or, with kv 0, [heads * key_dim] alone, rows row_stride apart; bias (float32, or null) has that layout; all of q and all of k
+ * are divided by the root mean square of the whole projection (eps inside the root) and multiplied by q_norm_w [heads * key_dim] and
+ * k_norm_w [kv heads * key_dim] (float32; q_norm_w null: no norm), then turned as by tqk_normed_rope_store.  gate_out [tokens, heads] (or null):
+ * the sigmoid of the row's elements gate_at .. gate_at + heads.  q goes to q_out, keys and values (kv != 0) into the pages. */
+int tqk_projection_store(const void* rows, int act_dtype, long long row_stride, const float* bias, const float* q_norm_w, const float* k_norm_w,
+                         float eps, const float* cos_table, const float* sin_table, int rot_dim, int style, int max_positions,
+                         const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* page_table, int table_width, void* keys, void* values,
+                         void* q_out, float* gate_out, long long gate_at, int n_tokens, int n_heads, int n_kv_heads, int key_dim, int value_dim,
+                         int kv, void* stream);
 
 /* Mixers with a fixed-size state (recurrent.hip).  A step is a packed batch: token t belongs to sequence tok_seq[t] of the step at position
  * tok_pos[t]; sequence s brings seq_new[s] tokens from packed row cu[s] on, had seq_start[s] positions before, and its state is row seq_slot[s]
@@ -460,7 +479,8 @@ int tqk_shift_remember(const float* n, float* state, long long state_stride, con
 /* Linear attention with a decaying state (linear_attention.hip): per head S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, the state
  * of a slot [heads][d][dv] float32, head_stride elements from head to head.  q, k, v: rows `stride` elements apart, heads side by side.  The decay: z [tokens, heads * d] float32
  * with z_bias gives a = sigmoid(z + bias)^inv_tau per key channel; z null: head_decay[h] for the whole head, or, with
- * log_decay [tokens, heads], its exponential (k then times exp(log_in), the output times out_scale, both [tokens, heads] or null).  q and k are turned by
+ * log_decay [tokens, heads], its exponential (k then times exp(log_in), the output times out_scale, both [tokens, heads] or null), or decay [tokens, heads * d] as it is.
+ * bonus [heads, d] (or null): o_t = S_(t-1)^T q_t + (sum_i bonus_i k_i q_i) v_t.  q and k are turned by
  * tok_pos through cos, sin [max_pos, rot_dim / 2] (style 1: halves, 2: pairs; cos null: not turned) and multiplied by q_scale, k_scale.
  * mode 0: every sequence's tokens in order from its state row, which is written back (cu, seq_new, seq_slot; n_items sequences).
  * mode 1 and 2: chunks as tqk_ssm_chunks takes them (chunk_row0, chunk_count; n_items chunks), between them tqk_chunk_carry with
@@ -470,7 +490,7 @@ int tqk_shift_remember(const float* n, float* state, long long state_stride, con
 int tqk_linear_attention_max_dim(void);
 int tqk_linear_attention(const void* q, const void* k, const void* v, int act_dtype, long long stride, const float* z, long long z_stride,
                          const float* z_bias, float inv_tau, const float* head_decay, const float* log_decay, const float* log_in,
-                         const float* out_scale, float q_scale, float k_scale, const float* cos,
+                         const float* out_scale, const float* decay, const float* bonus, float q_scale, float k_scale, const float* cos,
                          const float* sin, int rot_dim, int style, int max_pos, const int32_t* tok_pos, float* state, long long state_stride,
                          const int32_t* cu, const int32_t* seq_new, const int32_t* seq_slot, const int32_t* chunk_row0,
                          const int32_t* chunk_count, float* chunk_state, float* chunk_decay, float* out, int mode, int n_items, int heads,
@@ -478,6 +498,19 @@ int tqk_linear_attention(const void* q, const void* k, const void* v, int act_dt
 int tqk_head_norm_gate(const float* o, const float* weight, int weight_stride, float eps, const void* gate, int gate_dtype, long long gate_stride,
                        int sigmoid, void* out,
                        int out_dtype, int n_tokens, int heads, int dv, void* stream);
+
+/* What time mixing puts in front of its recurrence (time_mixing.hip).  tqk_token_mixes: out[s][t] = x[t] + (x[t - 1] - x[t]) mu[s] for n_mixes
+ * rows mu [n_mixes, width] float32, out [n_mixes][tokens][width] in x's type; the sequence's state row stands for x[t - 1] at the first token a
+ * step brings of it; remember != 0 (steps of one token a sequence) also leaves x[t] there.  tqk_rows_remember: the state of every sequence
+ * becomes x of the last token the step brings of it.  tqk_low_rank_decay: decay[t, c] = exp(-exp(sum_r w2[r, c] tanh(low[t, r]) + bias[c])), all
+ * float32, w2 [rank, channels]. */
+int tqk_token_mixes(const void* x, int dtype, const float* mu, int n_mixes, float* state, long long state_stride, const int32_t* tok_seq,
+                    const int32_t* tok_pos, const int32_t* seq_start, const int32_t* seq_slot, void* out, int n_tokens, int width, int remember,
+                    void* stream);
+int tqk_rows_remember(const void* x, int dtype, float* state, long long state_stride, const int32_t* cu, const int32_t* seq_new,
+                      const int32_t* seq_slot, int n_seqs, int width, void* stream);
+int tqk_low_rank_max(void);
+int tqk_low_rank_decay(const float* low, const float* w2, const float* bias, float* decay, int n_tokens, int rank, int channels, void* stream);
 
 /* The gates of a matrix memory (mlstm.hip): z [tokens] rows z_stride apart, [heads] input gates' products then [heads] forget gates', bias
  * [2 heads].  a = cap tanh((z_i + b) / cap), f = log sigmoid(cap tanh((z_f + b) / cap)); in the tokens' order m_t = max(f_t + m_(t-1), a_t), kappa
