@@ -25,6 +25,8 @@ Piditar shape of equal size.  `python bench.py --recurrent` does it for the
 Piditar design (layers of attention, of a real-gated linear recurrent unit and of a selective state-space mixer, each with a dense
 feed-forward).  `python bench.py --matrix-memory` does it for the Rasodra design (a matrix memory, latent attention with a sink and an
 element gate, chunked attention whose values are its keys, norms on both sides of every part) beside a Nikasun shape of equal size.
+`python bench.py --time-mixing` does it for the Kezasun design (time mixing, windowed attention with a norm over the projection and a gate per head,
+experts in groups) beside a Povipel shape of equal size.
 """
 import argparse
 import gc
@@ -56,6 +58,7 @@ def main():
     ap.add_argument("--recurrent", action="store_true", help="measure the Piditar design beside a Qwen2 shape of equal size instead of the default workload")
     ap.add_argument("--streams", action="store_true", help="measure the Povipel design beside a Piditar shape of equal size instead of the default workload")
     ap.add_argument("--matrix-memory", action="store_true", help="measure the Rasodra design beside a Nikasun shape of equal size instead of the default workload")
+    ap.add_argument("--time-mixing", action="store_true", help="measure the Kezasun design beside a Povipel shape of equal size instead of the default workload")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this library runs on one GPU; --gpus %d is not supported" % args.gpus)
@@ -171,6 +174,9 @@ def main():
 
     if args.matrix_memory:
         return design_comparison("rasodra", memory_shapes, args, torch, Model, Engine, note, timed_prefill, decode, random_prompts, release, beside="nikasun")
+
+    if args.time_mixing:
+        return design_comparison("kezasun", mixing_shapes, args, torch, Model, Engine, note, timed_prefill, decode, random_prompts, release, beside="povipel")
 
     # -- the headline shape -------------------------------------------------------------------------
     raw = dict(catalog.find(args.shape))
@@ -420,6 +426,33 @@ def memory_shapes(width, layers=4):
     return rasodra, nikasun, {"width": width, "layers": layers, "memory_heads": memory["heads"], "memory_dim": 128, "memory_vdim": 256, "heads": heads,
                               "kv_heads": kv_heads, "head_dim": dim, "kv_rank": 512, "rot_dim": 64, "chunk": 1024, "ff": ff, "beside_ff": gated["ff"],
                               "beside_q_rank": other["q_rank"]}
+
+
+def mixing_shapes(width, layers=4):
+    """A Kezasun configuration (attention, time mixing, attention on the first one's keys and values, time mixing; experts in every layer) and a
+    Povipel one of one copy of the stream (attention over a window and pooled blocks beside a gated linear attention, and retention, in turn;
+    experts in every layer) of the same width, depth, heads and experts."""
+    heads, dim = width // 128, 128
+    kv_heads = max(1, heads // 4)
+    rot = {"base": 10000.0, "dims": 64}
+    mixing = {"heads": width // 64, "dim": 64}
+    attention = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": 1024},
+                 "rot": dict(rot, scaling={"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192})}
+    moe = {"kind": "moe", "expert": {"ff": 3 * width // 4}, "router": {"experts": 30, "top": 4, "identity": 2, "groups": {"count": 4, "keep": 2}}}
+    kinds = [("attention", attention), ("wkv", mixing), ("attention", dict(attention, kv_from=0)), ("wkv", mixing)]
+    lay = [{"type": kinds[l % 4][0], "mixer": kinds[l % 4][1], "mlp": moe} for l in range(layers)]
+    kezasun = {"architecture": "Kezasun", "vocab": 32000, "width": width, "norm": {"eps": 1e-5}, "residual_mult": 0.7, "layers": lay, "max_positions": 8192}
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": 1024, "pool": 16}, "rot": rot}
+    right = {"heads": width // 256, "dim": 128, "vdim": 256, "tau": 16.0}
+    retention = {"heads": width // 64, "dim": 64, "vdim": 64, "rot": {"base": 10000.0, "dims": 64},
+                 "decay": [1.0 - 2.0 ** (-5.0 - 3.0 * h / max(1, width // 64 - 1)) for h in range(width // 64)]}
+    other = {"kind": "moe", "expert": {"ff": 3 * width // 4}, "router": {"experts": 32, "top": 4}}
+    kinds = [("parallel", {"left": left, "right": right}), ("retention", retention)]
+    povipel = {"architecture": "Povipel", "vocab": 32000, "width": width, "embedding": {"scale": width ** 0.5}, "norm": {"eps": 1e-5}, "max_positions": 8192,
+               "layers": [{"type": kinds[l % 2][0], "mixer": kinds[l % 2][1], "mlp": other} for l in range(layers)]}
+    return kezasun, povipel, {"width": width, "layers": layers, "mixing_heads": mixing["heads"], "mixing_dim": 64, "heads": heads, "kv_heads": kv_heads, "head_dim": dim,
+                              "window": 1024, "experts": 30, "identity_experts": 2, "top": 4, "groups": 4, "groups_kept": 2, "expert_ff": moe["expert"]["ff"],
+                              "beside_linear_heads": right["heads"], "beside_linear_dim": 128, "beside_linear_vdim": 256, "beside_retention_heads": retention["heads"]}
 
 
 def design_comparison(design, shapes, args, torch, Model, Engine, note, timed_prefill, decode, random_prompts, release, beside="qwen2"):

@@ -37,7 +37,7 @@ def test_host_library_is_clean_under_address_and_ub_sanitizers(tmp_path):
     os.environ.setdefault("CXX", cxx)
     build.compile_host(lib, extra_flags=["-O1", "-g", "-fsanitize=address,undefined", "-fno-sanitize-recover=undefined", "-fno-omit-frame-pointer"])
     tests = [os.path.join(ROOT, "tests", n) for n in ("test_cache.py", "test_step_plan.py", "test_generate_loop.py", "test_config.py",
-                                                      "test_weights.py", "test_dry_run.py", "test_sizudra_config.py", "test_rasodra_config.py")]
+                                                      "test_weights.py", "test_dry_run.py", "test_sizudra_config.py", "test_rasodra_config.py", "test_kezasun_config.py")]
     env = dict(os.environ, LD_PRELOAD=" ".join(runtimes), ASAN_OPTIONS="detect_leaks=0:abort_on_error=1",
                TQ_KERNEL_LIBRARY=build.find_library(), TQ_ENGINE_LIBRARY=lib)
     child = subprocess.run([sys.executable, "-c", CHILD.format(root=ROOT, lib=lib, tests=tests)], capture_output=True, text=True, env=env,

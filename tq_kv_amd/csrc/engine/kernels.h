@@ -123,7 +123,7 @@ TQ_QUERY(int, linear_attention_max_dim);
 TQ_KERNEL(linear_attention, cptr, cptr, cptr, int, long long, cf32, long long, cf32, float, cf32, cf32, cf32, cf32, cf32, cf32, float, float, cf32, cf32, int,
           int, int, ci32, float*, long long, ci32, ci32, ci32, ci32, ci32, float*, float*, float*, int, int, int, int, int, long long, void*);
 TQ_KERNEL(head_norm_gate, cf32, cf32, int, float, cptr, int, long long, int, void*, int, int, int, int, void*);
-TQ_KERNEL(token_mixes, cptr, int, cf32, int, float*, long long, ci32, ci32, ci32, ci32, void*, int, int, int, void*);
+TQ_KERNEL(token_mixes, cptr, int, cf32, int, float*, long long, ci32, ci32, ci32, ci32, void*, long long, int, int, int, void*);
 TQ_KERNEL(rows_remember, cptr, int, float*, long long, ci32, ci32, ci32, int, int, void*);
 TQ_QUERY(int, low_rank_max);
 TQ_KERNEL(low_rank_decay, cf32, cf32, cf32, float*, int, int, int, void*);

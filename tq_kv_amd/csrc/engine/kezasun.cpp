@@ -24,7 +24,7 @@ namespace tq {
 namespace {
 
 const long long DEFAULT_MAX_POSITIONS = 131072;
-const long long DEFAULT_DECAY_RANK = 16;        // what random weights get: the checkpoint's tensors give the rank
+const long long DEFAULT_DECAY_RANK = 64;        // what random weights get: the checkpoint's tensors give the rank
 const double SINK_SCORE = 0.0;                  // the denominator's extra exp(0): fixed by the design
 const double WEIGHT_FLOOR = 1e-20;              // added to the sum the chosen experts' scores are divided by
 

@@ -139,17 +139,16 @@ public:
         const long long row = entry.state.cols();
         float* state = (float*)entry.state.data + entry.state_offset;
         float* last = state + last_at();
-        Tensor mixes = c.alloc(dtype, {N_MIXES * n, hidden_});
-        K::token_mixes(x.x.data, dtype, (const float*)mu_->t.data, N_MIXES, last, row, c.dev.tok_seq, c.dev.tok_pos, c.dev.seq_start, c.dev.seq_slot, mixes.data, (int)n,
+        // (the mixes one behind the other, each beginning at a multiple of 16 bytes)
+        const int64_t mix_stride = (n * hidden_ + 7) / 8 * 8;
+        const Tensor mixes = c.alloc(dtype, {N_MIXES, mix_stride});
+        auto mix = [&](int i) { return Tensor((char*)mixes.data + (size_t)(i * mix_stride) * dtype_size(dtype), dtype, {n, hidden_}); };
+        K::token_mixes(x.x.data, dtype, (const float*)mu_->t.data, N_MIXES, last, row, c.dev.tok_seq, c.dev.tok_pos, c.dev.seq_start, c.dev.seq_slot, mixes.data, mix_stride, (int)n,
                        (int)hidden_, c.all_decode ? 1 : 0, c.stream);
         if (!c.all_decode) K::rows_remember(x.x.data, dtype, last, row, c.dev.cu, c.dev.seq_new, c.dev.seq_slot, c.n_seqs, (int)hidden_, c.stream);
-        Tensor in = c.alloc(dtype, {4 * n, hd});                             // r, k, v, g one behind the other
-        Tensor part[4];
-        for (int i = 0; i < 4; ++i) {
-            part[i] = in.slice(i * n, (i + 1) * n);
-            linear(c, mixes.slice(i * n, (i + 1) * n), w_in_[i], nullptr, dtype, false, &part[i]);
-        }
-        const Tensor low = linear(c, mixes.slice(4 * n, 5 * n), w_w1_, nullptr, F32).t;
+        Tensor part[4];                                                      // r, k, v, g
+        for (int i = 0; i < 4; ++i) part[i] = linear(c, mix(i), w_in_[i], nullptr, dtype).t;
+        const Tensor low = linear(c, mix(4), w_w1_, nullptr, F32).t;
         Tensor decay = c.alloc(F32, {n, hd});
         K::low_rank_decay((const float*)low.data, (const float*)w2_->t.data, (const float*)w0_->t.data, (float*)decay.data, (int)n, (int)rank_, (int)hd, c.stream);
         Tensor o = c.alloc(F32, {n, heads_, d_});

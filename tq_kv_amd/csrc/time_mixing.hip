@@ -42,7 +42,7 @@ template <typename T, int VEC>
 __global__ __launch_bounds__(256)
 void token_mixes_kernel(const T* __restrict__ x, const float* __restrict__ mu, int n_mixes, float* __restrict__ state, long long state_stride,
                         const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ seq_start,
-                        const int32_t* __restrict__ seq_slot, T* __restrict__ out, int n_tokens, int W, int remember) {
+                        const int32_t* __restrict__ seq_slot, T* __restrict__ out, long long mix_stride, int W, int remember) {
     const size_t t = blockIdx.x;
     const int e = (blockIdx.y * blockDim.x + threadIdx.x) * VEC;
     if (e >= W) return;
@@ -67,7 +67,7 @@ void token_mixes_kernel(const T* __restrict__ x, const float* __restrict__ mu, i
         load_piece<float, VEC>(mu + (size_t)s * W + e, m);
 #pragma unroll
         for (int j = 0; j < VEC; ++j) v[j] = fmaf(prev[j], m[j], cur[j]);
-        store_piece<T, VEC>(out + ((size_t)s * n_tokens + t) * W + e, v);
+        store_piece<T, VEC>(out + (size_t)s * mix_stride + t * W + e, v);
     }
 }
 
@@ -117,18 +117,19 @@ void low_rank_decay_kernel(const float* __restrict__ low, const float* __restric
 }
 
 extern "C" int tqk_token_mixes(const void* x, int dtype, const float* mu, int n_mixes, float* state, long long state_stride, const int32_t* tok_seq,
-                               const int32_t* tok_pos, const int32_t* seq_start, const int32_t* seq_slot, void* out, int n_tokens, int width,
-                               int remember, void* stream) {
+                               const int32_t* tok_pos, const int32_t* seq_start, const int32_t* seq_slot, void* out, long long mix_stride, int n_tokens,
+                               int width, int remember, void* stream) {
     TQK_REQUIRE(x && mu && state && tok_seq && tok_pos && seq_start && seq_slot && out, "tqk_token_mixes: null pointer");
     TQK_REQUIRE(n_tokens >= 0 && width > 0 && state_stride >= width, "tqk_token_mixes: bad sizes");
+    TQK_REQUIRE(mix_stride >= (long long)n_tokens * width, "tqk_token_mixes: the mixes overlap");
     TQK_REQUIRE(n_mixes > 0 && n_mixes <= TM_MAX_MIXES, "tqk_token_mixes: %d mixes, the kernel takes up to %d", n_mixes, TM_MAX_MIXES);
     if (n_tokens == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
-    const bool vec = width % 8 == 0 && state_stride % 4 == 0 && (((uintptr_t)x | (uintptr_t)out | (uintptr_t)mu | (uintptr_t)state) & 15) == 0;
+    const bool vec = width % 8 == 0 && mix_stride % 8 == 0 && state_stride % 4 == 0 && (((uintptr_t)x | (uintptr_t)out | (uintptr_t)mu | (uintptr_t)state) & 15) == 0;
     const int pieces = vec ? width / 8 : width;
     const int threads = pieces >= 256 ? 256 : (pieces + TQK_WAVE - 1) / TQK_WAVE * TQK_WAVE;
     dim3 grid(n_tokens, (pieces + threads - 1) / threads);
-#define TQK_TM(T, VEC) token_mixes_kernel<T, VEC><<<grid, threads, 0, s>>>((const T*)x, mu, n_mixes, state, state_stride, tok_seq, tok_pos, seq_start, seq_slot, (T*)out, n_tokens, width, remember)
+#define TQK_TM(T, VEC) token_mixes_kernel<T, VEC><<<grid, threads, 0, s>>>((const T*)x, mu, n_mixes, state, state_stride, tok_seq, tok_pos, seq_start, seq_slot, (T*)out, mix_stride, width, remember)
     if (dtype == TQK_F32) { if (vec) TQK_TM(float, 8); else TQK_TM(float, 1); }
     else if (dtype == TQK_BF16) { if (vec) TQK_TM(bf16_t, 8); else TQK_TM(bf16_t, 1); }
     else return tqk_fail("tqk_token_mixes: unknown dtype %d", dtype);

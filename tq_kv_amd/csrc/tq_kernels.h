@@ -500,13 +500,13 @@ int tqk_head_norm_gate(const float* o, const float* weight, int weight_stride, f
                        int out_dtype, int n_tokens, int heads, int dv, void* stream);
 
 /* What time mixing puts in front of its recurrence (time_mixing.hip).  tqk_token_mixes: out[s][t] = x[t] + (x[t - 1] - x[t]) mu[s] for n_mixes
- * rows mu [n_mixes, width] float32, out [n_mixes][tokens][width] in x's type; the sequence's state row stands for x[t - 1] at the first token a
+ * rows mu [n_mixes, width] float32, out [n_mixes][tokens][width] in x's type, mix_stride elements from mix to mix; the sequence's state row stands for x[t - 1] at the first token a
  * step brings of it; remember != 0 (steps of one token a sequence) also leaves x[t] there.  tqk_rows_remember: the state of every sequence
  * becomes x of the last token the step brings of it.  tqk_low_rank_decay: decay[t, c] = exp(-exp(sum_r w2[r, c] tanh(low[t, r]) + bias[c])), all
  * float32, w2 [rank, channels]. */
 int tqk_token_mixes(const void* x, int dtype, const float* mu, int n_mixes, float* state, long long state_stride, const int32_t* tok_seq,
-                    const int32_t* tok_pos, const int32_t* seq_start, const int32_t* seq_slot, void* out, int n_tokens, int width, int remember,
-                    void* stream);
+                    const int32_t* tok_pos, const int32_t* seq_start, const int32_t* seq_slot, void* out, long long mix_stride, int n_tokens, int width,
+                    int remember, void* stream);
 int tqk_rows_remember(const void* x, int dtype, float* state, long long state_stride, const int32_t* cu, const int32_t* seq_new,
                       const int32_t* seq_slot, int n_seqs, int width, void* stream);
 int tqk_low_rank_max(void);
