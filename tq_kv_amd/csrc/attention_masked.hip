@@ -449,9 +449,9 @@ template <> struct Piece<bf16_t, 8> {
 };
 
 template <typename TA, int VEC>
-__global__ __launch_bounds__(256)
+__global__ __launch_bounds__(1024)
 void projection_store_kernel(const ProjectionArgs a) {
-    __shared__ float scratch[4];
+    __shared__ float scratch[16];
     const int t = blockIdx.x;
     const int H = a.n_heads, G = a.n_kv_heads, dk = a.dk, dv = a.dv;
     const int nq = H * dk, nk = a.kv ? G * dk : 0;
@@ -716,20 +716,25 @@ extern "C" int tqk_projection_store(const void* rows, int act_dtype, long long r
     hipStream_t s = (hipStream_t)stream;
     ProjectionArgs a = {rows, row_stride, bias, q_norm_w, k_norm_w, eps, cos_table, sin_table, rot_dim, style, max_positions, tok_seq, tok_pos, page_table, table_width,
                         keys, values, q_out, gate_out, gate_at, n_heads, n_kv_heads, key_dim, value_dim, kv, 1};
+    // a thread a piece of the row, as far as blocks go (from the sizes alone: a row's sums have one order)
+    const auto threads_for = [&](int vec) {
+        const long long pieces = (nq + nk + vec - 1) / vec;
+        return (unsigned)(pieces >= 1024 ? 1024 : (pieces + TQK_WAVE - 1) / TQK_WAVE * TQK_WAVE);
+    };
     const bool aligned = row_stride % 8 == 0 && (((uintptr_t)rows | (uintptr_t)keys | (uintptr_t)q_out) & 15) == 0;
     if (act_dtype == TQK_BF16 && key_dim % 8 == 0 && (rot_dim == 0 || style == 2 || rot_dim % 16 == 0) && aligned) {
         // steps of many tokens: values with the lanes along the tokens
         const bool apart = kv && n_tokens > 64 && value_dim % 8 == 0;
         a.store_values = apart ? 0 : 1;
-        projection_store_kernel<bf16_t, 8><<<n_tokens, 256, 0, s>>>(a);
+        projection_store_kernel<bf16_t, 8><<<n_tokens, threads_for(8), 0, s>>>(a);
         if (apart) {
             const long long v_blocks = (long long)((n_tokens + TQK_WAVE - 1) / TQK_WAVE) * n_kv_heads;
             TQK_REQUIRE(v_blocks <= 0x7fffffff, "tqk_projection_store: too many tokens");
             biased_values_store_vec_kernel<float><<<(unsigned)v_blocks, 256, 0, s>>>((const bf16_t*)rows, bias, tok_seq, tok_pos, page_table, table_width, (bf16_t*)values,
                                                                                      n_tokens, n_kv_heads, value_dim, (size_t)row_stride, (size_t)(nq + nk));
         }
-    } else if (act_dtype == TQK_BF16) projection_store_kernel<bf16_t, 1><<<n_tokens, 256, 0, s>>>(a);
-    else if (act_dtype == TQK_F32) projection_store_kernel<float, 1><<<n_tokens, 256, 0, s>>>(a);
+    } else if (act_dtype == TQK_BF16) projection_store_kernel<bf16_t, 1><<<n_tokens, threads_for(1), 0, s>>>(a);
+    else if (act_dtype == TQK_F32) projection_store_kernel<float, 1><<<n_tokens, threads_for(1), 0, s>>>(a);
     else return tqk_fail("tqk_projection_store: unknown dtype %d", act_dtype);
     return tqk_check_launch("tqk_projection_store");
 }

@@ -77,11 +77,16 @@ TQ_KERNEL(moe_group, ci32, int, int, int, int, int32_t*, int32_t*, int32_t*, int
 TQ_KERNEL(moe_product, cptr, int, ci32, cptr, int, long long, void*, int, int, int, int, float, float, ci32, ci32, ci32, ci32, int, void*);
 TQ_KERNEL(moe_scale_rows, cptr, int, ci32, cf32, int, void*, float*, int, int, void*);
 TQ_KERNEL(moe_route_grouped, cptr, int, cptr, int, int, int, int, cf32, int, int, float, int32_t*, float*, int, void*);
+TQ_QUERY(int, moe_combine_norm_supported, int);
+TQ_KERNEL(moe_combine_norm, float*, cptr, int, ci32, cf32, int, cptr, cptr, cf32, cptr, float, cptr, int, float, void*, int, int, void*);
 TQ_KERNEL(moe_combine, cptr, int, ci32, cf32, int, cptr, cptr, cf32, cptr, float, void*, int, int, void*);
 TQ_KERNEL(pair_embed, cptr, int, int, long long, long long, ci32, ci32, ci32, ci32, ci32, int32_t*, float*, int, int, int, void*, int, void*);
 TQ_KERNEL(remember_tokens, ci32, ci32, ci32, ci32, int32_t*, int, void*);
 TQ_KERNEL(norm_add, float*, cptr, int, cptr, int, float, void*, int, int, void*);
 TQ_KERNEL(unary_act, cptr, void*, int, long long, int, float, float, void*);
+TQ_KERNEL(fused_store_groups, cptr, long long, int, cptr, int, void*, int, int, int, int, void*);
+TQ_QUERY(int, mid_takes_groups, int, int, int);
+TQ_KERNEL(mid_store_groups, cptr, long long, int, cptr, void*, int, int, int, int, void*, void*);
 TQ_KERNEL(scaled_sum, cptr, cptr, int, float, void*, long long, void*);
 TQ_KERNEL(row_gate, cptr, int, cptr, int, float*, int, int, void*);
 TQ_KERNEL(normed_rope_store, cptr, int, cptr, cptr, cptr, int, float, cf32, cf32, int, int, int, cptr, cptr, void*, ci32, ci32, ci32, int, void*, void*,
@@ -125,6 +130,9 @@ TQ_KERNEL(linear_attention, cptr, cptr, cptr, int, long long, cf32, long long, c
 TQ_KERNEL(head_norm_gate, cf32, cf32, int, float, cptr, int, long long, int, void*, int, int, int, int, void*);
 TQ_KERNEL(token_mixes, cptr, int, cf32, int, float*, long long, ci32, ci32, ci32, ci32, void*, long long, int, int, int, void*);
 TQ_KERNEL(rows_remember, cptr, int, float*, long long, ci32, ci32, ci32, int, int, void*);
+TQ_QUERY(int, decay_chunks_supported, int, int);
+TQ_KERNEL(decay_local, cptr, cptr, long long, cf32, ci32, ci32, int, float*, float*, int, int, int, void*);
+TQ_KERNEL(decay_apply, cptr, cptr, cptr, long long, cf32, cf32, ci32, ci32, int, float*, cf32, float, cptr, long long, void*, int, int, int, void*);
 TQ_QUERY(int, low_rank_max);
 TQ_KERNEL(low_rank_decay, cf32, cf32, cf32, float*, int, int, int, void*);
 TQ_QUERY(int, mlstm_chunks_supported, int, int);

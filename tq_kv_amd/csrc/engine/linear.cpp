@@ -210,6 +210,47 @@ Product linear(StepContext& c, const Tensor& x, const Weight& w, const Tensor* b
     return p;
 }
 
+bool takes_groups(int64_t x_rows, const Weight& w, int64_t group_rows) {
+    if (w.dtype != BF16 || w.k % 32 || group_rows % 32 || null_device()) return false;
+    if (policy().skinny && x_rows <= skinny_max_rows()) return true;
+    return leaves_sums(x_rows, w) && K::mid_takes_groups.raw((int)w.n, (int)w.k, (int)group_rows) != 0;
+}
+
+Tensor linear_groups(StepContext& c, const Tensor& x, int64_t x_group_stride, const Weight& w, int64_t group_rows, int out_dtype) {
+    const int64_t m = x.shape[0];
+    if (x.shape[1] != w.k || !takes_groups(m, w, group_rows)) raise(TQE_ERR_STATE, "linear_groups: the kernels do not take these groups");
+    Tensor out = c.alloc(out_dtype, {m, w.n});
+    if (m <= skinny_max_rows()) {
+        int packed = 0;
+        const void* wp = few_ptr(w, &packed);
+        K::fused_store_groups(x.data, x_group_stride, (int)group_rows, wp, packed, out.data, out_dtype, (int)m, (int)w.n, (int)w.k, c.stream);
+        return out;
+    }
+    const int splits = K::mid_splits.raw((int)w.n, (int)w.k, 0);
+    Tensor scratch;
+    if (splits > 1) scratch = c.alloc(F32, {splits, m, w.n});
+    K::mid_store_groups(x.data, x_group_stride, (int)group_rows, w.packed->t.data, out.data, out_dtype, (int)m, (int)w.n, (int)w.k, scratch.data, c.stream);
+    return out;
+}
+
+Weight weight_slice(const Weight& w, int64_t a, int64_t b) {
+    Weight s;
+    s.n = b - a;
+    s.k = w.k;
+    s.dtype = w.dtype;
+    auto view = [](const Tensor& t) {
+        OwnedPtr o = std::make_shared<Owned>();
+        o->t = t;
+        return o;
+    };
+    if (w.rows) s.rows = view(w.rows->t.slice(a, b));
+    if (w.packed) {
+        if (a % 16 || b % 16) raise(TQE_ERR_STATE, "a slice of a packed weight must begin and end at multiples of 16 rows");
+        s.packed = view(w.packed->t.slice(a / 16, b / 16));
+    }
+    return s;
+}
+
 Gate Gate::from_params(const KeyReader& r, const char* what) {
     Gate g;
     const std::string name = r.string_or("gate", "silu");

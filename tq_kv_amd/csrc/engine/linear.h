@@ -64,6 +64,12 @@ struct Product {
 // x [M, K] times weight^T -> [M, N] of out_dtype (into `out` if given, else workspace memory).
 // leave_sums: the caller also takes the product unfinished where the kernel cuts K into pieces.
 Product linear(StepContext& c, const Tensor& x, const Weight& w, const Tensor* bias, int out_dtype, bool leave_sums = false, Tensor* out = nullptr);
+// Several products in one launch, for the few-row and mid-sized kernels: the rows of the weight are groups of group_rows one behind the other,
+// and group i multiplies the rows of x + i * x_group_stride elements (x: the first group's [M, K]) -> [M, w.n], where takes_groups(M, ...).
+bool takes_groups(int64_t x_rows, const Weight& w, int64_t group_rows);
+Tensor linear_groups(StepContext& c, const Tensor& x, int64_t x_group_stride, const Weight& w, int64_t group_rows, int out_dtype);
+// Rows a .. b of a weight as a weight of its own (views: the whole one must outlive it); both multiples of 16 where it has a packed copy.
+Weight weight_slice(const Weight& w, int64_t a, int64_t b);
 // The same for a step of few rows whose input is a folded norm: the stream times the norm's weight goes in, and the kernel divides
 // its result by the rows' root mean square (where fusable(rows, w) holds).
 Tensor linear_of_norm(StepContext& c, const LazyNorm& norm, const Weight& w, int out_dtype);

@@ -109,9 +109,11 @@ struct Stream {
     Tensor copies;
     const float* copies_mix = nullptr;
     const float* copies_out = nullptr;
+    Tensor normed;                      // the norm normed_for of h, where the kernel that added to h also worked that out (valid while nothing is pending)
+    const Norm* normed_for = nullptr;
     Tensor copy;                        // h in the activation type, where a kernel that added to h also wrote it (valid while copy_valid)
     bool copy_valid = false;
-    void invalidate() { xw_for = nullptr; copy_valid = false; }
+    void invalidate() { xw_for = nullptr; copy_valid = false; normed_for = nullptr; }
 };
 
 // ---- building --------------------------------------------------------------------------------
@@ -217,8 +219,12 @@ public:
     virtual bool adds_to_stream(const StepContext& c) const { (void)c; return false; }
     virtual Tensor forward(StepContext& c, const Activation& x, Stream* stream) = 0;
     // Optional: scale (forward(x) + beside) out of the part's own last kernel (beside: [tokens, hidden], what another part made of the step).
+    // stream and next_norm given: the part may add the sum to the stream and leave next_norm of it there (normed); it then returns nothing.
     virtual bool takes_beside() const { return false; }
-    virtual Tensor forward_beside(StepContext& c, const Activation& x, const Tensor& beside, float scale) { (void)beside; (void)scale; return forward(c, x, nullptr); }
+    virtual Tensor forward_beside(StepContext& c, const Activation& x, const Tensor& beside, float scale, Stream* stream, const Norm* next_norm) {
+        (void)beside; (void)scale; (void)stream; (void)next_norm;
+        return forward(c, x, nullptr);
+    }
 };
 
 class Block : public Part {

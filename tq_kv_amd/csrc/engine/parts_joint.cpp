@@ -2,8 +2,8 @@
 //
 //   block joint   h = norm(x), x' = x + scale (mixer(h) + ff(h)); the feed-forward may be absent.
 //
-// The sum is formed in the feed-forward's own last kernel where it offers that (takes_beside), and is left pending on the stream for the next
-// norm's kernel.
+// The sum is formed in the feed-forward's own last kernel where it offers that (takes_beside), which may also add it to the stream and work out the
+// next block's norm; else it is left pending on the stream for the next norm's kernel.
 //
 // params: mixer, feed_forward (or null), norm (part specs), scale (1 unless given); names {mixer, feed_forward, norm}: prefixes of the parts' tensors.
 #include "kernels.h"
@@ -76,11 +76,14 @@ public:
     Norm* first_norm() override { return norm_.get(); }
     Mixer* mixer() override { return mixer_.get(); }
 
-    Stream* forward(StepContext& c, Stream* stream, const CacheEntry& entry, Norm*, bool last) override {
+    Stream* forward(StepContext& c, Stream* stream, const CacheEntry& entry, Norm* next_norm, bool last) override {
         // the model's last block goes on with the wanted rows alone: keys and values of all tokens, everything else of those rows
         const bool prune = last && c.prune_last && policy().prune_last && mixer_->takes_rows;
         Activation x;
-        {
+        if (stream->normed_for == norm_.get() && stream->pending.kind == Pending::Nothing && stream->normed.dtype == c.act_dtype) {
+            x.x = stream->normed;
+            stream->invalidate();
+        } else {
             Span span(norm_->trace_name());
             x.x = c.alloc(c.act_dtype, {stream->h.shape[0], stream->h.shape[1]});
             norm_->add_norm(c, stream->h, stream->pending, x.x);
@@ -109,7 +112,9 @@ public:
         Tensor out;
         if (feed_forward_ && feed_forward_->takes_beside()) {
             Span span(feed_forward_->trace_name());
-            out = feed_forward_->forward_beside(c, x, y, scale_);
+            // (what the head reads after the last block is chosen rows: their norm is the head's)
+            out = feed_forward_->forward_beside(c, x, y, scale_, last ? nullptr : stream, last ? nullptr : next_norm);
+            if (!out.defined()) return stream;
         } else {
             Tensor f;
             if (feed_forward_) {

@@ -160,16 +160,16 @@ public:
         if (shared_) shared_->product_shapes(out);
     }
 
-    Tensor forward(StepContext& c, const Activation& x, Stream*) override { return run(c, x, nullptr, 1.f); }
+    Tensor forward(StepContext& c, const Activation& x, Stream*) override { return run(c, x, nullptr, 1.f, nullptr, nullptr); }
     bool takes_beside() const override { return true; }
-    Tensor forward_beside(StepContext& c, const Activation& x, const Tensor& beside, float scale) override {
+    Tensor forward_beside(StepContext& c, const Activation& x, const Tensor& beside, float scale, Stream* stream, const Norm* next_norm) override {
         if (beside.dtype != x.x.dtype || beside.shape[0] != x.x.shape[0] || beside.cols() != hidden_)
             raise(TQE_ERR_STATE, "routed_experts: what is to be added is %s for a step of [%lld, %lld]", beside.describe().c_str(), (long long)x.x.shape[0], (long long)hidden_);
-        return run(c, x, beside.data, scale);
+        return run(c, x, beside.data, scale, stream, next_norm);
     }
 
 private:
-    Tensor run(StepContext& c, const Activation& x, const void* beside, float scale) {
+    Tensor run(StepContext& c, const Activation& x, const void* beside, float scale, Stream* stream, const Norm* next_norm) {
         if (x.lazy) raise(TQE_ERR_STATE, "routed_experts takes no folded norm");
         const int64_t n = x.x.shape[0];
         const int dtype = x.x.dtype;
@@ -235,8 +235,20 @@ private:
                            0, 0.f, 1.f, tile_expert, tile_row0, tile_rows, (const int32_t*)n_tiles.data, max_tiles, c.stream);
         }
         Tensor out = c.alloc(dtype, {n, hidden_});
+        const float* shared_by = shared_gate_ ? (const float*)shared_scale.data : nullptr;
+        // the sum into the stream and the next norm of it in one pass, where that norm is one the kernel knows
+        if (stream && next_norm && next_norm->foldable() && next_norm->size() == hidden_ && K::moe_combine_norm_supported.raw((int)hidden_)) {
+            const Tensor& w = *next_norm->fold_weight();
+            K::moe_combine_norm((float*)stream->h.data, y.data, dtype, (const int32_t*)pair_pos.data, sum_weight, top_, identity_ ? x.x.data : nullptr, shared_out.data,
+                                shared_by, beside, scale, w.data, w.dtype, next_norm->fold_eps(), out.data, (int)n, (int)hidden_, c.stream);
+            stream->pending = Pending();
+            stream->invalidate();
+            stream->normed = out;
+            stream->normed_for = next_norm;
+            return Tensor();
+        }
         K::moe_combine(y.data, dtype, (const int32_t*)pair_pos.data, sum_weight, top_, identity_ ? x.x.data : nullptr, shared_out.data,
-                       shared_gate_ ? (const float*)shared_scale.data : nullptr, beside, scale, out.data, (int)n, (int)hidden_, c.stream);
+                       shared_by, beside, scale, out.data, (int)n, (int)hidden_, c.stream);
         return out;
     }
 

@@ -9,8 +9,8 @@
 //
 // The cache's state row holds the state, [heads][head_dim][head_dim] float32, and behind it the last token's x (zero when a slot is taken).  The
 // decay's second product, its exponentials, the recurrence and the heads' norm are float32 whatever the activation type; the other products are
-// the framework's.  Steps that bring many tokens of a sequence run the recurrence in chunks (every chunk from a zero state, a carry over the
-// chunks, every chunk again with the outputs).
+// the framework's.  Steps that bring many tokens of a sequence run the recurrence in chunks: every chunk's own part of the state, a carry over the
+// chunks, then the outputs; on the matrix cores where they take the heads' size (decay_chunks.hip).
 //
 // params: hidden, heads, head_dim, decay_rank (what random weights get: the checkpoint's tensors give the rank), eps, names {mu (a prefix: the mixes'
 // weights are <mu>r, <mu>k, ...), r, k, v, g, o, w1, w2, w0, bonus, norm}.
@@ -94,7 +94,16 @@ public:
         OwnedPtr stacked = stack_rows(mu, stream);                       // [mixes * hidden]
         mu_ = as_floats(stacked, stream);
         const std::string* products[4] = {&n_r_, &n_k_, &n_v_, &n_g_};
-        for (int i = 0; i < 4; ++i) w_in_[i] = make_weight(take(t, *products[i]), 1, false, stream);
+        const int64_t hd = (int64_t)heads_ * d_;
+        std::vector<OwnedPtr> four;
+        for (int i = 0; i < 4; ++i) four.push_back(take(t, *products[i]));
+        if (hd % 32 == 0) {
+            // one behind the other, so that short steps run the four products in one launch
+            w_all_ = make_weight(stack_rows(four, stream), 1, false, stream);
+            for (int i = 0; i < 4; ++i) w_in_[i] = weight_slice(w_all_, i * hd, (i + 1) * hd);
+        } else {
+            for (int i = 0; i < 4; ++i) w_in_[i] = make_weight(four[(size_t)i], 1, false, stream);
+        }
         w_o_ = make_weight(take(t, n_o_), 1, false, stream);
         OwnedPtr w1 = take(t, n_w1_), w2 = take(t, n_w2_);
         if (w1->t.shape[0] != w2->t.shape[1])
@@ -146,19 +155,42 @@ public:
         K::token_mixes(x.x.data, dtype, (const float*)mu_->t.data, N_MIXES, last, row, c.dev.tok_seq, c.dev.tok_pos, c.dev.seq_start, c.dev.seq_slot, mixes.data, mix_stride, (int)n,
                        (int)hidden_, c.all_decode ? 1 : 0, c.stream);
         if (!c.all_decode) K::rows_remember(x.x.data, dtype, last, row, c.dev.cu, c.dev.seq_new, c.dev.seq_slot, c.n_seqs, (int)hidden_, c.stream);
-        Tensor part[4];                                                      // r, k, v, g
-        for (int i = 0; i < 4; ++i) part[i] = linear(c, mix(i), w_in_[i], nullptr, dtype).t;
+        // r, k, v, g: each a row of `stride` elements a token
+        const void* part[4];
+        long long stride = hd;
+        if (dtype == BF16 && w_all_.defined() && takes_groups(n, w_all_, hd)) {
+            const Tensor all = linear_groups(c, mix(0), mix_stride, w_all_, hd, dtype);
+            stride = 4 * hd;
+            for (int i = 0; i < 4; ++i) part[i] = (const char*)all.data + (size_t)(i * hd) * dtype_size(dtype);
+        } else {
+            for (int i = 0; i < 4; ++i) part[i] = linear(c, mix(i), w_in_[i], nullptr, dtype).t.data;
+        }
         const Tensor low = linear(c, mix(4), w_w1_, nullptr, F32).t;
-        Tensor decay = c.alloc(F32, {n, hd});
-        K::low_rank_decay((const float*)low.data, (const float*)w2_->t.data, (const float*)w0_->t.data, (float*)decay.data, (int)n, (int)rank_, (int)hd, c.stream);
+        Tensor log_decay = c.alloc(F32, {n, hd});
+        const float* logs = (const float*)log_decay.data;
+        K::low_rank_decay((const float*)low.data, (const float*)w2_->t.data, (const float*)w0_->t.data, (float*)log_decay.data, (int)n, (int)rank_, (int)hd, c.stream);
+        const float* u = (const float*)u_->t.data;
+        const float* norm_w = (const float*)norm_w_->t.data;
+        Tensor gated = c.alloc(dtype, {n, hd});
+        const bool many = dtype == BF16 && !c.all_decode && !c.capturing && !null_device();
+        if (many && c.max_new >= CORES_FROM && K::decay_chunks_supported.raw(d_, d_)) {
+            // on the matrix cores, the heads' norm and the gate in the last kernel
+            const Chunks ch = c.chunks(CHUNK);
+            Tensor cs = c.alloc(F32, {ch.n, hd * d_}), cd = c.alloc(F32, {ch.n, hd});
+            K::decay_local(part[1], part[2], stride, logs, ch.row0, ch.count, ch.n, (float*)cs.data, (float*)cd.data, heads_, d_, d_, c.stream);
+            K::chunk_carry((const float*)cd.data, hd, d_, (float*)cs.data, ch.seq_first, c.dev.seq_slot, state, row, c.n_seqs, hd * d_, c.stream);
+            K::decay_apply(part[0], part[1], part[2], stride, logs, u, ch.row0, ch.count, ch.n, (float*)cs.data, norm_w, eps_, part[3], stride, gated.data,
+                           heads_, d_, d_, c.stream);
+            return linear(c, gated, w_o_, nullptr, dtype).t;
+        }
         Tensor o = c.alloc(F32, {n, heads_, d_});
         auto run = [&](int mode, int items, const Chunks* ch, float* cs, float* cd) {
-            K::linear_attention(part[0].data, part[1].data, part[2].data, dtype, hd, nullptr, 0, nullptr, 0.f, nullptr, nullptr, nullptr, nullptr, (const float*)decay.data,
-                                (const float*)u_->t.data, 1.f, 1.f, nullptr, nullptr, 0, 0, 0, c.dev.tok_pos, state, row, c.dev.cu, c.dev.seq_new, c.dev.seq_slot,
-                                ch ? ch->row0 : nullptr, ch ? ch->count : nullptr, cs, cd, (float*)o.data, mode, items, heads_, d_, d_, (long long)d_ * d_, c.stream);
+            K::linear_attention(part[0], part[1], part[2], dtype, stride, nullptr, 0, nullptr, 0.f, nullptr, nullptr, nullptr, nullptr, logs, u, 1.f, 1.f, nullptr,
+                                nullptr, 0, 0, 0, c.dev.tok_pos, state, row, c.dev.cu, c.dev.seq_new, c.dev.seq_slot, ch ? ch->row0 : nullptr, ch ? ch->count : nullptr,
+                                cs, cd, (float*)o.data, mode, items, heads_, d_, d_, (long long)d_ * d_, c.stream);
         };
-        if (dtype == BF16 && !c.all_decode && !c.capturing && c.max_new >= CHUNKED_FROM && !null_device()) {
-            const Chunks ch = c.chunks(SCAN_CHUNK);
+        if (many && c.max_new >= CHUNKED_FROM) {
+            const Chunks ch = c.chunks(CHUNK);
             Tensor cs = c.alloc(F32, {ch.n, hd * d_}), cd = c.alloc(F32, {ch.n, hd});
             run(1, ch.n, &ch, (float*)cs.data, (float*)cd.data);
             K::chunk_carry((const float*)cd.data, hd, d_, (float*)cs.data, ch.seq_first, c.dev.seq_slot, state, row, c.n_seqs, hd * d_, c.stream);
@@ -166,13 +198,13 @@ public:
         } else {
             run(0, c.n_seqs, nullptr, nullptr, nullptr);
         }
-        Tensor gated = c.alloc(dtype, {n, hd});
-        K::head_norm_gate((const float*)o.data, (const float*)norm_w_->t.data, d_, eps_, part[3].data, dtype, hd, 0, gated.data, dtype, (int)n, heads_, d_, c.stream);
+        K::head_norm_gate((const float*)o.data, norm_w, d_, eps_, part[3], dtype, stride, 0, gated.data, dtype, (int)n, heads_, d_, c.stream);
         return linear(c, gated, w_o_, nullptr, dtype).t;
     }
 
 private:
-    static const int CHUNKED_FROM = 128, SCAN_CHUNK = 64, N_MIXES = 5;
+    // steps that bring so many tokens of some sequence run in chunks: on the matrix cores, or (sizes those do not take) on the vector units
+    static const int CORES_FROM = 32, CHUNKED_FROM = 128, CHUNK = 64, N_MIXES = 5;
     static constexpr const char* MIXES[N_MIXES] = {"r", "k", "v", "g", "w"};
     // where a state row keeps the last token's x: behind the state, at a multiple of four floats
     int64_t last_at() const { return ((int64_t)heads_ * d_ * d_ + 3) / 4 * 4; }
@@ -180,7 +212,7 @@ private:
     int heads_, d_;
     float eps_;
     std::string n_mu_, n_r_, n_k_, n_v_, n_g_, n_o_, n_w1_, n_w2_, n_w0_, n_u_, n_norm_;
-    Weight w_in_[4], w_o_, w_w1_;
+    Weight w_all_, w_in_[4], w_o_, w_w1_;      // the four products stacked (or not defined); each of them
     OwnedPtr mu_, w2_, w0_, u_, norm_w_;
     Loaded stored_;
 };

@@ -1,8 +1,8 @@
 // Linear attention with a decaying state: per head S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, with S of d rows (key
 // channels) and dv columns in float32.  The decay a_t is one number per head (fixed) or one per key channel and token, formed here
 // from a product z as sigmoid(z + bias)^(1/tau) = exp(logsigmoid(z + bias) / tau), or one number per head and token given by its
-// logarithm (log_decay; then k may be weighted by exp(log_in) and the output multiplied by out_scale, per head and token too), or given as it
-// is per key channel and token (decay).  With a bonus u [heads, d] a token's output reads the state in front of it, and the token itself through
+// logarithm (log_decay; then k may be weighted by exp(log_in) and the output multiplied by out_scale, per head and token too), or by its
+// logarithm per key channel and token (log_channels).  With a bonus u [heads, d] a token's output reads the state in front of it, and the token itself through
 // u instead of the state: o_t = S_(t-1)^T q_t + (sum_i u_i k_i q_i) v_t.  q and k may be turned by the position (tables of
 // cos and sin, in halves or neighbouring pairs over the first rot_dim elements) and scaled on their way in; everything after the
 // loads is float32.
@@ -32,7 +32,7 @@ struct LaArgs {
     float inv_tau;
     const float* head_decay;
     const float *log_decay, *log_in, *out_scale;        // [tokens, heads] or null
-    const float* decay;                                 // [tokens, heads * d], or null
+    const float* log_channels;                          // [tokens, heads * d], or null
     const float* bonus;                                 // [heads, d], or null
     float q_scale, k_scale;
     const float *cos, *sin;
@@ -114,8 +114,8 @@ void linear_attention_kernel(LaArgs a, int rg_shift) {
             lq[e] = qv * a.q_scale;
             lk[e] = kv * a.k_scale;
             float al;
-            if (a.decay) {
-                al = a.decay[(row * H + head) * d + i];
+            if (a.log_channels) {
+                al = expf(a.log_channels[(row * H + head) * d + i]);
             } else if (a.z) {
                 const float zz = a.z[row * a.z_stride + (size_t)head * d + i] + a.z_bias[(size_t)head * d + i];
                 const float ls = fminf(zz, 0.f) - log1pf(expf(-fabsf(zz)));
@@ -223,8 +223,8 @@ void linear_attention_block_kernel(LaArgs a, int rg_shift, int cb) {
                 }
                 qv *= a.q_scale;
                 kv *= a.k_scale;
-                if (a.decay) {
-                    al = a.decay[((size_t)row * H + head) * d + i];
+                if (a.log_channels) {
+                    al = expf(a.log_channels[((size_t)row * H + head) * d + i]);
                 } else if (a.z) {
                     const float zz = a.z[row * a.z_stride + (size_t)head * d + i] + a.z_bias[(size_t)head * d + i];
                     const float ls = fminf(zz, 0.f) - log1pf(expf(-fabsf(zz)));
@@ -329,13 +329,13 @@ extern "C" int tqk_linear_attention_max_dim(void) { return 512; }
 
 extern "C" int tqk_linear_attention(const void* q, const void* k, const void* v, int act_dtype, long long stride, const float* z, long long z_stride,
                                     const float* z_bias, float inv_tau, const float* head_decay, const float* log_decay, const float* log_in,
-                                    const float* out_scale, const float* decay, const float* bonus, float q_scale, float k_scale, const float* cos,
+                                    const float* out_scale, const float* log_channels, const float* bonus, float q_scale, float k_scale, const float* cos,
                                     const float* sin, int rot_dim, int style, int max_pos, const int32_t* tok_pos, float* state, long long state_stride,
                                     const int32_t* cu, const int32_t* seq_new, const int32_t* seq_slot, const int32_t* chunk_row0,
                                     const int32_t* chunk_count, float* chunk_state, float* chunk_decay, float* out, int mode, int n_items, int heads,
                                     int d, int dv, long long head_stride, void* stream) {
     TQK_REQUIRE(q && k && v, "tqk_linear_attention: null pointer");
-    TQK_REQUIRE((z && z_bias) || head_decay || log_decay || decay, "tqk_linear_attention: neither a decay per channel nor one per head");
+    TQK_REQUIRE((z && z_bias) || head_decay || log_decay || log_channels, "tqk_linear_attention: neither a decay per channel nor one per head");
     TQK_REQUIRE(head_stride >= (long long)d * dv, "tqk_linear_attention: heads' states overlap");
     TQK_REQUIRE(mode >= LA_SCAN && mode <= LA_APPLY, "tqk_linear_attention: unknown mode %d", mode);
     TQK_REQUIRE(mode == LA_SCAN ? (state && cu && seq_new && seq_slot) : (chunk_row0 && chunk_count && chunk_state && chunk_decay),
@@ -346,7 +346,7 @@ extern "C" int tqk_linear_attention(const void* q, const void* k, const void* v,
     TQK_REQUIRE(!cos || (sin && tok_pos && rot_dim > 0 && rot_dim % 2 == 0 && rot_dim <= d && max_pos > 0 && (style == LA_STYLE_HALVES || style == LA_STYLE_PAIRS)),
                 "tqk_linear_attention: bad rotation");
     if (n_items == 0) return 0;
-    LaArgs a = {q, k, v, stride, z, z_stride, z_bias, inv_tau, head_decay, log_decay, log_in, out_scale, decay, bonus, q_scale, k_scale, cos, sin, rot_dim, style, max_pos, tok_pos,
+    LaArgs a = {q, k, v, stride, z, z_stride, z_bias, inv_tau, head_decay, log_decay, log_in, out_scale, log_channels, bonus, q_scale, k_scale, cos, sin, rot_dim, style, max_pos, tok_pos,
                 state, state_stride, cu, seq_new, seq_slot, chunk_row0, chunk_count, chunk_state, chunk_decay, out, heads, d, dv, head_stride};
     hipStream_t s = (hipStream_t)stream;
     if (d % 4 == 0 && dv % 4 == 0 && dv >= 16 && (((uintptr_t)out) & 15) == 0) {

@@ -49,6 +49,8 @@ struct MidArgs {
     int gate;                   // gated: which gate (TQK_GATE_*), with its limit and alpha
     float gate_limit, gate_alpha;
     int activated;              // store: the gate's function of the product itself is applied (act_value)
+    int group_rows;             // store: features n of group n / group_rows read the rows of x + group * x_group_stride (0: one group)
+    long long x_group_stride;
 };
 
 __device__ __forceinline__ uint2 pack4_bf16(float a, float b, float c, float d) {
@@ -80,6 +82,8 @@ void mid_product_kernel(const MidArgs p) {
     const int n_waves = blockDim.x / TQK_WAVE;
     const int row = lane % 16, kgrp = lane / 16;
     const int K = p.K;
+    const bf16_t* px = p.x;
+    if (EPI == MID_STORE && p.group_rows) px += (size_t)((int)blockIdx.x * n_waves * TN * 16 / p.group_rows) * p.x_group_stride;
     const int k_begin = blockIdx.y * p.k_per_split, k_end = min(K, k_begin + p.k_per_split);
 
     const int n_out = EPI == MID_GATED ? p.N / 2 : p.N;             // features one part of the weight has
@@ -105,7 +109,7 @@ void mid_product_kernel(const MidArgs p) {
             const int s = min((int)threadIdx.x + i * (int)blockDim.x, SLOTS - 1);
             const int mt = s / 256, ks = (s / 64) % 4, ln = s % 64;
             xk[i] = ks * 32 + (ln / 16) * 8;
-            xsrc[i] = p.x + (size_t)min(mt * 16 + ln % 16, p.M - 1) * K;
+            xsrc[i] = px + (size_t)min(mt * 16 + ln % 16, p.M - 1) * K;
         }
     }
     // 8 row groups: the block's first 256 threads bring x in, thread t piece t ([k step][lane]) of
@@ -132,7 +136,7 @@ void mid_product_kernel(const MidArgs p) {
 #pragma unroll
             for (int i = 0; i < XS; ++i) {
                 const uint32_t r = (uint32_t)min((i * PAR + st_half) * 16 + st_row, p.M - 1);
-                xr[i] = *reinterpret_cast<const u32x4_t*>(p.x + (r * (uint32_t)K + kk));
+                xr[i] = *reinterpret_cast<const u32x4_t*>(px + (r * (uint32_t)K + kk));
             }
         } else {
 #pragma unroll
@@ -451,7 +455,7 @@ static int check_mid(const MidArgs& a, const void* scratch, bool gated, bool fin
  * (for tqk_add_rmsnorm_sums) and y is not written. */
 extern "C" int tqk_mid_store(const void* x, const void* w_packed, void* y, int y_dtype, int M, int N, int K,
                              void* scratch, int finish, void* stream) {
-    MidArgs a = {(const bf16_t*)x, (const bf16_t*)w_packed, y, (float*)scratch, M, N, K, 0, 0, 0.f, 1.f, 0};
+    MidArgs a = {(const bf16_t*)x, (const bf16_t*)w_packed, y, (float*)scratch, M, N, K, 0, 0, 0.f, 1.f, 0, 0, 0};
     if (check_mid(a, scratch, false, finish != 0, "tqk_mid_store")) return -1;
     TQK_REQUIRE(y_dtype == TQK_F32 || y_dtype == TQK_BF16, "tqk_mid_store: unknown output dtype %d", y_dtype);
     if (M == 0) return 0;
@@ -462,11 +466,32 @@ extern "C" int tqk_mid_store(const void* x, const void* w_packed, void* y, int y
                               : launch_rows<MID_STORE, bf16_t>(a, plan, finish != 0, s);
 }
 
+/* Several products in one launch: the rows n of w in groups of group_rows, group i taking x + i * x_group_stride; scratch as tqk_mid_store's for all
+ * N rows.  Where tqk_mid_takes_groups (a block's features belong to one group). */
+extern "C" int tqk_mid_takes_groups(int N, int K, int group_rows) {
+    if (N <= 0 || K <= 0 || group_rows <= 0 || N % group_rows) return 0;
+    const MidPlan plan = mid_plan(N, K, false);
+    return group_rows % (plan.waves * plan.tn * 16) == 0;
+}
+extern "C" int tqk_mid_store_groups(const void* x, long long x_group_stride, int group_rows, const void* w_packed, void* y, int y_dtype, int M, int N, int K,
+                                    void* scratch, void* stream) {
+    MidArgs a = {(const bf16_t*)x, (const bf16_t*)w_packed, y, (float*)scratch, M, N, K, 0, 0, 0.f, 1.f, 0, group_rows, x_group_stride};
+    if (check_mid(a, scratch, false, true, "tqk_mid_store_groups")) return -1;
+    TQK_REQUIRE(y_dtype == TQK_F32 || y_dtype == TQK_BF16, "tqk_mid_store_groups: unknown output dtype %d", y_dtype);
+    TQK_REQUIRE(tqk_mid_takes_groups(N, K, group_rows), "tqk_mid_store_groups: %d rows in groups of %d", N, group_rows);
+    TQK_REQUIRE(x_group_stride % 8 == 0 && x_group_stride >= (long long)M * K, "tqk_mid_store_groups: the groups' rows of x overlap or are not aligned");
+    if (M == 0) return 0;
+    const MidPlan plan = mid_plan(N, K, false);
+    a.k_per_split = plan.k_per_split;
+    hipStream_t s = (hipStream_t)stream;
+    return y_dtype == TQK_F32 ? launch_rows<MID_STORE, float>(a, plan, true, s) : launch_rows<MID_STORE, bf16_t>(a, plan, true, s);
+}
+
 /* y[M,N] = f(x w^T) in bfloat16, f a gate's function of one product (TQK_GATE_*: common.h). */
 extern "C" int tqk_mid_store_act(const void* x, const void* w_packed, void* y, int M, int N, int K, void* scratch, int gate, float limit, float alpha,
                                  void* stream) {
     TQK_REQUIRE(gate >= 0 && gate < TQK_GATE_KINDS, "tqk_mid_store_act: unknown activation %d", gate);
-    MidArgs a = {(const bf16_t*)x, (const bf16_t*)w_packed, y, (float*)scratch, M, N, K, 0, gate, limit, alpha, 1};
+    MidArgs a = {(const bf16_t*)x, (const bf16_t*)w_packed, y, (float*)scratch, M, N, K, 0, gate, limit, alpha, 1, 0, 0};
     if (check_mid(a, scratch, false, true, "tqk_mid_store_act")) return -1;
     if (M == 0) return 0;
     const MidPlan plan = mid_plan(N, K, false);
@@ -483,7 +508,7 @@ extern "C" int tqk_mid_gated(const void* x, const void* w_packed, void* y, int M
 extern "C" int tqk_mid_gated_act(const void* x, const void* w_packed, void* y, int M, int N, int K, void* scratch, int gate, float limit,
                                  float alpha, void* stream) {
     TQK_REQUIRE(gate >= 0 && gate < TQK_GATE_KINDS, "tqk_mid_gated: unknown gate %d", gate);
-    MidArgs a = {(const bf16_t*)x, (const bf16_t*)w_packed, y, (float*)scratch, M, N, K, 0, gate, limit, alpha, 0};
+    MidArgs a = {(const bf16_t*)x, (const bf16_t*)w_packed, y, (float*)scratch, M, N, K, 0, gate, limit, alpha, 0, 0, 0};
     if (check_mid(a, scratch, true, true, "tqk_mid_gated")) return -1;
     if (M == 0) return 0;
     const MidPlan plan = mid_plan(N, K, true);

@@ -22,66 +22,93 @@
 #include "tq_kernels.h"
 
 #define MOE_MAX_EXPERTS 512
-#define MOE_ROUTE_WAVES 8
+#define MOE_ROUTE_WAVES 16
+#define MOE_ROUTE_TOKENS 4     // tokens of a block in steps of many
 #define MOE_TM 32               // rows of a tile
 #define MOE_TN 64               // features of a block
 #define MOE_TK 16               // k per stage
 
 // ---- route -----------------------------------------------------------------------------------
-// A block per token: its waves share the experts out for the logits (each a dot product over the lanes, several loads
-// under way at once, added up in a fixed order), then the first wave takes the softmax and the largest.
-template <typename TA, typename TW>
-__device__ __forceinline__ void route_logits(const TA* __restrict__ xr, const TW* __restrict__ w, int n_experts, int hidden, const TW* __restrict__ gate_w,
-                                             float* __restrict__ gate_out, float* z) {
+// A block takes NT tokens: its waves share the experts out for the logits, two at once (dot products over the lanes, several loads under way
+// together, added up in an order that the row's length alone decides), then a wave per token takes the softmax and the largest.
+// Logit e of the block's token n goes to z[n * MOE_MAX_EXPERTS + e].  One row more where a gate is given: sigmoid(x . gate_w) per token, which
+// rides along with the experts' dot products.
+template <typename TA, typename TW, int NT>
+__device__ __forceinline__ void route_logits(const TA* __restrict__ x, int n_tokens, const TW* __restrict__ w, int n_experts, int hidden,
+                                             const TW* __restrict__ gate_w, float* __restrict__ gate_out, float* z) {
     const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
-    // one row more where a gate is given: sigmoid(x . gate_w) per token, which rides along with the experts' dot products
-    for (int e = wave; e < n_experts + (gate_w ? 1 : 0); e += MOE_ROUTE_WAVES) {
-        const TW* wr = e < n_experts ? w + (size_t)e * hidden : gate_w;
-        float d0 = 0.f, d1 = 0.f, d2 = 0.f, d3 = 0.f;
-        int i = lane;
+    const int t0 = blockIdx.x * NT, rows = n_experts + (gate_w ? 1 : 0);
+    const TA* xr[NT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) xr[n] = x + (size_t)min(t0 + n, n_tokens - 1) * hidden;
+    for (int e0 = wave; e0 < rows; e0 += 2 * MOE_ROUTE_WAVES) {
+        const int ee[2] = {e0, min(e0 + MOE_ROUTE_WAVES, rows - 1)};
+        const TW* wr[2];
+#pragma unroll
+        for (int j = 0; j < 2; ++j) wr[j] = ee[j] < n_experts ? w + (size_t)ee[j] * hidden : gate_w;
+        float d[2][NT][4];
+#pragma unroll
+        for (int j = 0; j < 2; ++j)
+#pragma unroll
+            for (int n = 0; n < NT; ++n) d[j][n][0] = d[j][n][1] = d[j][n][2] = d[j][n][3] = 0.f;
         if (sizeof(TA) == 2 && sizeof(TW) == 2 && hidden % 8 == 0) {
-            // bfloat16 rows whose length is a multiple of 8: 16 bytes a lane and load, in the same order of additions for
-            // every token
-            float d[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+            // bfloat16 rows whose length is a multiple of 8: 16 bytes a lane and load
+#pragma unroll 2
             for (int c = lane * 8; c < hidden; c += TQK_WAVE * 8) {
-                const uint4 xv = *reinterpret_cast<const uint4*>(xr + c), wv = *reinterpret_cast<const uint4*>(wr + c);
-                const uint32_t xw[4] = {xv.x, xv.y, xv.z, xv.w}, ww[4] = {wv.x, wv.y, wv.z, wv.w};
+                uint4 wv[2], xv[NT];
+#pragma unroll
+                for (int j = 0; j < 2; ++j) wv[j] = *reinterpret_cast<const uint4*>(wr[j] + c);
+#pragma unroll
+                for (int n = 0; n < NT; ++n) xv[n] = *reinterpret_cast<const uint4*>(xr[n] + c);
+#pragma unroll
+                for (int j = 0; j < 2; ++j)
+#pragma unroll
+                    for (int n = 0; n < NT; ++n) {
+                        const uint32_t xw[4] = {xv[n].x, xv[n].y, xv[n].z, xv[n].w}, ww[4] = {wv[j].x, wv[j].y, wv[j].z, wv[j].w};
+#pragma unroll
+                        for (int k = 0; k < 4; ++k) {
+                            d[j][n][k] = fmaf(__uint_as_float(xw[k] << 16), __uint_as_float(ww[k] << 16), d[j][n][k]);
+                            d[j][n][k] = fmaf(__uint_as_float(xw[k] & 0xffff0000u), __uint_as_float(ww[k] & 0xffff0000u), d[j][n][k]);
+                        }
+                    }
+            }
+        } else {
+            for (int c = lane; c < hidden; c += 4 * TQK_WAVE) {
 #pragma unroll
                 for (int k = 0; k < 4; ++k) {
-                    d[2 * k] = fmaf(__uint_as_float(xw[k] << 16), __uint_as_float(ww[k] << 16), d[2 * k]);
-                    d[2 * k + 1] = fmaf(__uint_as_float(xw[k] & 0xffff0000u), __uint_as_float(ww[k] & 0xffff0000u), d[2 * k + 1]);
+                    const int i = c + k * TQK_WAVE;
+                    if (i >= hidden) continue;
+#pragma unroll
+                    for (int j = 0; j < 2; ++j)
+#pragma unroll
+                        for (int n = 0; n < NT; ++n) d[j][n][k] = fmaf(to_float(xr[n][i]), to_float(wr[j][i]), d[j][n][k]);
                 }
             }
-            d0 = (d[0] + d[1]) + (d[2] + d[3]);
-            d1 = (d[4] + d[5]) + (d[6] + d[7]);
-            i = hidden;
         }
-        for (; i + 3 * TQK_WAVE < hidden; i += 4 * TQK_WAVE) {
-            d0 = fmaf(to_float(xr[i]), to_float(wr[i]), d0);
-            d1 = fmaf(to_float(xr[i + TQK_WAVE]), to_float(wr[i + TQK_WAVE]), d1);
-            d2 = fmaf(to_float(xr[i + 2 * TQK_WAVE]), to_float(wr[i + 2 * TQK_WAVE]), d2);
-            d3 = fmaf(to_float(xr[i + 3 * TQK_WAVE]), to_float(wr[i + 3 * TQK_WAVE]), d3);
-        }
-        for (; i < hidden; i += TQK_WAVE) d0 = fmaf(to_float(xr[i]), to_float(wr[i]), d0);
-        const float dot = wave_sum((d0 + d1) + (d2 + d3));
-        if (lane == 0) {
-            if (e < n_experts) z[e] = dot;
-            else *gate_out = 1.f / (1.f + expf(-dot));
-        }
+#pragma unroll
+        for (int j = 0; j < 2; ++j)
+#pragma unroll
+            for (int n = 0; n < NT; ++n) {
+                const float dot = wave_sum((d[j][n][0] + d[j][n][1]) + (d[j][n][2] + d[j][n][3]));
+                if (lane != 0 || e0 + j * MOE_ROUTE_WAVES >= rows || t0 + n >= n_tokens) continue;
+                if (ee[j] < n_experts) z[n * MOE_MAX_EXPERTS + ee[j]] = dot;
+                else gate_out[t0 + n] = 1.f / (1.f + expf(-dot));
+            }
     }
     __syncthreads();
 }
 
-template <typename TA, typename TW>
+template <typename TA, typename TW, int NT>
 __global__ __launch_bounds__(MOE_ROUTE_WAVES * TQK_WAVE)
-void moe_route_kernel(const TA* __restrict__ x, const TW* __restrict__ w, int n_experts, int hidden, int top, float scale, int mode,
+void moe_route_kernel(const TA* __restrict__ x, int n_tokens, const TW* __restrict__ w, int n_experts, int hidden, int top, float scale, int mode,
                       int32_t* __restrict__ idx, float* __restrict__ weight, const TW* __restrict__ gate_w, float* __restrict__ gate_out) {
     const int renormalize = mode & 1, sigmoid_scores = mode & 2;
-    __shared__ float z[MOE_MAX_EXPERTS];
+    __shared__ float logits[NT * MOE_MAX_EXPERTS];
     const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
-    const int t = blockIdx.x;
-    route_logits(x + (size_t)t * hidden, w, n_experts, hidden, gate_w, gate_w ? gate_out + t : nullptr, z);
-    if (wave != 0) return;
+    route_logits<TA, TW, NT>(x, n_tokens, w, n_experts, hidden, gate_w, gate_out, logits);
+    const int t = blockIdx.x * NT + wave;
+    if (wave >= NT || t >= n_tokens) return;
+    float* z = logits + wave * MOE_MAX_EXPERTS;
     float m = -INFINITY;
     for (int e = lane; e < n_experts; e += TQK_WAVE) m = fmaxf(m, z[e]);
     m = wave_max(m);
@@ -135,18 +162,21 @@ __device__ __forceinline__ int wave_argmax(const volatile float* z, int n, int l
     return at;
 }
 
-// Choice by score plus correction within the best groups of neighbours.  What the first wave keeps of the experts lies in LDS and is
+// Choice by score plus correction within the best groups of neighbours.  What a token's wave keeps of the experts lies in LDS and is
 // read and written by that wave alone, each element by one lane between two of the wave's exchanges.
-template <typename TA, typename TW>
+template <typename TA, typename TW, int NT>
 __global__ __launch_bounds__(MOE_ROUTE_WAVES * TQK_WAVE)
-void moe_route_grouped_kernel(const TA* __restrict__ x, const TW* __restrict__ w, int n_experts, int hidden, int top, const float* __restrict__ correction,
+void moe_route_grouped_kernel(const TA* __restrict__ x, int n_tokens, const TW* __restrict__ w, int n_experts, int hidden, int top, const float* __restrict__ correction,
                               int n_groups, int keep, float floor, int32_t* __restrict__ idx, float* __restrict__ weight) {
-    __shared__ float z[MOE_MAX_EXPERTS];
-    __shared__ volatile float score[MOE_MAX_EXPERTS], choice[MOE_MAX_EXPERTS], group[MOE_MAX_EXPERTS];
+    __shared__ float logits[NT * MOE_MAX_EXPERTS];
+    __shared__ volatile float choices[NT * MOE_MAX_EXPERTS], groups[NT * MOE_MAX_EXPERTS];
     const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
-    const int t = blockIdx.x;
-    route_logits(x + (size_t)t * hidden, w, n_experts, hidden, (const TW*)nullptr, (float*)nullptr, z);
-    if (wave != 0) return;
+    route_logits<TA, TW, NT>(x, n_tokens, w, n_experts, hidden, (const TW*)nullptr, (float*)nullptr, logits);
+    const int t = blockIdx.x * NT + wave;
+    if (wave >= NT || t >= n_tokens) return;
+    volatile float* z = logits + wave * MOE_MAX_EXPERTS;           // the logits, then the scores
+    volatile float* choice = choices + wave * MOE_MAX_EXPERTS;
+    volatile float* group = groups + wave * MOE_MAX_EXPERTS;
     float m = -INFINITY;
     for (int e = lane; e < n_experts; e += TQK_WAVE) m = fmaxf(m, z[e]);
     m = wave_max(m);
@@ -155,7 +185,7 @@ void moe_route_grouped_kernel(const TA* __restrict__ x, const TW* __restrict__ w
     sum = wave_sum(sum);
     for (int e = lane; e < n_experts; e += TQK_WAVE) {
         const float s = expf(z[e] - m) / sum;
-        score[e] = s;
+        z[e] = s;
         choice[e] = s + (correction ? correction[e] : 0.f);
     }
     __threadfence_block();
@@ -187,7 +217,7 @@ void moe_route_grouped_kernel(const TA* __restrict__ x, const TW* __restrict__ w
         int e = wave_argmax(choice, n_experts, lane, best);
         e = e < n_experts ? e : k;                          // (scores that are not numbers: some expert that is there)
         if (lane == e % TQK_WAVE) choice[e] = -INFINITY;
-        const float s = score[e];
+        const float s = z[e];
         chosen += s;
         if (lane == 0) {
             idx[(size_t)t * top + k] = e;
@@ -316,31 +346,123 @@ void moe_product_kernel(const TX* __restrict__ x, const int32_t* __restrict__ x_
 }
 
 // ---- combine ---------------------------------------------------------------------------------
+struct CombineArgs {
+    const void* y;
+    const int32_t* pair_pos;
+    const float* weight;
+    int top;
+    const void *x, *shared;         // x: the step's rows, for pairs without a row (or null); shared, beside: or null
+    const float* shared_scale;
+    const void* beside;
+    float scale;
+    void* out;                      // the sums, in the activation type; or, with h, the norm of the stream
+    float* h;                       // null, or the stream, which the sums are added to
+    const void* norm_w;
+    float eps;
+    int hidden;
+};
+
+template <typename TA> struct Four;
+template <> struct Four<float> {
+    __device__ static float4 load(const void* p, size_t at) { return *reinterpret_cast<const float4*>((const float*)p + at); }
+    __device__ static void store(void* p, size_t at, float4 v) { *reinterpret_cast<float4*>((float*)p + at) = v; }
+};
+template <> struct Four<bf16_t> {
+    __device__ static float4 load(const void* p, size_t at) {
+        const uint2 u = *reinterpret_cast<const uint2*>((const bf16_t*)p + at);
+        return make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16), __uint_as_float(u.y & 0xffff0000u));
+    }
+    __device__ static void store(void* p, size_t at, float4 v) {
+        *reinterpret_cast<uint2*>((bf16_t*)p + at) = make_uint2(float_to_bf16_bits(v.x) | ((uint32_t)float_to_bf16_bits(v.y) << 16),
+                                                               float_to_bf16_bits(v.z) | ((uint32_t)float_to_bf16_bits(v.w) << 16));
+    }
+};
+
+// A block per token, four neighbouring elements a thread VPT times.  NORM: the sum goes to the stream h in float32, and out is the stream's RMS
+// norm (h / rms(h) * norm_w), which the next layer reads.
+template <typename TA, typename TW, int VPT, bool NORM>
+__global__ __launch_bounds__(1024)
+void moe_combine_vec_kernel(const CombineArgs a) {
+    __shared__ int32_t row[MOE_MAX_EXPERTS];
+    __shared__ float wt[MOE_MAX_EXPERTS];
+    __shared__ float scratch[16];
+    const size_t t = blockIdx.x;
+    const int hidden = a.hidden, top = a.top;
+    for (int k = threadIdx.x; k < top; k += blockDim.x) {
+        row[k] = a.pair_pos[t * top + k];
+        wt[k] = a.weight[t * top + k];
+    }
+    __syncthreads();
+    const float ss = a.shared && a.shared_scale ? a.shared_scale[t] : 1.f;
+    float4 keep[VPT];
+    float sq = 0.f;
+#pragma unroll
+    for (int j = 0; j < VPT; ++j) {
+        const int i = (j * blockDim.x + threadIdx.x) * 4;
+        keep[j] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (i >= hidden) continue;
+        float4 v = make_float4(0.f, 0.f, 0.f, 0.f), hv = v;
+        if (NORM) hv = *reinterpret_cast<const float4*>(a.h + t * hidden + i);
+#pragma unroll 4
+        for (int k = 0; k < top; ++k) {
+            const int r = row[k];
+            const float4 u = Four<TA>::load(r >= 0 ? a.y : a.x, (r >= 0 ? (size_t)r : t) * hidden + i);
+            const float w = wt[k];
+            v.x = fmaf(w, u.x, v.x); v.y = fmaf(w, u.y, v.y); v.z = fmaf(w, u.z, v.z); v.w = fmaf(w, u.w, v.w);
+        }
+        if (a.shared) {
+            const float4 u = Four<TA>::load(a.shared, t * hidden + i);
+            v.x = fmaf(ss, u.x, v.x); v.y = fmaf(ss, u.y, v.y); v.z = fmaf(ss, u.z, v.z); v.w = fmaf(ss, u.w, v.w);
+        }
+        if (a.beside) {
+            const float4 u = Four<TA>::load(a.beside, t * hidden + i);
+            v.x += u.x; v.y += u.y; v.z += u.z; v.w += u.w;
+        }
+        if (!NORM) {
+            Four<TA>::store(a.out, t * hidden + i, make_float4(v.x * a.scale, v.y * a.scale, v.z * a.scale, v.w * a.scale));
+            continue;
+        }
+        hv.x = fmaf(a.scale, v.x, hv.x); hv.y = fmaf(a.scale, v.y, hv.y); hv.z = fmaf(a.scale, v.z, hv.z); hv.w = fmaf(a.scale, v.w, hv.w);
+        *reinterpret_cast<float4*>(a.h + t * hidden + i) = hv;
+        keep[j] = hv;
+        sq += (hv.x * hv.x + hv.y * hv.y) + (hv.z * hv.z + hv.w * hv.w);
+    }
+    if (!NORM) return;
+    const float rms = sqrtf(block_sum(sq, scratch) / (float)hidden + a.eps);
+#pragma unroll
+    for (int j = 0; j < VPT; ++j) {
+        const int i = (j * blockDim.x + threadIdx.x) * 4;
+        if (i >= hidden) continue;
+        const float4 w = Four<TW>::load(a.norm_w, i), v = keep[j];
+        Four<TA>::store(a.out, t * hidden + i, make_float4(v.x / rms * w.x, v.y / rms * w.y, v.z / rms * w.z, v.w / rms * w.w));
+    }
+}
+
+// rows of any length and alignment, element by element
 template <typename TA>
 __global__ __launch_bounds__(256)
-void moe_combine_kernel(const TA* __restrict__ y, const int32_t* __restrict__ pair_pos, const float* __restrict__ weight, int top,
-                        const TA* __restrict__ x, const TA* __restrict__ shared, const float* __restrict__ shared_scale, const TA* __restrict__ beside,
-                        float scale, TA* __restrict__ out, int hidden) {
+void moe_combine_kernel(const CombineArgs a) {
     // the token's rows and weights once, side by side, not one load after the other in front of every element
     __shared__ int32_t row[MOE_MAX_EXPERTS];
     __shared__ float wt[MOE_MAX_EXPERTS];
-    const int t = blockIdx.x;
+    const size_t t = blockIdx.x;
+    const int hidden = a.hidden, top = a.top;
     for (int k = threadIdx.x; k < top; k += blockDim.x) {
-        row[k] = pair_pos[(size_t)t * top + k];
-        wt[k] = weight[(size_t)t * top + k];
+        row[k] = a.pair_pos[t * top + k];
+        wt[k] = a.weight[t * top + k];
     }
     __syncthreads();
-    const float ss = shared && shared_scale ? shared_scale[t] : 1.f;
+    const float ss = a.shared && a.shared_scale ? a.shared_scale[t] : 1.f;
     for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
         float v = 0.f;
 #pragma unroll 4
         for (int k = 0; k < top; ++k) {
-            const TA* src = row[k] >= 0 || !x ? y + (size_t)row[k] * hidden : x + (size_t)t * hidden;
-            v = fmaf(wt[k], to_float(src[i]), v);
+            const int r = row[k];
+            v = fmaf(wt[k], to_float(((const TA*)(r >= 0 ? a.y : a.x))[(r >= 0 ? (size_t)r : t) * hidden + i]), v);
         }
-        if (shared) v = fmaf(ss, to_float(shared[(size_t)t * hidden + i]), v);
-        if (beside) v += to_float(beside[(size_t)t * hidden + i]);
-        out[(size_t)t * hidden + i] = from_float<TA>(v * scale);
+        if (a.shared) v = fmaf(ss, to_float(((const TA*)a.shared)[t * hidden + i]), v);
+        if (a.beside) v += to_float(((const TA*)a.beside)[t * hidden + i]);
+        ((TA*)a.out)[t * hidden + i] = from_float<TA>(v * a.scale);
     }
 }
 
@@ -386,7 +508,8 @@ extern "C" int tqk_moe_route(const void* x, int act_dtype, const void* w_router,
     if (n_tokens == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
 #define TQK_ROUTE(TA, TW) \
-    moe_route_kernel<TA, TW><<<n_tokens, MOE_ROUTE_WAVES * TQK_WAVE, 0, s>>>((const TA*)x, (const TW*)w_router, n_experts, hidden, top, scale, mode, idx, weight, (const TW*)gate_w, gate_out)
+    do { if (n_tokens >= 512) moe_route_kernel<TA, TW, MOE_ROUTE_TOKENS><<<(n_tokens + MOE_ROUTE_TOKENS - 1) / MOE_ROUTE_TOKENS, MOE_ROUTE_WAVES * TQK_WAVE, 0, s>>>((const TA*)x, n_tokens, (const TW*)w_router, n_experts, hidden, top, scale, mode, idx, weight, (const TW*)gate_w, gate_out); \
+        else moe_route_kernel<TA, TW, 1><<<n_tokens, MOE_ROUTE_WAVES * TQK_WAVE, 0, s>>>((const TA*)x, n_tokens, (const TW*)w_router, n_experts, hidden, top, scale, mode, idx, weight, (const TW*)gate_w, gate_out); } while (0)
     if (act_dtype == TQK_F32 && w_dtype == TQK_F32) TQK_ROUTE(float, float);
     else if (act_dtype == TQK_F32 && w_dtype == TQK_BF16) TQK_ROUTE(float, bf16_t);
     else if (act_dtype == TQK_BF16 && w_dtype == TQK_F32) TQK_ROUTE(bf16_t, float);
@@ -406,7 +529,8 @@ extern "C" int tqk_moe_route_grouped(const void* x, int act_dtype, const void* w
     if (n_tokens == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
 #define TQK_ROUTE(TA, TW) \
-    moe_route_grouped_kernel<TA, TW><<<n_tokens, MOE_ROUTE_WAVES * TQK_WAVE, 0, s>>>((const TA*)x, (const TW*)w_router, n_experts, hidden, top, correction, n_groups, keep, floor, idx, weight)
+    do { if (n_tokens >= 512) moe_route_grouped_kernel<TA, TW, MOE_ROUTE_TOKENS><<<(n_tokens + MOE_ROUTE_TOKENS - 1) / MOE_ROUTE_TOKENS, MOE_ROUTE_WAVES * TQK_WAVE, 0, s>>>((const TA*)x, n_tokens, (const TW*)w_router, n_experts, hidden, top, correction, n_groups, keep, floor, idx, weight); \
+        else moe_route_grouped_kernel<TA, TW, 1><<<n_tokens, MOE_ROUTE_WAVES * TQK_WAVE, 0, s>>>((const TA*)x, n_tokens, (const TW*)w_router, n_experts, hidden, top, correction, n_groups, keep, floor, idx, weight); } while (0)
     if (act_dtype == TQK_F32 && w_dtype == TQK_F32) TQK_ROUTE(float, float);
     else if (act_dtype == TQK_F32 && w_dtype == TQK_BF16) TQK_ROUTE(float, bf16_t);
     else if (act_dtype == TQK_BF16 && w_dtype == TQK_F32) TQK_ROUTE(bf16_t, float);
@@ -463,17 +587,58 @@ extern "C" int tqk_moe_product(const void* x, int act_dtype, const int32_t* x_ro
     return tqk_fail("tqk_moe_product: unknown dtypes %d, %d", act_dtype, w_dtype);
 }
 
-extern "C" int tqk_moe_combine(const void* y, int act_dtype, const int32_t* pair_pos, const float* weight, int top, const void* x, const void* shared,
-                               const float* shared_scale, const void* beside, float scale, void* out, int n_tokens, int hidden, void* stream) {
+static int combine_args(CombineArgs& a, const void* y, const int32_t* pair_pos, const float* weight, int top, const void* x, const void* shared,
+                        const float* shared_scale, const void* beside, float scale, void* out, int n_tokens, int hidden) {
     TQK_REQUIRE(y && pair_pos && weight && out, "tqk_moe_combine: null pointer");
     TQK_REQUIRE(top > 0 && top <= MOE_MAX_EXPERTS && hidden > 0 && n_tokens >= 0, "tqk_moe_combine: bad sizes");
+    // (without x no pair may be without a row: every pair_pos is then a row of y)
+    a = {y, pair_pos, weight, top, x ? x : y, shared, shared_scale, beside, scale, out, nullptr, nullptr, 0.f, hidden};
+    return 0;
+}
+// rows in pieces of four elements, each piece at its alignment; a thread takes up to two of them
+static bool combine_in_pieces(const CombineArgs& a) {
+    return a.hidden % 4 == 0 && a.hidden <= 8192 &&
+           ((((uintptr_t)a.y | (uintptr_t)a.x | (uintptr_t)a.shared | (uintptr_t)a.beside | (uintptr_t)a.out | (uintptr_t)a.h | (uintptr_t)a.norm_w)) & 15) == 0;
+}
+template <typename TA, typename TW, bool NORM>
+static void launch_combine(const CombineArgs& a, int n_tokens, hipStream_t s) {
+    const int pieces = a.hidden / 4;
+    const int threads = pieces >= 1024 ? 1024 : (pieces + TQK_WAVE - 1) / TQK_WAVE * TQK_WAVE;
+    if (pieces <= threads) moe_combine_vec_kernel<TA, TW, 1, NORM><<<n_tokens, threads, 0, s>>>(a);
+    else moe_combine_vec_kernel<TA, TW, 2, NORM><<<n_tokens, threads, 0, s>>>(a);
+}
+
+extern "C" int tqk_moe_combine(const void* y, int act_dtype, const int32_t* pair_pos, const float* weight, int top, const void* x, const void* shared,
+                               const float* shared_scale, const void* beside, float scale, void* out, int n_tokens, int hidden, void* stream) {
+    CombineArgs a;
+    if (combine_args(a, y, pair_pos, weight, top, x, shared, shared_scale, beside, scale, out, n_tokens, hidden)) return -1;
+    TQK_REQUIRE(act_dtype == TQK_F32 || act_dtype == TQK_BF16, "tqk_moe_combine: unknown dtype %d", act_dtype);
     if (n_tokens == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
-#define TQK_COMBINE(TA) \
-    moe_combine_kernel<TA><<<n_tokens, 256, 0, s>>>((const TA*)y, pair_pos, weight, top, (const TA*)x, (const TA*)shared, shared_scale, (const TA*)beside, scale, (TA*)out, hidden)
-    if (act_dtype == TQK_F32) TQK_COMBINE(float);
-    else if (act_dtype == TQK_BF16) TQK_COMBINE(bf16_t);
-    else return tqk_fail("tqk_moe_combine: unknown dtype %d", act_dtype);
-#undef TQK_COMBINE
+    if (combine_in_pieces(a)) {
+        if (act_dtype == TQK_F32) launch_combine<float, float, false>(a, n_tokens, s);
+        else launch_combine<bf16_t, float, false>(a, n_tokens, s);
+    } else if (act_dtype == TQK_F32) moe_combine_kernel<float><<<n_tokens, 256, 0, s>>>(a);
+    else moe_combine_kernel<bf16_t><<<n_tokens, 256, 0, s>>>(a);
     return tqk_check_launch("tqk_moe_combine");
+}
+
+extern "C" int tqk_moe_combine_norm_supported(int hidden) { return hidden > 0 && hidden % 4 == 0 && hidden <= 8192; }
+
+extern "C" int tqk_moe_combine_norm(float* h, const void* y, int act_dtype, const int32_t* pair_pos, const float* weight, int top, const void* x,
+                                    const void* shared, const float* shared_scale, const void* beside, float scale, const void* norm_w, int norm_w_dtype,
+                                    float eps, void* out, int n_tokens, int hidden, void* stream) {
+    CombineArgs a;
+    if (combine_args(a, y, pair_pos, weight, top, x, shared, shared_scale, beside, scale, out, n_tokens, hidden)) return -1;
+    TQK_REQUIRE(h && norm_w, "tqk_moe_combine_norm: null pointer");
+    a.h = h; a.norm_w = norm_w; a.eps = eps;
+    TQK_REQUIRE(combine_in_pieces(a), "tqk_moe_combine_norm: rows of %d elements, or operands that are not aligned", hidden);
+    if (n_tokens == 0) return 0;
+    hipStream_t s = (hipStream_t)stream;
+    if (act_dtype == TQK_F32 && norm_w_dtype == TQK_F32) launch_combine<float, float, true>(a, n_tokens, s);
+    else if (act_dtype == TQK_F32 && norm_w_dtype == TQK_BF16) launch_combine<float, bf16_t, true>(a, n_tokens, s);
+    else if (act_dtype == TQK_BF16 && norm_w_dtype == TQK_F32) launch_combine<bf16_t, float, true>(a, n_tokens, s);
+    else if (act_dtype == TQK_BF16 && norm_w_dtype == TQK_BF16) launch_combine<bf16_t, bf16_t, true>(a, n_tokens, s);
+    else return tqk_fail("tqk_moe_combine_norm: unknown dtypes %d, %d", act_dtype, norm_w_dtype);
+    return tqk_check_launch("tqk_moe_combine_norm");
 }

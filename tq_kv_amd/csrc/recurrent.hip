@@ -388,11 +388,27 @@ void chunk_carry_kernel(const float* __restrict__ chunk_p, long long p_stride, i
     if (c1 <= c0) return;
     float* st = state + (size_t)seq_slot[s] * state_stride + e;
     float S = *st;
-    for (int c = c0; c < c1; ++c) {
+    const float* p = chunk_p + e / p_div;
+    int c = c0;
+    // eight chunks' values asked for together, then used in order
+    for (; c + 8 <= c1; c += 8) {
+        float local[8], decay[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+            local[j] = chunk_l[(size_t)(c + j) * per_seq + e];
+            decay[j] = p[(size_t)(c + j) * p_stride];
+        }
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+            chunk_l[(size_t)(c + j) * per_seq + e] = S;
+            S = fmaf(decay[j], S, local[j]);
+        }
+    }
+    for (; c < c1; ++c) {
         float* l = chunk_l + (size_t)c * per_seq + e;
         const float local = *l;
         *l = S;
-        S = fmaf(chunk_p[(size_t)c * p_stride + e / p_div], S, local);
+        S = fmaf(p[(size_t)c * p_stride], S, local);
     }
     *st = S;
 }

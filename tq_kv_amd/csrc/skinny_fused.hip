@@ -76,6 +76,8 @@ struct FusedArgs {
     const bf16_t* w;            // [N, K], or packed (see below)
     int w_packed;
     int M, N, K;
+    int group_rows;             // store: features n of group n / group_rows read the rows of x + group * x_group_stride (0: one group)
+    long long x_group_stride;
     // store / gated
     void* y;
     int gate;                   // gated: which gate (TQK_GATE_*), with its limit and alpha
@@ -163,6 +165,7 @@ void skinny_fused_kernel(const FusedArgs p) {
     // row 0 and their results are dropped.
     const int xr = row < p.M ? (GATHER ? p.x_rows[row] : row) : 0;
     const bf16_t* xrow = p.x + (size_t)xr * K + kgrp * 8;
+    if (EPI == EPI_STORE && p.group_rows) xrow += (size_t)(n_lo0 / p.group_rows) * p.x_group_stride;
 
     // The sums of squares [n_ss_parts, 16 rows] as float4s: thread t takes the float4s t, t + threads, ...,
     // which all hold rows 4*(t%4) .. +3.  The first is asked for here and used after the product.
@@ -473,6 +476,22 @@ extern "C" int tqk_fused_store(const void* x, const int32_t* x_rows, const float
         return y_dtype == TQK_F32 ? launch_tiled<false, EPI_STORE, float, true>(a, s) : launch_tiled<false, EPI_STORE, bf16_t, true>(a, s);
     }
     if (ss_parts) return y_dtype == TQK_F32 ? launch_tiled<true, EPI_STORE, float>(a, s) : launch_tiled<true, EPI_STORE, bf16_t>(a, s);
+    return y_dtype == TQK_F32 ? launch_tiled<false, EPI_STORE, float>(a, s) : launch_tiled<false, EPI_STORE, bf16_t>(a, s);
+}
+
+/* Several products in one launch: the rows n of w in groups of group_rows (a multiple of 32), group i taking x + i * x_group_stride. */
+extern "C" int tqk_fused_store_groups(const void* x, long long x_group_stride, int group_rows, const void* w, int w_packed, void* y, int y_dtype, int M, int N,
+                                      int K, void* stream) {
+    FusedArgs a = {};
+    a.x = (const bf16_t*)x; a.w = (const bf16_t*)w; a.w_packed = w_packed; a.M = M; a.N = N; a.K = K; a.y = y;
+    a.group_rows = group_rows; a.x_group_stride = x_group_stride;
+    if (check_common(a, "tqk_fused_store_groups")) return -1;
+    TQK_REQUIRE(y, "tqk_fused_store_groups: null output");
+    TQK_REQUIRE(y_dtype == TQK_F32 || y_dtype == TQK_BF16, "tqk_fused_store_groups: unknown output dtype %d", y_dtype);
+    TQK_REQUIRE(group_rows > 0 && group_rows % 32 == 0 && N % group_rows == 0, "tqk_fused_store_groups: %d rows in groups of %d", N, group_rows);
+    TQK_REQUIRE(x_group_stride % 8 == 0 && x_group_stride >= (long long)M * K, "tqk_fused_store_groups: the groups' rows of x overlap or are not aligned");
+    if (M == 0) return 0;
+    hipStream_t s = (hipStream_t)stream;
     return y_dtype == TQK_F32 ? launch_tiled<false, EPI_STORE, float>(a, s) : launch_tiled<false, EPI_STORE, bf16_t>(a, s);
 }
 

@@ -1,11 +1,11 @@
 // What time mixing puts in front of its recurrence (the recurrence itself is tqk_linear_attention with a decay of its own per key channel and
-// token, and a bonus).
+// token, and a bonus; in steps of many tokens decay_chunks.hip).
 //
 //   tqk_token_mixes     out[s][t] = x[t] + (x[t - 1] - x[t]) mu[s]: what each of the products that follow reads.  The row before a sequence's
 //                       first token of the step comes from the sequence's state (zeros before its first token); `remember` (steps of one
 //                       token a sequence) also leaves x[t] there
 //   tqk_rows_remember   state of sequence s = x[last token the step brings of s]
-//   tqk_low_rank_decay  decay[t, c] = exp(-exp(sum_r w2[r, c] tanh(low[t, r]) + bias[c]))
+//   tqk_low_rank_decay  log_decay[t, c] = -exp(sum_r w2[r, c] tanh(low[t, r]) + bias[c]), the logarithm of the decay
 //
 // float32 arithmetic; what comes and goes in the activation type is rounded once.
 #include "common.h"
@@ -86,7 +86,7 @@ void rows_remember_kernel(const T* __restrict__ x, float* __restrict__ state, lo
 // [rank][TT].  A decay's sum runs over the rank in order, whatever the step holds.
 template <int TT>
 __global__ __launch_bounds__(256)
-void low_rank_decay_kernel(const float* __restrict__ low, const float* __restrict__ w2, const float* __restrict__ bias, float* __restrict__ decay,
+void low_rank_decay_kernel(const float* __restrict__ low, const float* __restrict__ w2, const float* __restrict__ bias, float* __restrict__ log_decay,
                            int n_tokens, int rank, int channels) {
     extern __shared__ __attribute__((aligned(16))) float tanh_low[];
     const int t0 = blockIdx.y * TT, nt = min(TT, n_tokens - t0);
@@ -113,7 +113,7 @@ void low_rank_decay_kernel(const float* __restrict__ low, const float* __restric
         }
     }
     const float b = bias[c];
-    for (int tt = 0; tt < nt; ++tt) decay[(size_t)(t0 + tt) * channels + c] = expf(-expf(acc[tt] + b));
+    for (int tt = 0; tt < nt; ++tt) log_decay[(size_t)(t0 + tt) * channels + c] = -expf(acc[tt] + b);
 }
 
 extern "C" int tqk_token_mixes(const void* x, int dtype, const float* mu, int n_mixes, float* state, long long state_stride, const int32_t* tok_seq,
@@ -152,19 +152,19 @@ extern "C" int tqk_rows_remember(const void* x, int dtype, float* state, long lo
 
 extern "C" int tqk_low_rank_max(void) { return TM_MAX_RANK; }
 
-extern "C" int tqk_low_rank_decay(const float* low, const float* w2, const float* bias, float* decay, int n_tokens, int rank, int channels, void* stream) {
-    TQK_REQUIRE(low && w2 && bias && decay, "tqk_low_rank_decay: null pointer");
+extern "C" int tqk_low_rank_decay(const float* low, const float* w2, const float* bias, float* log_decay, int n_tokens, int rank, int channels, void* stream) {
+    TQK_REQUIRE(low && w2 && bias && log_decay, "tqk_low_rank_decay: null pointer");
     TQK_REQUIRE(n_tokens >= 0 && rank > 0 && channels > 0, "tqk_low_rank_decay: bad sizes");
     TQK_REQUIRE(rank <= TM_MAX_RANK, "tqk_low_rank_decay: a rank of %d, the kernel takes up to %d", rank, TM_MAX_RANK);
     if (n_tokens == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
     if (n_tokens <= 16) {
         dim3 grid((channels + TQK_WAVE - 1) / TQK_WAVE, (n_tokens + 3) / 4);
-        low_rank_decay_kernel<4><<<grid, TQK_WAVE, (size_t)rank * 4 * sizeof(float), s>>>(low, w2, bias, decay, n_tokens, rank, channels);
+        low_rank_decay_kernel<4><<<grid, TQK_WAVE, (size_t)rank * 4 * sizeof(float), s>>>(low, w2, bias, log_decay, n_tokens, rank, channels);
     } else {
         dim3 grid((channels + 255) / 256, (n_tokens + 15) / 16);
         TQK_REQUIRE(grid.y <= 65535, "tqk_low_rank_decay: %d tokens are more than the grid takes", n_tokens);
-        low_rank_decay_kernel<16><<<grid, 256, (size_t)rank * 16 * sizeof(float), s>>>(low, w2, bias, decay, n_tokens, rank, channels);
+        low_rank_decay_kernel<16><<<grid, 256, (size_t)rank * 16 * sizeof(float), s>>>(low, w2, bias, log_decay, n_tokens, rank, channels);
     }
     return tqk_check_launch("tqk_low_rank_decay");
 }

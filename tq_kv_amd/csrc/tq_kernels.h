@@ -285,6 +285,11 @@ int tqk_head_product(const void* x, int x_f32, long long x_row_stride, long long
                      void* stream);
 int tqk_moe_combine(const void* y, int act_dtype, const int32_t* pair_pos, const float* weight, int top, const void* x, const void* shared,
                     const float* shared_scale, const void* beside, float scale, void* out, int n_tokens, int hidden, void* stream);
+/* The same sum added to the stream h [tokens, hidden] float32 (not rounded), and out = h / sqrt(mean(h^2) + eps) * norm_w in one pass. */
+int tqk_moe_combine_norm_supported(int hidden);
+int tqk_moe_combine_norm(float* h, const void* y, int act_dtype, const int32_t* pair_pos, const float* weight, int top, const void* x,
+                         const void* shared, const float* shared_scale, const void* beside, float scale, const void* norm_w, int norm_w_dtype,
+                         float eps, void* out, int n_tokens, int hidden, void* stream);
 
 /* Around the residual stream (stream_ops.hip).  tqk_pair_embed: h[t] += table[(prev * mul_prev + token * mul_cur) mod buckets],
  * table [buckets + 1, hidden], the last row for a sequence's first token; prev is the token before it in the step or, for the
@@ -302,6 +307,13 @@ int tqk_remember_tokens(const int32_t* tokens, const int32_t* cu, const int32_t*
 int tqk_norm_add(float* h, const void* y, int act_dtype, const void* weight, int weight_dtype, float eps, void* copy, int n_tokens,
                  int hidden, void* stream);
 int tqk_unary_act(const void* x, void* out, int act_dtype, long long n, int kind, float limit, float alpha, void* stream);
+/* Several products in one launch, for few and for 17 to 128 rows: the rows n of w in groups of group_rows, group i taking the rows of x + i *
+ * x_group_stride; y [M, N].  tqk_fused_store_groups takes groups of a multiple of 32 rows, tqk_mid_store_groups what tqk_mid_takes_groups says. */
+int tqk_fused_store_groups(const void* x, long long x_group_stride, int group_rows, const void* w, int w_packed, void* y, int y_dtype, int M, int N,
+                           int K, void* stream);
+int tqk_mid_takes_groups(int N, int K, int group_rows);
+int tqk_mid_store_groups(const void* x, long long x_group_stride, int group_rows, const void* w_packed, void* y, int y_dtype, int M, int N, int K,
+                         void* scratch, void* stream);
 /* out = scale (a + b) over n elements of the activation type (b may be null) */
 int tqk_scaled_sum(const void* a, const void* b, int act_dtype, float scale, void* out, long long n, void* stream);
 int tqk_row_gate(const void* x, int act_dtype, const void* w, int w_dtype, float* out, int n_tokens, int hidden, void* stream);
@@ -479,7 +491,7 @@ int tqk_shift_remember(const float* n, float* state, long long state_stride, con
 /* Linear attention with a decaying state (linear_attention.hip): per head S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, the state
  * of a slot [heads][d][dv] float32, head_stride elements from head to head.  q, k, v: rows `stride` elements apart, heads side by side.  The decay: z [tokens, heads * d] float32
  * with z_bias gives a = sigmoid(z + bias)^inv_tau per key channel; z null: head_decay[h] for the whole head, or, with
- * log_decay [tokens, heads], its exponential (k then times exp(log_in), the output times out_scale, both [tokens, heads] or null), or decay [tokens, heads * d] as it is.
+ * log_decay [tokens, heads], its exponential (k then times exp(log_in), the output times out_scale, both [tokens, heads] or null), or the exponential of log_channels [tokens, heads * d].
  * bonus [heads, d] (or null): o_t = S_(t-1)^T q_t + (sum_i bonus_i k_i q_i) v_t.  q and k are turned by
  * tok_pos through cos, sin [max_pos, rot_dim / 2] (style 1: halves, 2: pairs; cos null: not turned) and multiplied by q_scale, k_scale.
  * mode 0: every sequence's tokens in order from its state row, which is written back (cu, seq_new, seq_slot; n_items sequences).
@@ -490,7 +502,7 @@ int tqk_shift_remember(const float* n, float* state, long long state_stride, con
 int tqk_linear_attention_max_dim(void);
 int tqk_linear_attention(const void* q, const void* k, const void* v, int act_dtype, long long stride, const float* z, long long z_stride,
                          const float* z_bias, float inv_tau, const float* head_decay, const float* log_decay, const float* log_in,
-                         const float* out_scale, const float* decay, const float* bonus, float q_scale, float k_scale, const float* cos,
+                         const float* out_scale, const float* log_channels, const float* bonus, float q_scale, float k_scale, const float* cos,
                          const float* sin, int rot_dim, int style, int max_pos, const int32_t* tok_pos, float* state, long long state_stride,
                          const int32_t* cu, const int32_t* seq_new, const int32_t* seq_slot, const int32_t* chunk_row0,
                          const int32_t* chunk_count, float* chunk_state, float* chunk_decay, float* out, int mode, int n_items, int heads,
@@ -502,7 +514,7 @@ int tqk_head_norm_gate(const float* o, const float* weight, int weight_stride, f
 /* What time mixing puts in front of its recurrence (time_mixing.hip).  tqk_token_mixes: out[s][t] = x[t] + (x[t - 1] - x[t]) mu[s] for n_mixes
  * rows mu [n_mixes, width] float32, out [n_mixes][tokens][width] in x's type, mix_stride elements from mix to mix; the sequence's state row stands for x[t - 1] at the first token a
  * step brings of it; remember != 0 (steps of one token a sequence) also leaves x[t] there.  tqk_rows_remember: the state of every sequence
- * becomes x of the last token the step brings of it.  tqk_low_rank_decay: decay[t, c] = exp(-exp(sum_r w2[r, c] tanh(low[t, r]) + bias[c])), all
+ * becomes x of the last token the step brings of it.  tqk_low_rank_decay: log_decay[t, c] = -exp(sum_r w2[r, c] tanh(low[t, r]) + bias[c]), all
  * float32, w2 [rank, channels]. */
 int tqk_token_mixes(const void* x, int dtype, const float* mu, int n_mixes, float* state, long long state_stride, const int32_t* tok_seq,
                     const int32_t* tok_pos, const int32_t* seq_start, const int32_t* seq_slot, void* out, long long mix_stride, int n_tokens, int width,
@@ -510,7 +522,18 @@ int tqk_token_mixes(const void* x, int dtype, const float* mu, int n_mixes, floa
 int tqk_rows_remember(const void* x, int dtype, float* state, long long state_stride, const int32_t* cu, const int32_t* seq_new,
                       const int32_t* seq_slot, int n_seqs, int width, void* stream);
 int tqk_low_rank_max(void);
-int tqk_low_rank_decay(const float* low, const float* w2, const float* bias, float* decay, int n_tokens, int rank, int channels, void* stream);
+int tqk_low_rank_decay(const float* low, const float* w2, const float* bias, float* log_decay, int n_tokens, int rank, int channels, void* stream);
+
+/* That recurrence for steps of many tokens, bfloat16, on the matrix cores (decay_chunks.hip), where tqk_decay_chunks_supported(d, dv).  Chunks of up
+ * to 64 tokens as tqk_ssm_chunks takes them: tqk_decay_local leaves a chunk's own part of the state [chunks][heads][d][dv] and its decays
+ * [chunks][heads * d]; tqk_chunk_carry (p_stride heads * d, p_div dv) turns that into the state every chunk starts from; tqk_decay_apply gives
+ * out [tokens, heads * dv] = the heads' outputs divided by their root mean square, times norm_weight [heads * dv], times silu(gate). */
+int tqk_decay_chunks_supported(int d, int dv);
+int tqk_decay_local(const void* k, const void* v, long long stride, const float* log_decay, const int32_t* chunk_row0, const int32_t* chunk_count,
+                    int n_chunks, float* chunk_state, float* chunk_decay, int heads, int d, int dv, void* stream);
+int tqk_decay_apply(const void* r, const void* k, const void* v, long long stride, const float* log_decay, const float* bonus,
+                    const int32_t* chunk_row0, const int32_t* chunk_count, int n_chunks, float* chunk_state, const float* norm_weight, float eps,
+                    const void* gate, long long gate_stride, void* out, int heads, int d, int dv, void* stream);
 
 /* The gates of a matrix memory (mlstm.hip): z [tokens] rows z_stride apart, [heads] input gates' products then [heads] forget gates', bias
  * [2 heads].  a = cap tanh((z_i + b) / cap), f = log sigmoid(cap tanh((z_f + b) / cap)); in the tokens' order m_t = max(f_t + m_(t-1), a_t), kappa
