@@ -196,7 +196,7 @@ def test_attention_on_another_runs_keys_and_values(window, borrowed, dtype):
 
 
 ROUTERS = [C.moe(40, 9, 3, 3, 4, 2), C.moe(8, 1, 1), C.moe(8, 1, 2, 1), C.moe(22, 3, 2, 2, 5, 3), C.moe(16, 6, 6, 2, 1, 1), C.moe(32, 60, 4, 4, 16, 3), C.moe(16, 2, 1, 6, 4, 1),
-           C.moe(64, 100, 8, 28, 128, 100), C.moe(24, 130, 5, 6, 2, 1), C.moe(64, 16, 4)]
+           C.moe(64, 100, 8, 28, 128, 100), C.moe(24, 130, 5, 6, 2, 1), C.moe(64, 16, 4), C.moe(192, 5, 3, 3, 4, 2), C.moe(64, 2, 2)]
 
 
 def router_ids(m):
@@ -223,7 +223,7 @@ def test_experts_alone(mlp, hidden, dtype):
     ff.load({k: v.to(DT[dtype]).to(DEV) for k, v in w.items()})
     cache = Cache([], [], 64, 1, DT[dtype], DEV)
     f = C.as_float(w)
-    for rows in (1, 5, 130):
+    for rows in (1, 5, 130) + ((700,) if mlp["expert"]["ff"] >= 64 else ()):          # (up to experts of several tiles of every size)
         x = torch.randn(rows, hidden).to(DT[dtype])
         ctx = StepContext([(0, 0, [0] * rows)], [[]], cache, DEV)
         got = ff.forward(x.to(DEV), ctx)

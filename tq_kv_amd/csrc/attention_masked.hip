@@ -448,6 +448,14 @@ template <> struct Piece<bf16_t, 8> {
     }
 };
 
+// VEC neighbouring float32 numbers (at a multiple of 16 bytes where VEC is 8)
+template <int VEC> __device__ __forceinline__ void float_piece(const float* p, float* v) {
+    if constexpr (VEC == 8) {
+        const float4 a = reinterpret_cast<const float4*>(p)[0], b = reinterpret_cast<const float4*>(p)[1];
+        v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
+    } else v[0] = p[0];
+}
+
 template <typename TA, int VEC>
 __global__ __launch_bounds__(1024)
 void projection_store_kernel(const ProjectionArgs a) {
@@ -459,8 +467,10 @@ void projection_store_kernel(const ProjectionArgs a) {
     auto load = [&](int at, float* v) {
         Piece<TA, VEC>::load(row + at, v);
         if (a.bias) {
+            float b[VEC];
+            float_piece<VEC>(a.bias + at, b);
 #pragma unroll
-            for (int j = 0; j < VEC; ++j) v[j] += a.bias[at + j];
+            for (int j = 0; j < VEC; ++j) v[j] += b[j];
         }
     };
     if (a.gate_out)
@@ -492,8 +502,11 @@ void projection_store_kernel(const ProjectionArgs a) {
         const float inv = is_q ? inv_q : inv_k;
         auto normed = [&](int at, float* v) {
             load(at, v);
+            if (!w) return;
+            float f[VEC];
+            float_piece<VEC>(w + (at - part_at), f);
 #pragma unroll
-            for (int j = 0; j < VEC; ++j) v[j] *= w ? inv * w[at - part_at + j] : 1.f;
+            for (int j = 0; j < VEC; ++j) v[j] *= inv * f[j];
         };
         float x[VEC];
         normed(e, x);
@@ -514,11 +527,11 @@ void projection_store_kernel(const ProjectionArgs a) {
                 const int angle = a.style == 2 ? off / 2 : first ? off : off - half;
                 float y[VEC];
                 normed(e - off + partner, y);
+                float c[VEC], s[VEC];
+                float_piece<VEC>(ct + angle, c);
+                float_piece<VEC>(st + angle, s);
 #pragma unroll
-                for (int j = 0; j < VEC; ++j) {
-                    const float c = ct[angle + j], s = st[angle + j];
-                    x[j] = first ? x[j] * c - y[j] * s : x[j] * c + y[j] * s;
-                }
+                for (int j = 0; j < VEC; ++j) x[j] = first ? x[j] * c[j] - y[j] * s[j] : x[j] * c[j] + y[j] * s[j];
             }
         }
         TA* dst = is_q ? (TA*)a.q_out + (size_t)t * nq + in_part
@@ -721,7 +734,8 @@ extern "C" int tqk_projection_store(const void* rows, int act_dtype, long long r
         const long long pieces = (nq + nk + vec - 1) / vec;
         return (unsigned)(pieces >= 1024 ? 1024 : (pieces + TQK_WAVE - 1) / TQK_WAVE * TQK_WAVE);
     };
-    const bool aligned = row_stride % 8 == 0 && (((uintptr_t)rows | (uintptr_t)keys | (uintptr_t)q_out) & 15) == 0;
+    const bool aligned = row_stride % 8 == 0 && (((uintptr_t)rows | (uintptr_t)keys | (uintptr_t)q_out | (uintptr_t)bias | (uintptr_t)q_norm_w | (uintptr_t)k_norm_w |
+                                                  (uintptr_t)cos_table | (uintptr_t)sin_table) & 15) == 0;
     if (act_dtype == TQK_BF16 && key_dim % 8 == 0 && (rot_dim == 0 || style == 2 || rot_dim % 16 == 0) && aligned) {
         // steps of many tokens: values with the lanes along the tokens
         const bool apart = kv && n_tokens > 64 && value_dim % 8 == 0;

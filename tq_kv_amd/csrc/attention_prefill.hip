@@ -103,6 +103,9 @@ struct PrefillArgs {
     int window, chunk;       // chunk > 0: positions fall into chunks and see nothing of an earlier one
     float scale;
     float cap;               // > 0: scores become cap tanh(scale s / cap)
+    const void* sink;        // [heads] or null: exp(sink_h) joins the softmax's denominator
+    int sink_f32;
+    const float* head_scale; // [tokens, heads] or null: the heads' outputs are multiplied by it
     bf16_t* out;
     int n_heads, n_kv_heads, n_tiles;
     int tq_shift;            // log2 of the queries per tile
@@ -461,6 +464,7 @@ void attention_prefill_kernel(const PrefillArgs p) {
                     mine = m0 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m0 - m);
                     theirs = m1 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m1 - m);
                     w.l = w.l * mine + l1 * theirs;
+                    w.m = m;
                 }
 #pragma unroll
                 for (int i = 0; i < 16; ++i) w.o[dt][i] = w.o[dt][i] * mine + hand[i * STEP] * theirs;
@@ -472,7 +476,12 @@ void attention_prefill_kernel(const PrefillArgs p) {
     if (live && w.set == 0) {
         // out^T[element 32 dt + 8 (i/4) + 4 h + i%4][this column]
         bf16_t* orow = p.out + ((size_t)(tok0 + qi) * p.n_heads + head) * D;
-        const float inv = 1.f / l;
+        // (a live column has seen a key: what the sums are set against is a score, in powers of two)
+        if (p.sink) {
+            const float sink = p.sink_f32 ? ((const float*)p.sink)[head] : to_float(((const bf16_t*)p.sink)[head]);
+            l += __builtin_amdgcn_exp2f(sink * 1.44269504088896340736f - w.m);
+        }
+        const float inv = (p.head_scale ? p.head_scale[(size_t)(tok0 + qi) * p.n_heads + head] : 1.f) / l;
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
@@ -541,9 +550,10 @@ extern "C" int tqk_attention_prefill_capped(const void* q, const void* keys, con
                                             const int32_t* page_table, int table_width, int n_seqs, int n_pages,
                                             const int32_t* tile_seq, const int32_t* tile_tok0, const int32_t* tile_count,
                                             int n_tiles, int tile_queries, const int32_t* seq_start, const int32_t* seq_new,
-                                            int window, int chunk, float scale, float cap, void* out, int n_tokens, int n_heads, int n_kv_heads,
-                                            int head_dim, void* stream) {
-    TQK_REQUIRE(cap >= 0.f, "tqk_attention_prefill: negative cap");
+                                            int window, int chunk, float scale, float cap, const void* sink, int sink_dtype, const float* head_scale,
+                                            void* out, int n_tokens, int n_heads, int n_kv_heads, int head_dim, void* stream) {
+    TQK_REQUIRE(cap >= 0.f && scale > 0.f, "tqk_attention_prefill: negative cap, or a scale that is not positive");
+    TQK_REQUIRE(!sink || sink_dtype == TQK_F32 || sink_dtype == TQK_BF16, "tqk_attention_prefill: unknown dtype %d of the sink", sink_dtype);
     TQK_REQUIRE(q && keys && values && tok_pos && page_table && tile_seq && tile_tok0 && tile_count && seq_start && seq_new && out,
                 "tqk_attention_prefill: null pointer");
     TQK_REQUIRE(n_tokens >= 0 && n_tiles >= 0 && n_heads > 0 && n_kv_heads > 0, "tqk_attention_prefill: bad sizes");
@@ -561,6 +571,7 @@ extern "C" int tqk_attention_prefill_capped(const void* q, const void* keys, con
     a.tok_pos = tok_pos; a.page_table = page_table; a.table_width = table_width;
     a.tile_seq = tile_seq; a.tile_tok0 = tile_tok0; a.tile_count = tile_count;
     a.seq_start = seq_start; a.seq_new = seq_new; a.window = window; a.chunk = chunk; a.scale = scale; a.cap = cap;
+    a.sink = sink; a.sink_f32 = sink_dtype == TQK_F32; a.head_scale = head_scale;
     a.out = (bf16_t*)out; a.n_heads = n_heads; a.n_kv_heads = n_kv_heads; a.n_tiles = n_tiles;
     a.tq_shift = tile_queries == 16 ? 4 : (tile_queries == 32 ? 5 : (tile_queries == 64 ? 6 : 7));
     prefill_heads(n_heads / n_kv_heads, tile_queries, &a.heads_per_block, &a.head_chunks);
@@ -603,5 +614,5 @@ extern "C" int tqk_attention_prefill(const void* q, const void* keys, const void
                                      int window, float scale, void* out, int n_tokens, int n_heads, int n_kv_heads,
                                      int head_dim, void* stream) {
     return tqk_attention_prefill_capped(q, keys, values, tok_pos, page_table, table_width, n_seqs, n_pages, tile_seq, tile_tok0, tile_count, n_tiles,
-                                        tile_queries, seq_start, seq_new, window, 0, scale, 0.f, out, n_tokens, n_heads, n_kv_heads, head_dim, stream);
+                                        tile_queries, seq_start, seq_new, window, 0, scale, 0.f, nullptr, 0, nullptr, out, n_tokens, n_heads, n_kv_heads, head_dim, stream);
 }

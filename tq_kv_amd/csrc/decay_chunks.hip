@@ -18,7 +18,7 @@
 
 #define DC_CHUNK 64
 #define DC_MAX_D 128
-#define DC_PROW 72                  // numbers between rows of P in LDS (16 bytes more than a row, against bank conflicts)
+#define DC_P_NUMBERS (32 * 40 + 32 * 72)
 #define DC_LOG_FLOOR -40.f
 #define DC_LOG2E 1.4426950408889634f
 
@@ -38,6 +38,9 @@ __device__ __forceinline__ void two_parts(float x, uint16_t& hi, uint16_t& lo) {
 __device__ __forceinline__ dc_floatx4_t mfma(const dc_pack8& a, const dc_pack8& b, dc_floatx4_t c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, b.v, c, 0, 0, 0);
 }
+
+// Where row t of P begins in LDS: the first 32 tokens see 32 keys at most, the others 64; rows are 16 bytes longer than that, against bank conflicts.
+__device__ __forceinline__ int p_row(int t) { return t < 32 ? 40 * t : 32 * 40 + 72 * (t - 32); }
 
 struct DecayChunkArgs {
     const bf16_t *r, *k, *v;
@@ -171,8 +174,8 @@ void decay_apply_kernel(const DecayChunkArgs a) {
     float* L = reinterpret_cast<float*>(dc_lds);                    // [64][ls]
     uint16_t* rl = reinterpret_cast<uint16_t*>(L + DC_CHUNK * ls);  // [64][rs]
     uint16_t* kl = rl + DC_CHUNK * rs;                              // [64][rs]
-    uint16_t* p_hi = kl + DC_CHUNK * rs;                            // [64][DC_PROW]
-    uint16_t* p_lo = p_hi + DC_CHUNK * DC_PROW;
+    uint16_t* p_hi = kl + DC_CHUNK * rs;                            // rows at p_row(t)
+    uint16_t* p_lo = p_hi + DC_P_NUMBERS;
     const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
     const int g = lane / 16, r = lane % 16;
     const int head = blockIdx.x, chunk = blockIdx.y;
@@ -248,7 +251,7 @@ void decay_apply_kernel(const DecayChunkArgs a) {
     }
     // P: the earlier sets' part (a lane has token r, keys 4 g ..), zeros for the keys behind, then the set's own pairs
     {
-        const int at = (first + r) * DC_PROW + 4 * g;
+        const int at = p_row(first + r) + 4 * g;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             if (j > (wave | 1)) continue;
@@ -285,7 +288,7 @@ void decay_apply_kernel(const DecayChunkArgs a) {
             sum = fmaf(bits_float(ra.y & 0xffff) * bits_float(ka.y & 0xffff), __builtin_amdgcn_exp2f(x.z - y.z), sum);
             sum = fmaf(bits_float(ra.y >> 16) * bits_float(ka.y >> 16), __builtin_amdgcn_exp2f(x.w - y.w), sum);
         }
-        two_parts(sum, p_hi[(first + t) * DC_PROW + first + q], p_lo[(first + t) * DC_PROW + first + q]);
+        two_parts(sum, p_hi[p_row(first + t) + first + q], p_lo[p_row(first + t) + first + q]);
     }
     {
         // the diagonal: the bonus, a token's channels in pieces of four dealt out to its four lanes
@@ -301,7 +304,7 @@ void decay_apply_kernel(const DecayChunkArgs a) {
         }
         sum += __shfl_xor(sum, 16, TQK_WAVE);
         sum += __shfl_xor(sum, 32, TQK_WAVE);
-        if (g == 0) two_parts(sum, p_hi[(first + r) * DC_PROW + first + r], p_lo[(first + r) * DC_PROW + first + r]);
+        if (g == 0) two_parts(sum, p_hi[p_row(first + r) + first + r], p_lo[p_row(first + r) + first + r]);
     }
     __builtin_amdgcn_wave_barrier();
 
@@ -353,7 +356,7 @@ void decay_apply_kernel(const DecayChunkArgs a) {
     for (int ks = 0; ks < 2; ++ks) {
         if (32 * ks > first + 15) continue;                         // keys behind all of the wave's tokens
         dc_pack8 ph, pl;
-        const int at = (first + r) * DC_PROW + 32 * ks + 8 * g;
+        const int at = p_row(first + r) + 32 * ks + 8 * g;
         ph.q = *reinterpret_cast<const uint4*>(p_hi + at);
         pl.q = *reinterpret_cast<const uint4*>(p_lo + at);
 #pragma unroll
@@ -444,7 +447,7 @@ extern "C" int tqk_decay_apply(const void* r, const void* k, const void* v, long
                 "tqk_decay_apply: operands are not aligned");
     if (n_chunks == 0) return 0;
     a.r = (const bf16_t*)r; a.bonus = bonus; a.norm_w = norm_weight; a.eps = eps; a.gate = (const bf16_t*)gate; a.gate_stride = gate_stride; a.out = (bf16_t*)out;
-    const size_t lds = (size_t)DC_CHUNK * ((d + 4) * sizeof(float) + 2 * (d + 8) * sizeof(uint16_t) + 2 * DC_PROW * sizeof(uint16_t));
+    const size_t lds = (size_t)DC_CHUNK * ((d + 4) * sizeof(float) + 2 * (d + 8) * sizeof(uint16_t)) + 2 * DC_P_NUMBERS * sizeof(uint16_t);
     dim3 grid(heads, n_chunks);
     hipStream_t s = (hipStream_t)stream;
 #define TQK_DA(NG, KB) do { \

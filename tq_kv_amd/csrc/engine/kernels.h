@@ -47,7 +47,7 @@ TQ_QUERY(int, attention_prefill_supported, int);
 TQ_QUERY(int, attention_prefill_tile, int, int, int, int);
 TQ_KERNEL(attention_prefill, cptr, cptr, cptr, ci32, ci32, int, int, int, ci32, ci32, ci32, int, int, ci32, ci32, int, float, void*, int, int,
           int, int, void*);
-TQ_KERNEL(attention_prefill_capped, cptr, cptr, cptr, ci32, ci32, int, int, int, ci32, ci32, ci32, int, int, ci32, ci32, int, int, float, float, void*, int,
+TQ_KERNEL(attention_prefill_capped, cptr, cptr, cptr, ci32, ci32, int, int, int, ci32, ci32, ci32, int, int, ci32, ci32, int, int, float, float, cptr, int, cf32, void*, int,
           int, int, int, void*);
 TQ_KERNEL(swiglu, cptr, void*, int, int, int, void*);
 TQ_KERNEL(gated_act, cptr, void*, int, int, int, int, float, float, void*);
@@ -70,6 +70,7 @@ TQ_QUERY(int, moe_max_experts);
 TQ_QUERY(int, moe_max_tiles, int, int, int);
 TQ_QUERY(int, moe_tile_rows);
 TQ_QUERY(int, grouped_supported, int);
+TQ_QUERY(int, grouped_max_tile, int, int);
 TQ_KERNEL(moe_product_mfma, cptr, ci32, cptr, long long, void*, int, int, int, int, float, float, ci32, ci32, ci32, ci32, int, int, void*);
 TQ_KERNEL(head_product, cptr, int, long long, long long, cptr, void*, int, long long, long long, cf32, cptr, int, long long, int, int, int, int, void*);
 TQ_KERNEL(moe_route, cptr, int, cptr, int, int, int, int, float, int, int32_t*, float*, cptr, float*, int, void*);
@@ -77,6 +78,7 @@ TQ_KERNEL(moe_group, ci32, int, int, int, int, int32_t*, int32_t*, int32_t*, int
 TQ_KERNEL(moe_product, cptr, int, ci32, cptr, int, long long, void*, int, int, int, int, float, float, ci32, ci32, ci32, ci32, int, void*);
 TQ_KERNEL(moe_scale_rows, cptr, int, ci32, cf32, int, void*, float*, int, int, void*);
 TQ_KERNEL(moe_route_grouped, cptr, int, cptr, int, int, int, int, cf32, int, int, float, int32_t*, float*, int, void*);
+TQ_KERNEL(moe_choose_grouped, cf32, int, int, cf32, int, int, float, int32_t*, float*, int, void*);
 TQ_QUERY(int, moe_combine_norm_supported, int);
 TQ_KERNEL(moe_combine_norm, float*, cptr, int, ci32, cf32, int, cptr, cptr, cf32, cptr, float, cptr, int, float, void*, int, int, void*);
 TQ_KERNEL(moe_combine, cptr, int, ci32, cf32, int, cptr, cptr, cf32, cptr, float, void*, int, int, void*);
@@ -133,6 +135,8 @@ TQ_KERNEL(rows_remember, cptr, int, float*, long long, ci32, ci32, ci32, int, in
 TQ_QUERY(int, decay_chunks_supported, int, int);
 TQ_KERNEL(decay_local, cptr, cptr, long long, cf32, ci32, ci32, int, float*, float*, int, int, int, void*);
 TQ_KERNEL(decay_apply, cptr, cptr, cptr, long long, cf32, cf32, ci32, ci32, int, float*, cf32, float, cptr, long long, void*, int, int, int, void*);
+TQ_QUERY(int, low_rank_mfma_supported, int, int);
+TQ_KERNEL(low_rank_decay_mfma, cf32, cptr, cf32, float*, int, int, int, void*);
 TQ_QUERY(int, low_rank_max);
 TQ_KERNEL(low_rank_decay, cf32, cf32, cf32, float*, int, int, int, void*);
 TQ_QUERY(int, mlstm_chunks_supported, int, int);

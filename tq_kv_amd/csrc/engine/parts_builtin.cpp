@@ -634,15 +634,15 @@ private:
                                          n_kv_heads_, head_dim_, value_dim_, c.stream);
                 return;
             }
-            // keys and values of one size, every earlier position visible (or a plain window), no sink: the prompt kernel of the
-            // plain attention takes the cap as an option
-            if (!rows && policy().prefill_mfma && value_dim_ == head_dim_ && keep_first_ == 0 && !sink_ && !hs &&
+            // keys and values of one size, every earlier position visible (or a plain window): the prompt kernel of the plain
+            // attention takes the cap, the sink and the heads' gates as options
+            if (!rows && policy().prefill_mfma && value_dim_ == head_dim_ && keep_first_ == 0 && scale_ > 0.f &&
                 K::attention_prefill_supported.raw(head_dim_)) {
                 const int tile = tile_for(c);
                 const Tiles t = last_rows ? c.last_tiles(tile) : c.query_tiles(tile);
                 K::attention_prefill_capped(q.data, entry.keys.data, entry.values.data, tok_pos, table.dev, table.width, c.n_seqs, n_pages, t.seq, t.tok0,
-                                            t.count, t.n, tile, c.dev.seq_start, c.dev.seq_new, window_, chunk_, scale_, cap_, out.data, n, n_heads_, n_kv_heads_,
-                                            head_dim_, c.stream);
+                                            t.count, t.n, tile, c.dev.seq_start, c.dev.seq_new, window_, chunk_, scale_, cap_, sink, sink_dtype, hs, out.data, n,
+                                            n_heads_, n_kv_heads_, head_dim_, c.stream);
                 return;
             }
             if (!rows && policy().prefill_mfma) {
@@ -756,7 +756,7 @@ private:
             return decode_kernel(c, q, entry, c.dev.tok_pos, table.dev, table.width, out);
         // (not for steps of one token per sequence: tiles of one query are what the plain kernel does anyway,
         // and such a step may be replayed from a graph, which cannot carry the tiles' upload)
-        if (q.dtype == BF16 && !c.all_decode && policy().prefill_mfma && K::attention_prefill_supported.raw(head_dim_)) {
+        if (q.dtype == BF16 && !c.all_decode && policy().prefill_mfma && scale_ > 0.f && K::attention_prefill_supported.raw(head_dim_)) {
             const int tile = tile_for(c);
             const Tiles t = c.query_tiles(tile);
             K::attention_prefill(q.data, entry.keys.data, entry.values.data, c.dev.tok_pos, table.dev, table.width, c.n_seqs, n_pages, t.seq, t.tok0,
@@ -781,7 +781,7 @@ private:
             k_gather_rows(c, whole, c.dev.last_seq, n, rows_table);
             return decode_kernel(c, q, entry, c.dev.last_pos, (const int32_t*)rows_table.data, table.width, out);
         }
-        if (q.dtype == BF16 && policy().prefill_mfma && K::attention_prefill_supported.raw(head_dim_)) {
+        if (q.dtype == BF16 && policy().prefill_mfma && scale_ > 0.f && K::attention_prefill_supported.raw(head_dim_)) {
             const int tile = tile_for(c);
             const Tiles t = c.last_tiles(tile);
             K::attention_prefill(q.data, entry.keys.data, entry.values.data, c.dev.last_pos, table.dev, table.width, c.n_seqs, n_pages, t.seq, t.tok0,

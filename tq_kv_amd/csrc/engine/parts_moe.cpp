@@ -128,6 +128,7 @@ public:
     }
     void load(Loaded& t, hipStream_t stream) override {
         router_ = take(t, n_router_);
+        if (by_choice_) w_router_ = make_weight(router_, 1, true, stream);
         if (!n_correction_.empty()) correction_ = as_floats(stored_correction_ = take(t, n_correction_), stream);
         // all experts' weights in two tensors: [experts, gate rows then up rows, hidden] and [experts, hidden, inter]
         std::vector<OwnedPtr> gu, down;
@@ -178,7 +179,8 @@ private:
         const bool on_cores = dtype == BF16 && gate_up_->t.dtype == BF16 && down_->t.dtype == BF16 && policy().skinny && hidden_ % 8 == 0 &&
                               inter_ % 8 == 0 && K::grouped_supported.raw((int)hidden_) != 0;
         const int64_t per_expert = pairs / n_experts_;
-        const int tile_m = !on_cores ? K::moe_tile_rows.raw() : per_expert >= 48 ? 64 : per_expert >= 24 ? 32 : 16;
+        const bool big = on_cores && per_expert >= 96 && K::grouped_max_tile.raw((int)inter_, (int)hidden_) >= 128 && K::grouped_max_tile.raw((int)hidden_, (int)inter_) >= 128;
+        const int tile_m = !on_cores ? K::moe_tile_rows.raw() : big ? 128 : per_expert >= 48 ? 64 : per_expert >= 24 ? 32 : 16;
         const int max_tiles = K::moe_max_tiles.raw((int)pairs, n_experts_, tile_m);
         Tensor idx = c.alloc(I32, {n, top_}), weight = c.alloc(F32, {n, top_});
         Tensor pair_pos = c.alloc(I32, {pairs}), sorted_tok = c.alloc(I32, {pairs});
@@ -190,9 +192,15 @@ private:
         Tensor shared_scale;
         const bool gate_in_route = shared_gate_ && shared_gate_->t.dtype == router_->t.dtype;
         if (shared_gate_) shared_scale = c.alloc(F32, {n});
-        if (by_choice_)
-            K::moe_route_grouped(x.x.data, dtype, router_->t.data, router_->t.dtype, n_experts_ + identity_, (int)hidden_, top_,
-                                 correction_ ? (const float*)correction_->t.data : nullptr, n_groups_, keep_groups_, weight_floor_, (int32_t*)idx.data,
+        const float* correction = correction_ ? (const float*)correction_->t.data : nullptr;
+        const int outputs = n_experts_ + identity_;
+        if (by_choice_ && dtype == BF16 && router_->t.dtype == BF16 && n > mid_max_rows() && outputs % 8 == 0 && hidden_ % 8 == 0 && policy().library && !null_device()) {
+            // steps of many tokens: the logits as a product of bfloat16 operands with float32 sums (which is what the kernel below forms too)
+            const Tensor z = linear(c, x.x, w_router_, nullptr, F32).t;
+            K::moe_choose_grouped((const float*)z.data, outputs, top_, correction, n_groups_, keep_groups_, weight_floor_, (int32_t*)idx.data, (float*)weight.data, (int)n,
+                                  c.stream);
+        } else if (by_choice_)
+            K::moe_route_grouped(x.x.data, dtype, router_->t.data, router_->t.dtype, outputs, (int)hidden_, top_, correction, n_groups_, keep_groups_, weight_floor_, (int32_t*)idx.data,
                                  (float*)weight.data, (int)n, c.stream);
         else
             K::moe_route(x.x.data, dtype, router_->t.data, router_->t.dtype, n_experts_, (int)hidden_, top_, router_scale_, (renormalize_ ? 1 : 0) | (sigmoid_scores_ ? 2 : 0), (int32_t*)idx.data,
@@ -265,6 +273,7 @@ private:
     std::string n_router_, n_expert_, n_gate_, n_up_, n_down_, n_shared_;
     std::shared_ptr<FeedForward> shared_;
     OwnedPtr router_, gate_up_, down_;
+    Weight w_router_;
 };
 
 }  // namespace

@@ -111,6 +111,9 @@ public:
         rank_ = w1->t.shape[0];
         if (rank_ > K::low_rank_max.raw()) raise(TQE_ERR_WEIGHTS, "time_mixing: a decay of rank %lld is more than the kernel takes (%d)", (long long)rank_, K::low_rank_max.raw());
         w_w1_ = make_weight(w1, 1, false, stream);
+        // (bfloat16 on the matrix cores takes the matrix as it is)
+        on_cores_ = w2->t.dtype == BF16 && K::low_rank_mfma_supported.raw((int)rank_, (int)hd) != 0;
+        if (on_cores_) w2_rows_ = w2;
         w2_ = transposed(as_floats(w2, stream), stream);
         w0_ = as_floats(take(t, n_w0_), stream);
         u_ = as_floats(take(t, n_u_), stream);
@@ -168,7 +171,10 @@ public:
         const Tensor low = linear(c, mix(4), w_w1_, nullptr, F32).t;
         Tensor log_decay = c.alloc(F32, {n, hd});
         const float* logs = (const float*)log_decay.data;
-        K::low_rank_decay((const float*)low.data, (const float*)w2_->t.data, (const float*)w0_->t.data, (float*)log_decay.data, (int)n, (int)rank_, (int)hd, c.stream);
+        if (dtype == BF16 && on_cores_)
+            K::low_rank_decay_mfma((const float*)low.data, w2_rows_->t.data, (const float*)w0_->t.data, (float*)log_decay.data, (int)n, (int)rank_, (int)hd, c.stream);
+        else
+            K::low_rank_decay((const float*)low.data, (const float*)w2_->t.data, (const float*)w0_->t.data, (float*)log_decay.data, (int)n, (int)rank_, (int)hd, c.stream);
         const float* u = (const float*)u_->t.data;
         const float* norm_w = (const float*)norm_w_->t.data;
         Tensor gated = c.alloc(dtype, {n, hd});
@@ -213,7 +219,8 @@ private:
     float eps_;
     std::string n_mu_, n_r_, n_k_, n_v_, n_g_, n_o_, n_w1_, n_w2_, n_w0_, n_u_, n_norm_;
     Weight w_all_, w_in_[4], w_o_, w_w1_;      // the four products stacked (or not defined); each of them
-    OwnedPtr mu_, w2_, w0_, u_, norm_w_;
+    OwnedPtr mu_, w2_, w2_rows_, w0_, u_, norm_w_;      // w2_: [rank, channels] float32; w2_rows_: as the checkpoint has it
+    bool on_cores_ = false;
     Loaded stored_;
 };
 constexpr const char* TimeMixing::MIXES[];

@@ -226,6 +226,105 @@ void grouped_mfma_kernel(GroupedArgs p) {
         }
 }
 
+// Tiles of up to 128 rows (prompts: experts that get so many): both operands staged in LDS.  A block of four waves takes 128 rows of x and 128 rows of
+// the weight (gated: 64 gate rows and the 64 up rows that go with them), a wave 64 of each: every piece a wave reads from LDS serves four
+// products.  K in steps of 64, the next step's pieces on their way into registers while the block multiplies; rows in LDS are 16 bytes longer than a
+// step, so that the 16 rows a load of the matrix cores' operands touches fall on different banks.  The weight goes in as A and x as B, so a lane
+// holds four neighbouring features of one row and stores them together.
+#define GRP_BIG_ROWS 128
+#define GRP_BIG_K 64
+#define GRP_BIG_STRIDE (GRP_BIG_K + 8)
+template <bool GATED>
+__global__ __launch_bounds__(GRP_WAVES * TQK_WAVE)
+void grouped_big_kernel(GroupedArgs p) {
+    __shared__ __attribute__((aligned(16))) uint16_t x_lds[GRP_BIG_ROWS * GRP_BIG_STRIDE], w_lds[GRP_BIG_ROWS * GRP_BIG_STRIDE];
+    const int tile = blockIdx.y;
+    if (tile >= *p.n_tiles) return;
+    const int group = p.tile_group[tile], row0 = p.tile_row0[tile], n_rows = p.tile_rows[tile];
+    const int tid = threadIdx.x, wave = tid / TQK_WAVE, lane = tid % TQK_WAVE;
+    const int g = lane / 16, r16 = lane % 16;
+    constexpr int FEATURES = GATED ? 64 : 128;          // output features of a block
+    const int n0 = blockIdx.x * FEATURES;
+    const bf16_t* wg = p.w + (size_t)group * p.w_group_stride;
+    // where the thread's pieces of a step come from: row tid / 8 + 32 j, 16-byte piece tid % 8 (rows beyond the tile or the weight: one that is there)
+    const int piece = tid % 8, prow = tid / 8;
+    const bf16_t* x_src[4];
+    const bf16_t* w_src[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int r = prow + 32 * j;
+        const int rr = row0 + min(r, n_rows - 1);
+        x_src[j] = (const bf16_t*)p.x + (size_t)(p.x_rows ? p.x_rows[rr] : rr) * p.x_row_stride + piece * 8;
+        const int f = GATED ? min(n0 + (r & 63), p.N - 1) + (r >= 64 ? p.N : 0) : min(n0 + r, p.N - 1);
+        w_src[j] = wg + (size_t)f * p.K + piece * 8;
+    }
+    grp_bf16x8_t xr[4], wr[4];
+    // the wave's 64 rows of x, and its 64 rows of the weight: gated, 32 gate rows and the 32 up rows that go with them
+    const int xb = (wave & 1) * 64, wb = (wave >> 1) * (GATED ? 32 : 64);
+    grp_floatx4_t acc[4][4];                            // [weight tile][x tile]
+#pragma unroll
+    for (int a = 0; a < 4; ++a)
+#pragma unroll
+        for (int b = 0; b < 4; ++b) acc[a][b] = grp_floatx4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        xr[j] = *reinterpret_cast<const grp_bf16x8_t*>(x_src[j]);
+        wr[j] = *reinterpret_cast<const grp_bf16x8_t*>(w_src[j]);
+    }
+    for (int k0 = 0; k0 < p.K; k0 += GRP_BIG_K) {
+        __syncthreads();                                // everyone has done with the step before
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            *reinterpret_cast<grp_bf16x8_t*>(x_lds + (prow + 32 * j) * GRP_BIG_STRIDE + piece * 8) = xr[j];
+            *reinterpret_cast<grp_bf16x8_t*>(w_lds + (prow + 32 * j) * GRP_BIG_STRIDE + piece * 8) = wr[j];
+        }
+        __syncthreads();
+        const int next = min(k0 + GRP_BIG_K, p.K - GRP_BIG_K);      // (after the last step: the last step's again, dropped)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            xr[j] = *reinterpret_cast<const grp_bf16x8_t*>(x_src[j] + next);
+            wr[j] = *reinterpret_cast<const grp_bf16x8_t*>(w_src[j] + next);
+        }
+        __builtin_amdgcn_sched_barrier(0);              // (asked for in front of the products, not behind them)
+#pragma unroll
+        for (int ks = 0; ks < 2; ++ks) {
+            grp_pack8 wa[4], xa[4];
+#pragma unroll
+            for (int a = 0; a < 4; ++a) {
+                const int wrow = GATED ? wb + (a & 1) * 16 + (a >> 1) * 64 : wb + a * 16;
+                wa[a].q = *reinterpret_cast<const uint4*>(w_lds + (wrow + r16) * GRP_BIG_STRIDE + ks * 32 + g * 8);
+                xa[a].q = *reinterpret_cast<const uint4*>(x_lds + (xb + a * 16 + r16) * GRP_BIG_STRIDE + ks * 32 + g * 8);
+            }
+#pragma unroll
+            for (int a = 0; a < 4; ++a)
+#pragma unroll
+                for (int b = 0; b < 4; ++b) acc[a][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wa[a].v, xa[b].v, acc[a][b], 0, 0, 0);
+        }
+    }
+    // the lane holds features 4 g + i of a weight tile, for row r16 of an x tile
+#pragma unroll
+    for (int b = 0; b < 4; ++b) {
+        const int r = xb + 16 * b + r16;
+        if (r >= n_rows) continue;
+        bf16_t* out = (bf16_t*)p.y + (size_t)(row0 + r) * p.y_row_stride;
+#pragma unroll
+        for (int a = 0; a < (GATED ? 2 : 4); ++a) {
+            const int n = n0 + wb + 16 * a + 4 * g;
+            uint16_t v[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                float f = acc[a][b][i];
+                if (GATED) {
+                    // gate and up rounded as stored products would be, then the gate in float32
+                    f = gate_value(p.gate, p.gate_limit, p.gate_alpha, to_float(from_float<bf16_t>(f)), to_float(from_float<bf16_t>(acc[GATED ? a + 2 : a][b][i])));
+                } else if (p.activated) f = act_value(p.gate, p.gate_limit, p.gate_alpha, to_float(from_float<bf16_t>(f)));
+                v[i] = float_to_bf16_bits(f);
+            }
+            if (n + 4 <= p.N) *reinterpret_cast<uint2*>(out + n) = make_uint2(v[0] | ((uint32_t)v[1] << 16), v[2] | ((uint32_t)v[3] << 16));
+        }
+    }
+}
+
 template <bool GATED>
 static int launch_grouped(const GroupedArgs& a, int tiles, hipStream_t s) {
     // rows of a tile: up to 16, 32 or 64; features of a wave: 16 or 32 (32 where there are enough of them to fill the chip)
@@ -244,14 +343,16 @@ static int launch_grouped(const GroupedArgs& a, int tiles, hipStream_t s) {
 }
 
 extern "C" int tqk_grouped_supported(int K) { return K % 8 == 0; }
+/* the most rows of a tile that a product of these sizes takes */
+extern "C" int tqk_grouped_max_tile(int N, int K) { return K % GRP_BIG_K == 0 && N % 4 == 0 ? GRP_BIG_ROWS : 64; }
 
-/* The experts' products over tiles of up to tile_m rows (16, 32 or 64: what tqk_moe_group was given). */
+/* The experts' products over tiles of up to tile_m rows (16, 32, 64 or, where tqk_grouped_max_tile says so, 128: what tqk_moe_group was given). */
 extern "C" int tqk_moe_product_mfma(const void* x, const int32_t* x_rows, const void* w, long long expert_stride, void* y, int N, int K,
                                     int gated, int gate, float limit, float alpha, const int32_t* tile_expert, const int32_t* tile_row0,
                                     const int32_t* tile_rows, const int32_t* n_tiles, int max_tiles, int tile_m, void* stream) {
     TQK_REQUIRE(x && w && y && tile_expert && tile_row0 && tile_rows && n_tiles, "tqk_moe_product_mfma: null pointer");
     TQK_REQUIRE(N > 0 && K > 0 && K % 8 == 0 && max_tiles >= 0 && max_tiles <= 65535, "tqk_moe_product_mfma: bad sizes (N %d, K %d, %d tiles)", N, K, max_tiles);
-    TQK_REQUIRE(tile_m == 16 || tile_m == 32 || tile_m == 64, "tqk_moe_product_mfma: tiles of %d rows", tile_m);
+    TQK_REQUIRE(tile_m == 16 || tile_m == 32 || tile_m == 64 || (tile_m == GRP_BIG_ROWS && tqk_grouped_max_tile(N, K) >= tile_m), "tqk_moe_product_mfma: tiles of %d rows", tile_m);
     TQK_REQUIRE(gated >= 0 && gated <= 2, "tqk_moe_product_mfma: gated must be 0, 1 or 2, got %d", gated);
     TQK_REQUIRE(!gated || (gate >= 0 && gate < TQK_GATE_KINDS), "tqk_moe_product_mfma: unknown gate %d", gate);
     TQK_REQUIRE(expert_stride >= (long long)(gated == 1 ? 2 : 1) * N * K && expert_stride % 8 == 0, "tqk_moe_product_mfma: experts overlap or are not aligned");
@@ -263,6 +364,14 @@ extern "C" int tqk_moe_product_mfma(const void* x, const int32_t* x_rows, const 
     a.y = y; a.y_row_stride = N;
     a.N = N; a.K = K; a.gate = gate; a.gate_limit = limit; a.gate_alpha = alpha; a.activated = gated == 2;
     a.tile_group = tile_expert; a.tile_row0 = tile_row0; a.tile_rows = tile_rows; a.n_tiles = n_tiles; a.tile_rows_max = tile_m;
+    if (tile_m == GRP_BIG_ROWS) {
+        TQK_REQUIRE(((uintptr_t)y & 7) == 0, "tqk_moe_product_mfma: y must be 8-byte aligned");
+        const int features = gated == 1 ? 64 : 128;
+        dim3 grid((N + features - 1) / features, max_tiles);
+        if (gated == 1) grouped_big_kernel<true><<<grid, GRP_WAVES * TQK_WAVE, 0, (hipStream_t)stream>>>(a);
+        else grouped_big_kernel<false><<<grid, GRP_WAVES * TQK_WAVE, 0, (hipStream_t)stream>>>(a);
+        return tqk_check_launch("tqk_moe_product_mfma");
+    }
     return gated == 1 ? launch_grouped<true>(a, max_tiles, (hipStream_t)stream) : launch_grouped<false>(a, max_tiles, (hipStream_t)stream);
 }
 

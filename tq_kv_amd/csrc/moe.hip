@@ -145,38 +145,43 @@ void moe_route_kernel(const TA* __restrict__ x, int n_tokens, const TW* __restri
     }
 }
 
+// The wave's largest value, by moves between the lanes' registers (inside rows of 16 lanes, then from row to row): no trip through LDS.
+template <int CTRL, int ROWS> __device__ __forceinline__ float lanes_max(float v) {
+    return fmaxf(v, __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(__builtin_bit_cast(int, -INFINITY), __builtin_bit_cast(int, v), CTRL, ROWS, 0xf, false)));
+}
+__device__ __forceinline__ float lanes_wave_max(float v) {
+    v = lanes_max<0x111, 0xf>(v);           // from the lane 1, 2, 4, 8 places before
+    v = lanes_max<0x112, 0xf>(v);
+    v = lanes_max<0x114, 0xf>(v);
+    v = lanes_max<0x118, 0xf>(v);
+    v = lanes_max<0x142, 0xa>(v);           // a row's last lane to the row behind it, then the second row's to the upper two
+    v = lanes_max<0x143, 0xc>(v);
+    return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), TQK_WAVE - 1));
+}
 // The lane's largest of z[lane], z[lane + 64], ... below n, then the wave's: the lower index wins a tie.  In every lane of the wave.
 __device__ __forceinline__ int wave_argmax(const volatile float* z, int n, int lane, float& best) {
     int at = 0x7fffffff;
-    best = -INFINITY;
+    float mine = -INFINITY;
     for (int e = lane; e < n; e += TQK_WAVE) {
         const float v = z[e];
-        if (v > best) { best = v; at = e; }
+        if (v > mine) { mine = v; at = e; }
     }
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-        const float ov = __shfl_xor(best, o, TQK_WAVE);
-        const int oe = __shfl_xor(at, o, TQK_WAVE);
-        if (ov > best || (ov == best && oe < at)) { best = ov; at = oe; }
+    best = lanes_wave_max(mine);
+    uint64_t who = __ballot(mine == best && at != 0x7fffffff);
+    int first = 0x7fffffff;
+    while (who) {                           // (one lane, but for equal values)
+        const int l = __builtin_ctzll(who);
+        first = min(first, __builtin_amdgcn_readlane(at, l));
+        who &= who - 1;
     }
-    return at;
+    return first;
 }
 
-// Choice by score plus correction within the best groups of neighbours.  What a token's wave keeps of the experts lies in LDS and is
-// read and written by that wave alone, each element by one lane between two of the wave's exchanges.
-template <typename TA, typename TW, int NT>
-__global__ __launch_bounds__(MOE_ROUTE_WAVES * TQK_WAVE)
-void moe_route_grouped_kernel(const TA* __restrict__ x, int n_tokens, const TW* __restrict__ w, int n_experts, int hidden, int top, const float* __restrict__ correction,
-                              int n_groups, int keep, float floor, int32_t* __restrict__ idx, float* __restrict__ weight) {
-    __shared__ float logits[NT * MOE_MAX_EXPERTS];
-    __shared__ volatile float choices[NT * MOE_MAX_EXPERTS], groups[NT * MOE_MAX_EXPERTS];
-    const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
-    route_logits<TA, TW, NT>(x, n_tokens, w, n_experts, hidden, (const TW*)nullptr, (float*)nullptr, logits);
-    const int t = blockIdx.x * NT + wave;
-    if (wave >= NT || t >= n_tokens) return;
-    volatile float* z = logits + wave * MOE_MAX_EXPERTS;           // the logits, then the scores
-    volatile float* choice = choices + wave * MOE_MAX_EXPERTS;
-    volatile float* group = groups + wave * MOE_MAX_EXPERTS;
+// Choice by score plus correction within the best groups of neighbours, by a token's wave.  What it keeps of the experts lies in LDS (z: the logits,
+// then the scores; choice; group) and is read and written by that wave alone, each element by one lane between two of the wave's exchanges.
+__device__ __forceinline__ void choose_grouped(volatile float* z, volatile float* choice, volatile float* group, int n_experts, int top,
+                                               const float* __restrict__ correction, int n_groups, int keep, float floor, int lane, int32_t* __restrict__ idx,
+                                               float* __restrict__ weight) {
     float m = -INFINITY;
     for (int e = lane; e < n_experts; e += TQK_WAVE) m = fmaxf(m, z[e]);
     m = wave_max(m);
@@ -220,12 +225,40 @@ void moe_route_grouped_kernel(const TA* __restrict__ x, int n_tokens, const TW* 
         const float s = z[e];
         chosen += s;
         if (lane == 0) {
-            idx[(size_t)t * top + k] = e;
-            weight[(size_t)t * top + k] = s;
+            idx[k] = e;
+            weight[k] = s;
         }
     }
     if (lane == 0)
-        for (int k = 0; k < top; ++k) weight[(size_t)t * top + k] /= chosen + floor;
+        for (int k = 0; k < top; ++k) weight[k] /= chosen + floor;
+}
+
+template <typename TA, typename TW, int NT>
+__global__ __launch_bounds__(MOE_ROUTE_WAVES * TQK_WAVE)
+void moe_route_grouped_kernel(const TA* __restrict__ x, int n_tokens, const TW* __restrict__ w, int n_experts, int hidden, int top, const float* __restrict__ correction,
+                              int n_groups, int keep, float floor, int32_t* __restrict__ idx, float* __restrict__ weight) {
+    __shared__ float logits[NT * MOE_MAX_EXPERTS];
+    __shared__ volatile float choices[NT * MOE_MAX_EXPERTS], groups[NT * MOE_MAX_EXPERTS];
+    const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
+    route_logits<TA, TW, NT>(x, n_tokens, w, n_experts, hidden, (const TW*)nullptr, (float*)nullptr, logits);
+    const int t = blockIdx.x * NT + wave;
+    if (wave >= NT || t >= n_tokens) return;
+    choose_grouped(logits + wave * MOE_MAX_EXPERTS, choices + wave * MOE_MAX_EXPERTS, groups + wave * MOE_MAX_EXPERTS, n_experts, top, correction, n_groups, keep, floor,
+                   lane, idx + (size_t)t * top, weight + (size_t)t * top);
+}
+
+// the same from logits that a product has left, [tokens, n_experts] float32: a wave a token
+__global__ __launch_bounds__(MOE_ROUTE_TOKENS * TQK_WAVE)
+void moe_choose_grouped_kernel(const float* __restrict__ logits, int n_tokens, int n_experts, int top, const float* __restrict__ correction, int n_groups, int keep,
+                               float floor, int32_t* __restrict__ idx, float* __restrict__ weight) {
+    __shared__ volatile float zs[MOE_ROUTE_TOKENS * MOE_MAX_EXPERTS], choices[MOE_ROUTE_TOKENS * MOE_MAX_EXPERTS], groups[MOE_ROUTE_TOKENS * MOE_MAX_EXPERTS];
+    const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
+    const int t = blockIdx.x * MOE_ROUTE_TOKENS + wave;
+    if (t >= n_tokens) return;
+    volatile float* z = zs + wave * MOE_MAX_EXPERTS;
+    for (int e = lane; e < n_experts; e += TQK_WAVE) z[e] = logits[(size_t)t * n_experts + e];
+    choose_grouped(z, choices + wave * MOE_MAX_EXPERTS, groups + wave * MOE_MAX_EXPERTS, n_experts, top, correction, n_groups, keep, floor, lane, idx + (size_t)t * top,
+                   weight + (size_t)t * top);
 }
 
 // ---- group -----------------------------------------------------------------------------------
@@ -538,6 +571,18 @@ extern "C" int tqk_moe_route_grouped(const void* x, int act_dtype, const void* w
     else return tqk_fail("tqk_moe_route_grouped: unknown dtypes %d, %d", act_dtype, w_dtype);
 #undef TQK_ROUTE
     return tqk_check_launch("tqk_moe_route_grouped");
+}
+
+extern "C" int tqk_moe_choose_grouped(const float* logits, int n_experts, int top, const float* correction, int n_groups, int keep, float floor, int32_t* idx,
+                                      float* weight, int n_tokens, void* stream) {
+    TQK_REQUIRE(logits && idx && weight, "tqk_moe_choose_grouped: null pointer");
+    TQK_REQUIRE(n_experts > 0 && n_experts <= MOE_MAX_EXPERTS, "tqk_moe_choose_grouped: %d experts, the kernel takes 1 to %d", n_experts, MOE_MAX_EXPERTS);
+    TQK_REQUIRE(n_groups > 0 && n_experts % n_groups == 0 && keep > 0 && keep <= n_groups && top > 0 && top <= keep * (n_experts / n_groups) && n_tokens >= 0,
+                "tqk_moe_choose_grouped: top %d of %d of %d groups of %d experts", top, keep, n_groups, n_experts);
+    if (n_tokens == 0) return 0;
+    moe_choose_grouped_kernel<<<(n_tokens + MOE_ROUTE_TOKENS - 1) / MOE_ROUTE_TOKENS, MOE_ROUTE_TOKENS * TQK_WAVE, 0, (hipStream_t)stream>>>(
+        logits, n_tokens, n_experts, top, correction, n_groups, keep, floor, idx, weight);
+    return tqk_check_launch("tqk_moe_choose_grouped");
 }
 
 extern "C" int tqk_moe_group(const int32_t* idx, int n_tokens, int top, int n_experts, int tile_m, int32_t* pair_pos, int32_t* sorted_tok,

@@ -82,9 +82,9 @@ void rows_remember_kernel(const T* __restrict__ x, float* __restrict__ state, lo
     state[(size_t)seq_slot[s] * state_stride + e] = to_float(x[t * W + e]);
 }
 
-// A block takes TT tokens and blockDim.x channels, a thread one channel of all of them; tanh(low) of the block's tokens lies in LDS,
-// [rank][TT].  A decay's sum runs over the rank in order, whatever the step holds.
-template <int TT>
+// A block takes TT tokens and CH blockDim.x channels, a thread CH channels (blockDim.x apart) of all of them; tanh(low) of the block's tokens lies in
+// LDS, [rank][TT].  A decay's sum runs over the rank in order, whatever the step holds.
+template <int TT, int CH>
 __global__ __launch_bounds__(256)
 void low_rank_decay_kernel(const float* __restrict__ low, const float* __restrict__ w2, const float* __restrict__ bias, float* __restrict__ log_decay,
                            int n_tokens, int rank, int channels) {
@@ -95,25 +95,111 @@ void low_rank_decay_kernel(const float* __restrict__ low, const float* __restric
         tanh_low[i] = tt < nt ? tanhf(low[(size_t)(t0 + tt) * rank + r]) : 0.f;
     }
     __syncthreads();
-    const int c = blockIdx.x * blockDim.x + threadIdx.x;
-    if (c >= channels) return;
-    float acc[TT];
+    const int c0 = blockIdx.x * CH * blockDim.x + threadIdx.x;
+    int c[CH];
 #pragma unroll
-    for (int tt = 0; tt < TT; ++tt) acc[tt] = 0.f;
-#pragma unroll 8
+    for (int k = 0; k < CH; ++k) c[k] = min(c0 + k * (int)blockDim.x, channels - 1);
+    float acc[CH][TT];
+#pragma unroll
+    for (int k = 0; k < CH; ++k)
+#pragma unroll
+        for (int tt = 0; tt < TT; ++tt) acc[k][tt] = 0.f;
+#pragma unroll 4
     for (int r = 0; r < rank; ++r) {
-        const float w = w2[(size_t)r * channels + c];
+        float w[CH];
+#pragma unroll
+        for (int k = 0; k < CH; ++k) w[k] = w2[(size_t)r * channels + c[k]];
 #pragma unroll
         for (int tt = 0; tt < TT; tt += 4) {
             const float4 z = *reinterpret_cast<const float4*>(tanh_low + r * TT + tt);
-            acc[tt] = fmaf(w, z.x, acc[tt]);
-            acc[tt + 1] = fmaf(w, z.y, acc[tt + 1]);
-            acc[tt + 2] = fmaf(w, z.z, acc[tt + 2]);
-            acc[tt + 3] = fmaf(w, z.w, acc[tt + 3]);
+#pragma unroll
+            for (int k = 0; k < CH; ++k) {
+                acc[k][tt] = fmaf(w[k], z.x, acc[k][tt]);
+                acc[k][tt + 1] = fmaf(w[k], z.y, acc[k][tt + 1]);
+                acc[k][tt + 2] = fmaf(w[k], z.z, acc[k][tt + 2]);
+                acc[k][tt + 3] = fmaf(w[k], z.w, acc[k][tt + 3]);
+            }
         }
     }
-    const float b = bias[c];
-    for (int tt = 0; tt < nt; ++tt) log_decay[(size_t)(t0 + tt) * channels + c] = -expf(acc[tt] + b);
+#pragma unroll
+    for (int k = 0; k < CH; ++k) {
+        if (c0 + k * (int)blockDim.x >= channels) continue;
+        const float b = bias[c[k]];
+#pragma unroll
+        for (int tt = 0; tt < TT; ++tt)
+            if (tt < nt) log_decay[(size_t)(t0 + tt) * channels + c[k]] = -expf(acc[k][tt] + b);
+    }
+}
+
+// The same on the matrix cores, for a second matrix w2 [channels, rank] of bfloat16 numbers (which go in exactly; tanh(low) goes in as the sum of two).
+// v_mfma_f32_16x16x32_bf16: A a tile of 16 channels, B 16 tokens, so a lane holds four neighbouring channels of one token.  A block of four
+// waves takes 16 tokens and 64 TILES channels.
+typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 tm_bf16x8_t;
+typedef __attribute__((__vector_size__(4 * sizeof(float)))) float tm_floatx4_t;
+union tm_pack8 {
+    tm_bf16x8_t v;
+    uint16_t u[8];
+};
+#define TM_MAX_CORE_RANK 256
+template <int KB>
+__global__ __launch_bounds__(256)
+void low_rank_decay_mfma_kernel(const float* __restrict__ low, const bf16_t* __restrict__ w2, const float* __restrict__ bias, float* __restrict__ log_decay,
+                                int n_tokens, int rank, int channels, int tiles) {
+    const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
+    const int g = lane / 16, r = lane % 16;
+    const int t = blockIdx.y * 16 + r;
+    const float* lr = low + (size_t)min(t, n_tokens - 1) * rank;
+    tm_pack8 hi[KB], lo[KB];
+#pragma unroll
+    for (int kb = 0; kb < KB; ++kb) {
+        const int e0 = 32 * kb + 8 * g, at = e0 < rank ? e0 : 0;
+        const float4 a = *reinterpret_cast<const float4*>(lr + at), b = *reinterpret_cast<const float4*>(lr + at + 4);
+        const float z[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            const float y = e0 < rank ? tanhf(z[e]) : 0.f;
+            hi[kb].u[e] = float_to_bf16_bits(y);
+            lo[kb].u[e] = float_to_bf16_bits(y - __uint_as_float((uint32_t)hi[kb].u[e] << 16));
+        }
+    }
+    for (int j = 0; j < tiles; ++j) {
+        const int c0 = ((blockIdx.x * tiles + j) * 4 + wave) * 16;
+        if (c0 >= channels) break;
+        const bf16_t* wr = w2 + (size_t)min(c0 + r, channels - 1) * rank;
+        tm_floatx4_t acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int kb = 0; kb < KB; ++kb) {
+            const int e0 = 32 * kb + 8 * g;
+            const tm_bf16x8_t w = *reinterpret_cast<const tm_bf16x8_t*>(wr + (e0 < rank ? e0 : 0));     // (beyond the rank tanh(low) is zero)
+            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, hi[kb].v, acc, 0, 0, 0);
+            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, lo[kb].v, acc, 0, 0, 0);
+        }
+        const int c = c0 + 4 * g;
+        if (t < n_tokens && c < channels) {                 // (channels: a multiple of four)
+            const float4 b = *reinterpret_cast<const float4*>(bias + c);
+            *reinterpret_cast<float4*>(log_decay + (size_t)t * channels + c) = make_float4(-expf(acc[0] + b.x), -expf(acc[1] + b.y), -expf(acc[2] + b.z), -expf(acc[3] + b.w));
+        }
+    }
+}
+
+extern "C" int tqk_low_rank_mfma_supported(int rank, int channels) { return rank > 0 && rank % 8 == 0 && rank <= TM_MAX_CORE_RANK && channels > 0 && channels % 4 == 0; }
+
+extern "C" int tqk_low_rank_decay_mfma(const float* low, const void* w2, const float* bias, float* log_decay, int n_tokens, int rank, int channels, void* stream) {
+    TQK_REQUIRE(low && w2 && bias && log_decay, "tqk_low_rank_decay_mfma: null pointer");
+    TQK_REQUIRE(n_tokens >= 0 && tqk_low_rank_mfma_supported(rank, channels), "tqk_low_rank_decay_mfma: rank %d and %d channels are not taken", rank, channels);
+    TQK_REQUIRE((((uintptr_t)low | (uintptr_t)w2 | (uintptr_t)bias | (uintptr_t)log_decay) & 15) == 0, "tqk_low_rank_decay_mfma: operands must be 16-byte aligned");
+    if (n_tokens == 0) return 0;
+    const int token_tiles = (n_tokens + 15) / 16, channel_blocks = (channels + 63) / 64;
+    TQK_REQUIRE(token_tiles <= 65535, "tqk_low_rank_decay_mfma: %d tokens are more than the grid takes", n_tokens);
+    // few tokens: a block per 64 channels; many: a block keeps its tokens' numbers for up to eight times as many
+    int tiles = 1;
+    while (tiles < 8 && (long long)token_tiles * (channel_blocks / (2 * tiles)) >= 512) tiles *= 2;
+    dim3 grid((channel_blocks + tiles - 1) / tiles, token_tiles);
+    hipStream_t s = (hipStream_t)stream;
+#define TQK_LRM(KB) low_rank_decay_mfma_kernel<KB><<<grid, 256, 0, s>>>(low, (const bf16_t*)w2, bias, log_decay, n_tokens, rank, channels, tiles)
+    if (rank <= 32) TQK_LRM(1); else if (rank <= 64) TQK_LRM(2); else if (rank <= 128) TQK_LRM(4); else TQK_LRM(8);
+#undef TQK_LRM
+    return tqk_check_launch("tqk_low_rank_decay_mfma");
 }
 
 extern "C" int tqk_token_mixes(const void* x, int dtype, const float* mu, int n_mixes, float* state, long long state_stride, const int32_t* tok_seq,
@@ -158,13 +244,13 @@ extern "C" int tqk_low_rank_decay(const float* low, const float* w2, const float
     TQK_REQUIRE(rank <= TM_MAX_RANK, "tqk_low_rank_decay: a rank of %d, the kernel takes up to %d", rank, TM_MAX_RANK);
     if (n_tokens == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
-    if (n_tokens <= 16) {
+    if (n_tokens <= 256) {
         dim3 grid((channels + TQK_WAVE - 1) / TQK_WAVE, (n_tokens + 3) / 4);
-        low_rank_decay_kernel<4><<<grid, TQK_WAVE, (size_t)rank * 4 * sizeof(float), s>>>(low, w2, bias, log_decay, n_tokens, rank, channels);
+        low_rank_decay_kernel<4, 1><<<grid, TQK_WAVE, (size_t)rank * 4 * sizeof(float), s>>>(low, w2, bias, log_decay, n_tokens, rank, channels);
     } else {
-        dim3 grid((channels + 255) / 256, (n_tokens + 15) / 16);
+        dim3 grid((channels + 511) / 512, (n_tokens + 15) / 16);
         TQK_REQUIRE(grid.y <= 65535, "tqk_low_rank_decay: %d tokens are more than the grid takes", n_tokens);
-        low_rank_decay_kernel<16><<<grid, 256, (size_t)rank * 16 * sizeof(float), s>>>(low, w2, bias, log_decay, n_tokens, rank, channels);
+        low_rank_decay_kernel<16, 2><<<grid, 256, (size_t)rank * 16 * sizeof(float), s>>>(low, w2, bias, log_decay, n_tokens, rank, channels);
     }
     return tqk_check_launch("tqk_low_rank_decay");
 }

@@ -174,13 +174,14 @@ int tqk_attention_prefill(const void* q, const void* keys, const void* values, c
                           int window, float scale, void* out, int n_tokens, int n_heads, int n_kv_heads,
                           int head_dim, void* stream);
 /* The same with a cap on the scores: cap > 0 makes them cap tanh(scale q.k / cap) before the softmax; chunk > 0: a query sees no
- * position of an earlier chunk of `chunk` positions than its own. */
+ * position of an earlier chunk of `chunk` positions than its own; sink [heads] (or null) adds exp(sink_h) to the softmax's denominator; head_scale
+ * [tokens, heads] float32 (or null) multiplies the heads' outputs.  The scale must be positive. */
 int tqk_attention_prefill_capped(const void* q, const void* keys, const void* values, const int32_t* tok_pos,
                                  const int32_t* page_table, int table_width, int n_seqs, int n_pages,
                                  const int32_t* tile_seq, const int32_t* tile_tok0, const int32_t* tile_count,
                                  int n_tiles, int tile_queries, const int32_t* seq_start, const int32_t* seq_new,
-                                 int window, int chunk, float scale, float cap, void* out, int n_tokens, int n_heads, int n_kv_heads,
-                                 int head_dim, void* stream);
+                                 int window, int chunk, float scale, float cap, const void* sink, int sink_dtype, const float* head_scale,
+                                 void* out, int n_tokens, int n_heads, int n_kv_heads, int head_dim, void* stream);
 
 /* out[t, i] = silu(gate_up[t, i]) * gate_up[t, inter + i] */
 int tqk_swiglu(const void* gate_up, void* out, int act_dtype, int n_tokens, int inter, void* stream);
@@ -266,16 +267,21 @@ int tqk_moe_route(const void* x, int act_dtype, const void* w_router, int w_dtyp
                   int mode, int32_t* idx, float* weight, const void* gate_w, float* gate_out, int n_tokens, void* stream);
 int tqk_moe_route_grouped(const void* x, int act_dtype, const void* w_router, int w_dtype, int n_experts, int hidden, int top, const float* correction,
                           int n_groups, int keep, float floor, int32_t* idx, float* weight, int n_tokens, void* stream);
+/* the same choice from logits [tokens, n_experts] float32 that a product has left */
+int tqk_moe_choose_grouped(const float* logits, int n_experts, int top, const float* correction, int n_groups, int keep, float floor, int32_t* idx,
+                           float* weight, int n_tokens, void* stream);
 int tqk_moe_group(const int32_t* idx, int n_tokens, int top, int n_experts, int tile_m, int32_t* pair_pos, int32_t* sorted_tok,
                   int32_t* tile_expert, int32_t* tile_row0, int32_t* tile_rows, int32_t* n_tiles, void* stream);
 int tqk_moe_product(const void* x, int act_dtype, const int32_t* x_rows, const void* w, int w_dtype, long long expert_stride, void* y,
                     int N, int K, int gated, int gate, float limit, float alpha, const int32_t* tile_expert,
                     const int32_t* tile_row0, const int32_t* tile_rows, const int32_t* n_tiles, int max_tiles, void* stream);
 /* Many small products on the matrix cores (grouped.hip), bfloat16 weights, K a multiple of 8: the experts' products over
- * tiles of up to tile_m rows (16, 32 or 64, what tqk_moe_group was given; tqk_moe_product takes tqk_moe_tile_rows()), and
+ * tiles of up to tile_m rows (16, 32, 64, or 128 where tqk_grouped_max_tile(N, K) of the product says so; what tqk_moe_group was given;
+ * tqk_moe_product takes tqk_moe_tile_rows()), and
  * y[t, h, :N] = scale[t, h] * W_h x[t, h, :K] for every token and head (x bfloat16 or float32, w [heads][N][K], y
  * bfloat16 or float32, strides in values, scale float32 [tokens, heads] or null). */
 int tqk_grouped_supported(int K);
+int tqk_grouped_max_tile(int N, int K);
 int tqk_moe_product_mfma(const void* x, const int32_t* x_rows, const void* w, long long expert_stride, void* y, int N, int K,
                          int gated, int gate, float limit, float alpha, const int32_t* tile_expert, const int32_t* tile_row0,
                          const int32_t* tile_rows, const int32_t* n_tiles, int max_tiles, int tile_m, void* stream);
@@ -523,6 +529,10 @@ int tqk_rows_remember(const void* x, int dtype, float* state, long long state_st
                       const int32_t* seq_slot, int n_seqs, int width, void* stream);
 int tqk_low_rank_max(void);
 int tqk_low_rank_decay(const float* low, const float* w2, const float* bias, float* log_decay, int n_tokens, int rank, int channels, void* stream);
+
+/* The same on the matrix cores with w2 [channels, rank] bfloat16 as the checkpoint has it (tanh(low) in two bfloat16 parts). */
+int tqk_low_rank_mfma_supported(int rank, int channels);
+int tqk_low_rank_decay_mfma(const float* low, const void* w2, const float* bias, float* log_decay, int n_tokens, int rank, int channels, void* stream);
 
 /* That recurrence for steps of many tokens, bfloat16, on the matrix cores (decay_chunks.hip), where tqk_decay_chunks_supported(d, dv).  Chunks of up
  * to 64 tokens as tqk_ssm_chunks takes them: tqk_decay_local leaves a chunk's own part of the state [chunks][heads][d][dv] and its decays

@@ -405,7 +405,7 @@ def attention_prefill(q, keys, values, tok_pos, page_table, tile_seq, tile_tok0,
         _dev(tile_seq, "tile_seq", torch.int32, (n_tiles,)), _dev(tile_tok0, "tile_tok0", torch.int32, (n_tiles,)),
         _dev(tile_count, "tile_count", torch.int32, (n_tiles,)), n_tiles, int(tile_queries),
         _dev(seq_start, "seq_start", torch.int32, (n_seqs,)), _dev(seq_new, "seq_new", torch.int32, (n_seqs,)),
-        int(window or 0), int(chunk), ctypes.c_float(scale), ctypes.c_float(cap), _dev(out, "out", torch.bfloat16, (n, n_heads * head_dim)),
+        int(window or 0), int(chunk), ctypes.c_float(scale), ctypes.c_float(cap), None, 0, None, _dev(out, "out", torch.bfloat16, (n, n_heads * head_dim)),
         n, n_heads, n_kv_heads, head_dim, _stream()), "attention_prefill")
     return out
 
