@@ -42,10 +42,10 @@ def mixer_spec(kind, m, hidden, eps, own_kv=True, cache_window=None):
 
 
 SC = C.scaled(8.0, 1.0, 4.0, 64)
-MIXERS = [C.wkv(3, 20), C.wkv(1, 1), C.wkv(2, 2), C.wkv(3, 10), C.wkv(4, 64), C.wkv(2, 128), C.wkv(1, 200), C.wkv(2, 68), C.wkv(5, 7), C.wkv(1, 300), C.wkv(6, 32),
+MIXERS = [C.wkv(3, 20), C.wkv(1, 1), C.wkv(2, 2), C.wkv(3, 10), C.wkv(5, 64), C.wkv(2, 128), C.wkv(1, 200), C.wkv(2, 68), C.wkv(5, 7), C.wkv(1, 300), C.wkv(6, 32),
           C.attention(6, 3, 24, 40, 37, 16, base=300.0, scale=0.35, scaling=SC), C.attention(1, 1, 2, 1, 1, 0), C.attention(3, 3, 10, 14, 9, 6, scaling=SC),
           C.attention(8, 2, 64, 64, 64, 64, scaling=C.scaled(4.0, 0.5, 8.0, 200)), C.attention(16, 2, 128, 128, 100, 32), C.attention(2, 1, 160, 200, 200, 40, scale=0.05),
-          C.attention(5, 5, 32, 32, 130, 2), C.attention(6, 2, 96, 64, 1000, 96, scale=0.2), C.attention(40, 2, 32, 48, 63, 32), C.attention(4, 2, 64, 64, 129, 20),
+          C.attention(5, 5, 32, 32, 130, 2), C.attention(6, 2, 96, 64, 1000, 96, scale=0.2), C.attention(40, 2, 32, 48, 63, 32), C.attention(6, 2, 64, 64, 129, 20),
           C.attention(4, 1, 16, 24, 65, 16, scale=-0.3)]
 
 
@@ -254,7 +254,10 @@ def test_a_group_is_kept_for_its_best_choice_score_and_choices_stay_inside():
 # ---- whole models ----------------------------------------------------------------------------------------
 _MODELS = {}
 MAKERS = {"mixed": C.config_mixed, "ones": C.config_ones, "odd": C.config_odd, "wkv": lambda: C.config_single("wkv"), "slow": lambda: C.config_single("wkv"),
-          "attention": lambda: C.config_single("attention")}
+          "attention": lambda: C.config_single("attention"),
+          "wide1030": lambda: C.config(61, 1030, [(C.attention(2, 1, 16, 16, 40, 8), C.moe(24, 3, 2, 1)), (C.wkv(2, 8), C.moe(16, 2, 1))]),
+          "wide4160": lambda: C.config(61, 4160, [(C.wkv(2, 16), C.moe(32, 3, 2, 1)), (C.attention(2, 1, 16, 16, 40, 8), None), (C.wkv(2, 16), C.moe(32, 2, 2))]),
+          "wide9000": lambda: C.config(61, 9000, [(C.wkv(2, 16), C.moe(32, 2, 1)), (C.attention(2, 2, 32, 32, 50, 32), C.moe(16, 2, 1, 1))])}
 
 
 def model(name, tmp_path_factory):
@@ -344,6 +347,26 @@ def test_whole_prompts_and_every_cut(name, dtype, tmp_path_factory):
         close(got, want, dtype, "cuts %s" % cuts[:4])
         if dtype == "float32":          # no sum depends on the cut: states are carried exactly
             assert torch.equal(got, whole), "float32 logits depend on the cut %s" % cuts[:4]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["wide1030", "wide4160", "wide9000"])
+def test_streams_of_other_widths(name, dtype, tmp_path_factory):
+    """Widths that take the kernels between the layers in all their shapes (experts' sum, stream and next norm in one pass of one or two pieces a
+    thread, or in two kernels), in prompts and in steps of few and of many sequences."""
+    cfg, w, eng = engine(name, dtype, tmp_path_factory, slots=24)
+    toks = C.tokens(60, cfg["vocab"], 5)
+    want = wanted(name, cfg, w, toks)
+    for cuts in ([], [40], list(range(50, 60))):
+        close(run_cut(eng, toks, cuts), want, dtype, "cuts %s" % cuts[:3])
+    reqs = [C.tokens(2 + i % 3, cfg["vocab"], 300 + i) for i in range(20)]
+    slots = [eng.open() for _ in reqs]
+    eng.step([(s, r[:-1], []) for s, r in zip(slots, reqs)])
+    got = eng.step([(s, r[-1:], [0]) for s, r in zip(slots, reqs)])
+    for i in (0, 1, 2, 19):
+        close(got[i:i + 1], wanted(name, cfg, w, reqs[i]), dtype, "sequence %d" % i, [len(reqs[i]) - 1])
+    for s in slots:
+        eng.close(s)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)

@@ -19,7 +19,7 @@ def draw(seed):
     layers = []
     for i in range(r.randint(1, 6)):
         lenders = [k for k, ((t, m), _) in enumerate(layers) if t == "attention" and "kv_from" not in m]
-        window = r.choice([1, 3, 16, 40, 64, 100, 128, 136, 200, 1000])
+        window = r.choice([1, 3, 16, 40, 64, 100, 128, 139, 200, 1000])
         if r.random() < 0.4:
             mix = C.wkv(r.choice([1, 2, 3, 6]), r.choice([3, 4, 8, 12, 32, 48, 64, 96, 128]))
         elif lenders and r.random() < 0.5:

@@ -133,52 +133,66 @@ void low_rank_decay_kernel(const float* __restrict__ low, const float* __restric
 
 // The same on the matrix cores, for a second matrix w2 [channels, rank] of bfloat16 numbers (which go in exactly; tanh(low) goes in as the sum of two).
 // v_mfma_f32_16x16x32_bf16: A a tile of 16 channels, B 16 tokens, so a lane holds four neighbouring channels of one token.  A block of four
-// waves takes 16 tokens and 64 TILES channels.
+// waves takes 16 tokens and 64 `tiles` channels.
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 tm_bf16x8_t;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float tm_floatx4_t;
-union tm_pack8 {
-    tm_bf16x8_t v;
-    uint16_t u[8];
-};
 #define TM_MAX_CORE_RANK 256
 template <int KB>
 __global__ __launch_bounds__(256)
 void low_rank_decay_mfma_kernel(const float* __restrict__ low, const bf16_t* __restrict__ w2, const float* __restrict__ bias, float* __restrict__ log_decay,
                                 int n_tokens, int rank, int channels, int tiles) {
+    __shared__ __attribute__((aligned(16))) uint2 hi_half[KB * TQK_WAVE * 2], lo_half[KB * TQK_WAVE * 2];       // tanh(low) in the lanes' order: [32 of the rank][lane][half of its eight]
     const int wave = threadIdx.x / TQK_WAVE, lane = threadIdx.x % TQK_WAVE;
     const int g = lane / 16, r = lane % 16;
-    const int t = blockIdx.y * 16 + r;
-    const float* lr = low + (size_t)min(t, n_tokens - 1) * rank;
-    tm_pack8 hi[KB], lo[KB];
+    for (int i = threadIdx.x; i < KB * TQK_WAVE * 2; i += 256) {
+        const int ln = i / 2 % TQK_WAVE, e0 = 32 * (i / (2 * TQK_WAVE)) + 8 * (ln / 16) + 4 * (i % 2);
+        const float4 a = *reinterpret_cast<const float4*>(low + (size_t)min(blockIdx.y * 16 + ln % 16, n_tokens - 1) * rank + (e0 < rank ? e0 : 0));
+        const float z[4] = {a.x, a.y, a.z, a.w};
+        uint32_t hi[4], lo[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const float y = e0 < rank ? tanhf(z[e]) : 0.f;
+            hi[e] = float_to_bf16_bits(y);
+            lo[e] = float_to_bf16_bits(y - __uint_as_float(hi[e] << 16));
+        }
+        hi_half[i] = make_uint2(hi[0] | hi[1] << 16, hi[2] | hi[3] << 16);
+        lo_half[i] = make_uint2(lo[0] | lo[1] << 16, lo[2] | lo[3] << 16);
+    }
+    __syncthreads();
+    tm_bf16x8_t hi[KB], lo[KB];
 #pragma unroll
     for (int kb = 0; kb < KB; ++kb) {
-        const int e0 = 32 * kb + 8 * g, at = e0 < rank ? e0 : 0;
-        const float4 a = *reinterpret_cast<const float4*>(lr + at), b = *reinterpret_cast<const float4*>(lr + at + 4);
-        const float z[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
-#pragma unroll
-        for (int e = 0; e < 8; ++e) {
-            const float y = e0 < rank ? tanhf(z[e]) : 0.f;
-            hi[kb].u[e] = float_to_bf16_bits(y);
-            lo[kb].u[e] = float_to_bf16_bits(y - __uint_as_float((uint32_t)hi[kb].u[e] << 16));
-        }
+        hi[kb] = *reinterpret_cast<const tm_bf16x8_t*>(hi_half + (kb * TQK_WAVE + lane) * 2);
+        lo[kb] = *reinterpret_cast<const tm_bf16x8_t*>(lo_half + (kb * TQK_WAVE + lane) * 2);
     }
-    for (int j = 0; j < tiles; ++j) {
-        const int c0 = ((blockIdx.x * tiles + j) * 4 + wave) * 16;
-        if (c0 >= channels) break;
+    const int t = blockIdx.y * 16 + r, first = (blockIdx.x * tiles * 4 + wave) * 16;
+    auto weights = [&](int c0, tm_bf16x8_t (&w)[KB]) {
         const bf16_t* wr = w2 + (size_t)min(c0 + r, channels - 1) * rank;
-        tm_floatx4_t acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int kb = 0; kb < KB; ++kb) {
             const int e0 = 32 * kb + 8 * g;
-            const tm_bf16x8_t w = *reinterpret_cast<const tm_bf16x8_t*>(wr + (e0 < rank ? e0 : 0));     // (beyond the rank tanh(low) is zero)
-            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, hi[kb].v, acc, 0, 0, 0);
-            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, lo[kb].v, acc, 0, 0, 0);
+            w[kb] = *reinterpret_cast<const tm_bf16x8_t*>(wr + (e0 < rank ? e0 : 0));     // (beyond the rank tanh(low) is zero)
+        }
+    };
+    tm_bf16x8_t w[KB], ahead[KB];
+    weights(first, w);
+    for (int j = 0; j < tiles; ++j) {
+        const int c0 = first + 64 * j;
+        if (c0 >= channels) break;
+        if (j + 1 < tiles) weights(c0 + 64, ahead);
+        tm_floatx4_t acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int kb = 0; kb < KB; ++kb) {
+            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[kb], hi[kb], acc, 0, 0, 0);
+            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[kb], lo[kb], acc, 0, 0, 0);
         }
         const int c = c0 + 4 * g;
         if (t < n_tokens && c < channels) {                 // (channels: a multiple of four)
             const float4 b = *reinterpret_cast<const float4*>(bias + c);
             *reinterpret_cast<float4*>(log_decay + (size_t)t * channels + c) = make_float4(-expf(acc[0] + b.x), -expf(acc[1] + b.y), -expf(acc[2] + b.z), -expf(acc[3] + b.w));
         }
+#pragma unroll
+        for (int kb = 0; kb < KB; ++kb) w[kb] = ahead[kb];
     }
 }
 
@@ -193,7 +207,7 @@ extern "C" int tqk_low_rank_decay_mfma(const float* low, const void* w2, const f
     TQK_REQUIRE(token_tiles <= 65535, "tqk_low_rank_decay_mfma: %d tokens are more than the grid takes", n_tokens);
     // few tokens: a block per 64 channels; many: a block keeps its tokens' numbers for up to eight times as many
     int tiles = 1;
-    while (tiles < 8 && (long long)token_tiles * (channel_blocks / (2 * tiles)) >= 512) tiles *= 2;
+    while (tiles < 8 && (long long)token_tiles * (channel_blocks / (2 * tiles)) >= 1024) tiles *= 2;
     dim3 grid((channel_blocks + tiles - 1) / tiles, token_tiles);
     hipStream_t s = (hipStream_t)stream;
 #define TQK_LRM(KB) low_rank_decay_mfma_kernel<KB><<<grid, 256, 0, s>>>(low, (const bf16_t*)w2, bias, log_decay, n_tokens, rank, channels, tiles)
