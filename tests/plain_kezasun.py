@@ -12,13 +12,13 @@ Notation: T tokens, D the model's width, m the layer's share of what it computes
 
 Mixers:
 
-    time mixing   h^-_t = h_(t-1) (zero in front of the first token); each of r, k, v, g, w reads h + (h^- - h) mu of its own.
+    time mixing   h^-_t = h_(t-1) (0 where there is none); the input of r is h + (h^- - h) mu_r, and so for k, v, g and w.
                r = W_r ., k = W_k ., v = W_v . per head; a_t = exp(-exp(A_2 tanh(A_1 .) + b)) per head and key channel;
                o_t = S_(t-1)^T r_t + (sum_i u_i k_i r_i) v_t,  S_t = diag(a_t) S_(t-1) + k_t v_t^T from S = 0;
                o is divided per head by its root mean square, times a weight over all heads' elements, times silu(W_g .), W_o
     attention  q = W_q h + b_q, k = W_k h + b_k, v = W_v h + b_v; all of q at once, and all of k at once, are divided by their root mean
                square and multiplied by a weight; then the heads are turned.  Position i sees positions i - M < j <= i; the softmax's
-               denominator has one more 1; head n's output is multiplied by sigmoid(W_g h)_n, W_o.  A layer may read the keys and
+               denominator has one more 1; o_n <- o_n sigmoid(W_g h)_n for head n, then W_o.  A layer may read the keys and
                values of an earlier layer instead of its own.
 
 Turning is in halves: (e_i, e_(i+r/2)) by p f_i with f_i = base^(-2i/r), and f scaled by its wavelength l = 2 pi / f: kept where

@@ -2,10 +2,9 @@
 // number per key channel and token, and whose current token is read through a bonus instead of the state.
 //
 //   time_mixing   with x' the previous token's x (zeros for a sequence's first), m_s = x + (x' - x) mu_s for s in r, k, v, g, w;
-//                 r, k, v = W_r m_r, W_k m_k, W_v m_v (heads of head_dim elements), a = exp(-exp(W_w2 tanh(W_w1 m_w) + w0)) per head and key
-//                 channel; o_t = S_(t-1)^T r_t + (sum_i u_i k_i r_i) v_t, then S_t = diag(a_t) S_(t-1) + k_t v_t^T.  Each head's output is
-//                 divided by its root mean square and multiplied by a weight over all heads' elements, the heads side by side by
-//                 silu(W_g m_g), and W_o projects back.
+//                 r, k, v = W_r m_r, W_k m_k, W_v m_v (heads of head_dim elements), a = exp(-exp(W_w2 tanh(W_w1 m_w) + w0)) for all of
+//                 their key channels; o_t = S_(t-1)^T r_t + (sum_i u_i k_i r_i) v_t, then S_t = diag(a_t) S_(t-1) + k_t v_t^T.  y = W_o (w_norm
+//                 * [rms_norm(o) of every head] * silu(W_g m_g)), w_norm over all heads' elements.
 //
 // The cache's state row holds the state, [heads][head_dim][head_dim] float32, and behind it the last token's x (zero when a slot is taken).  The
 // decay's second product, its exponentials, the recurrence and the heads' norm are float32 whatever the activation type; the other products are
